@@ -1,4 +1,5 @@
-"""Builds libqm_attn.so (HIP kernels + C ABI) for gfx950 with hipcc, in-tree.
+"""Builds the libraries for gfx950 with hipcc, in-tree: libqm_attn.so (HIP kernels + C ABI), libqm_engine.so (the engine
+shell over it) and libqm_decoder.so (the decoder language models: their kernels and their engine).
 
 Usage: python build.py            (from anywhere; also called by __graft_entry__.build())
 hipcc cross-compiles without a GPU.  The flags are part of the product: fp contraction is
@@ -14,6 +15,7 @@ CSRC = os.path.join(HERE, "csrc")
 LIB_DIR = os.path.join(HERE, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libqm_attn.so")
 ENGINE_LIB_PATH = os.path.join(LIB_DIR, "libqm_engine.so")
+DECODER_LIB_PATH = os.path.join(LIB_DIR, "libqm_decoder.so")
 
 SOURCES = ["qm_lib.hip", "qm_norm_rope.hip", "qm_decode.hip", "qm_prefill.hip", "qm_predictor.hip", "qm_predictor_layout.hip", "qm_predictor_mfma.hip", "qm_predictor_frame.hip", "qm_talker_chain.hip", "qm_linear.hip", "qm_rmsnorm.hip", "qm_sampler.hip", "qm_linear_rows.hip", "qm_linear_rows_mfma.hip"]
 
@@ -27,23 +29,57 @@ FLAGS = [
 
 def build(verbose=True, jobs=4):
     os.makedirs(LIB_DIR, exist_ok=True)
-    objs, procs = [], []
-    for src in SOURCES:
-        obj = os.path.join(LIB_DIR, src.replace(".hip", ".o"))
-        objs.append(obj)
-        cmd = ["hipcc", *FLAGS, "-c", os.path.join(CSRC, src), "-o", obj]
+    objs = _compile(SOURCES + DECODER_SOURCES, verbose, jobs)
+    _link(LIB_PATH, [objs[src] for src in SOURCES], verbose)
+    build_engine(verbose)
+    _link_decoder(objs, verbose)
+    return LIB_PATH
+
+
+# The decoder language models' library stands alone: its kernels, the kernels it shares with libqm_attn.so (their objects)
+# and its engine, so that a first run of such a model compiles no other model's kernels.
+DECODER_SOURCES = ["decoder/qm_decoder_ops.hip", "decoder/qm_decoder_norm.hip", "decoder/qm_decoder_linear.hip",
+                   "decoder/qm_decoder_attention.hip", "decoder/qm_decoder_recurrent.hip"]
+DECODER_SHARED = ["qm_lib.hip", "qm_sampler.hip", "qm_linear_rows_mfma.hip"]
+DECODER_ENGINE_SOURCES = ["engine/qm_safetensors.cpp", "engine/qm_decoder_config.cpp", "engine/qm_decoder.cpp"]
+
+
+def build_decoder(verbose=True, jobs=8):
+    """libqm_decoder.so and nothing else."""
+    os.makedirs(LIB_DIR, exist_ok=True)
+    _link_decoder(_compile(DECODER_SHARED + DECODER_SOURCES, verbose, jobs), verbose)
+    return DECODER_LIB_PATH
+
+
+def _compile(sources, verbose, jobs):
+    """{source: object}, compiled `jobs` at a time."""
+    objs, procs = {}, []
+    for src in sources:
+        objs[src] = os.path.join(LIB_DIR, os.path.basename(src).replace(".hip", ".o"))
+        cmd = ["hipcc", *FLAGS, "-c", os.path.join(CSRC, src), "-o", objs[src]]
         if verbose:
             print(" ".join(cmd), flush=True)
         procs.append((src, subprocess.Popen(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)))
         if len(procs) >= jobs:
             _drain(procs, verbose)
     _drain(procs, verbose)
-    link = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_PATH, *objs]
+    return objs
+
+
+def _link(path, objs, verbose, extra=()):
+    cmd = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", "-o", path, *objs, *extra]
     if verbose:
-        print(" ".join(link), flush=True)
-    subprocess.run(link, check=True)
-    build_engine(verbose)
-    return LIB_PATH
+        print(" ".join(cmd), flush=True)
+    subprocess.run(cmd, check=True)
+
+
+def _link_decoder(objs, verbose):
+    # (host-only C++, compiled on the link line; symbols stay the library's own where libqm_attn.so has the same)
+    part = DECODER_LIB_PATH + ".part"
+    _link(part, [objs[src] for src in DECODER_SHARED + DECODER_SOURCES], verbose,
+          ["-O2", "-std=c++17", "-Wall", "-Wextra", "-Wno-unused-parameter", "-Wl,-Bsymbolic",
+           *[os.path.join(CSRC, src) for src in DECODER_ENGINE_SOURCES]])
+    os.replace(part, DECODER_LIB_PATH)
 
 
 ENGINE_SOURCES = ["engine/qm_safetensors.cpp", "engine/qm_engine.cpp", "engine/qm_frame_engine.cpp"]

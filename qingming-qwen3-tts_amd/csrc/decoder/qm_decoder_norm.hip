@@ -1,0 +1,44 @@
+// qm_decoder_norm.hip — row operators around the decoder language models' mixers: the residual sum with the norm that
+// reads it, and the gated norm behind a recurrent mixer.  One block of 256 threads per row; a row is a few tens of KB, so
+// both are bound by memory latency for few rows and by bandwidth for a prompt.
+#include "qm_decoder_device.h"
+#include "../qm_host.h"
+
+namespace qm {
+
+template <class T>
+__global__ __launch_bounds__(kDecThreads) void residual_norm_kernel(ResidualParams prm) {
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    __shared__ float sh_red[16];
+    const int row = static_cast<int>(blockIdx.x);
+    residual_norm_row<T>(prm, row, reinterpret_cast<float*>(smem), sh_red, static_cast<T*>(prm.h) + row * prm.ld_h, true);
+}
+
+template <class T>
+__global__ __launch_bounds__(kDecThreads) void gated_norm_kernel(GatedNormParams prm) {
+    __shared__ float sh_red[4];
+    const int64_t row = blockIdx.x;
+    gated_norm_row<T>(prm, row, sh_red, static_cast<T*>(prm.out) + row * prm.ld_out);
+}
+
+int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream) {
+    if (rows < 0 || prm.width <= 0 || prm.ld_h < prm.width || prm.terms < 0 || prm.terms > 3) return QM_ERR_ARGUMENT;
+    if (!prm.h || !prm.norm_w || (!prm.x_in && (!prm.embed || !prm.tokens))) return QM_ERR_NULL;
+    if (prm.width > kDecMaxWidth) return QM_ERR_GEOMETRY;
+    if (rows == 0) return QM_OK;
+    const size_t lds = static_cast<size_t>(prm.width) * sizeof(float);
+    if (f32) hipLaunchKernelGGL(residual_norm_kernel<float>, dim3(rows), dim3(kDecThreads), lds, stream, prm);
+    else hipLaunchKernelGGL(residual_norm_kernel<uint16_t>, dim3(rows), dim3(kDecThreads), lds, stream, prm);
+    return launch_status();
+}
+
+int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStream_t stream) {
+    if (rows < 0 || prm.groups <= 0 || prm.size <= 0 || prm.ld_out < static_cast<int64_t>(prm.groups) * prm.size) return QM_ERR_ARGUMENT;
+    if (!prm.o || !prm.weight || !prm.gate || !prm.out) return QM_ERR_NULL;
+    if (rows == 0) return QM_OK;
+    if (f32) hipLaunchKernelGGL(gated_norm_kernel<float>, dim3(rows), dim3(kDecThreads), 0, stream, prm);
+    else hipLaunchKernelGGL(gated_norm_kernel<uint16_t>, dim3(rows), dim3(kDecThreads), 0, stream, prm);
+    return launch_status();
+}
+
+}  // namespace qm

@@ -1,0 +1,47 @@
+// qm_decoder_ops.h — launch parameters and launchers of the decoder language models' kernels, as the engine calls them.
+// Every launcher checks its arguments on the host, enqueues on `stream` and returns a QM_* code.  `f32` chooses the
+// activation type: 0 bf16, 1 fp32.
+#pragma once
+
+#include <hip/hip_runtime.h>
+
+#include "../../../include/qm_attn.h"
+#include "../../../include/qm_decoder.h"
+
+namespace qm {
+
+constexpr int kDecMaxWidth = 12288;       // columns of the residual stream (a row lives in LDS)
+constexpr int kDecMaxSplits = 64;         // key splits of one attention (a wave's lanes combine them)
+constexpr int kDecMaxHead = 256;          // channels of a head
+constexpr int kDecGroups = 3;             // linears in one launch
+constexpr int kDotLdsMost = 159 * 1024;   // dynamic LDS of one block
+
+// Linears of one launch.
+struct DecLinearParams {
+    qm_decoder_linear group[kDecGroups];
+    int groups, rows;
+};
+using ResidualParams = qm_residual_norm;
+using GatedNormParams = qm_gated_norm;
+using AttentionPartials = qm_attention_partials;
+using DecLinearGroup = qm_decoder_linear;
+using ChunkAttentionParams = qm_chunk_attention;
+using DecayAttentionParams = qm_decay_attention;
+using DeltaParams = qm_general_delta;
+constexpr int kDecayChunk = QM_DECAY_CHUNK;
+constexpr int kDecayPowers = QM_DECAY_POWERS;
+
+int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream);
+int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStream_t stream);
+// Many rows of bf16 go to the matrix cores (linears of one launch in one grid, a gate/up pair in its own), few rows and
+// fp32 to the streaming kernel.
+int32_t launch_decoder_linears(const DecLinearParams& prm, int f32, hipStream_t stream);
+// Rotation and cache write, then the attention.
+int32_t launch_chunk_attention(const ChunkAttentionParams& prm, int f32, hipStream_t stream);
+int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stream);
+// Floats of scratch with which a pass of `rows` tokens is computed in chunks (0: it is not).
+int64_t decay_scratch_floats(int rows, int heads, int dim, int vdim);
+int64_t delta_scratch_floats(int rows, int heads, int dim);
+int32_t launch_general_delta(const DeltaParams& prm, hipStream_t stream);
+
+}  // namespace qm

@@ -1,0 +1,175 @@
+// qm_decoder_recurrent.h — the two recurrences, token by token: a head's state [dim][columns] is cut along its columns
+// (value channels), which never interact.  A wave owns 16 columns; its four lane groups of 16 hold a quarter of the
+// state's rows each, in registers, so a sum over the rows is RD fmafs and two exchanges between lanes.  The vectors that
+// all columns share are put into LDS a few tokens at a time.
+#pragma once
+
+#include "qm_decoder_device.h"
+
+namespace qm {
+
+constexpr int kRecTokens = 8;                  // tokens whose vectors are in LDS at once
+constexpr int kRecColumns = 64;                // state columns of a block
+// a lane group's quarter of a vector starts 4 floats further on than the last one ended: the four quarters of one read lie
+// in different banks
+__host__ __device__ inline int rec_stride(int rd) { return 4 * (rd + 4); }
+template <int RD>
+__device__ __forceinline__ int rec_at(int channel) { return (channel / RD) * (RD + 4) + channel % RD; }
+
+template <int RD>
+__device__ __forceinline__ void load_state(float (&s)[RD], const float* state, int dim, int columns, int sub, int column) {
+#pragma unroll
+    for (int i = 0; i < RD; ++i) {
+        const int d = sub * RD + i;
+        s[i] = d < dim && column < columns ? state[static_cast<int64_t>(d) * columns + column] : 0.0f;
+    }
+}
+template <int RD>
+__device__ __forceinline__ void store_state(const float (&s)[RD], float* state, int dim, int columns, int sub, int column) {
+#pragma unroll
+    for (int i = 0; i < RD; ++i) {
+        const int d = sub * RD + i;
+        if (d < dim && column < columns) state[static_cast<int64_t>(d) * columns + column] = s[i];
+    }
+}
+__device__ __forceinline__ float quarter_sum(float v) {
+    v += __shfl_xor(v, 16, 64);
+    v += __shfl_xor(v, 32, 64);
+    return v;
+}
+
+__host__ __device__ inline int decay_lds_floats(int rd) { return kRecTokens * 2 * rec_stride(rd); }
+
+// Linear attention with decay: head `head`, state columns [64 slice, 64 slice + 64).
+template <int RD>
+__device__ __forceinline__ void decay_attention_block(const DecayAttentionParams& prm, int head, int slice, float* lds) {
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = lane >> 4;
+    const int column = slice * kRecColumns + wave * 16 + (lane & 15);
+    constexpr int kStride = 4 * (RD + 4);
+    float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.vdim;
+    const float decay = prm.powers[head * kDecayPowers + 1];
+    float s[RD];
+    load_state<RD>(s, state, prm.dim, prm.vdim, sub, column);
+    for (int t0 = 0; t0 < prm.rows; t0 += kRecTokens) {
+        const int tokens = min(kRecTokens, prm.rows - t0);
+        __syncthreads();
+        for (int i = tid; i < tokens * 4 * RD; i += kDecThreads) {
+            const int t = i / (4 * RD), c = i % (4 * RD);
+            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim + c;
+            float* to = lds + t * 2 * kStride + rec_at<RD>(c);
+            to[0] = c < prm.dim ? silu_f32(p[prm.q_column]) : 0.0f;
+            to[kStride] = c < prm.dim ? silu_f32(p[prm.k_column]) : 0.0f;
+        }
+        float v[kRecTokens];
+#pragma unroll
+        for (int t = 0; t < kRecTokens; ++t)
+            v[t] = t < tokens && column < prm.vdim ? silu_f32(prm.proj[(t0 + t) * prm.ld_proj + prm.v_column + head * prm.vdim + column]) : 0.0f;
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < kRecTokens; ++t) {
+            if (t >= tokens) break;
+            const float* q = lds + t * 2 * kStride + sub * (RD + 4);
+            const float* k = q + kStride;
+            float o = 0.0f;
+#pragma unroll
+            for (int i = 0; i < RD; i += 4) {
+                const float4 kk = *reinterpret_cast<const float4*>(k + i), qq = *reinterpret_cast<const float4*>(q + i);
+                s[i] = fmaf(kk.x, v[t], decay * s[i]); o = fmaf(qq.x, s[i], o);
+                s[i + 1] = fmaf(kk.y, v[t], decay * s[i + 1]); o = fmaf(qq.y, s[i + 1], o);
+                s[i + 2] = fmaf(kk.z, v[t], decay * s[i + 2]); o = fmaf(qq.z, s[i + 2], o);
+                s[i + 3] = fmaf(kk.w, v[t], decay * s[i + 3]); o = fmaf(qq.w, s[i + 3], o);
+            }
+            o = quarter_sum(o);
+            if (sub == 0 && column < prm.vdim) prm.out[static_cast<int64_t>(t0 + t) * prm.heads * prm.vdim + head * prm.vdim + column] = o;
+        }
+    }
+    store_state<RD>(s, state, prm.dim, prm.vdim, sub, column);
+}
+
+__host__ __device__ inline int delta_lds_floats(int rd, int rank) { return kRecTokens * (5 * rec_stride(rd) + rank); }
+
+// What enters the delta rule's recurrence for channel c of a head at one token, given tanh of the token's rank-sized
+// projection in LDS: the decay of the channel and the removal rate.
+__device__ __forceinline__ float delta_channel_decay(const DeltaParams& prm, const float* tanh_z, int at) {
+    float z = prm.w0[at];
+    const int all = prm.heads * prm.dim;
+    for (int r = 0; r < prm.rank; ++r) z = fmaf(prm.w2[static_cast<int64_t>(r) * all + at], tanh_z[r], z);
+    return expf(-0.60653065971263342f * sigmoid_f32(z));          // exp(-1/2) = 0.6065...
+}
+
+// Generalized delta rule: head `head`, state columns [64 slice, 64 slice + 64).
+template <int RD>
+__device__ __forceinline__ void general_delta_block(const DeltaParams& prm, int head, int slice, float* lds) {
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = lane >> 4;
+    const int column = slice * kRecColumns + wave * 16 + (lane & 15);
+    constexpr int kStride = 4 * (RD + 4);
+    float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.dim;
+    float* tanh_z = lds + kRecTokens * 5 * kStride;
+    float s[RD];
+    load_state<RD>(s, state, prm.dim, prm.dim, sub, column);
+    for (int t0 = 0; t0 < prm.rows; t0 += kRecTokens) {
+        const int tokens = min(kRecTokens, prm.rows - t0);
+        __syncthreads();
+        for (int i = tid; i < tokens * prm.rank; i += kDecThreads) {
+            const int t = i / prm.rank, r = i - t * prm.rank;
+            tanh_z[i] = tanhf(prm.proj[(t0 + t) * prm.ld_proj + prm.z_column + r]);
+        }
+        __syncthreads();
+        for (int t = wave; t < tokens; t += 4) {                   // a wave per token: w, a u, u, k, r of the head
+            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim;
+            float* to = lds + t * 5 * kStride;
+            float sq = 0.0f;
+            for (int c = lane; c < prm.dim; c += 64) {
+                const float k = p[prm.k_column + c];
+                sq = fmaf(k, k, sq);
+            }
+            const float inverse = 1.0f / sqrtf(wave_sum(sq) + prm.unit_eps);
+            for (int c = lane; c < 4 * RD; c += 64) {
+                float w = 0.0f, au = 0.0f, u = 0.0f, k = 0.0f, r = 0.0f;
+                if (c < prm.dim) {
+                    const int at = head * prm.dim + c;
+                    w = delta_channel_decay(prm, tanh_z + t * prm.rank, at);
+                    k = p[prm.k_column + c];
+                    r = p[prm.r_column + c];
+                    u = k * inverse;
+                    au = sigmoid_f32(p[prm.a_column + c] + prm.a_bias[at]) * u;
+                }
+                float* put = to + rec_at<RD>(c);
+                put[0] = w; put[kStride] = au; put[2 * kStride] = u; put[3 * kStride] = k; put[4 * kStride] = r;
+            }
+        }
+        float v[kRecTokens];
+#pragma unroll
+        for (int t = 0; t < kRecTokens; ++t)
+            v[t] = t < tokens && column < prm.dim ? prm.proj[(t0 + t) * prm.ld_proj + prm.v_column + head * prm.dim + column] : 0.0f;
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < kRecTokens; ++t) {
+            if (t >= tokens) break;
+            const float* w = lds + t * 5 * kStride + sub * (RD + 4);
+            float seen = 0.0f;
+#pragma unroll
+            for (int i = 0; i < RD; i += 4) {
+                const float4 u = *reinterpret_cast<const float4*>(w + 2 * kStride + i);
+                seen = fmaf(u.x, s[i], seen); seen = fmaf(u.y, s[i + 1], seen);
+                seen = fmaf(u.z, s[i + 2], seen); seen = fmaf(u.w, s[i + 3], seen);
+            }
+            seen = quarter_sum(seen);
+            float o = 0.0f;
+#pragma unroll
+            for (int i = 0; i < RD; i += 4) {
+                const float4 ww = *reinterpret_cast<const float4*>(w + i), au = *reinterpret_cast<const float4*>(w + kStride + i);
+                const float4 k = *reinterpret_cast<const float4*>(w + 3 * kStride + i), r = *reinterpret_cast<const float4*>(w + 4 * kStride + i);
+                s[i] = fmaf(k.x, v[t], fmaf(-au.x, seen, ww.x * s[i])); o = fmaf(r.x, s[i], o);
+                s[i + 1] = fmaf(k.y, v[t], fmaf(-au.y, seen, ww.y * s[i + 1])); o = fmaf(r.y, s[i + 1], o);
+                s[i + 2] = fmaf(k.z, v[t], fmaf(-au.z, seen, ww.z * s[i + 2])); o = fmaf(r.z, s[i + 2], o);
+                s[i + 3] = fmaf(k.w, v[t], fmaf(-au.w, seen, ww.w * s[i + 3])); o = fmaf(r.w, s[i + 3], o);
+            }
+            o = quarter_sum(o);
+            if (sub == 0 && column < prm.dim) prm.out[static_cast<int64_t>(t0 + t) * prm.heads * prm.dim + head * prm.dim + column] = o;
+        }
+    }
+    store_state<RD>(s, state, prm.dim, prm.dim, sub, column);
+}
+
+}  // namespace qm

@@ -51,6 +51,8 @@ private:
 class ModelDirectory {
 public:
     explicit ModelDirectory(const std::string& directory);
+    // The tensor of exactly this name; nullptr if there is none.
+    const TensorView* find(const std::string& name) const;
     // The one tensor whose name ends in `suffix`; nullptr if none; TensorError if several.
     const TensorView* maybe_suffix(const std::string& suffix) const;
     const TensorView& suffix(const std::string& suffix) const;

@@ -159,13 +159,15 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int wave_n = BM == 128 ? (wave & 1) : wave;
     const int wave_m = BM == 128 ? (wave >> 1) : 0;
-    const int K = prm.reduction;
+    int K = prm.reduction;
     const int m0 = static_cast<int>(blockIdx.y) * BM;
     // (several linears of one input in one grid: which of them this block's column tile belongs to)
     int tile = static_cast<int>(blockIdx.x);
     const uint16_t* weight0 = prm.weight[0];
+    const uint16_t* input = prm.input;
     const uint16_t* bias = prm.bias;
     uint16_t* output = prm.output;
+    float* sums = prm.sums;
     int columns = prm.columns;
     if (!DUAL && prm.groups > 1) {
         const int g = (tile >= prm.group_first_tile[0]) + (prm.groups > 2 && tile >= prm.group_first_tile[1]);
@@ -174,7 +176,10 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
             weight0 = prm.group_weight[g - 1];
             bias = prm.group_bias[g - 1];
             output = prm.group_output[g - 1];
+            sums = prm.group_sums[g - 1];
             columns = prm.group_columns[g - 1];
+            if (prm.group_input[g - 1]) input = prm.group_input[g - 1];
+            if (prm.group_reduction[g - 1]) K = prm.group_reduction[g - 1];
         }
     }
     const int n0 = tile * BN;
@@ -188,7 +193,7 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
     const uint32_t row_bytes = static_cast<uint32_t>(K) * 2u;
     const int x_rows = min(prm.rows - m0, BM);
     const __amdgpu_buffer_rsrc_t x_rsrc = __builtin_amdgcn_make_buffer_rsrc(
-        const_cast<uint16_t*>(prm.input + static_cast<int64_t>(m0) * K), 0, static_cast<int>(x_rows * row_bytes), 0x00020000);
+        const_cast<uint16_t*>(input + static_cast<int64_t>(m0) * K), 0, static_cast<int>(x_rows * row_bytes), 0x00020000);
     const __amdgpu_buffer_rsrc_t w_rsrc = __builtin_amdgcn_make_buffer_rsrc(
         const_cast<uint16_t*>(weight0 + static_cast<int64_t>(n0) * K), 0, static_cast<int>(BN * row_bytes), 0x00020000);
     const __amdgpu_buffer_rsrc_t u_rsrc = __builtin_amdgcn_make_buffer_rsrc(
@@ -432,6 +437,23 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
                     if (DUAL)
                         *reinterpret_cast<float4*>(at + plane) =
                             make_float4(acc_up[a][b][4 * g], acc_up[a][b][4 * g + 1], acc_up[a][b][4 * g + 2], acc_up[a][b][4 * g + 3]);
+                }
+            }
+        }
+        return;
+    }
+    if (!DUAL && sums) {
+#pragma unroll
+        for (int a = 0; a < kTn; ++a) {
+#pragma unroll
+            for (int b = 0; b < kTm; ++b) {
+                const int m = m0 + 32 * (kTm * wave_m + b) + (lane & 31);
+                if (m >= prm.rows) continue;
+#pragma unroll
+                for (int g = 0; g < 4; ++g) {
+                    const int n = n0 + 32 * (kTn * wave_n + a) + 8 * g + 4 * (lane >> 5);
+                    *reinterpret_cast<float4*>(sums + static_cast<int64_t>(m) * columns + n) =
+                        make_float4(acc[a][b][4 * g], acc[a][b][4 * g + 1], acc[a][b][4 * g + 2], acc[a][b][4 * g + 3]);
                 }
             }
         }

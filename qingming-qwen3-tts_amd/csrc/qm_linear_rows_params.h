@@ -28,6 +28,13 @@ struct LinearRowsParams {
     const uint16_t* group_bias[2];
     uint16_t* group_output[2];
     int group_columns[2];
+    // (matrix cores, no gate/up pair, reduction uncut) sums != NULL: the fp32 sums as they are go to sums /
+    // group_sums[g - 1] ([rows][columns] floats) and nothing to the outputs; bias and residual are not read.
+    float* sums;
+    float* group_sums[2];
+    // a linear of its own input and reduction (a multiple of 128 as well): NULL / 0 = the first one's
+    const uint16_t* group_input[2];
+    int group_reduction[2];
 };
 
 // The row linears on the matrix cores (qm_linear_rows_mfma.hip).  `dual`: weight[0] / weight[1] are the gate and up
