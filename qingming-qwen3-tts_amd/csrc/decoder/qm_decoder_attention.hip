@@ -58,7 +58,7 @@ __global__ __launch_bounds__(kDecThreads) void merge_attention_kernel(ChunkAtten
                            static_cast<T*>(prm.out) + row * prm.ld_out, prm.ld_out);
 }
 
-static int32_t check_attention(const ChunkAttentionParams& p) {
+int32_t check_attention(const ChunkAttentionParams& p) {
     if (p.rows < 0 || p.position < 0) return QM_ERR_ARGUMENT;
     if (!p.proj || !p.k_cache || !p.v_cache || !p.out || !p.part.ml || !p.part.acc || (p.rot_dims > 0 && !p.frequency)) return QM_ERR_NULL;
     if (p.heads <= 0 || p.kv_heads <= 0 || p.heads % p.kv_heads || p.dim <= 0 || p.vdim <= 0 || p.dim > kDecMaxHead || p.vdim > kDecMaxHead)

@@ -2,7 +2,7 @@
 // prompt) and for the 32-bit mode: weight-streaming dot products; many bf16 rows are handed to the matrix-core kernel.
 //
 // Bound by HBM: every weight is read once per group of R rows.  A wave owns NR weight rows and streams them 16 bytes a
-// lane, `kAhead` pieces of each row requested before the first is used; the input rows live in LDS as T.  Sums are fp32
+// lane, `kDotAhead` pieces of each row requested before the first is used; the input rows live in LDS as T.  Sums are fp32
 // (packed bf16 dot products, or fmaf in the 32-bit mode), combined over the wave's lanes at the end.
 #include "qm_decoder_device.h"
 #include "../qm_host.h"
@@ -11,18 +11,21 @@
 
 namespace qm {
 
+constexpr int kLinearRows = 4;                 // weight rows a wave streams at once
+
 template <class T, int R>
 __global__ __launch_bounds__(kDecThreads) void decoder_linear_kernel(DecLinearParams prm) {
     request_arguments(prm);
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     T* xs = reinterpret_cast<T*>(smem);
     int tile = static_cast<int>(blockIdx.x);
-    int g = 0;
-    while (g + 1 < prm.groups && tile >= dot_tiles(prm.group[g])) tile -= dot_tiles(prm.group[g++]);
-    const DecLinearGroup& group = prm.group[g];
+    const DecLinearGroup& group = prm.group[dot_group<kLinearRows>(prm, tile)];
     const int row0 = static_cast<int>(blockIdx.y) * R;
     const int rows = min(R, prm.rows - row0);
     const int k = group.k;
+    const DotRows<kLinearRows> d = dot_rows<kLinearRows>(group, tile);
+    uint4 piece[kDotAhead][kLinearRows];
+    dot_request<kLinearRows>(d, k, piece);
     constexpr int kVec = 16 / sizeof(T);
     for (int r = 0; r < R; ++r) {
         const int src = row0 + min(r, rows - 1);               // (a row past the end repeats the last one, never stored)
@@ -31,16 +34,14 @@ __global__ __launch_bounds__(kDecThreads) void decoder_linear_kernel(DecLinearPa
             *reinterpret_cast<uint4*>(xs + r * k + c) = *reinterpret_cast<const uint4*>(x + c);
     }
     __syncthreads();
-    dot_tile<T, R>(group, xs, tile, row0, rows);
+    dot_finish<T, R, kLinearRows>(group, d, piece, xs, row0, rows);
 }
 
 template <class T, int R>
 static int32_t launch_streaming(const DecLinearParams& prm, hipStream_t stream) {
-    int tiles = 0, k = 0;
-    for (int g = 0; g < prm.groups; ++g) {
-        tiles += dot_tiles(prm.group[g]);
-        k = prm.group[g].k > k ? prm.group[g].k : k;
-    }
+    int k = 0;
+    for (int g = 0; g < prm.groups; ++g) k = prm.group[g].k > k ? prm.group[g].k : k;
+    const int tiles = dot_tiles_of<kLinearRows>(prm);
     static std::atomic<bool> raised[kMaxDevices];
     const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(decoder_linear_kernel<T, R>), kDotLdsMost, raised);
     if (rc != QM_OK) return rc;

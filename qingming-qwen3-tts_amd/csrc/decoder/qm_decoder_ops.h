@@ -31,6 +31,9 @@ using DeltaParams = qm_general_delta;
 constexpr int kDecayChunk = QM_DECAY_CHUNK;
 constexpr int kDecayPowers = QM_DECAY_POWERS;
 
+// Whether the kernels take these arguments.
+int32_t check_attention(const ChunkAttentionParams& prm);
+int32_t check_decay_attention(const DecayAttentionParams& prm);
 int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream);
 int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStream_t stream);
 // Many rows of bf16 go to the matrix cores (linears of one launch in one grid, a gate/up pair in its own), few rows and
@@ -43,5 +46,30 @@ int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stre
 int64_t decay_scratch_floats(int rows, int heads, int dim, int vdim);
 int64_t delta_scratch_floats(int rows, int heads, int dim);
 int32_t launch_general_delta(const DeltaParams& prm, hipStream_t stream);
+
+// ---- one token: a layer run in three launches -----------------------------------------------------------------------
+// Residual sum and norm by every block for itself, then the linears that read it (row 0 of everything).
+struct LayerInParams {
+    ResidualParams residual;
+    DecLinearParams linears;
+};
+// The output linears, each block preparing the input of its own: 0 as it is in memory, 1 the attention's key splits
+// combined, 2 the gated norm.
+struct LayerOutParams {
+    DecLinearParams linears;
+    int input[kDecGroups];
+    int chunk;                       // of the attention (input 1)
+    AttentionPartials part;
+    const int32_t* position_dev;
+    GatedNormParams gated;           // (input 2)
+};
+int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream);
+// The attention (rotation and cache write included) beside the decayed linear attention, one token each.
+int32_t launch_mixer_step(const ChunkAttentionParams& attention, const DecayAttentionParams& decay, int f32, hipStream_t stream);
+int32_t launch_layer_out(const LayerOutParams& prm, int f32, hipStream_t stream);
+// step = {position, token, emitted}: the token of the highest of `vocab` scores (lowest id among equals) into step[1]
+int32_t launch_argmax(const float* scores, int vocab, int32_t* step, hipStream_t stream);
+// out[step[2]++] = step[1], and the position moves on by `advance`
+int32_t launch_emit(int32_t* step, int32_t* out, int advance, hipStream_t stream);
 
 }  // namespace qm

@@ -24,11 +24,16 @@ static int32_t decay_as(const DecayAttentionParams& prm, hipStream_t stream) {
     return launch_status();
 }
 
-int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stream) {
+int32_t check_decay_attention(const DecayAttentionParams& prm) {
     if (!prm.proj || !prm.powers || !prm.state || !prm.out) return QM_ERR_NULL;
     if (prm.rows < 0) return QM_ERR_ARGUMENT;
     if (prm.heads <= 0 || prm.heads > 65535 || prm.dim <= 0 || prm.vdim <= 0 || prm.dim > kDecMaxHead || prm.vdim > kDecMaxHead) return QM_ERR_GEOMETRY;
-    if (prm.rows == 0) return QM_OK;
+    return QM_OK;
+}
+
+int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stream) {
+    const int32_t rc = check_decay_attention(prm);
+    if (rc != QM_OK || prm.rows == 0) return rc;
     if (prm.dim <= 32) return decay_as<8>(prm, stream);
     if (prm.dim <= 64) return decay_as<16>(prm, stream);
     if (prm.dim <= 128) return decay_as<32>(prm, stream);

@@ -38,7 +38,7 @@ namespace {
 
 constexpr float kUnitEps = 1.0e-6f;       // inside the root of the delta rule's unit key
 constexpr int kLogitRows = 256;           // rows of the head at once
-constexpr int kStepWords = 4;             // device words of a one-token step: position, token
+constexpr int kStepWords = 4;             // device words of a one-token step: position, token, tokens emitted
 
 int padded(int n, int to) { return (n + to - 1) / to * to; }
 
@@ -89,6 +89,7 @@ struct qm_decoder {
     qm_engine::DeviceBuffer embed, final_norm, loop_step;
     qm_engine::Matrix head;
     int capacity = 0, max_rows = 0, f32 = 0, path = 0;
+    bool warm = false;
     int width_p = 0, vocab_p = 0;
     hipStream_t stream = nullptr;
     bool own_stream = false;
@@ -552,6 +553,105 @@ void run_head(qm_decoder& d, const float* x, const Pending& pending, const int32
     }
 }
 
+// ---- one token -----------------------------------------------------------------------------------------------------------
+
+int32_t* step_words(const qm_decoder& d) { return static_cast<int32_t*>(d.step_words.raw()); }
+
+// The token and position that the step words name, through every layer run and the head: logits in row 0 of d.logits.
+void enqueue_one(qm_decoder& d, int sequence) {
+    hipStream_t s = d.stream;
+    const float* x = nullptr;
+    int next = 0;
+    Pending pending;
+    auto residual = [&](float* x_new, const float* step_vec, const float* norm) {
+        qm_residual_norm p = residual_of(d, pending, x, x_new, step_vec, norm, nullptr);
+        p.tokens = step_words(d) + 1;
+        return p;
+    };
+    for (size_t i = 0; i < d.runs.size(); ++i) {
+        const LayerRun& run = d.runs[i];
+        const DecoderLayer& w = d.layers[static_cast<size_t>(run.layer)];
+        float* x_new = f32_of(d.x[next]);
+        qm::LayerInParams in = {};
+        in.residual = residual(x_new, step_vec_of(d, run), f32_of(w.norm1));
+        in.linears = linears_in(d, w, 1);
+        op_check(qm::launch_layer_in(in, d.f32, s), "residual + norm + input projections");
+        x = x_new;
+        next ^= 1;
+        qm::LayerOutParams out = {};
+        out.linears = linears_out(d, w, 1, pending);
+        out.gated = gated_of(d, w);
+        out.position_dev = step_words(d);
+        if (w.config.mixer == MixerKind::AttentionBesideDecay) {
+            qm_chunk_attention a = attention_of(d, w, d.states[i], sequence, 1, 0);
+            a.position_dev = step_words(d);
+            op_check(qm::launch_mixer_step(a, decay_of(d, w, d.states[i], sequence, 1), d.f32, s), "attention beside decayed attention");
+            out.part = a.part;
+            out.chunk = a.chunk;
+            out.input[0] = 1;
+            out.input[1] = 2;
+        } else {
+            op_check(qm::launch_general_delta(delta_of(d, w, d.states[i], sequence, 1), s), "generalized delta rule");
+            out.input[0] = 2;
+        }
+        op_check(qm::launch_layer_out(out, d.f32, s), "output projections");
+    }
+    qm::LayerInParams head = {};
+    head.residual = residual(nullptr, nullptr, f32_of(d.final_norm));
+    head.linears.rows = 1;
+    head.linears.group[head.linears.groups++] = linear_of(d.head, nullptr, f32_of(d.logits));
+    op_check(qm::launch_layer_in(head, d.f32, s), "final norm + head");
+}
+
+// The same by the operators of the prompt pass.
+void enqueue_one_by_operators(qm_decoder& d, int sequence, int position) {
+    hip_check(hipMemcpyAsync(d.tokens.raw(), step_words(d) + 1, 4, hipMemcpyDeviceToDevice, d.stream), "token");
+    const float* x = nullptr;
+    Pending pending;
+    run_layers(d, sequence, 1, position, &x, pending, nullptr);
+    op_check(qm::launch_residual_norm(residual_of(d, pending, x, nullptr, nullptr, f32_of(d.final_norm), d.head_h.raw()), 1, d.f32, d.stream), "final norm");
+    qm::DecLinearParams l = {};
+    l.rows = 1;
+    l.group[l.groups++] = linear_of(d.head, d.head_h.raw(), f32_of(d.logits));
+    op_check(qm::launch_decoder_linears(l, d.f32, d.stream), "head");
+}
+
+// One token of the sequence, whose words are in place; logits in row 0 of d.logits.
+void run_one(qm_decoder& d, int sequence) {
+    int& length = d.length[static_cast<size_t>(sequence)];
+    if (length >= d.capacity) throw ApiError(QM_ERR_SLOT_RANGE, "the sequence exceeds its capacity");
+    hipGraphExec_t& graph = d.graphs[static_cast<size_t>(sequence)];
+    if ((d.path & 3) == 2) {
+        enqueue_one_by_operators(d, sequence, length);
+    } else if ((d.path & 3) == 1 || !d.warm) {
+        enqueue_one(d, sequence);          // (the first of all sets the kernels' attributes, outside of any capture)
+        d.warm = true;
+    } else {
+        if (!graph) {
+            hipGraph_t captured = nullptr;
+            hip_check(hipStreamBeginCapture(d.stream, hipStreamCaptureModeThreadLocal), "step capture");
+            try {
+                enqueue_one(d, sequence);
+            } catch (...) {
+                (void)hipStreamEndCapture(d.stream, &captured);
+                if (captured) (void)hipGraphDestroy(captured);
+                throw;
+            }
+            hip_check(hipStreamEndCapture(d.stream, &captured), "step capture");
+            const hipError_t e = hipGraphInstantiate(&graph, captured, nullptr, nullptr, 0);
+            (void)hipGraphDestroy(captured);
+            hip_check(e, "step graph");
+        }
+        hip_check(hipGraphLaunch(graph, d.stream), "step graph launch");
+    }
+    ++length;
+}
+
+void put_step_words(qm_decoder& d, int position, int token) {
+    const int32_t words[3] = {position, token, 0};
+    hip_check(hipMemcpyAsync(d.step_words.raw(), words, sizeof words, hipMemcpyHostToDevice, d.stream), "step words");
+}
+
 void check_tokens(const qm_decoder& d, const int32_t* tokens, int count) {
     if (!tokens) throw ApiError(QM_ERR_NULL, "no tokens");
     for (int i = 0; i < count; ++i)
@@ -564,7 +664,8 @@ int& length_of(qm_decoder& d, int sequence) {
     return d.length[static_cast<size_t>(sequence)];
 }
 
-void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const int32_t* want, int wanted, float* logits, float* streams) {
+void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const int32_t* want, int wanted, float* logits, float* streams,
+          bool read_back = true) {
     int& length = length_of(d, sequence);
     if (count <= 0) throw ApiError(QM_ERR_ARGUMENT, "a step has at least one token");
     check_tokens(d, tokens, count);
@@ -576,6 +677,15 @@ void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const i
     if (streams && !d.tap.raw()) {
         d.tap = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.config.width * 4);
         d.tap_h = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.width_p * 4);
+    }
+    if (count == 1 && !streams) {
+        put_step_words(d, length, tokens[0]);
+        run_one(d, sequence);
+        for (int i = 0; i < wanted; ++i)
+            hip_check(hipMemcpyAsync(logits + static_cast<size_t>(i) * d.config.vocab, d.logits.raw(), static_cast<size_t>(d.config.vocab) * 4,
+                                     hipMemcpyDeviceToHost, d.stream), "logits read");
+        if (read_back) hip_check(hipStreamSynchronize(d.stream), "step");
+        return;
     }
     for (int first = 0; first < count; first += d.max_rows) {
         const int rows = std::min(d.max_rows, count - first);
@@ -599,7 +709,47 @@ void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const i
                             static_cast<size_t>(d.config.vocab) * 4);
         }
     }
-    hip_check(hipStreamSynchronize(d.stream), "step");
+    if (read_back) hip_check(hipStreamSynchronize(d.stream), "step");
+}
+
+// The prompt, then token by token: the head's scores, the token they give into the step words, the step that reads it.
+int generate(qm_decoder& d, int sequence, const int32_t* prompt, int count, int maximum, int stop_token, int top_k, float temperature, uint64_t seed,
+             int32_t* out) {
+    int& length = length_of(d, sequence);
+    if (maximum <= 0 || !out) throw ApiError(QM_ERR_ARGUMENT, "no room for the tokens");
+    if (count <= 0) throw ApiError(QM_ERR_ARGUMENT, "a prompt has at least one token");
+    if (top_k > 0 && (d.config.vocab > 4096 || top_k > 256 || !(temperature > 0.0f)))
+        throw ApiError(QM_ERR_GEOMETRY, "the sampler takes a vocabulary of at most 4096, top_k <= 256 and a positive temperature");
+    // (the last token emitted is not fed back)
+    if (static_cast<int64_t>(length) + count + maximum - 1 > d.capacity) throw ApiError(QM_ERR_SLOT_RANGE, "prompt and tokens exceed the capacity");
+    std::vector<float> last(static_cast<size_t>(d.config.vocab));
+    const int32_t want = count - 1;
+    step(d, sequence, prompt, count, &want, 1, last.data(), nullptr);    // leaves the scores in row 0 of d.logits
+    DeviceBuffer emitted(static_cast<size_t>(maximum) * 4), generator(8);
+    hip_check(hipMemcpyAsync(generator.raw(), &seed, 8, hipMemcpyHostToDevice, d.stream), "generator state");
+    put_step_words(d, length, 0);
+    StreamDrain drain(d.stream);          // (the two buffers outlive what reads them, also on an error)
+    int produced = 0;
+    for (;;) {
+        if (top_k > 0)
+            op_check(qm_sample_topk(d.logits.raw(), 0, 0, d.config.vocab, top_k, temperature, static_cast<uint64_t*>(generator.raw()),
+                                    step_words(d) + 1, d.stream), "sampler");
+        else
+            op_check(qm::launch_argmax(f32_of(d.logits), d.config.vocab, step_words(d), d.stream), "arg-max");
+        op_check(qm::launch_emit(step_words(d), static_cast<int32_t*>(emitted.raw()), produced > 0, d.stream), "emit");
+        ++produced;
+        if (stop_token >= 0) {
+            int32_t token = 0;
+            hip_check(hipMemcpyAsync(&token, step_words(d) + 1, 4, hipMemcpyDeviceToHost, d.stream), "token read");
+            hip_check(hipStreamSynchronize(d.stream), "token read");
+            if (token == stop_token) break;
+        }
+        if (produced == maximum) break;
+        run_one(d, sequence);
+    }
+    hip_check(hipMemcpyAsync(out, emitted.raw(), static_cast<size_t>(produced) * 4, hipMemcpyDeviceToHost, d.stream), "tokens read");
+    hip_check(hipStreamSynchronize(d.stream), "tokens read");
+    return produced;
 }
 
 }  // namespace
@@ -676,9 +826,12 @@ extern "C" int32_t qm_decoder_set_path(qm_decoder* d, int32_t path) {
 
 extern "C" int32_t qm_decoder_enqueue(qm_decoder* d, int32_t sequence, const int32_t* tokens, int32_t count) {
     if (!d) return QM_ERR_NULL;
-    return guarded([&] { step(*d, sequence, tokens, count, nullptr, 0, nullptr, nullptr); });
+    return guarded([&] { step(*d, sequence, tokens, count, nullptr, 0, nullptr, nullptr, false); });
 }
+
 extern "C" int32_t qm_decoder_generate(qm_decoder* d, int32_t sequence, const int32_t* prompt, int32_t count, int32_t maximum, int32_t stop_token,
                                        int32_t top_k, float temperature, uint64_t seed, int32_t* tokens_out, int32_t* produced) {
-    return QM_ERR_ARGUMENT;
+    if (!d || !produced) return QM_ERR_NULL;
+    *produced = 0;
+    return guarded([&] { *produced = generate(*d, sequence, prompt, count, maximum, stop_token, top_k, temperature, seed, tokens_out); });
 }
