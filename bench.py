@@ -1061,6 +1061,185 @@ class PredictorLoop:
         return {"all": dt * self.units / n}, err, "first %d of %d units, time scaled" % (n, self.units), ok
 
 
+DECODER_SIZES = {
+    # name: width, (query heads, kv heads, dim, value dim), chunk, (decay heads, dim, value dim), (delta heads, dim), ff
+    "w1024": dict(width=1024, left=(16, 8, 64, 64), chunk=512, right=(8, 64, 128), delta=(16, 64), ff=3072),
+    "w2048": dict(width=2048, left=(16, 8, 128, 128), chunk=1024, right=(16, 64, 128), delta=(16, 128), ff=6144),
+    "w4096": dict(width=4096, left=(32, 8, 128, 128), chunk=2048, right=(32, 64, 128), delta=(32, 128), ff=12288),
+}
+
+
+def write_decoder_model(directory, width, left, chunk, right, delta, ff, vocab=4096, types=("parallel", "parallel", "parallel", "general_delta"),
+                        seed=1, dev="cpu"):
+    """A Vabevik model directory of random weights (normal, 1/sqrt(inputs)): config.json and model.safetensors."""
+    import torch
+    from safetensors.torch import save_file
+    gen = torch.Generator(device=dev).manual_seed(seed)
+    tensors = {}
+
+    def linear(name, n, k):
+        tensors[name] = (torch.randn(n, k, generator=gen, device=dev) * k ** -0.5).to(torch.bfloat16).cpu()
+
+    def norm(name, n):
+        tensors[name] = (1 + 0.1 * torch.randn(n, generator=gen, device=dev)).to(torch.bfloat16).cpu()
+
+    linear("embed", vocab, width)
+    linear("head", vocab, width)
+    norm("final.norm", width)
+    layers = []
+    for i, kind in enumerate(types):
+        base = f"l{i}."
+        norm(base + "norm1", width)
+        if kind == "parallel":
+            h, g, d, e = left
+            rh, rd, re = right
+            for name, n in (("left.q", h * d), ("left.k", g * d), ("left.v", g * e), ("right.q", rh * rd), ("right.k", rh * rd),
+                            ("right.v", rh * re), ("right.g", rh * re)):
+                linear(base + "mix." + name, n, width)
+            linear(base + "mix.left.o", width, h * e)
+            linear(base + "mix.right.o", width, rh * re)
+            norm(base + "mix.right.norm", rh * re)
+            norm(base + "mix.left.out", width)
+            norm(base + "mix.right.out", width)
+            mixer = {"left": {"heads": h, "kv_heads": g, "dim": d, "vdim": e, "mask": {"size": chunk}, "rot": {"base": 1e6, "dims": d},
+                              "scale": d ** -0.5},
+                     "right": {"heads": rh, "dim": rd, "vdim": re, "decay": [1.0 - 2.0 ** -(1 + 8 * (j + 1) / rh) for j in range(rh)]}}
+        else:
+            dh, dd = delta
+            for name in ("r", "k", "v", "a", "g"):
+                linear(base + "mix." + name, dh * dd, width)
+            linear(base + "mix.w1", 64, width)
+            linear(base + "mix.w2", dh * dd, 64)
+            linear(base + "mix.o", width, dh * dd)
+            for name in ("a.b", "w0"):
+                tensors[base + "mix." + name] = torch.randn(dh * dd, generator=gen, device=dev).to(torch.bfloat16).cpu()
+            norm(base + "mix.norm", dh * dd)
+            mixer = {"heads": dh, "dim": dd}
+        linear(base + "mlp.gate", ff, width)
+        linear(base + "mlp.up", ff, width)
+        linear(base + "mlp.down", width, ff)
+        layers.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    config = {"architecture": "Vabevik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": layers}
+    with open(os.path.join(directory, "config.json"), "w") as f:
+        json.dump(config, f)
+    save_file(tensors, os.path.join(directory, "model.safetensors"))
+    return sum(t.numel() * 2 for name, t in tensors.items() if name not in ("embed", "head"))
+
+
+def decoder_throughput(size, dev, rows=1024, steps=64, kinds=None):
+    """Prefill of `rows` tokens and decoding behind them for a decoder language model of one of DECODER_SIZES; microseconds are
+    per layer run (head included in the total it is divided from)."""
+    import tempfile
+    module = importlib.import_module("qingming-qwen3-tts_amd.decoder")
+    out = {}
+    for name, types in (("mixed", ("parallel", "parallel", "parallel", "general_delta")), ("parallel", ("parallel",) * 4),
+                        ("general_delta", ("general_delta",) * 4)):
+        if kinds and name not in kinds:
+            continue
+        with tempfile.TemporaryDirectory() as directory:
+            weight_bytes = write_decoder_model(directory, types=types, dev=dev, **DECODER_SIZES[size])
+            model = module.Decoder(directory, capacity=rows + 2 * steps + 8, max_rows=rows)
+        tokens = np.arange(rows, dtype=np.int32) * 7 % model.vocab
+
+        def prefill():
+            sequence = model.open()
+            model.enqueue(sequence, tokens)
+            return sequence
+
+        for _ in range(3):
+            model.close(prefill())
+        model.synchronize()
+        started, repeats = time.perf_counter(), 10
+        for _ in range(repeats):
+            model.close(prefill())
+        model.synchronize()
+        prefill_s = (time.perf_counter() - started) / repeats
+        sequence = prefill()
+        for _ in range(steps // 4):
+            model.enqueue(sequence, [1])
+        model.synchronize()
+        started = time.perf_counter()
+        for _ in range(steps):
+            model.enqueue(sequence, [1])
+        model.synchronize()
+        decode_s = (time.perf_counter() - started) / steps
+        out[name] = {"prefill_tokens_per_s": rows / prefill_s, "prefill_us_per_layer": prefill_s * 1e6 / model.runs,
+                     "decode_tokens_per_s": 1 / decode_s, "decode_us_per_layer": decode_s * 1e6 / model.runs,
+                     "decode_weight_TBps": weight_bytes / decode_s / 1e12,
+                     "prefill_weight_TFLOPps": weight_bytes * rows / prefill_s / 1e12}
+        model.close_model()
+    return out
+
+
+def talker_throughput(dev, rows=1024, steps=64, layers=4):
+    """The same for the talker (hidden 2048, 16/8 heads of 128, intermediate 6144), the framework's closest model: prompt pass
+    and decode step through the engine shell, per layer."""
+    import tempfile
+    import torch
+    from safetensors.torch import save_file
+    module = importlib.import_module("qingming-qwen3-tts_amd.engine")
+    gen = torch.Generator(device=dev).manual_seed(2)
+    tensors = {"talker.model.norm.weight": torch.ones(2048, dtype=torch.bfloat16)}
+    for i in range(layers):
+        base = f"talker.model.layers.{i}."
+        for name, n, k in (("self_attn.q_proj", 2048, 2048), ("self_attn.k_proj", 1024, 2048), ("self_attn.v_proj", 1024, 2048),
+                           ("self_attn.o_proj", 2048, 2048), ("mlp.gate_proj", 6144, 2048), ("mlp.up_proj", 6144, 2048), ("mlp.down_proj", 2048, 6144)):
+            tensors[base + name + ".weight"] = (torch.randn(n, k, generator=gen, device=dev) * k ** -0.5).to(torch.bfloat16).cpu()
+        for name, n in (("input_layernorm", 2048), ("post_attention_layernorm", 2048), ("self_attn.q_norm", 128), ("self_attn.k_norm", 128)):
+            tensors[base + name + ".weight"] = torch.ones(n, dtype=torch.bfloat16)
+    weight_bytes = sum(t.numel() * 2 for t in tensors.values())
+    with tempfile.TemporaryDirectory() as directory:
+        save_file(tensors, os.path.join(directory, "model.safetensors"))
+        talker = module.Talker(directory, rows + 2 * steps + 8)
+    x = torch.randn(rows, 2048, generator=gen, device=dev).to(torch.bfloat16)
+    cos, sin = module.rope_rows(rows + 2 * steps + 8, 0)
+    torch.cuda.synchronize()
+    for _ in range(3):
+        talker.prefill(x, cos[:rows], sin[:rows], rows)
+    talker.synchronize()
+    started, repeats = time.perf_counter(), 10
+    for _ in range(repeats):
+        talker.prefill(x, cos[:rows], sin[:rows], rows)
+    talker.synchronize()
+    prefill_s = (time.perf_counter() - started) / repeats
+    device_rope = torch.from_numpy(np.stack([cos[rows:rows + 1], sin[rows:rows + 1]]).view(np.int16)).to(dev)
+    torch.cuda.synchronize()
+    import ctypes
+
+    def step(i):
+        final = ctypes.c_void_p()
+        rc = module.lib().qm_talker_decode_device_rope(talker._handle, x.data_ptr(), device_rope[0].data_ptr(), device_rope[1].data_ptr(), i,
+                                                       ctypes.byref(final))
+        assert rc == 0, rc
+
+    for i in range(steps // 4):
+        step(i)
+    talker.synchronize()
+    started = time.perf_counter()
+    for i in range(steps):
+        step(steps // 4 + i)
+    talker.synchronize()
+    decode_s = (time.perf_counter() - started) / steps
+    talker.close()
+    return {"prefill_tokens_per_s": rows / prefill_s, "prefill_us_per_layer": prefill_s * 1e6 / layers, "decode_tokens_per_s": 1 / decode_s,
+            "decode_us_per_layer": decode_s * 1e6 / layers, "decode_weight_TBps": weight_bytes / decode_s / 1e12,
+            "prefill_weight_TFLOPps": weight_bytes * rows / prefill_s / 1e12}
+
+
+def decoder_report(which, dev):
+    """Every size (or the one named), and the talker at the size they share."""
+    report = {}
+    for size in DECODER_SIZES if which == "all" else [which.split(":")[0]]:
+        kinds = which.split(":")[1].split(",") if ":" in which else None
+        for name, r in decoder_throughput(size, dev, kinds=kinds).items():
+            report[f"vabevik_{size}_{name}"] = r
+            print(f"vabevik_{size}_{name} " + json.dumps({k: round(v, 2) for k, v in r.items()}), flush=True)
+    if ":" not in which:
+        report["talker_w2048"] = talker_throughput(dev)
+        print("talker_w2048 " + json.dumps({k: round(v, 2) for k, v in report["talker_w2048"].items()}), flush=True)
+    return report
+
+
 def _within_rule(oracle, got_bits, want_bits, tol=1e-2):
     """The tolerance rule of the parity tests, per element: |got - want| <= max(tol, one bf16 ulp of the oracle's
     value) (beyond |x| = 2 one bf16 step is 1.56e-2, more than tol).  Returns (max abs error, elements outside the
@@ -1132,6 +1311,10 @@ def main():
     ap.add_argument("--layers", type=int, default=28,
                     help="with --only layer / layer1 / layer2: distinct weight sets and caches in rotation (a profiler that "
                          "records counters for every dispatch is spared most of the input generation with a small number)")
+    ap.add_argument("--decoder", nargs="?", const="all", default=None, metavar="SIZE[:KINDS]",
+                    help="prefill and decode throughput of the decoder language models (" + ", ".join(DECODER_SIZES) + ", or all) beside the "
+                         "talker's, instead of the attention workloads; SIZE:KINDS times that size's layer kinds alone (mixed, parallel, "
+                         "general_delta)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run three plain 512 MiB device-to-device copies (for scaling rocprofv3's "
                          "FETCH_SIZE / WRITE_SIZE counters against a kernel of known traffic)")
@@ -1159,6 +1342,11 @@ def main():
         del src, dst
         torch.cuda.empty_cache()
 
+    if args.decoder:
+        report = decoder_report(args.decoder, dev)
+        print(json.dumps({"metric": "decoder_language_models", "unit": "per entry", "dtype": "bf16, f32 accumulate", "data": "synthetic",
+                          "results": report}))
+        return
     if args.only == "generate":
         print(json.dumps(generate_end_to_end(qm, dev)))
         return

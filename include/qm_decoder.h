@@ -21,23 +21,24 @@ extern "C" {
 
 /* ---- residual sum and norm --------------------------------------------------------------------------------------- */
 /* x = x_in (or embed[token]) + sum_i scale_i * y_i + step_vec, where a y with a norm weight is first divided by its own
- * root mean square and weighted;  h = x / sqrt(mean(x^2) + eps) * norm_w. */
+ * root mean square and weighted;  h = x / sqrt(mean(x^2) + eps) * norm_w.  Every row and vector here has ld_h columns (a
+ * multiple of 4), zeros behind the first `width`; means are over `width`. */
 typedef struct {
-    const float* y;          /* [rows][ld] */
-    const float* norm_w;     /* [width], or NULL: y as it is */
+    const float* y;          /* [rows][ld], ld >= ld_h */
+    const float* norm_w;     /* [ld_h], or NULL: y as it is */
     int64_t ld;
     float scale;
     int32_t reserved;
 } qm_residual_term;
 typedef struct {
-    const float* x_in;       /* [rows][width]; NULL: the embedding of tokens[row] */
-    const uint16_t* embed;   /* [vocab][width] bf16 */
+    const float* x_in;       /* [rows][ld_h]; NULL: the embedding of tokens[row] */
+    const uint16_t* embed;   /* [vocab][ld_h] bf16 */
     const int32_t* tokens;
     const int32_t* row_map;  /* NULL, or each row's source row in x_in, tokens and the terms */
-    const float* step_vec;   /* [width], or NULL */
-    const float* norm_w;     /* [width] */
-    float* x_out;            /* [rows][width], or NULL */
-    void* h;                 /* [rows][ld_h] bf16 or fp32; columns width .. ld_h - 1 become zero */
+    const float* step_vec;   /* [ld_h], or NULL */
+    const float* norm_w;     /* [ld_h] */
+    float* x_out;            /* [rows][ld_h], or NULL */
+    void* h;                 /* [rows][ld_h] bf16 or fp32 */
     int64_t ld_h;
     int32_t width, vocab, terms;
     float eps;
@@ -97,7 +98,10 @@ typedef struct {
     int32_t heads, kv_heads, dim, vdim, k_stride, v_stride, ring, chunk, rot_dims;
     int32_t k_column, v_column;
     float scale;
+    int32_t options;         /* QM_ATTENTION_ROWS: keep many rows off the matrix cores */
+    int32_t reserved;
 } qm_chunk_attention;
+#define QM_ATTENTION_ROWS 1
 int32_t qm_chunk_attention_rows(const qm_chunk_attention* op, int32_t f32, void* hip_stream);
 
 /* ---- linear attention with a per-head decay ------------------------------------------------------------------------ */

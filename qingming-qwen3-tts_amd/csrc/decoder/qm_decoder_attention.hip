@@ -27,6 +27,7 @@ __global__ __launch_bounds__(kDecThreads) void rope_cache_kernel(ChunkAttentionP
         const float u = head[pair], v = head[pair + half], cosine = sh_turn[pair], sine = sh_turn[half + pair];
         return c < half ? u * cosine - v * sine : v * cosine + u * sine;
     };
+#pragma unroll 4
     for (int i = tid; i < prm.heads * prm.k_stride; i += kDecThreads) {
         const int h = i / prm.k_stride, c = i - h * prm.k_stride;
         static_cast<T*>(prm.q_rot)[static_cast<int64_t>(row) * prm.heads * prm.k_stride + i] = from_f32<T>(channel(proj + h * prm.dim, c));
@@ -102,6 +103,8 @@ int32_t launch_chunk_attention(const ChunkAttentionParams& prm, int f32, hipStre
     if (!prm.q_rot) return QM_ERR_NULL;
     rc = launch_rope_cache(prm, f32, stream);
     if (rc != QM_OK) return rc;
+    // (positions that only the device knows belong to one-token steps)
+    if (!f32 && prm.rows >= kAttentionMatrixRows && !prm.position_dev && !(prm.options & QM_ATTENTION_ROWS)) return launch_chunk_attention_mfma(prm, stream);
     return f32 ? attention_rows<float>(prm, stream) : attention_rows<uint16_t>(prm, stream);
 }
 

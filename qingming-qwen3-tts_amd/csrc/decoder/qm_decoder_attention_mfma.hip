@@ -1,0 +1,269 @@
+// qm_decoder_attention_mfma.hip — the chunked attention of a prompt's rows on the bf16 matrix cores (gfx950).
+//
+// A block of four waves takes 64 query rows of one key/value head (a query row is a position and one of the head's query
+// heads: they share keys and values) and walks the keys that any of them sees in tiles of 64.  Waves work in pairs on 32 of
+// the rows, each wave of a pair on half of every tile, and combine at the end: a prompt of a thousand tokens gives a grid
+// that fills the chip, and a wave needs nothing from another while it walks.
+//
+// Scores are S^T = K Q^T (v_mfma_f32_32x32x16_bf16): a lane then holds sixteen keys of one query, the softmax is in the lane
+// but for one exchange with the other half of the wave, and the weights stand where the second product O^T = V^T P^T wants
+// its operand, if it takes the keys of a block in the order the scores left them.  Scores and weights are fp32; the second
+// product takes a weight as the sum of two bf16 numbers (its rounding and the rounding of what is left: 16 bits).  Values
+// are transposed on their way into LDS.  Bound: bf16 MFMA and the vector work per score; flops 2 (dim + vdim) per visible
+// key and query (the second product's doubled weights not counted).
+#include "../qm_host.h"
+#include "qm_decoder_device.h"
+
+namespace qm {
+
+typedef float dec_f32x16 __attribute__((ext_vector_type(16)));
+
+constexpr int kFlashKeys = 64;                 // keys per tile
+constexpr int kFlashRows = 64;                 // query rows per block
+constexpr int kFlashVStride = kFlashKeys + 4;  // bf16 per value channel in LDS: the 32 rows of a fragment lie in different banks
+
+// C: channels of a head, rounded up to 32, 64, 128 or 256 (the larger of the key and the value size)
+template <int C>
+struct FlashShape {
+    static constexpr int kKStride = C + 8;
+    static constexpr int kKBytes = kFlashKeys * kKStride * 2;
+    static constexpr int kVBytes = C * kFlashVStride * 2;
+    static constexpr int kCombineBytes = 2 * (C / 32) * 16 * 64 * 4 + 2 * 2 * 32 * 4;
+    static constexpr int kLds = kKBytes + kVBytes > kCombineBytes ? kKBytes + kVBytes : kCombineBytes;
+};
+
+template <int C>
+__global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(ChunkAttentionParams prm) {
+    using Shape = FlashShape<C>;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    uint16_t* ks = reinterpret_cast<uint16_t*>(smem);                          // [keys][kKStride]
+    uint16_t* vt = reinterpret_cast<uint16_t*>(smem + Shape::kKBytes);         // [C][kFlashVStride]
+    constexpr int kKb = C / 16, kVt = C / 32;
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int pair = wave >> 1, part = wave & 1, half = lane >> 5;
+    const int kv_head = static_cast<int>(blockIdx.y);
+    const int group = prm.heads / prm.kv_heads;
+    const int total = prm.rows * group;
+    const int row0 = static_cast<int>(blockIdx.x) * kFlashRows;
+    auto position_at = [&](int query_row) { return prm.position + min(query_row, total - 1) / group; };
+    auto chunk_start = [&](int position) { return position - position % prm.chunk; };
+    // what the block, this wave and this lane see: keys [.., ..]
+    const int block_lo = chunk_start(position_at(row0)), block_hi = position_at(row0 + kFlashRows - 1);
+    const int wave_first = position_at(row0 + 32 * pair), wave_last = position_at(row0 + 32 * pair + 31);
+    const int wave_lo = chunk_start(wave_first), wave_lo_most = chunk_start(wave_last);
+    const int query_row = row0 + 32 * pair + (lane & 31);
+    const int local = min(query_row, total - 1) / group;
+    const int head = kv_head * group + min(query_row, total - 1) % group;
+    const int position = prm.position + local;
+    const int lo = chunk_start(position);
+    const int key_blocks = (prm.dim + 15) / 16, value_tiles = (prm.vdim + 31) / 32;
+
+    uint4 q[kKb];
+    const uint16_t* q_row = static_cast<const uint16_t*>(prm.q_rot) + (static_cast<int64_t>(local) * prm.heads + head) * prm.k_stride;
+#pragma unroll
+    for (int kb = 0; kb < kKb; ++kb) {
+        const int c = kb * 16 + 8 * half;
+        q[kb] = c < prm.k_stride ? *reinterpret_cast<const uint4*>(q_row + c) : make_uint4(0, 0, 0, 0);
+    }
+    dec_f32x16 o[kVt];
+#pragma unroll
+    for (int t = 0; t < kVt; ++t)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[t][r] = 0.0f;
+    float m = -INFINITY, l = 0.0f;
+    const float to_log2 = prm.scale * kLog2e;
+
+    const uint16_t* k_head = static_cast<const uint16_t*>(prm.k_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.k_stride;
+    const uint16_t* v_head = static_cast<const uint16_t*>(prm.v_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.v_stride;
+    constexpr int kKPieces = kFlashKeys * (C / 8) / kDecThreads;                // 16-byte pieces of keys per thread
+    constexpr int kVBlocks = (16 * (C / 4) + kDecThreads - 1) / kDecThreads;    // blocks of 4 keys x 4 channels per thread
+    uint4 k_piece[kKPieces];
+    uint2 v_piece[kVBlocks][4];
+    // (keys past the last one that the block sees are not read: zeros, whose weights are zero as well)
+    auto request = [&](int tile) {
+        const int base = tile % prm.ring;
+        auto slot_of = [&](int key) {
+            const int s = base + key;
+            return static_cast<int64_t>(s >= prm.ring ? s - prm.ring : s);
+        };
+#pragma unroll
+        for (int i = 0; i < kKPieces; ++i) {
+            const int at = tid + i * kDecThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            k_piece[i] = tile + key <= block_hi && c < prm.k_stride ? *reinterpret_cast<const uint4*>(k_head + slot_of(key) * prm.k_stride + c)
+                                                                    : make_uint4(0, 0, 0, 0);
+        }
+#pragma unroll
+        for (int i = 0; i < kVBlocks; ++i) {
+            const int at = tid + i * kDecThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                v_piece[i][j] = at < 16 * (C / 4) && tile + key + j <= block_hi && c < prm.v_stride
+                                    ? *reinterpret_cast<const uint2*>(v_head + slot_of(key + j) * prm.v_stride + c) : make_uint2(0, 0);
+        }
+    };
+    auto deposit = [&]() {
+#pragma unroll
+        for (int i = 0; i < kKPieces; ++i) {
+            const int at = tid + i * kDecThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            *reinterpret_cast<uint4*>(ks + key * Shape::kKStride + c) = k_piece[i];
+        }
+#pragma unroll
+        for (int i = 0; i < kVBlocks; ++i) {
+            const int at = tid + i * kDecThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
+            if (at >= 16 * (C / 4)) break;
+            const uint2 *p = v_piece[i];
+            uint16_t* to = vt + c * kFlashVStride + key;
+            *reinterpret_cast<uint2*>(to) = make_uint2(__builtin_amdgcn_perm(p[1].x, p[0].x, 0x05040100U), __builtin_amdgcn_perm(p[3].x, p[2].x, 0x05040100U));
+            *reinterpret_cast<uint2*>(to + kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].x, p[0].x, 0x07060302U), __builtin_amdgcn_perm(p[3].x, p[2].x, 0x07060302U));
+            *reinterpret_cast<uint2*>(to + 2 * kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].y, p[0].y, 0x05040100U), __builtin_amdgcn_perm(p[3].y, p[2].y, 0x05040100U));
+            *reinterpret_cast<uint2*>(to + 3 * kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].y, p[0].y, 0x07060302U), __builtin_amdgcn_perm(p[3].y, p[2].y, 0x07060302U));
+        }
+    };
+
+    request(block_lo);
+    for (int tile = block_lo; tile <= block_hi; tile += kFlashKeys) {
+        __syncthreads();                                           // the tile before has been read
+        deposit();
+        __syncthreads();
+        if (tile + kFlashKeys <= block_hi) request(tile + kFlashKeys);
+        const int k0 = tile + 32 * part;
+        if (k0 > wave_last || k0 + 31 < wave_lo) continue;         // nothing here for this wave's rows
+        dec_f32x16 s;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) s[r] = 0.0f;
+        const uint16_t* k_row = ks + (32 * part + (lane & 31)) * Shape::kKStride + 8 * half;
+#pragma unroll
+        for (int kb = 0; kb < kKb; ++kb) {
+            if (kb >= key_blocks) break;
+            const uint4 a = *reinterpret_cast<const uint4*>(k_row + kb * 16);
+            s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, q[kb]), s, 0, 0, 0);
+        }
+        // register r is key k0 + 8 (r / 4) + 4 half + r % 4
+        float p[16];
+        const bool whole = k0 >= wave_lo_most && k0 + 31 <= wave_first;
+        float largest = -INFINITY;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            p[r] = s[r] * to_log2;
+            if (!whole) {
+                const int key = k0 + 8 * (r / 4) + 4 * half + r % 4;
+                if (key < lo || key > position) p[r] = -INFINITY;
+            }
+            largest = fmaxf(largest, p[r]);
+        }
+        largest = fmaxf(largest, __shfl_xor(largest, 32, 64));
+        const float before = m;
+        m = fmaxf(m, largest);
+        const float reference = m == -INFINITY ? 0.0f : m;         // (a row that has seen no key yet: all its weights are zero)
+        const float alpha = fast_exp2(before - reference);
+        float sum = 0.0f;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            p[r] = fast_exp2(p[r] - reference);
+            sum += p[r];
+        }
+        l = l * alpha + sum;
+        if (__any(alpha != 1.0f)) {
+#pragma unroll
+            for (int t = 0; t < kVt; ++t)
+#pragma unroll
+                for (int r = 0; r < 16; ++r) o[t][r] *= alpha;
+        }
+        uint4 high[2], low[2];
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+            uint32_t h4[4], l4[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const float x = p[8 * b + 2 * e], y = p[8 * b + 2 * e + 1];
+                h4[e] = pack_bf16_pair(x, y);
+                l4[e] = pack_bf16_pair(x - lo_bf16(h4[e]), y - hi_bf16(h4[e]));
+            }
+            high[b] = make_uint4(h4[0], h4[1], h4[2], h4[3]);
+            low[b] = make_uint4(l4[0], l4[1], l4[2], l4[3]);
+        }
+#pragma unroll
+        for (int t = 0; t < kVt; ++t) {
+            if (t >= value_tiles) break;
+            const uint16_t* v_row = vt + (32 * t + (lane & 31)) * kFlashVStride + 32 * part + 4 * half;
+#pragma unroll
+            for (int b = 0; b < 2; ++b) {
+                const uint2 first = *reinterpret_cast<const uint2*>(v_row + 16 * b), second = *reinterpret_cast<const uint2*>(v_row + 16 * b + 8);
+                const uint4 a = make_uint4(first.x, first.y, second.x, second.y);
+                o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, high[b]), o[t], 0, 0, 0);
+                o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, low[b]), o[t], 0, 0, 0);
+            }
+        }
+    }
+
+    // the pair's two halves of the keys, combined by its first wave
+    l += __shfl_xor(l, 32, 64);
+    __syncthreads();
+    float* other_o = reinterpret_cast<float*>(smem) + pair * kVt * 16 * 64;
+    float* other_ml = reinterpret_cast<float*>(smem) + 2 * kVt * 16 * 64 + pair * 64;
+    if (part == 1) {
+#pragma unroll
+        for (int t = 0; t < kVt; ++t)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) other_o[(t * 16 + r) * 64 + lane] = o[t][r];
+        if (lane < 32) {
+            other_ml[lane] = m;
+            other_ml[32 + lane] = l;
+        }
+    }
+    __syncthreads();
+    if (part == 0 && query_row < total) {
+        const float m1 = other_ml[lane & 31], l1 = other_ml[32 + (lane & 31)];
+        const float most = fmaxf(m, m1);
+        const float f0 = fast_exp2(m - most), f1 = fast_exp2(m1 - most);
+        const float scale = 1.0f / (l * f0 + l1 * f1);
+        uint16_t* out = static_cast<uint16_t*>(prm.out) + local * prm.ld_out + head * prm.vdim;
+#pragma unroll
+        for (int t = 0; t < kVt; ++t) {
+#pragma unroll
+            for (int g = 0; g < 4; ++g) {
+                const int c = 32 * t + 8 * g + 4 * half;
+                float v[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) v[e] = (o[t][4 * g + e] * f0 + other_o[(t * 16 + 4 * g + e) * 64 + lane] * f1) * scale;
+                if (prm.vdim % 4 == 0) {
+                    if (c < prm.vdim) *reinterpret_cast<uint2*>(out + c) = make_uint2(pack_bf16_pair(v[0], v[1]), pack_bf16_pair(v[2], v[3]));
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (c + e < prm.vdim) out[c + e] = f2bf(v[e]);
+                }
+            }
+        }
+    }
+    // zeros behind the heads' columns, by the last head's blocks
+    if (kv_head == prm.kv_heads - 1) {
+        const int first = row0 / group, last = min(row0 + kFlashRows - 1, total - 1) / group;
+        const int from = prm.heads * prm.vdim, behind = static_cast<int>(prm.ld_out) - from;
+        for (int i = tid; i < (last - first + 1) * behind; i += kDecThreads)
+            static_cast<uint16_t*>(prm.out)[(first + i / behind) * prm.ld_out + from + i % behind] = 0;
+    }
+}
+
+template <int C>
+static int32_t flash_as(const ChunkAttentionParams& prm, hipStream_t stream) {
+    static std::atomic<bool> raised[kMaxDevices];
+    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(chunk_attention_mfma_kernel<C>), FlashShape<C>::kLds, raised);
+    if (rc != QM_OK) return rc;
+    const int64_t total = static_cast<int64_t>(prm.rows) * (prm.heads / prm.kv_heads);
+    hipLaunchKernelGGL((chunk_attention_mfma_kernel<C>), dim3(static_cast<unsigned>((total + kFlashRows - 1) / kFlashRows), prm.kv_heads),
+                       dim3(kDecThreads), FlashShape<C>::kLds, stream, prm);
+    return launch_status();
+}
+
+int32_t launch_chunk_attention_mfma(const ChunkAttentionParams& prm, hipStream_t stream) {
+    if (prm.ld_out % 4 || (reinterpret_cast<uintptr_t>(prm.out) & 7)) return QM_ERR_GEOMETRY;
+    const int c = prm.dim > prm.vdim ? prm.dim : prm.vdim;
+    if (c <= 32) return flash_as<32>(prm, stream);
+    if (c <= 64) return flash_as<64>(prm, stream);
+    if (c <= 128) return flash_as<128>(prm, stream);
+    return flash_as<256>(prm, stream);
+}
+
+}  // namespace qm

@@ -1,0 +1,334 @@
+// qm_decoder_delta_chunks.hip — the generalized delta rule over a prompt's rows, in chunks of 32 tokens (gfx950).
+//
+// S_t = diag(w_t) S_{t-1} - (a_t u_t)(u_t^T S_{t-1}) + k_t v_t^T,  o_t = S_t^T r_t.  Let W_t be the product of the decays of
+// the chunk's tokens up to t (per channel, W before the first token 1), S the state before the chunk, and
+//   U_t = u_t W_{t-1},  A_t = a_t u_t / W_t,  K_t = k_t / W_t,  R_t = r_t W_t   (rows of [32][dim] matrices).
+// What the removal terms read, p_t = u_t^T S_{t-1}, solves a triangular system:  (I + L_A) P = U S + L_K V  with
+// L_A[t][s] = U_t . A_s and L_K[t][s] = U_t . K_s for s < t.  So P = M S + N V with M = (I + L_A)^-1 U, N = (I + L_A)^-1 L_K,
+// and with the lower triangles (diagonal included) D_A[t][s] = R_t . A_s, D_K[t][s] = R_t . K_s:
+//   O = (R - D_A M) S + (D_K - D_A N) V,      S' = diag(W) (S - A^T P + K^T V),  W the whole chunk's product.
+// M, N, R - D_A M, D_K - D_A N do not depend on S: one launch computes them for every chunk and head at once.  A second one
+// walks the chunks; columns of S never interact, so its blocks take 16 columns each, four waves sharing the rows.  A decay is
+// never below exp(-e^(-1/2)) = 0.545, so 1 / W stays under 3e8 and everything fits fp32; A and K enter the state already
+// multiplied by W.  All products are fp32 (matrix cores, or fmaf for the triangular solve).
+// Bound: the walk, a chain of rows / 32 dependent steps.
+#include "../qm_host.h"
+#include "qm_decoder_mfma32.h"
+#include "qm_decoder_recurrent.h"
+
+namespace qm {
+
+constexpr int kDeltaChunk = 32;
+constexpr int kDeltaMat = kDeltaChunk + 4;     // row stride of a [32][32] matrix in LDS
+
+// Scratch of a (chunk, head), floats: M, X [32][dp], -A^T W, K^T W [dp][32], N, Y [32][32], W [dp].
+struct DeltaScratch {
+    int m, x, at, kt, n, y, w, floats;
+};
+__host__ __device__ inline DeltaScratch delta_scratch(int dim) {
+    const int dp = mfma32_pad(dim), rows = kDeltaChunk * dp, square = kDeltaChunk * kDeltaChunk;
+    DeltaScratch s;
+    s.m = 0; s.x = rows; s.at = 2 * rows; s.kt = 3 * rows; s.n = 4 * rows; s.y = s.n + square; s.w = s.y + square;
+    s.floats = s.w + (dp + 63) / 64 * 64;
+    return s;
+}
+__host__ __device__ inline int delta_z_stride(int rank) { return (rank + 3) / 4 * 4; }
+inline int delta_prepare_lds(int dim) { return 4 * kDeltaChunk * mfma32_stride(dim) + 4 * kDeltaChunk * kDeltaMat + kDeltaChunk; }
+
+__global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaParams prm) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l16 = lane & 15;
+    const int chunk = static_cast<int>(blockIdx.x), head = static_cast<int>(blockIdx.y);
+    const int t0 = chunk * kDeltaChunk, tokens = min(kDeltaChunk, prm.rows - t0);
+    const int dim = prm.dim, dp = mfma32_pad(dim), stride = mfma32_stride(dim);
+    const DeltaScratch at = delta_scratch(dim);
+    float* scratch = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * at.floats;
+    float* us = lds;                           // [32][stride] each; us holds the decays first
+    float* as = us + kDeltaChunk * stride;
+    float* ks = as + kDeltaChunk * stride;
+    float* rs = ks + kDeltaChunk * stride;
+    float* mats = rs + kDeltaChunk * stride;   // L_A, L_K, D_A, D_K, each [32][kDeltaMat]
+    float* inverse = mats + 4 * kDeltaChunk * kDeltaMat;
+    float* zs = as;                            // tanh of the rank-sized projection, [32][z_stride], until the decays are there
+    const int z_stride = delta_z_stride(prm.rank);
+
+    for (int i = tid; i < kDeltaChunk * z_stride; i += kDecThreads) {
+        const int t = i / z_stride, r = i - t * z_stride;
+        zs[i] = t < tokens && r < prm.rank ? tanhf(prm.proj[(t0 + t) * prm.ld_proj + prm.z_column + r]) : 0.0f;
+    }
+    for (int t = wave; t < tokens; t += 4) {
+        const float* k = prm.proj + (t0 + t) * prm.ld_proj + prm.k_column + head * dim;
+        float sq = 0.0f;
+        for (int c = lane; c < dim; c += 64) sq = fmaf(k[c], k[c], sq);
+        sq = wave_sum(sq);
+        if (lane == 0) inverse[t] = 1.0f / sqrtf(sq + prm.unit_eps);
+    }
+    __syncthreads();
+    const int all = prm.heads * dim;
+    for (int i = tid; i < 2 * dp; i += kDecThreads) {              // decays: a thread takes a channel of sixteen tokens
+        const int c = i % dp, first = i / dp * 16;
+        float z[16];
+        const float bias = c < dim ? prm.w0[head * dim + c] : 0.0f;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) z[t] = bias;
+        if (c < dim) {
+            const float* w2 = prm.w2 + head * dim + c;
+#pragma unroll 2
+            for (int r = 0; r < prm.rank; r += 4) {
+                float w[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) w[e] = r + e < prm.rank ? w2[static_cast<int64_t>(r + e) * all] : 0.0f;
+#pragma unroll
+                for (int t = 0; t < 16; ++t) {
+                    const float4 x = *reinterpret_cast<const float4*>(zs + (first + t) * z_stride + r);
+                    z[t] = fmaf(w[0], x.x, z[t]); z[t] = fmaf(w[1], x.y, z[t]);
+                    z[t] = fmaf(w[2], x.z, z[t]); z[t] = fmaf(w[3], x.w, z[t]);
+                }
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < 16; ++t) us[(first + t) * stride + c] = first + t < tokens && c < dim ? delta_decay_of(z[t]) : 1.0f;
+    }
+    __syncthreads();
+    if (tid < dp) {                                                // a channel's products of decays, and what they scale
+        const int c = tid;
+        const float bias = c < dim ? prm.a_bias[head * dim + c] : 0.0f;
+        float before = 1.0f;
+#pragma unroll 8
+        for (int t = 0; t < kDeltaChunk; ++t) {
+            const bool in = t < tokens && c < dim;
+            const float* p = prm.proj + (t0 + min(t, tokens - 1)) * prm.ld_proj + head * dim + min(c, dim - 1);
+            const float k = in ? p[prm.k_column] : 0.0f, r = in ? p[prm.r_column] : 0.0f;
+            const float u = in ? k * inverse[t] : 0.0f;
+            const float a = in ? sigmoid_f32(p[prm.a_column] + bias) * u : 0.0f;
+            const float after = before * us[t * stride + c];
+            const float over = 1.0f / after;
+            us[t * stride + c] = u * before;
+            as[t * stride + c] = a * over;
+            ks[t * stride + c] = k * over;
+            rs[t * stride + c] = r * after;
+            before = after;
+        }
+        scratch[at.w + c] = before;
+#pragma unroll
+        for (int t = 0; t < kDeltaChunk; t += 4) {
+            float4 a, k;
+            a.x = -before * as[t * stride + c]; a.y = -before * as[(t + 1) * stride + c];
+            a.z = -before * as[(t + 2) * stride + c]; a.w = -before * as[(t + 3) * stride + c];
+            k.x = before * ks[t * stride + c]; k.y = before * ks[(t + 1) * stride + c];
+            k.z = before * ks[(t + 2) * stride + c]; k.w = before * ks[(t + 3) * stride + c];
+            *reinterpret_cast<float4*>(scratch + at.at + c * kDeltaChunk + t) = a;
+            *reinterpret_cast<float4*>(scratch + at.kt + c * kDeltaChunk + t) = k;
+        }
+    }
+    __syncthreads();
+    {                                                              // wave 0: L_A, 1: L_K, 2: D_A, 3: D_K
+        const float* left = wave < 2 ? us : rs;
+        const float* right = wave & 1 ? ks : as;
+        f32x4_t acc[2][2] = {};
+        for (int d0 = 0; d0 < dp; d0 += 16) {
+            float4 a[2], b[2];
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                a[i] = *reinterpret_cast<const float4*>(left + (16 * i + l16) * stride + d0 + 4 * g);
+                b[i] = *reinterpret_cast<const float4*>(right + (16 * i + l16) * stride + d0 + 4 * g);
+            }
+            acc[0][0] = mfma32_block(a[0], b[0], acc[0][0]);
+            acc[1][0] = mfma32_block(a[1], b[0], acc[1][0]);
+            acc[1][1] = mfma32_block(a[1], b[1], acc[1][1]);
+        }
+        float* mat = mats + wave * kDeltaChunk * kDeltaMat;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int j = 0; j < 2; ++j)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int t = 16 * i + 4 * g + r, s = 16 * j + l16;
+                    mat[t * kDeltaMat + s] = s < t || (s == t && wave >= 2) ? acc[i][j][r] : 0.0f;
+                }
+    }
+    __syncthreads();
+    const float* l_a = mats;
+    const float* d_a = mats + 2 * kDeltaChunk * kDeltaMat;
+    for (int c = tid; c < dp + kDeltaChunk; c += kDecThreads) {    // columns of (U, L_K) solved, and of (R, D_K) less D_A times them
+        const bool wide = c < dp;
+        const float* y = wide ? us + c : mats + kDeltaChunk * kDeltaMat + (c - dp);
+        const float* z = wide ? rs + c : mats + 3 * kDeltaChunk * kDeltaMat + (c - dp);
+        const int step = wide ? stride : kDeltaMat, out_step = wide ? dp : kDeltaChunk;
+        float* solved_out = scratch + (wide ? at.m + c : at.n + c - dp);
+        float* rest_out = scratch + (wide ? at.x + c : at.y + c - dp);
+        float solved[kDeltaChunk];
+#pragma unroll
+        for (int t = 0; t < kDeltaChunk; ++t) {
+            float v = y[t * step], x = z[t * step];
+#pragma unroll
+            for (int s = 0; s < t; s += 4) {
+                const float4 m = *reinterpret_cast<const float4*>(l_a + t * kDeltaMat + s);
+                v = fmaf(-m.x, solved[s], v);
+                if (s + 1 < t) v = fmaf(-m.y, solved[s + 1], v);
+                if (s + 2 < t) v = fmaf(-m.z, solved[s + 2], v);
+                if (s + 3 < t) v = fmaf(-m.w, solved[s + 3], v);
+            }
+            solved[t] = v;
+#pragma unroll
+            for (int s = 0; s <= t; s += 4) {
+                const float4 m = *reinterpret_cast<const float4*>(d_a + t * kDeltaMat + s);
+                x = fmaf(-m.x, solved[s], x);
+                if (s + 1 <= t) x = fmaf(-m.y, solved[s + 1], x);
+                if (s + 2 <= t) x = fmaf(-m.z, solved[s + 2], x);
+                if (s + 3 <= t) x = fmaf(-m.w, solved[s + 3], x);
+            }
+            solved_out[t * out_step] = v;
+            rest_out[t * out_step] = x;
+        }
+    }
+}
+
+// What a wave needs of a chunk besides the state: its shares of the prepared matrices, and the values of the block's columns.
+template <int TW>
+struct DeltaStep {
+    float4 m[2][TW], x[2][TW], at[TW][2], kt[TW][2], w[TW];
+    float2 n[2], y[2];
+    float v[2][4];
+};
+
+// TW: 16-row tiles of the state per wave (tile = wave + 4 i)
+template <int TW>
+__global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaParams prm, int chunks) {
+    constexpr int kStride = 20;                                    // the four row groups of a store lie in different banks
+    __shared__ float sh[2][4][2][kDeltaChunk * kStride];           // by turns: each wave's share of P and of O
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l16 = lane & 15;
+    const int head = static_cast<int>(blockIdx.y), column = static_cast<int>(blockIdx.x) * 16 + l16;
+    const int dim = prm.dim, dp = mfma32_pad(dim);
+    const DeltaScratch at = delta_scratch(dim);
+    float* state = prm.state + static_cast<int64_t>(head) * dim * dim;
+    const int part = wave >> 1, pair = 2 * (wave & 1);             // the wave's terms of N V and Y V: tokens 16 part + 4 g + pair, + 1
+    f32x4_t s[TW];
+#pragma unroll
+    for (int i = 0; i < TW; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int d = 16 * (wave + 4 * i) + 4 * g + r;
+            s[i][r] = d < dim && column < dim ? state[static_cast<int64_t>(d) * dim + column] : 0.0f;
+        }
+    const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    auto request = [&](int chunk, DeltaStep<TW>& f) __attribute__((always_inline)) {
+        const float* from = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * at.floats;
+#pragma unroll
+        for (int i = 0; i < TW; ++i) {
+            const int tile = wave + 4 * i;
+            const bool in = 16 * tile < dp;
+#pragma unroll
+            for (int b = 0; b < 2; ++b) {
+                const int row = (16 * b + l16) * dp + 16 * tile + 4 * g, channel = (16 * tile + l16) * kDeltaChunk + 16 * b + 4 * g;
+                f.m[b][i] = in ? *reinterpret_cast<const float4*>(from + at.m + row) : zero;
+                f.x[b][i] = in ? *reinterpret_cast<const float4*>(from + at.x + row) : zero;
+                f.at[i][b] = in ? *reinterpret_cast<const float4*>(from + at.at + channel) : zero;
+                f.kt[i][b] = in ? *reinterpret_cast<const float4*>(from + at.kt + channel) : zero;
+            }
+            f.w[i] = in ? *reinterpret_cast<const float4*>(from + at.w + 16 * tile + 4 * g) : zero;
+        }
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+            const int row = (16 * b + l16) * kDeltaChunk + 16 * part + 4 * g + pair;
+            f.n[b] = *reinterpret_cast<const float2*>(from + at.n + row);
+            f.y[b] = *reinterpret_cast<const float2*>(from + at.y + row);
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const int token = chunk * kDeltaChunk + 16 * b + 4 * g + t;
+                f.v[b][t] = token < prm.rows && column < dim ? prm.proj[token * prm.ld_proj + prm.v_column + head * dim + column] : 0.0f;
+            }
+        }
+    };
+    auto walk = [&](int chunk, DeltaStep<TW>& f, DeltaStep<TW>& next) __attribute__((always_inline)) {
+        if (chunk + 1 < chunks) request(chunk + 1, next);
+        f32x4_t p[2] = {}, o[2] = {};
+#pragma unroll
+        for (int i = 0; i < TW; ++i) {
+            const float4 b = make_float4(s[i][0], s[i][1], s[i][2], s[i][3]);
+#pragma unroll
+            for (int half = 0; half < 2; ++half) {
+                p[half] = mfma32_block(f.m[half][i], b, p[half]);
+                o[half] = mfma32_block(f.x[half][i], b, o[half]);
+            }
+        }
+        const float v0 = part ? (pair ? f.v[1][2] : f.v[1][0]) : (pair ? f.v[0][2] : f.v[0][0]);
+        const float v1 = part ? (pair ? f.v[1][3] : f.v[1][1]) : (pair ? f.v[0][3] : f.v[0][1]);
+        float (*mine)[kDeltaChunk * kStride] = sh[chunk & 1][wave];
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+            p[half] = mfma32(f.n[half].y, v1, mfma32(f.n[half].x, v0, p[half]));
+            o[half] = mfma32(f.y[half].y, v1, mfma32(f.y[half].x, v0, o[half]));
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                mine[0][(16 * half + 4 * g + r) * kStride + l16] = p[half][r];
+                mine[1][(16 * half + 4 * g + r) * kStride + l16] = o[half][r];
+            }
+        }
+        // (what does not need P, while the others arrive)
+#pragma unroll
+        for (int i = 0; i < TW; ++i) {
+            s[i][0] *= f.w[i].x; s[i][1] *= f.w[i].y; s[i][2] *= f.w[i].z; s[i][3] *= f.w[i].w;
+#pragma unroll
+            for (int b = 0; b < 2; ++b) s[i] = mfma32_block(f.kt[i][b], make_float4(f.v[b][0], f.v[b][1], f.v[b][2], f.v[b][3]), s[i]);
+        }
+        __syncthreads();
+        float read[2][4];
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const int from = (16 * b + 4 * g + t) * kStride + l16;
+                read[b][t] = (sh[chunk & 1][0][0][from] + sh[chunk & 1][1][0][from]) + (sh[chunk & 1][2][0][from] + sh[chunk & 1][3][0][from]);
+            }
+#pragma unroll
+        for (int i = 0; i < TW; ++i)
+#pragma unroll
+            for (int b = 0; b < 2; ++b) s[i] = mfma32_block(f.at[i][b], make_float4(read[b][0], read[b][1], read[b][2], read[b][3]), s[i]);
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+            const int t = 8 * wave + 4 * j + g, from = t * kStride + l16, token = chunk * kDeltaChunk + t;
+            const float out = (sh[chunk & 1][0][1][from] + sh[chunk & 1][1][1][from]) + (sh[chunk & 1][2][1][from] + sh[chunk & 1][3][1][from]);
+            if (token < prm.rows && column < dim) prm.out[static_cast<int64_t>(token) * prm.heads * dim + head * dim + column] = out;
+        }
+    };
+    DeltaStep<TW> even, odd;
+    request(0, even);
+    for (int chunk = 0; chunk < chunks; chunk += 2) {
+        walk(chunk, even, odd);
+        if (chunk + 1 < chunks) walk(chunk + 1, odd, even);
+    }
+#pragma unroll
+    for (int i = 0; i < TW; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int d = 16 * (wave + 4 * i) + 4 * g + r;
+            if (d < dim && column < dim) state[static_cast<int64_t>(d) * dim + column] = s[i][r];
+        }
+}
+
+int64_t delta_scratch_floats(int rows, int heads, int dim) {
+    if (rows < kChunkedRows || heads <= 0 || dim <= 0) return 0;
+    return static_cast<int64_t>((rows + kDeltaChunk - 1) / kDeltaChunk) * heads * delta_scratch(dim).floats;
+}
+
+// (the rank-sized projection's tanh shares the LDS of three matrices)
+bool delta_chunks_fit(const DeltaParams& prm) { return delta_z_stride(prm.rank) <= 3 * mfma32_stride(prm.dim); }
+
+int32_t launch_delta_chunks(const DeltaParams& prm, hipStream_t stream) {
+    const int chunks = (prm.rows + kDeltaChunk - 1) / kDeltaChunk;
+    const int lds = static_cast<int>(sizeof(float)) * delta_prepare_lds(prm.dim);
+    static std::atomic<bool> raised[kMaxDevices];
+    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(delta_chunk_prepare_kernel), kDotLdsMost, raised);
+    if (rc != QM_OK) return rc;
+    if (lds > kDotLdsMost || prm.scratch_floats < delta_scratch_floats(prm.rows, prm.heads, prm.dim)) return QM_ERR_WORKSPACE;
+    hipLaunchKernelGGL(delta_chunk_prepare_kernel, dim3(chunks, prm.heads), dim3(kDecThreads), lds, stream, prm);
+    const dim3 grid((prm.dim + 15) / 16, prm.heads);
+    if (prm.dim <= 64) hipLaunchKernelGGL(delta_chunk_walk_kernel<1>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
+    else if (prm.dim <= 128) hipLaunchKernelGGL(delta_chunk_walk_kernel<2>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
+    else hipLaunchKernelGGL(delta_chunk_walk_kernel<4>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
+    return launch_status();
+}
+
+}  // namespace qm

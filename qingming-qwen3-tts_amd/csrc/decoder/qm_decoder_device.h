@@ -52,52 +52,86 @@ __device__ __forceinline__ void block_sums(float (&v)[N], float* sh) {
 // A position is known to the host, or lives in device memory where a captured graph finds it.
 __device__ __forceinline__ int position_of(const int32_t* device, int host) { return device ? *device : host; }
 
-// One row by a block of 256 threads.  sh_x: width floats, sh_red: 16 floats, both LDS; h may be LDS or global memory.
-// The caller puts a barrier between this and any use of sh_x, sh_red or h by other threads.
-template <class T>
-__device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int row, float* sh_x, float* sh_red, T* h, bool write_x) {
+// The residual sum and its norm for one row by a block of 256 threads.  Rows are padded with zeros to ld_h columns, and a
+// thread owns the float4s tid, tid + 256, ... of a row (NV of them): everything the row needs is requested before the first
+// sum waits.  sh_red: 16 floats of LDS; h may be LDS or global memory.  The caller puts a barrier between this and any use
+// of sh_red or h by other threads.
+__device__ __forceinline__ float4 load4(const float* p, int v) { return reinterpret_cast<const float4*>(p)[v]; }
+__device__ __forceinline__ float4 load4(const uint16_t* p, int v) {
+    const uint2 w = reinterpret_cast<const uint2*>(p)[v];
+    return make_float4(lo_bf16(w.x), hi_bf16(w.x), lo_bf16(w.y), hi_bf16(w.y));
+}
+__device__ __forceinline__ void store4(float* p, int v, float a, float b, float c, float d) { reinterpret_cast<float4*>(p)[v] = make_float4(a, b, c, d); }
+__device__ __forceinline__ void store4(uint16_t* p, int v, float a, float b, float c, float d) {
+    reinterpret_cast<uint2*>(p)[v] = make_uint2(pack_bf16_pair(a, b), pack_bf16_pair(c, d));
+}
+__device__ __forceinline__ float square_sum(float4 v, float sum) { return fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, sum)))); }
+// acc + f * y * w
+__device__ __forceinline__ float4 weighted(float4 acc, float f, float4 y, float4 w) {
+    return make_float4(fmaf(f * y.x, w.x, acc.x), fmaf(f * y.y, w.y, acc.y), fmaf(f * y.z, w.z, acc.z), fmaf(f * y.w, w.w, acc.w));
+}
+
+template <class T, int NV>
+__device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int row, float* sh_red, T* h, bool write_x) {
     const int tid = threadIdx.x;
-    const int width = prm.width;
     const int64_t src = prm.row_map ? prm.row_map[row] : row;
-    const float* y0 = prm.terms > 0 ? prm.term[0].y + src * prm.term[0].ld : nullptr;
-    const float* y1 = prm.terms > 1 ? prm.term[1].y + src * prm.term[1].ld : nullptr;
-    const float* y2 = prm.terms > 2 ? prm.term[2].y + src * prm.term[2].ld : nullptr;
-    float sq[3] = {0.0f, 0.0f, 0.0f};
-    const bool n0 = y0 && prm.term[0].norm_w, n1 = y1 && prm.term[1].norm_w, n2 = y2 && prm.term[2].norm_w;
-    if (n0 || n1 || n2) {
-        for (int c = tid; c < width; c += kDecThreads) {
-            if (n0) sq[0] = fmaf(y0[c], y0[c], sq[0]);
-            if (n1) sq[1] = fmaf(y1[c], y1[c], sq[1]);
-            if (n2) sq[2] = fmaf(y2[c], y2[c], sq[2]);
-        }
-        block_sums<3>(sq, sh_red);
+    const int vectors = static_cast<int>(prm.ld_h >> 2);
+    const float* y_row[3];
+    bool normed[3];
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+        y_row[i] = i < prm.terms ? prm.term[i].y + src * prm.term[i].ld : nullptr;
+        normed[i] = i < prm.terms && prm.term[i].norm_w;
     }
-    const float inv_width = 1.0f / static_cast<float>(width);
-    const float f0 = y0 ? prm.term[0].scale * (n0 ? 1.0f / sqrtf(sq[0] * inv_width + prm.eps) : 1.0f) : 0.0f;
-    const float f1 = y1 ? prm.term[1].scale * (n1 ? 1.0f / sqrtf(sq[1] * inv_width + prm.eps) : 1.0f) : 0.0f;
-    const float f2 = y2 ? prm.term[2].scale * (n2 ? 1.0f / sqrtf(sq[2] * inv_width + prm.eps) : 1.0f) : 0.0f;
     const uint16_t* embedding = nullptr;
-    if (!prm.x_in) {
-        const int token = min(max(prm.tokens[src], 0), prm.vocab - 1);
-        embedding = prm.embed + static_cast<int64_t>(token) * width;
+    if (!prm.x_in) embedding = prm.embed + min(max(prm.tokens[src], 0), prm.vocab - 1) * prm.ld_h;
+    const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f), one = make_float4(1.0f, 1.0f, 1.0f, 1.0f);
+    float4 x[NV], y[3][NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int v = tid + i * kDecThreads;
+        const bool in = v < vectors;
+        x[i] = !in ? zero : embedding ? load4(embedding, v) : load4(prm.x_in + src * prm.ld_h, v);
+#pragma unroll
+        for (int t = 0; t < 3; ++t) y[t][i] = in && y_row[t] ? load4(y_row[t], v) : zero;
+    }
+    const float inv_width = 1.0f / static_cast<float>(prm.width);
+    float factor[3] = {0.0f, 0.0f, 0.0f};
+    if (normed[0] || normed[1] || normed[2]) {
+#pragma unroll
+        for (int t = 0; t < 3; ++t)
+#pragma unroll
+            for (int i = 0; i < NV; ++i) factor[t] = square_sum(y[t][i], factor[t]);
+        block_sums<3>(factor, sh_red);
+    }
+#pragma unroll
+    for (int t = 0; t < 3; ++t) {
+        const float inverse = normed[t] ? 1.0f / sqrtf(factor[t] * inv_width + prm.eps) : 1.0f;
+        factor[t] = t < prm.terms ? prm.term[t].scale * inverse : 0.0f;
     }
     float total[1] = {0.0f};
-    for (int c = tid; c < width; c += kDecThreads) {
-        float x = embedding ? bf2f(embedding[c]) : prm.x_in[src * width + c];
-        float add = 0.0f;
-        if (y0) add = fmaf(f0 * y0[c], n0 ? prm.term[0].norm_w[c] : 1.0f, add);
-        if (y1) add = fmaf(f1 * y1[c], n1 ? prm.term[1].norm_w[c] : 1.0f, add);
-        if (y2) add = fmaf(f2 * y2[c], n2 ? prm.term[2].norm_w[c] : 1.0f, add);
-        x += add;
-        if (prm.step_vec) x += prm.step_vec[c];
-        sh_x[c] = x;
-        if (write_x && prm.x_out) prm.x_out[static_cast<int64_t>(row) * width + c] = x;
-        total[0] = fmaf(x, x, total[0]);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int v = tid + i * kDecThreads;
+        if (v >= vectors) continue;
+        float4 add = zero;
+#pragma unroll
+        for (int t = 0; t < 3; ++t)
+            if (y_row[t]) add = weighted(add, factor[t], y[t][i], normed[t] ? load4(prm.term[t].norm_w, v) : one);
+        x[i] = weighted(x[i], 1.0f, add, one);
+        if (prm.step_vec) x[i] = weighted(x[i], 1.0f, load4(prm.step_vec, v), one);
+        if (write_x && prm.x_out) reinterpret_cast<float4*>(prm.x_out + static_cast<int64_t>(row) * prm.ld_h)[v] = x[i];
+        total[0] = square_sum(x[i], total[0]);
     }
     block_sums<1>(total, sh_red + 12);
     const float inverse = 1.0f / sqrtf(total[0] * inv_width + prm.eps);
-    for (int c = tid; c < prm.ld_h; c += kDecThreads)
-        h[c] = c < width ? from_f32<T>(sh_x[c] * inverse * prm.norm_w[c]) : from_f32<T>(0.0f);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int v = tid + i * kDecThreads;
+        if (v >= vectors) continue;
+        const float4 w = load4(prm.norm_w, v);
+        store4(h, v, x[i].x * inverse * w.x, x[i].y * inverse * w.y, x[i].z * inverse * w.z, x[i].w * inverse * w.w);
+    }
 }
 
 // One row of the gated norm by a block of 256 threads; sh_red: 4 floats of LDS.
@@ -108,7 +142,30 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
     const float* gate = prm.gate + row * prm.ld_gate;
     const int total = prm.groups * prm.size;
     const float inv_size = 1.0f / static_cast<float>(prm.size);
-    if (prm.groups == 1) {
+    constexpr int kHeld = 4;                   // float4s a thread holds between its two uses of a value
+    if (prm.groups == 1 && total % 4 == 0 && prm.ld_o % 4 == 0 && total <= kHeld * 4 * kDecThreads) {
+        const int vectors = total >> 2;
+        float4 held[kHeld], g[kHeld];
+        float sq[1] = {0.0f};
+#pragma unroll
+        for (int i = 0; i < kHeld; ++i) {
+            const int v = tid + i * kDecThreads;
+            if (v >= vectors) continue;
+            held[i] = load4(o, v);
+            g[i] = load4(gate, v);
+            sq[0] = square_sum(held[i], sq[0]);
+        }
+        block_sums<1>(sq, sh_red);
+        const float inverse = 1.0f / sqrtf(sq[0] * inv_size + prm.eps);
+#pragma unroll
+        for (int i = 0; i < kHeld; ++i) {
+            const int v = tid + i * kDecThreads;
+            if (v >= vectors) continue;
+            const float4 w = load4(prm.weight, v);
+            store4(out, v, held[i].x * inverse * w.x * sigmoid_f32(g[i].x), held[i].y * inverse * w.y * sigmoid_f32(g[i].y),
+                   held[i].z * inverse * w.z * sigmoid_f32(g[i].z), held[i].w * inverse * w.w * sigmoid_f32(g[i].w));
+        }
+    } else if (prm.groups == 1) {
         float sq[1] = {0.0f};
         for (int c = tid; c < total; c += kDecThreads) sq[0] = fmaf(o[c], o[c], sq[0]);
         block_sums<1>(sq, sh_red);
@@ -116,14 +173,25 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
         for (int c = tid; c < total; c += kDecThreads)
             out[c] = from_f32<T>(o[c] * inverse * prm.weight[c] * sigmoid_f32(gate[c]));
     } else {
+        // a wave per slice, a slice of up to 256 values held by its lanes
         for (int g = wave; g < prm.groups; g += kDecThreads / 64) {
-            float sq = 0.0f;
-            for (int c = lane; c < prm.size; c += 64) {
-                const float v = o[g * prm.size + c];
-                sq = fmaf(v, v, sq);
+            float held[4], gates[4], sq = 0.0f;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int c = lane + 64 * i;
+                const bool in = c < prm.size;
+                held[i] = in ? o[g * prm.size + c] : 0.0f;
+                gates[i] = in ? gate[g * prm.size + c] : 0.0f;
+                sq = fmaf(held[i], held[i], sq);
             }
+            for (int c = lane + 256; c < prm.size; c += 64) sq = fmaf(o[g * prm.size + c], o[g * prm.size + c], sq);
             const float inverse = 1.0f / sqrtf(wave_sum(sq) * inv_size + prm.eps);
-            for (int c = lane; c < prm.size; c += 64) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int c = lane + 64 * i, at = g * prm.size + c;
+                if (c < prm.size) out[at] = from_f32<T>(held[i] * inverse * prm.weight[at] * sigmoid_f32(gates[i]));
+            }
+            for (int c = lane + 256; c < prm.size; c += 64) {
                 const int at = g * prm.size + c;
                 out[at] = from_f32<T>(o[at] * inverse * prm.weight[at] * sigmoid_f32(gate[at]));
             }

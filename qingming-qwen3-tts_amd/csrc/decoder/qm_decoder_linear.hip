@@ -4,6 +4,8 @@
 // Bound by HBM: every weight is read once per group of R rows.  A wave owns NR weight rows and streams them 16 bytes a
 // lane, `kDotAhead` pieces of each row requested before the first is used; the input rows live in LDS as T.  Sums are fp32
 // (packed bf16 dot products, or fmaf in the 32-bit mode), combined over the wave's lanes at the end.
+#include <algorithm>
+
 #include "qm_decoder_device.h"
 #include "../qm_host.h"
 #include "../qm_linear_rows_params.h"
@@ -77,8 +79,10 @@ int32_t launch_decoder_linears(const DecLinearParams& prm, int f32, hipStream_t 
     for (int g = 0; g < prm.groups; ++g) matrix = matrix && prm.group[g].ldx == prm.group[g].k && prm.group[g].ldo == prm.group[g].n;
     if (!matrix) return streaming<uint16_t>(prm, stream);
     LinearRowsParams plain = {};
-    for (int g = 0; g < prm.groups; ++g) {
-        const DecLinearGroup& d = prm.group[g];
+    int order[kDecGroups] = {0, 1, 2};         // long reductions first
+    std::stable_sort(order, order + prm.groups, [&](int a, int b) { return prm.group[a].k > prm.group[b].k; });
+    for (int i = 0; i < prm.groups; ++i) {
+        const DecLinearGroup& d = prm.group[order[i]];
         if (d.w_up) {
             LinearRowsParams pair = {};
             pair.input = static_cast<const uint16_t*>(d.x);
@@ -108,6 +112,7 @@ int32_t launch_decoder_linears(const DecLinearParams& prm, int f32, hipStream_t 
         }
         ++plain.groups;
     }
+    plain.linear_by_linear = plain.groups > 1;
     return plain.groups ? launch_rows_mfma(plain, false, stream) : QM_OK;
 }
 

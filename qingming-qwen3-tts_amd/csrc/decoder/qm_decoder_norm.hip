@@ -6,12 +6,11 @@
 
 namespace qm {
 
-template <class T>
+template <class T, int NV>
 __global__ __launch_bounds__(kDecThreads) void residual_norm_kernel(ResidualParams prm) {
-    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     __shared__ float sh_red[16];
     const int row = static_cast<int>(blockIdx.x);
-    residual_norm_row<T>(prm, row, reinterpret_cast<float*>(smem), sh_red, static_cast<T*>(prm.h) + row * prm.ld_h, true);
+    residual_norm_row<T, NV>(prm, row, sh_red, static_cast<T*>(prm.h) + row * prm.ld_h, true);
 }
 
 template <class T>
@@ -21,15 +20,35 @@ __global__ __launch_bounds__(kDecThreads) void gated_norm_kernel(GatedNormParams
     gated_norm_row<T>(prm, row, sh_red, static_cast<T*>(prm.out) + row * prm.ld_out);
 }
 
-int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream) {
-    if (rows < 0 || prm.width <= 0 || prm.ld_h < prm.width || prm.terms < 0 || prm.terms > 3) return QM_ERR_ARGUMENT;
-    if (!prm.h || !prm.norm_w || (!prm.x_in && (!prm.embed || !prm.tokens))) return QM_ERR_NULL;
-    if (prm.width > kDecMaxWidth) return QM_ERR_GEOMETRY;
-    if (rows == 0) return QM_OK;
-    const size_t lds = static_cast<size_t>(prm.width) * sizeof(float);
-    if (f32) hipLaunchKernelGGL(residual_norm_kernel<float>, dim3(rows), dim3(kDecThreads), lds, stream, prm);
-    else hipLaunchKernelGGL(residual_norm_kernel<uint16_t>, dim3(rows), dim3(kDecThreads), lds, stream, prm);
+int32_t check_residual(const ResidualParams& prm) {
+    if (prm.width <= 0 || prm.ld_h < prm.width || prm.terms < 0 || prm.terms > 3) return QM_ERR_ARGUMENT;
+    if (!prm.norm_w || (!prm.x_in && (!prm.embed || !prm.tokens))) return QM_ERR_NULL;
+    if (prm.ld_h % 4 || prm.ld_h > kDecMaxWidth) return QM_ERR_GEOMETRY;
+    for (int i = 0; i < prm.terms; ++i) {
+        if (!prm.term[i].y) return QM_ERR_NULL;
+        if (prm.term[i].ld < prm.ld_h || prm.term[i].ld % 4) return QM_ERR_GEOMETRY;
+    }
+    return QM_OK;
+}
+
+template <class T>
+static int32_t residual_as(const ResidualParams& prm, int rows, hipStream_t stream) {
+    switch (row_vectors(prm.ld_h)) {
+        case 1: hipLaunchKernelGGL((residual_norm_kernel<T, 1>), dim3(rows), dim3(kDecThreads), 0, stream, prm); break;
+        case 2: hipLaunchKernelGGL((residual_norm_kernel<T, 2>), dim3(rows), dim3(kDecThreads), 0, stream, prm); break;
+        case 4: hipLaunchKernelGGL((residual_norm_kernel<T, 4>), dim3(rows), dim3(kDecThreads), 0, stream, prm); break;
+        default: hipLaunchKernelGGL((residual_norm_kernel<T, 12>), dim3(rows), dim3(kDecThreads), 0, stream, prm); break;
+    }
     return launch_status();
+}
+
+int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream) {
+    const int32_t rc = check_residual(prm);
+    if (rc != QM_OK) return rc;
+    if (rows < 0) return QM_ERR_ARGUMENT;
+    if (!prm.h) return QM_ERR_NULL;
+    if (rows == 0) return QM_OK;
+    return f32 ? residual_as<float>(prm, rows, stream) : residual_as<uint16_t>(prm, rows, stream);
 }
 
 int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStream_t stream) {

@@ -10,9 +10,11 @@
 
 namespace qm {
 
-constexpr int kDecMaxWidth = 12288;       // columns of the residual stream (a row lives in LDS)
+constexpr int kDecMaxWidth = 12288;       // columns of the residual stream (a block's threads hold a row)
 constexpr int kDecMaxSplits = 64;         // key splits of one attention (a wave's lanes combine them)
 constexpr int kDecMaxHead = 256;          // channels of a head
+constexpr int kAttentionMatrixRows = 16;  // rows from which bf16 attention goes to the matrix cores
+constexpr int kChunkedRows = 16;          // rows from which a recurrence is computed in chunks (given scratch)
 constexpr int kDecGroups = 3;             // linears in one launch
 constexpr int kDotLdsMost = 159 * 1024;   // dynamic LDS of one block
 
@@ -31,7 +33,11 @@ using DeltaParams = qm_general_delta;
 constexpr int kDecayChunk = QM_DECAY_CHUNK;
 constexpr int kDecayPowers = QM_DECAY_POWERS;
 
+// float4s of a row that each of a block's 256 threads holds: the kernels' choices for a row of ld columns.
+inline int row_vectors(int64_t ld) { return ld <= 1024 ? 1 : ld <= 2048 ? 2 : ld <= 4096 ? 4 : 12; }
+
 // Whether the kernels take these arguments.
+int32_t check_residual(const ResidualParams& prm);
 int32_t check_attention(const ChunkAttentionParams& prm);
 int32_t check_decay_attention(const DecayAttentionParams& prm);
 int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipStream_t stream);
@@ -41,10 +47,14 @@ int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStre
 int32_t launch_decoder_linears(const DecLinearParams& prm, int f32, hipStream_t stream);
 // Rotation and cache write, then the attention.
 int32_t launch_chunk_attention(const ChunkAttentionParams& prm, int f32, hipStream_t stream);
+int32_t launch_chunk_attention_mfma(const ChunkAttentionParams& prm, hipStream_t stream);
 int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stream);
 // Floats of scratch with which a pass of `rows` tokens is computed in chunks (0: it is not).
 int64_t decay_scratch_floats(int rows, int heads, int dim, int vdim);
 int64_t delta_scratch_floats(int rows, int heads, int dim);
+bool delta_chunks_fit(const DeltaParams& prm);
+int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream);
+int32_t launch_delta_chunks(const DeltaParams& prm, hipStream_t stream);
 int32_t launch_general_delta(const DeltaParams& prm, hipStream_t stream);
 
 // ---- one token: a layer run in three launches -----------------------------------------------------------------------

@@ -86,15 +86,18 @@ __device__ __forceinline__ void decay_attention_block(const DecayAttentionParams
     store_state<RD>(s, state, prm.dim, prm.vdim, sub, column);
 }
 
-__host__ __device__ inline int delta_lds_floats(int rd, int rank) { return kRecTokens * (5 * rec_stride(rd) + rank); }
+__host__ __device__ inline int delta_lds_floats(int rd, int rank) { return kRecTokens * (5 * rec_stride(rd) + 1 + rank); }
 
-// What enters the delta rule's recurrence for channel c of a head at one token, given tanh of the token's rank-sized
-// projection in LDS: the decay of the channel and the removal rate.
+// exp(-exp(-1/2) sigmoid(z))
+__device__ __forceinline__ float delta_decay_of(float z) { return expf(-0.60653065971263342f * sigmoid_f32(z)); }
+
+// The decay of channel `at` (of all heads') at one token, given tanh of the token's rank-sized projection in LDS.
 __device__ __forceinline__ float delta_channel_decay(const DeltaParams& prm, const float* tanh_z, int at) {
     float z = prm.w0[at];
     const int all = prm.heads * prm.dim;
+#pragma unroll 16
     for (int r = 0; r < prm.rank; ++r) z = fmaf(prm.w2[static_cast<int64_t>(r) * all + at], tanh_z[r], z);
-    return expf(-0.60653065971263342f * sigmoid_f32(z));          // exp(-1/2) = 0.6065...
+    return delta_decay_of(z);
 }
 
 // Generalized delta rule: head `head`, state columns [64 slice, 64 slice + 64).
@@ -104,7 +107,8 @@ __device__ __forceinline__ void general_delta_block(const DeltaParams& prm, int 
     const int column = slice * kRecColumns + wave * 16 + (lane & 15);
     constexpr int kStride = 4 * (RD + 4);
     float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.dim;
-    float* tanh_z = lds + kRecTokens * 5 * kStride;
+    float* inverse = lds + kRecTokens * 5 * kStride;              // [kRecTokens]
+    float* tanh_z = inverse + kRecTokens;                          // [kRecTokens][rank]
     float s[RD];
     load_state<RD>(s, state, prm.dim, prm.dim, sub, column);
     for (int t0 = 0; t0 < prm.rows; t0 += kRecTokens) {
@@ -115,28 +119,28 @@ __device__ __forceinline__ void general_delta_block(const DeltaParams& prm, int 
             tanh_z[i] = tanhf(prm.proj[(t0 + t) * prm.ld_proj + prm.z_column + r]);
         }
         __syncthreads();
-        for (int t = wave; t < tokens; t += 4) {                   // a wave per token: w, a u, u, k, r of the head
-            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim;
-            float* to = lds + t * 5 * kStride;
+        for (int t = wave; t < tokens; t += 4) {                   // a wave per token: the unit key's factor
+            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim + prm.k_column;
             float sq = 0.0f;
-            for (int c = lane; c < prm.dim; c += 64) {
-                const float k = p[prm.k_column + c];
-                sq = fmaf(k, k, sq);
+            for (int c = lane; c < prm.dim; c += 64) sq = fmaf(p[c], p[c], sq);
+            sq = wave_sum(sq);
+            if (lane == 0) inverse[t] = 1.0f / sqrtf(sq + prm.unit_eps);
+        }
+        __syncthreads();
+        for (int i = tid; i < tokens * 4 * RD; i += kDecThreads) { // w, a u, u, k, r of every token and channel of the head
+            const int t = i / (4 * RD), c = i % (4 * RD);
+            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim + c;
+            float w = 0.0f, au = 0.0f, u = 0.0f, k = 0.0f, r = 0.0f;
+            if (c < prm.dim) {
+                const int at = head * prm.dim + c;
+                k = p[prm.k_column];
+                r = p[prm.r_column];
+                u = k * inverse[t];
+                au = sigmoid_f32(p[prm.a_column] + prm.a_bias[at]) * u;
+                w = delta_channel_decay(prm, tanh_z + t * prm.rank, at);
             }
-            const float inverse = 1.0f / sqrtf(wave_sum(sq) + prm.unit_eps);
-            for (int c = lane; c < 4 * RD; c += 64) {
-                float w = 0.0f, au = 0.0f, u = 0.0f, k = 0.0f, r = 0.0f;
-                if (c < prm.dim) {
-                    const int at = head * prm.dim + c;
-                    w = delta_channel_decay(prm, tanh_z + t * prm.rank, at);
-                    k = p[prm.k_column + c];
-                    r = p[prm.r_column + c];
-                    u = k * inverse;
-                    au = sigmoid_f32(p[prm.a_column + c] + prm.a_bias[at]) * u;
-                }
-                float* put = to + rec_at<RD>(c);
-                put[0] = w; put[kStride] = au; put[2 * kStride] = u; put[3 * kStride] = k; put[4 * kStride] = r;
-            }
+            float* put = lds + t * 5 * kStride + rec_at<RD>(c);
+            put[0] = w; put[kStride] = au; put[2 * kStride] = u; put[3 * kStride] = k; put[4 * kStride] = r;
         }
         float v[kRecTokens];
 #pragma unroll

@@ -34,6 +34,7 @@ int32_t check_decay_attention(const DecayAttentionParams& prm) {
 int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stream) {
     const int32_t rc = check_decay_attention(prm);
     if (rc != QM_OK || prm.rows == 0) return rc;
+    if (prm.scratch && prm.rows >= kChunkedRows) return launch_decay_chunks(prm, stream);
     if (prm.dim <= 32) return decay_as<8>(prm, stream);
     if (prm.dim <= 64) return decay_as<16>(prm, stream);
     if (prm.dim <= 128) return decay_as<32>(prm, stream);
@@ -56,13 +57,11 @@ int32_t launch_general_delta(const DeltaParams& prm, hipStream_t stream) {
     if (prm.rows < 0) return QM_ERR_ARGUMENT;
     if (prm.heads <= 0 || prm.heads > 65535 || prm.dim <= 0 || prm.dim > kDecMaxHead || prm.rank <= 0 || prm.rank > 1024) return QM_ERR_GEOMETRY;
     if (prm.rows == 0) return QM_OK;
+    if (prm.scratch && prm.rows >= kChunkedRows && delta_chunks_fit(prm)) return launch_delta_chunks(prm, stream);
     if (prm.dim <= 32) return delta_as<8>(prm, stream);
     if (prm.dim <= 64) return delta_as<16>(prm, stream);
     if (prm.dim <= 128) return delta_as<32>(prm, stream);
     return delta_as<64>(prm, stream);
 }
-
-int64_t decay_scratch_floats(int rows, int heads, int dim, int vdim) { return 0; }
-int64_t delta_scratch_floats(int rows, int heads, int dim) { return 0; }
 
 }  // namespace qm

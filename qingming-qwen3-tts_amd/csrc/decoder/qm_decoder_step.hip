@@ -15,19 +15,18 @@ constexpr int kInRows = 4;                     // weight rows per wave: input li
 constexpr int kOutRows = 2;                    // output linears (few, long rows)
 constexpr int kInBlocks = 1024;                // most blocks of the input launch: each repeats the norm
 
-template <class T>
+template <class T, int NV>
 __global__ __launch_bounds__(kDecThreads) void layer_in_kernel(LayerInParams prm, int tiles) {
     request_arguments(prm);
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     __shared__ float sh_red[16];
     T* hs = reinterpret_cast<T*>(smem);                                        // [ld_h]
-    float* sh_x = reinterpret_cast<float*>(hs + prm.residual.ld_h);            // [width]
     int tile = static_cast<int>(blockIdx.x);
     int g = dot_group<kInRows>(prm.linears, tile);
     DotRows<kInRows> d = dot_rows<kInRows>(prm.linears.group[g], tile);
     uint4 piece[kDotAhead][kInRows];
     dot_request<kInRows>(d, prm.linears.group[g].k, piece);
-    residual_norm_row<T>(prm.residual, 0, sh_x, sh_red, hs, blockIdx.x == 0);
+    residual_norm_row<T, NV>(prm.residual, 0, sh_red, hs, blockIdx.x == 0);
     __syncthreads();
     for (int next = static_cast<int>(blockIdx.x) + static_cast<int>(gridDim.x);; next += static_cast<int>(gridDim.x)) {
         dot_finish<T, 1, kInRows>(prm.linears.group[g], d, piece, hs, 0, 1);
@@ -132,16 +131,21 @@ static int most_k(const DecLinearParams& prm) {
     return k;
 }
 
-template <class T>
+template <class T, int NV>
 static int32_t layer_in_as(const LayerInParams& prm, hipStream_t stream) {
     const int tiles = dot_tiles_of<kInRows>(prm.linears);
-    const size_t lds = static_cast<size_t>(prm.residual.ld_h) * sizeof(T) + static_cast<size_t>(prm.residual.width) * sizeof(float);
-    static std::atomic<bool> raised[kMaxDevices];
-    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(layer_in_kernel<T>), kDotLdsMost, raised);
-    if (rc != QM_OK) return rc;
-    if (lds > static_cast<size_t>(kDotLdsMost)) return QM_ERR_GEOMETRY;
-    hipLaunchKernelGGL(layer_in_kernel<T>, dim3(tiles < kInBlocks ? tiles : kInBlocks), dim3(kDecThreads), lds, stream, prm, tiles);
+    const size_t lds = static_cast<size_t>(prm.residual.ld_h) * sizeof(T);
+    hipLaunchKernelGGL((layer_in_kernel<T, NV>), dim3(tiles < kInBlocks ? tiles : kInBlocks), dim3(kDecThreads), lds, stream, prm, tiles);
     return launch_status();
+}
+template <class T>
+static int32_t layer_in(const LayerInParams& prm, hipStream_t stream) {
+    switch (row_vectors(prm.residual.ld_h)) {
+        case 1: return layer_in_as<T, 1>(prm, stream);
+        case 2: return layer_in_as<T, 2>(prm, stream);
+        case 4: return layer_in_as<T, 4>(prm, stream);
+        default: return layer_in_as<T, 12>(prm, stream);
+    }
 }
 
 int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream) {
@@ -151,8 +155,9 @@ int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream) {
         if (!d.w || (d.w_up ? !d.out : !d.out32)) return QM_ERR_NULL;
         if (d.n <= 0 || d.n % 128 || d.k % 128 || d.k != prm.residual.ld_h) return QM_ERR_GEOMETRY;
     }
-    if (prm.residual.width > kDecMaxWidth || prm.residual.width > prm.residual.ld_h) return QM_ERR_GEOMETRY;
-    return f32 ? layer_in_as<float>(prm, stream) : layer_in_as<uint16_t>(prm, stream);
+    const int32_t rc = check_residual(prm.residual);
+    if (rc != QM_OK) return rc;
+    return f32 ? layer_in<float>(prm, stream) : layer_in<uint16_t>(prm, stream);
 }
 
 template <class T>

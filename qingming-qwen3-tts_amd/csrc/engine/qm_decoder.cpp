@@ -86,8 +86,8 @@ struct qm_decoder {
     std::vector<qm_engine::DeviceBuffer> memory;    // one per sequence
     std::vector<int> length;                        // tokens of each live sequence, -1: free
     size_t sequence_bytes = 0;
-    qm_engine::DeviceBuffer embed, final_norm, loop_step;
-    qm_engine::Matrix head;
+    qm_engine::DeviceBuffer final_norm, loop_step;
+    qm_engine::Matrix embed, head;
     int capacity = 0, max_rows = 0, f32 = 0, path = 0;
     bool warm = false;
     int width_p = 0, vocab_p = 0;
@@ -127,9 +127,15 @@ public:
     }
     // a vector, or a small matrix, as fp32
     DeviceBuffer floats(const std::string& name, const std::vector<int64_t>& shape) const {
+        return padded_floats(name, shape, static_cast<int>(shape.back()));
+    }
+    // the same with zeros behind each row, up to `columns`
+    DeviceBuffer padded_floats(const std::string& name, const std::vector<int64_t>& shape, int columns) const {
         const TensorView& t = get(name, shape);
-        std::vector<float> host(t.elements());
-        for (size_t i = 0; i < host.size(); ++i) host[i] = element(t, i);
+        const size_t from = static_cast<size_t>(shape.back()), rows = t.elements() / from;
+        std::vector<float> host(rows * columns, 0.0f);
+        for (size_t r = 0; r < rows; ++r)
+            for (size_t c = 0; c < from; ++c) host[r * columns + c] = element(t, r * from + c);
         return upload(host.data(), host.size() * sizeof(float));
     }
     DeviceBuffer transposed_floats(const std::string& name, int64_t rows, int64_t columns) const {
@@ -185,7 +191,7 @@ DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, in
     DecoderLayer w;
     w.config = config;
     const std::string base = "l" + std::to_string(index) + ".", mix = base + "mix.";
-    w.norm1 = from.floats(base + "norm1", {width});
+    w.norm1 = from.padded_floats(base + "norm1", {width}, padded(width, 128));
     if (config.mixer == MixerKind::AttentionBesideDecay) {
         const ChunkAttentionConfig& a = config.attention;
         const DecayAttentionConfig& d = config.decay;
@@ -196,8 +202,8 @@ DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, in
         w.o_left = from.matrix(mix + "left.o", width, a.heads * a.vdim);
         w.o_right = from.matrix(mix + "right.o", width, d.heads * d.vdim);
         w.mix_norm = from.floats(mix + "right.norm", {d.heads * d.vdim});
-        w.out_left = from.floats(mix + "left.out", {width});
-        w.out_right = from.floats(mix + "right.out", {width});
+        w.out_left = from.padded_floats(mix + "left.out", {width}, padded(width, 128));
+        w.out_right = from.padded_floats(mix + "right.out", {width}, padded(width, 128));
         std::vector<double> frequency(static_cast<size_t>(std::max(1, a.rot_dims / 2)), 0.0);
         for (int i = 0; i < a.rot_dims / 2; ++i) frequency[static_cast<size_t>(i)] = std::pow(a.rot_base, -2.0 * i / a.rot_dims);
         w.frequency = Loader::upload(frequency.data(), frequency.size() * sizeof(double));
@@ -241,7 +247,7 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
     d->max_rows = std::min(capacity, max_rows ? max_rows : 2048);
     d->f32 = f32;
     const int width = d->config.width;
-    if (width > qm::kDecMaxWidth) throw ApiError(QM_ERR_GEOMETRY, "model width beyond the kernels' limit");
+    if (padded(width, 128) > qm::kDecMaxWidth) throw ApiError(QM_ERR_GEOMETRY, "model width beyond the kernels' limit");
     d->stream = stream;
     if (!stream) {
         hip_check(hipStreamCreateWithFlags(&d->stream, hipStreamNonBlocking), "decoder stream");
@@ -250,13 +256,10 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
     const Loader from(dir);
     d->width_p = padded(width, 128);
     d->vocab_p = padded(d->config.vocab, 128);
-    {
-        const TensorView& t = from.get("embed", {d->config.vocab, width});
-        d->embed = Loader::upload(t.data, t.bytes);
-    }
-    d->final_norm = from.floats("final.norm", {width});
+    d->embed = from.matrix("embed", d->config.vocab, width);
+    d->final_norm = from.padded_floats("final.norm", {width}, d->width_p);
     d->head = from.matrix("head", d->config.vocab, width);
-    if (d->config.loop_times) d->loop_step = from.floats("loop.step", {d->config.loop_times, width});
+    if (d->config.loop_times) d->loop_step = from.padded_floats("loop.step", {d->config.loop_times, width}, d->width_p);
     for (size_t i = 0; i < d->config.layers.size(); ++i)
         d->layers.push_back(load_layer(from, d->config.layers[i], static_cast<int>(i), width));
 
@@ -317,7 +320,7 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
         hip_check(hipMemset(b.raw(), 0, b.bytes()), "activation reset");
         return b;
     };
-    const size_t stream_floats = rows * static_cast<size_t>(width);
+    const size_t stream_floats = rows * static_cast<size_t>(d->width_p);
     d->x[0] = zeros(stream_floats * 4);
     d->x[1] = zeros(stream_floats * 4);
     d->h = zeros(rows * d->width_p * item);
@@ -371,7 +374,7 @@ float* f32_of(const DeviceBuffer& b) { return static_cast<float*>(b.raw()); }
 char* at_of(const DeviceBuffer& b, size_t offset) { return static_cast<char*>(b.raw()) + offset; }
 
 const float* step_vec_of(const qm_decoder& d, const LayerRun& run) {
-    return run.opens_pass < 0 ? nullptr : f32_of(d.loop_step) + static_cast<size_t>(run.opens_pass) * d.config.width;
+    return run.opens_pass < 0 ? nullptr : f32_of(d.loop_step) + static_cast<size_t>(run.opens_pass) * d.width_p;
 }
 
 qm_chunk_attention attention_of(const qm_decoder& d, const DecoderLayer& w, const RunState& s, int sequence, int rows, int position) {
@@ -395,6 +398,7 @@ qm_chunk_attention attention_of(const qm_decoder& d, const DecoderLayer& w, cons
     p.rot_dims = a.rot_dims;
     p.k_column = w.k.at; p.v_column = w.v.at;
     p.scale = static_cast<float>(a.scale);
+    p.options = d.path & 4 ? QM_ATTENTION_ROWS : 0;
     p.part.ml = f32_of(d.ml);
     p.part.acc = f32_of(d.acc);
     p.part.heads = a.heads; p.part.vdim = a.vdim;
@@ -523,8 +527,9 @@ void run_layers(qm_decoder& d, int sequence, int rows, int position, const float
             // the stream behind this run, before anything is added ahead of the next one
             op_check(qm::launch_residual_norm(residual_of(d, pending, x, f32_of(d.tap), nullptr, f32_of(d.final_norm), d.tap_h.raw()), rows, d.f32, s),
                      "stream");
-            const size_t floats = static_cast<size_t>(rows) * d.config.width;
-            hip_check(hipMemcpyAsync(taps + i * floats, d.tap.raw(), floats * 4, hipMemcpyDeviceToHost, s), "stream read");
+            const size_t row_bytes = static_cast<size_t>(d.config.width) * 4;
+            hip_check(hipMemcpy2DAsync(taps + i * rows * d.config.width, row_bytes, d.tap.raw(), static_cast<size_t>(d.width_p) * 4, row_bytes,
+                                       static_cast<size_t>(rows), hipMemcpyDeviceToHost, s), "stream read");
             hip_check(hipStreamSynchronize(s), "stream read");
         }
     }
@@ -675,7 +680,7 @@ void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const i
         if (want[i] < 0 || want[i] >= count) throw ApiError(QM_ERR_ARGUMENT, "a wanted place is outside the step");
     if (streams && count > d.max_rows) throw ApiError(QM_ERR_ARGUMENT, "streams of one pass only");
     if (streams && !d.tap.raw()) {
-        d.tap = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.config.width * 4);
+        d.tap = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.width_p * 4);
         d.tap_h = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.width_p * 4);
     }
     if (count == 1 && !streams) {

@@ -160,9 +160,19 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
     const int wave_n = BM == 128 ? (wave & 1) : wave;
     const int wave_m = BM == 128 ? (wave >> 1) : 0;
     int K = prm.reduction;
-    const int m0 = static_cast<int>(blockIdx.y) * BM;
+    int m0 = static_cast<int>(blockIdx.y) * BM;
     // (several linears of one input in one grid: which of them this block's column tile belongs to)
     int tile = static_cast<int>(blockIdx.x);
+    if (!DUAL && prm.linear_by_linear) {
+        int at = static_cast<int>(blockIdx.y * gridDim.x + blockIdx.x), first = 0, next = prm.group_first_tile[0];
+        for (int g = 1; g < prm.groups && at >= static_cast<int>(gridDim.y) * (next - first); ++g) {
+            at -= static_cast<int>(gridDim.y) * (next - first);
+            first = next;
+            next = g + 1 < prm.groups ? prm.group_first_tile[g] : static_cast<int>(gridDim.x);
+        }
+        tile = first + at % (next - first);
+        m0 = at / (next - first) * BM;
+    }
     const uint16_t* weight0 = prm.weight[0];
     const uint16_t* input = prm.input;
     const uint16_t* bias = prm.bias;

@@ -35,6 +35,9 @@ struct LinearRowsParams {
     // a linear of its own input and reduction (a multiple of 128 as well): NULL / 0 = the first one's
     const uint16_t* group_input[2];
     int group_reduction[2];
+    // blocks in the order linear by linear (all row tiles of the first, then of the next) instead of row tile by row
+    // tile: the linears with the long reductions first, so that none of them starts late
+    int linear_by_linear;
 };
 
 // The row linears on the matrix cores (qm_linear_rows_mfma.hip).  `dual`: weight[0] / weight[1] are the gate and up

@@ -29,7 +29,7 @@ DecoderLinear = _structure("DecoderLinear", *_same(_P, "x w w_up out32 out"), *_
 AttentionPartials = _structure("AttentionPartials", *_same(_P, "ml acc"), *_same(_I32, "heads vdim splits keys_per_split"))
 ChunkAttention = _structure("ChunkAttention", *_same(_P, "proj frequency q_rot k_cache v_cache out"), ("part", AttentionPartials),
                             ("position_dev", _P), *_same(_I64, "ld_proj ld_out"), *_same(_I32, "position rows"),
-                            *_same(_I32, "heads kv_heads dim vdim k_stride v_stride ring chunk rot_dims k_column v_column"), ("scale", _F))
+                            *_same(_I32, "heads kv_heads dim vdim k_stride v_stride ring chunk rot_dims k_column v_column"), ("scale", _F), ("options", _I32), ("reserved", _I32))
 DecayAttention = _structure("DecayAttention", *_same(_P, "proj powers state out scratch"), *_same(_I64, "ld_proj scratch_floats"),
                             *_same(_I32, "rows heads dim vdim q_column k_column v_column reserved"))
 GeneralDelta = _structure("GeneralDelta", *_same(_P, "proj w2 w0 a_bias state out scratch"), *_same(_I64, "ld_proj scratch_floats"),
