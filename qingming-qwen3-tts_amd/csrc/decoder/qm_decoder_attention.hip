@@ -9,39 +9,61 @@
 
 namespace qm {
 
-// Rotation of the rows' queries and keys, keys and values into the ring: one block per row.
+// Rotation of the rows' queries and keys, keys and values into the ring: one block per row.  The row's projections pass
+// through LDS; a thread puts out eight channels at a time.
+__device__ __forceinline__ void store8(uint16_t* to, const float (&v)[8]) {
+    *reinterpret_cast<uint4*>(to) = make_uint4(pack_bf16_pair(v[0], v[1]), pack_bf16_pair(v[2], v[3]), pack_bf16_pair(v[4], v[5]), pack_bf16_pair(v[6], v[7]));
+}
+__device__ __forceinline__ void store8(float* to, const float (&v)[8]) {
+    reinterpret_cast<float4*>(to)[0] = make_float4(v[0], v[1], v[2], v[3]);
+    reinterpret_cast<float4*>(to)[1] = make_float4(v[4], v[5], v[6], v[7]);
+}
+
 template <class T>
 __global__ __launch_bounds__(kDecThreads) void rope_cache_kernel(ChunkAttentionParams prm) {
-    extern __shared__ float sh_turn[];         // [rot_dims / 2] cosines, then sines
+    extern __shared__ __attribute__((aligned(16))) float sh_row[];             // q, k, v; cosines; sines
     const int tid = threadIdx.x;
     const int row = static_cast<int>(blockIdx.x);
     const int position = position_of(prm.position_dev, prm.position) + row;
-    const int half = prm.rot_dims >> 1;
-    for (int i = tid; i < half; i += kDecThreads) rotary(position, prm.frequency[i], sh_turn[i], sh_turn[half + i]);
-    __syncthreads();
+    const int half = prm.rot_dims >> 1, q_n = prm.heads * prm.dim, k_n = prm.kv_heads * prm.dim, v_n = prm.kv_heads * prm.vdim;
+    float* sh_cos = sh_row + q_n + k_n + v_n;
+    float* sh_sin = sh_cos + half;
     const float* proj = prm.proj + row * prm.ld_proj;
-    auto channel = [&](const float* head, int c) {
-        if (c >= prm.dim) return 0.0f;
-        if (c >= prm.rot_dims) return head[c];
-        const int pair = c < half ? c : c - half;
-        const float u = head[pair], v = head[pair + half], cosine = sh_turn[pair], sine = sh_turn[half + pair];
-        return c < half ? u * cosine - v * sine : v * cosine + u * sine;
-    };
 #pragma unroll 4
-    for (int i = tid; i < prm.heads * prm.k_stride; i += kDecThreads) {
-        const int h = i / prm.k_stride, c = i - h * prm.k_stride;
-        static_cast<T*>(prm.q_rot)[static_cast<int64_t>(row) * prm.heads * prm.k_stride + i] = from_f32<T>(channel(proj + h * prm.dim, c));
-    }
+    for (int i = tid; i < q_n; i += kDecThreads) sh_row[i] = proj[i];
+#pragma unroll 4
+    for (int i = tid; i < k_n; i += kDecThreads) sh_row[q_n + i] = proj[prm.k_column + i];
+#pragma unroll 4
+    for (int i = tid; i < v_n; i += kDecThreads) sh_row[q_n + k_n + i] = proj[prm.v_column + i];
+    for (int i = tid; i < half; i += kDecThreads) rotary(position, prm.frequency[i], sh_cos[i], sh_sin[i]);
+    __syncthreads();
+    auto rotated = [&](const float* head, int c0, float (&v)[8]) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const int c = c0 + e;
+            const int pair = c < half ? c : c - half;
+            const bool turns = c < prm.rot_dims;
+            const float own = c < prm.dim ? head[c] : 0.0f;
+            const float other = turns ? head[c < half ? c + half : pair] : 0.0f;
+            const float cosine = turns ? sh_cos[pair] : 1.0f, sine = turns ? sh_sin[pair] : 0.0f;
+            v[e] = c < half ? own * cosine - other * sine : own * cosine + other * sine;
+        }
+    };
     const int64_t slot = position % prm.ring;
-    for (int i = tid; i < prm.kv_heads * prm.k_stride; i += kDecThreads) {
-        const int h = i / prm.k_stride, c = i - h * prm.k_stride;
-        static_cast<T*>(prm.k_cache)[(static_cast<int64_t>(h) * prm.ring + slot) * prm.k_stride + c] =
-            from_f32<T>(channel(proj + prm.k_column + h * prm.dim, c));
+    const int k_pieces = prm.k_stride >> 3, v_pieces = prm.v_stride >> 3;
+    for (int i = tid; i < (prm.heads + prm.kv_heads) * k_pieces; i += kDecThreads) {
+        const int h = i / k_pieces, c = (i - h * k_pieces) * 8;
+        float v[8];
+        rotated(sh_row + h * prm.dim, c, v);                                   // (the key heads follow the query heads)
+        store8(h < prm.heads ? static_cast<T*>(prm.q_rot) + (static_cast<int64_t>(row) * prm.heads + h) * prm.k_stride + c
+                             : static_cast<T*>(prm.k_cache) + (static_cast<int64_t>(h - prm.heads) * prm.ring + slot) * prm.k_stride + c, v);
     }
-    for (int i = tid; i < prm.kv_heads * prm.v_stride; i += kDecThreads) {
-        const int h = i / prm.v_stride, c = i - h * prm.v_stride;
-        static_cast<T*>(prm.v_cache)[(static_cast<int64_t>(h) * prm.ring + slot) * prm.v_stride + c] =
-            from_f32<T>(c < prm.vdim ? proj[prm.v_column + h * prm.vdim + c] : 0.0f);
+    for (int i = tid; i < prm.kv_heads * v_pieces; i += kDecThreads) {
+        const int h = i / v_pieces, c = (i - h * v_pieces) * 8;
+        float v[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = c + e < prm.vdim ? sh_row[q_n + k_n + h * prm.vdim + c + e] : 0.0f;
+        store8(static_cast<T*>(prm.v_cache) + (static_cast<int64_t>(h) * prm.ring + slot) * prm.v_stride + c, v);
     }
 }
 
@@ -72,10 +94,14 @@ int32_t check_attention(const ChunkAttentionParams& p) {
     return QM_OK;
 }
 
-int32_t launch_rope_cache(const ChunkAttentionParams& prm, int f32, hipStream_t stream) {
-    const size_t lds = static_cast<size_t>(prm.rot_dims + 2) * sizeof(float);
-    if (f32) hipLaunchKernelGGL(rope_cache_kernel<float>, dim3(prm.rows), dim3(kDecThreads), lds, stream, prm);
-    else hipLaunchKernelGGL(rope_cache_kernel<uint16_t>, dim3(prm.rows), dim3(kDecThreads), lds, stream, prm);
+template <class T>
+static int32_t rope_cache(const ChunkAttentionParams& prm, hipStream_t stream) {
+    const size_t lds = sizeof(float) * (static_cast<size_t>(prm.heads + prm.kv_heads) * prm.dim + static_cast<size_t>(prm.kv_heads) * prm.vdim + prm.rot_dims);
+    static std::atomic<bool> raised[kMaxDevices];
+    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(rope_cache_kernel<T>), kDotLdsMost, raised);
+    if (rc != QM_OK) return rc;
+    if (lds > static_cast<size_t>(kDotLdsMost)) return QM_ERR_GEOMETRY;
+    hipLaunchKernelGGL(rope_cache_kernel<T>, dim3(prm.rows), dim3(kDecThreads), lds, stream, prm);
     return launch_status();
 }
 
@@ -101,7 +127,7 @@ int32_t launch_chunk_attention(const ChunkAttentionParams& prm, int f32, hipStre
     int32_t rc = check_attention(prm);
     if (rc != QM_OK || prm.rows == 0) return rc;
     if (!prm.q_rot) return QM_ERR_NULL;
-    rc = launch_rope_cache(prm, f32, stream);
+    rc = f32 ? rope_cache<float>(prm, stream) : rope_cache<uint16_t>(prm, stream);
     if (rc != QM_OK) return rc;
     // (positions that only the device knows belong to one-token steps)
     if (!f32 && prm.rows >= kAttentionMatrixRows && !prm.position_dev && !(prm.options & QM_ATTENTION_ROWS)) return launch_chunk_attention_mfma(prm, stream);

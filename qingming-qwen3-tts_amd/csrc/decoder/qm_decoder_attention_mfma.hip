@@ -1,9 +1,10 @@
 // qm_decoder_attention_mfma.hip — the chunked attention of a prompt's rows on the bf16 matrix cores (gfx950).
 //
-// A block of four waves takes 64 query rows of one key/value head (a query row is a position and one of the head's query
-// heads: they share keys and values) and walks the keys that any of them sees in tiles of 64.  Waves work in pairs on 32 of
-// the rows, each wave of a pair on half of every tile, and combine at the end: a prompt of a thousand tokens gives a grid
-// that fills the chip, and a wave needs nothing from another while it walks.
+// A block of eight waves takes 64 query rows of one key/value head (a query row is a position and one of the head's query
+// heads: they share keys and values) and walks the keys that any of them sees in tiles of 128.  Four waves work on the same
+// 32 rows, each on a quarter of every tile, and combine at the end: a prompt of a thousand tokens gives a grid that fills the
+// chip, its longest block walks eight tiles, and a wave needs nothing from another while it walks.  Blocks of one key/value
+// head share a die's L2 (block numbers go round the dies).
 //
 // Scores are S^T = K Q^T (v_mfma_f32_32x32x16_bf16): a lane then holds sixteen keys of one query, the softmax is in the lane
 // but for one exchange with the other half of the wave, and the weights stand where the second product O^T = V^T P^T wants
@@ -18,7 +19,9 @@ namespace qm {
 
 typedef float dec_f32x16 __attribute__((ext_vector_type(16)));
 
-constexpr int kFlashKeys = 64;                 // keys per tile
+constexpr int kFlashKeys = 128;                // keys per tile
+constexpr int kFlashParts = kFlashKeys / 32;   // waves that share 32 query rows
+constexpr int kFlashThreads = 2 * kFlashParts * 64;
 constexpr int kFlashRows = 64;                 // query rows per block
 constexpr int kFlashVStride = kFlashKeys + 4;  // bf16 per value channel in LDS: the 32 rows of a fragment lie in different banks
 
@@ -28,12 +31,14 @@ struct FlashShape {
     static constexpr int kKStride = C + 8;
     static constexpr int kKBytes = kFlashKeys * kKStride * 2;
     static constexpr int kVBytes = C * kFlashVStride * 2;
-    static constexpr int kCombineBytes = 2 * (C / 32) * 16 * 64 * 4 + 2 * 2 * 32 * 4;
+    // (the other parts' sums arrive two channel tiles at a time)
+    static constexpr int kCombineTiles = C / 32 < 2 ? 1 : 2;
+    static constexpr int kCombineBytes = 2 * (kFlashParts - 1) * (kCombineTiles * 16 * 64 + 2 * 32) * 4;
     static constexpr int kLds = kKBytes + kVBytes > kCombineBytes ? kKBytes + kVBytes : kCombineBytes;
 };
 
 template <int C>
-__global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(ChunkAttentionParams prm) {
+__global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(ChunkAttentionParams prm) {
     using Shape = FlashShape<C>;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     uint16_t* ks = reinterpret_cast<uint16_t*>(smem);                          // [keys][kKStride]
@@ -41,11 +46,11 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(Chunk
     constexpr int kKb = C / 16, kVt = C / 32;
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int pair = wave >> 1, part = wave & 1, half = lane >> 5;
-    const int kv_head = static_cast<int>(blockIdx.y);
+    const int pair = wave / kFlashParts, part = wave % kFlashParts, half = lane >> 5;
+    const int kv_head = static_cast<int>(blockIdx.x);
     const int group = prm.heads / prm.kv_heads;
     const int total = prm.rows * group;
-    const int row0 = static_cast<int>(blockIdx.x) * kFlashRows;
+    const int row0 = static_cast<int>(gridDim.y - 1 - blockIdx.y) * kFlashRows;      // (late rows, which may see more keys, first)
     auto position_at = [&](int query_row) { return prm.position + min(query_row, total - 1) / group; };
     auto chunk_start = [&](int position) { return position - position % prm.chunk; };
     // what the block, this wave and this lane see: keys [.., ..]
@@ -76,8 +81,8 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(Chunk
 
     const uint16_t* k_head = static_cast<const uint16_t*>(prm.k_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.k_stride;
     const uint16_t* v_head = static_cast<const uint16_t*>(prm.v_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.v_stride;
-    constexpr int kKPieces = kFlashKeys * (C / 8) / kDecThreads;                // 16-byte pieces of keys per thread
-    constexpr int kVBlocks = (16 * (C / 4) + kDecThreads - 1) / kDecThreads;    // blocks of 4 keys x 4 channels per thread
+    constexpr int kKPieces = kFlashKeys * (C / 8) / kFlashThreads;                // 16-byte pieces of keys per thread
+    constexpr int kVBlocks = (kFlashKeys / 4 * (C / 4) + kFlashThreads - 1) / kFlashThreads;    // blocks of 4 keys x 4 channels per thread
     uint4 k_piece[kKPieces];
     uint2 v_piece[kVBlocks][4];
     // (keys past the last one that the block sees are not read: zeros, whose weights are zero as well)
@@ -89,29 +94,29 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(Chunk
         };
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
-            const int at = tid + i * kDecThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
             k_piece[i] = tile + key <= block_hi && c < prm.k_stride ? *reinterpret_cast<const uint4*>(k_head + slot_of(key) * prm.k_stride + c)
                                                                     : make_uint4(0, 0, 0, 0);
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
-            const int at = tid + i * kDecThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
+            const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-                v_piece[i][j] = at < 16 * (C / 4) && tile + key + j <= block_hi && c < prm.v_stride
+                v_piece[i][j] = at < kFlashKeys / 4 * (C / 4) && tile + key + j <= block_hi && c < prm.v_stride
                                     ? *reinterpret_cast<const uint2*>(v_head + slot_of(key + j) * prm.v_stride + c) : make_uint2(0, 0);
         }
     };
     auto deposit = [&]() {
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
-            const int at = tid + i * kDecThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
             *reinterpret_cast<uint4*>(ks + key * Shape::kKStride + c) = k_piece[i];
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
-            const int at = tid + i * kDecThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
-            if (at >= 16 * (C / 4)) break;
+            const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
+            if (at >= kFlashKeys / 4 * (C / 4)) break;
             const uint2 *p = v_piece[i];
             uint16_t* to = vt + c * kFlashVStride + key;
             *reinterpret_cast<uint2*>(to) = make_uint2(__builtin_amdgcn_perm(p[1].x, p[0].x, 0x05040100U), __builtin_amdgcn_perm(p[3].x, p[2].x, 0x05040100U));
@@ -197,36 +202,57 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(Chunk
         }
     }
 
-    // the pair's two halves of the keys, combined by its first wave
+    // the four parts of the keys, combined by the first
     l += __shfl_xor(l, 32, 64);
-    __syncthreads();
-    float* other_o = reinterpret_cast<float*>(smem) + pair * kVt * 16 * 64;
-    float* other_ml = reinterpret_cast<float*>(smem) + 2 * kVt * 16 * 64 + pair * 64;
-    if (part == 1) {
+    constexpr int kAtOnce = Shape::kCombineTiles;
+    float* shared = reinterpret_cast<float*>(smem);
+    float* sh_ml = shared + 2 * (kFlashParts - 1) * kAtOnce * 16 * 64;         // [2 pairs][parts - 1][2][32]
+    auto sums_of = [&](int p) { return shared + (pair * (kFlashParts - 1) + p - 1) * kAtOnce * 16 * 64; };
+    auto ml_of = [&](int p) { return sh_ml + (pair * (kFlashParts - 1) + p - 1) * 64; };
+    float factor[kFlashParts], scale = 0.0f;
 #pragma unroll
-        for (int t = 0; t < kVt; ++t)
+    for (int t0 = 0; t0 < kVt; t0 += kAtOnce) {
+        __syncthreads();
+        if (part > 0) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) other_o[(t * 16 + r) * 64 + lane] = o[t][r];
-        if (lane < 32) {
-            other_ml[lane] = m;
-            other_ml[32 + lane] = l;
+            for (int t = 0; t < kAtOnce; ++t)
+#pragma unroll
+                for (int r = 0; r < 16; ++r) sums_of(part)[(t * 16 + r) * 64 + lane] = o[t0 + t][r];
+            if (t0 == 0 && lane < 32) {
+                ml_of(part)[lane] = m;
+                ml_of(part)[32 + lane] = l;
+            }
         }
-    }
-    __syncthreads();
-    if (part == 0 && query_row < total) {
-        const float m1 = other_ml[lane & 31], l1 = other_ml[32 + (lane & 31)];
-        const float most = fmaxf(m, m1);
-        const float f0 = fast_exp2(m - most), f1 = fast_exp2(m1 - most);
-        const float scale = 1.0f / (l * f0 + l1 * f1);
+        __syncthreads();
+        if (part > 0) continue;
+        if (t0 == 0) {
+            float most = m;
+#pragma unroll
+            for (int p = 1; p < kFlashParts; ++p) most = fmaxf(most, ml_of(p)[lane & 31]);
+            factor[0] = fast_exp2(m - most);
+            float total_l = l * factor[0];
+#pragma unroll
+            for (int p = 1; p < kFlashParts; ++p) {
+                factor[p] = fast_exp2(ml_of(p)[lane & 31] - most);
+                total_l = fmaf(ml_of(p)[32 + (lane & 31)], factor[p], total_l);
+            }
+            scale = 1.0f / total_l;
+        }
+        if (query_row >= total) continue;
         uint16_t* out = static_cast<uint16_t*>(prm.out) + local * prm.ld_out + head * prm.vdim;
 #pragma unroll
-        for (int t = 0; t < kVt; ++t) {
+        for (int t = 0; t < kAtOnce; ++t) {
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
-                const int c = 32 * t + 8 * g + 4 * half;
+                const int c = 32 * (t0 + t) + 8 * g + 4 * half;
                 float v[4];
 #pragma unroll
-                for (int e = 0; e < 4; ++e) v[e] = (o[t][4 * g + e] * f0 + other_o[(t * 16 + 4 * g + e) * 64 + lane] * f1) * scale;
+                for (int e = 0; e < 4; ++e) {
+                    v[e] = o[t0 + t][4 * g + e] * factor[0];
+#pragma unroll
+                    for (int p = 1; p < kFlashParts; ++p) v[e] = fmaf(sums_of(p)[(t * 16 + 4 * g + e) * 64 + lane], factor[p], v[e]);
+                    v[e] *= scale;
+                }
                 if (prm.vdim % 4 == 0) {
                     if (c < prm.vdim) *reinterpret_cast<uint2*>(out + c) = make_uint2(pack_bf16_pair(v[0], v[1]), pack_bf16_pair(v[2], v[3]));
                 } else {
@@ -241,7 +267,7 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_mfma_kernel(Chunk
     if (kv_head == prm.kv_heads - 1) {
         const int first = row0 / group, last = min(row0 + kFlashRows - 1, total - 1) / group;
         const int from = prm.heads * prm.vdim, behind = static_cast<int>(prm.ld_out) - from;
-        for (int i = tid; i < (last - first + 1) * behind; i += kDecThreads)
+        for (int i = tid; i < (last - first + 1) * behind; i += kFlashThreads)
             static_cast<uint16_t*>(prm.out)[(first + i / behind) * prm.ld_out + from + i % behind] = 0;
     }
 }
@@ -252,8 +278,9 @@ static int32_t flash_as(const ChunkAttentionParams& prm, hipStream_t stream) {
     const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(chunk_attention_mfma_kernel<C>), FlashShape<C>::kLds, raised);
     if (rc != QM_OK) return rc;
     const int64_t total = static_cast<int64_t>(prm.rows) * (prm.heads / prm.kv_heads);
-    hipLaunchKernelGGL((chunk_attention_mfma_kernel<C>), dim3(static_cast<unsigned>((total + kFlashRows - 1) / kFlashRows), prm.kv_heads),
-                       dim3(kDecThreads), FlashShape<C>::kLds, stream, prm);
+    if ((total + kFlashRows - 1) / kFlashRows > 65535) return QM_ERR_GEOMETRY;
+    hipLaunchKernelGGL((chunk_attention_mfma_kernel<C>), dim3(prm.kv_heads, static_cast<unsigned>((total + kFlashRows - 1) / kFlashRows)),
+                       dim3(kFlashThreads), FlashShape<C>::kLds, stream, prm);
     return launch_status();
 }
 

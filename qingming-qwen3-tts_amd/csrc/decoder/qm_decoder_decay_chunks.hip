@@ -14,12 +14,33 @@ namespace qm {
 constexpr int kDecaySlice = 64;                // value channels staged at once
 constexpr int kDecayVStride = kDecaySlice + 4;
 
-// Rows [t0, t0 + 64) of a head's q, k or v columns into LDS as silu(x) (zeros past the rows or the head), times factor(j).
+// Rows [t0, t0 + 64) of a head's q, k or v columns into LDS as silu(x) (zeros past the rows or the head), times factor(j):
+// sixteen threads take 64 columns of a row, four each.  `padded`: a multiple of 16.
 template <class F>
 __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, float* to, int stride, int t0, int column, int columns, int padded, F factor) {
-    for (int i = threadIdx.x; i < kDecayChunk * padded; i += kDecThreads) {
-        const int j = i / padded, c = i - j * padded;
-        to[j * stride + c] = t0 + j < prm.rows && c < columns ? silu_f32(prm.proj[(t0 + j) * prm.ld_proj + column + c]) * factor(j) : 0.0f;
+    const int c4 = (threadIdx.x & 15) * 4, row = threadIdx.x >> 4;
+    for (int c = c4; c < padded; c += 64) {
+        float4 x[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int j = row + 16 * i;
+            const bool in = t0 + j < prm.rows;
+            const float* p = prm.proj + (t0 + j) * prm.ld_proj + column + c;
+            if (in && c + 3 < columns && ((column | prm.ld_proj) & 3) == 0) {
+                x[i] = *reinterpret_cast<const float4*>(p);
+            } else {
+                x[i].x = in && c < columns ? p[0] : 0.0f;
+                x[i].y = in && c + 1 < columns ? p[1] : 0.0f;
+                x[i].z = in && c + 2 < columns ? p[2] : 0.0f;
+                x[i].w = in && c + 3 < columns ? p[3] : 0.0f;
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int j = row + 16 * i;
+            const float f = t0 + j < prm.rows ? factor(j) : 0.0f;
+            *reinterpret_cast<float4*>(to + j * stride + c) = make_float4(silu_f32(x[i].x) * f, silu_f32(x[i].y) * f, silu_f32(x[i].z) * f, silu_f32(x[i].w) * f);
+        }
     }
 }
 
@@ -83,7 +104,7 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, l16 = lane & 15;
     const int chunk = static_cast<int>(blockIdx.x), head = static_cast<int>(blockIdx.y);
-    const int t0 = chunk * kDecayChunk;
+    const int t0 = chunk * kDecayChunk, e0 = static_cast<int>(blockIdx.z) * kDecaySlice;
     const int dp = mfma32_pad(prm.dim), stride = mfma32_stride(prm.dim);
     const float* powers = prm.powers + head * kDecayPowers;
     float* qs = lds;                           // [64][stride]
@@ -93,6 +114,7 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
     auto one = [](int) { return 1.0f; };
     stage_rows(prm, qs, stride, t0, prm.q_column + head * prm.dim, prm.dim, dp, one);
     stage_rows(prm, ks, stride, t0, prm.k_column + head * prm.dim, prm.dim, dp, one);
+    stage_rows(prm, vs, kDecayVStride, t0, prm.v_column + head * prm.vdim + e0, prm.vdim - e0, kDecaySlice, one);
     __syncthreads();
     f32x4_t score[4] = {};                     // rows of tile `wave`, column tiles 0 .. wave
     for (int d0 = 0; d0 < dp; d0 += 16) {
@@ -115,43 +137,39 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
 #pragma unroll
     for (int i = 0; i < 4; ++i) decayed[i] = powers[16 * i + l16 + 1];
     const float* before = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * prm.dim * prm.vdim;
-    for (int e0 = 0; e0 < prm.vdim; e0 += kDecaySlice) {
-        __syncthreads();
-        stage_rows(prm, vs, kDecayVStride, t0, prm.v_column + head * prm.vdim + e0, prm.vdim - e0, kDecaySlice, one);
-        __syncthreads();
-        const int column = e0 + 16 * wave + l16;
-        f32x4_t acc[4] = {};
-        for (int d0 = 0; d0 < dp; d0 += 16) {
-            float s[4];
+    __syncthreads();
+    const int column = e0 + 16 * wave + l16;
+    f32x4_t acc[4] = {};
+    for (int d0 = 0; d0 < dp; d0 += 16) {
+        float s[4];
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                const int d = d0 + 4 * g + t;
-                s[t] = d < prm.dim && column < prm.vdim ? before[static_cast<int64_t>(d) * prm.vdim + column] : 0.0f;
-            }
-            const float4 b = make_float4(s[0], s[1], s[2], s[3]);
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                float4 a = *reinterpret_cast<const float4*>(qs + (16 * i + l16) * stride + d0 + 4 * g);
-                a.x *= decayed[i]; a.y *= decayed[i]; a.z *= decayed[i]; a.w *= decayed[i];
-                acc[i] = mfma32_block(a, b, acc[i]);
-            }
+        for (int t = 0; t < 4; ++t) {
+            const int d = d0 + 4 * g + t;
+            s[t] = d < prm.dim && column < prm.vdim ? before[static_cast<int64_t>(d) * prm.vdim + column] : 0.0f;
         }
+        const float4 b = make_float4(s[0], s[1], s[2], s[3]);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            const float* v = vs + (16 * j + 4 * g) * kDecayVStride + 16 * wave + l16;
-            const float4 b = make_float4(v[0], v[kDecayVStride], v[2 * kDecayVStride], v[3 * kDecayVStride]);
-#pragma unroll
-            for (int i = j; i < 4; ++i)
-                acc[i] = mfma32_block(*reinterpret_cast<const float4*>(ps + (16 * i + l16) * kDecayVStride + 16 * j + 4 * g), b, acc[i]);
+        for (int i = 0; i < 4; ++i) {
+            float4 a = *reinterpret_cast<const float4*>(qs + (16 * i + l16) * stride + d0 + 4 * g);
+            a.x *= decayed[i]; a.y *= decayed[i]; a.z *= decayed[i]; a.w *= decayed[i];
+            acc[i] = mfma32_block(a, b, acc[i]);
         }
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = t0 + 16 * i + 4 * g + r;
-                if (t < prm.rows && column < prm.vdim) prm.out[static_cast<int64_t>(t) * prm.heads * prm.vdim + head * prm.vdim + column] = acc[i][r];
-            }
     }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const float* v = vs + (16 * j + 4 * g) * kDecayVStride + 16 * wave + l16;
+        const float4 b = make_float4(v[0], v[kDecayVStride], v[2 * kDecayVStride], v[3 * kDecayVStride]);
+#pragma unroll
+        for (int i = j; i < 4; ++i)
+            acc[i] = mfma32_block(*reinterpret_cast<const float4*>(ps + (16 * i + l16) * kDecayVStride + 16 * j + 4 * g), b, acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = t0 + 16 * i + 4 * g + r;
+            if (t < prm.rows && column < prm.vdim) prm.out[static_cast<int64_t>(t) * prm.heads * prm.vdim + head * prm.vdim + column] = acc[i][r];
+        }
 }
 
 int64_t decay_scratch_floats(int rows, int heads, int dim, int vdim) {
@@ -173,7 +191,7 @@ int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream)
     const int64_t plane = static_cast<int64_t>(prm.heads) * prm.dim * prm.vdim;
     hipLaunchKernelGGL(decay_chunk_walk_kernel, dim3(static_cast<unsigned>((plane + kDecThreads - 1) / kDecThreads)), dim3(kDecThreads), 0, stream, prm,
                        chunks);
-    hipLaunchKernelGGL(decay_chunk_output_kernel, dim3(chunks, prm.heads), dim3(kDecThreads), output_lds, stream, prm);
+    hipLaunchKernelGGL(decay_chunk_output_kernel, dim3(chunks, prm.heads, slices), dim3(kDecThreads), output_lds, stream, prm);
     return launch_status();
 }
 

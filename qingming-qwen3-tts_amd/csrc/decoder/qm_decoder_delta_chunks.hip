@@ -10,7 +10,7 @@
 // M, N, R - D_A M, D_K - D_A N do not depend on S: one launch computes them for every chunk and head at once.  A second one
 // walks the chunks; columns of S never interact, so its blocks take 16 columns each, four waves sharing the rows.  A decay is
 // never below exp(-e^(-1/2)) = 0.545, so 1 / W stays under 3e8 and everything fits fp32; A and K enter the state already
-// multiplied by W.  All products are fp32 (matrix cores, or fmaf for the triangular solve).
+// multiplied by W.  All products are fp32 on the matrix cores.
 // Bound: the walk, a chain of rows / 32 dependent steps.
 #include "../qm_host.h"
 #include "qm_decoder_mfma32.h"
@@ -33,7 +33,7 @@ __host__ __device__ inline DeltaScratch delta_scratch(int dim) {
     return s;
 }
 __host__ __device__ inline int delta_z_stride(int rank) { return (rank + 3) / 4 * 4; }
-inline int delta_prepare_lds(int dim) { return 4 * kDeltaChunk * mfma32_stride(dim) + 4 * kDeltaChunk * kDeltaMat + kDeltaChunk; }
+inline int delta_prepare_lds(int dim) { return 4 * kDeltaChunk * mfma32_stride(dim) + 5 * kDeltaChunk * kDeltaMat + kDeltaChunk; }
 
 __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaParams prm) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -48,7 +48,8 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
     float* ks = as + kDeltaChunk * stride;
     float* rs = ks + kDeltaChunk * stride;
     float* mats = rs + kDeltaChunk * stride;   // L_A, L_K, D_A, D_K, each [32][kDeltaMat]
-    float* inverse = mats + 4 * kDeltaChunk * kDeltaMat;
+    float* inverted = mats + 4 * kDeltaChunk * kDeltaMat;          // (I + L_A)^-1
+    float* inverse = inverted + kDeltaChunk * kDeltaMat;
     float* zs = as;                            // tanh of the rank-sized projection, [32][z_stride], until the decays are there
     const int z_stride = delta_z_stride(prm.rank);
 
@@ -73,7 +74,7 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
         for (int t = 0; t < 16; ++t) z[t] = bias;
         if (c < dim) {
             const float* w2 = prm.w2 + head * dim + c;
-#pragma unroll 2
+#pragma unroll 4
             for (int r = 0; r < prm.rank; r += 4) {
                 float w[4];
 #pragma unroll
@@ -90,35 +91,57 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
         for (int t = 0; t < 16; ++t) us[(first + t) * stride + c] = first + t < tokens && c < dim ? delta_decay_of(z[t]) : 1.0f;
     }
     __syncthreads();
-    if (tid < dp) {                                                // a channel's products of decays, and what they scale
-        const int c = tid;
-        const float bias = c < dim ? prm.a_bias[head * dim + c] : 0.0f;
-        float before = 1.0f;
+    if (tid < dp) {                                                // products of decays, into rs
+        float product = 1.0f;
 #pragma unroll 8
         for (int t = 0; t < kDeltaChunk; ++t) {
-            const bool in = t < tokens && c < dim;
-            const float* p = prm.proj + (t0 + min(t, tokens - 1)) * prm.ld_proj + head * dim + min(c, dim - 1);
-            const float k = in ? p[prm.k_column] : 0.0f, r = in ? p[prm.r_column] : 0.0f;
-            const float u = in ? k * inverse[t] : 0.0f;
-            const float a = in ? sigmoid_f32(p[prm.a_column] + bias) * u : 0.0f;
-            const float after = before * us[t * stride + c];
-            const float over = 1.0f / after;
-            us[t * stride + c] = u * before;
-            as[t * stride + c] = a * over;
-            ks[t * stride + c] = k * over;
-            rs[t * stride + c] = r * after;
-            before = after;
+            product *= us[t * stride + tid];
+            rs[t * stride + tid] = product;
         }
-        scratch[at.w + c] = before;
+        scratch[at.w + tid] = product;
+    }
+    __syncthreads();
+    // a thread takes a channel of sixteen tokens, last token first: a token needs the products up to it and up to the one
+    // before, and leaves its row of R in the product's place
+    float edge[2], whole[2];
 #pragma unroll
-        for (int t = 0; t < kDeltaChunk; t += 4) {
-            float4 a, k;
-            a.x = -before * as[t * stride + c]; a.y = -before * as[(t + 1) * stride + c];
-            a.z = -before * as[(t + 2) * stride + c]; a.w = -before * as[(t + 3) * stride + c];
-            k.x = before * ks[t * stride + c]; k.y = before * ks[(t + 1) * stride + c];
-            k.z = before * ks[(t + 2) * stride + c]; k.w = before * ks[(t + 3) * stride + c];
-            *reinterpret_cast<float4*>(scratch + at.at + c * kDeltaChunk + t) = a;
-            *reinterpret_cast<float4*>(scratch + at.kt + c * kDeltaChunk + t) = k;
+    for (int n = 0; n < 2; ++n) {
+        const int i = tid + n * kDecThreads, c = i % dp, first = i / dp * 16;
+        const bool in = i < 2 * dp;
+        edge[n] = in && first > 0 ? rs[(first - 1) * stride + c] : 1.0f;
+        whole[n] = in ? rs[(kDeltaChunk - 1) * stride + c] : 1.0f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int n = 0; n < 2; ++n) {
+        const int i = tid + n * kDecThreads, c = i % dp, first = i / dp * 16;
+        if (i >= 2 * dp) break;
+        const float bias = c < dim ? prm.a_bias[head * dim + c] : 0.0f;
+        for (int t1 = first + 12; t1 >= first; t1 -= 4) {
+            float k[4], r[4], a[4], at_[4], kt_[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const bool in = t1 + e < tokens && c < dim;
+                const float* p = prm.proj + (t0 + t1 + e) * prm.ld_proj + head * dim + c;
+                k[e] = in ? p[prm.k_column] : 0.0f;
+                r[e] = in ? p[prm.r_column] : 0.0f;
+                a[e] = in ? p[prm.a_column] : 0.0f;
+            }
+#pragma unroll
+            for (int e = 3; e >= 0; --e) {
+                const int t = t1 + e;
+                const float after = rs[t * stride + c], before = t > first ? rs[(t - 1) * stride + c] : edge[n];
+                const float u = t < tokens ? k[e] * inverse[t] : 0.0f;
+                const float removal = sigmoid_f32(a[e] + bias) * u, over = reciprocal(after);
+                us[t * stride + c] = u * before;
+                as[t * stride + c] = removal * over;
+                ks[t * stride + c] = k[e] * over;
+                rs[t * stride + c] = r[e] * after;
+                at_[e] = -whole[n] * removal * over;
+                kt_[e] = whole[n] * k[e] * over;
+            }
+            *reinterpret_cast<float4*>(scratch + at.at + c * kDeltaChunk + t1) = make_float4(at_[0], at_[1], at_[2], at_[3]);
+            *reinterpret_cast<float4*>(scratch + at.kt + c * kDeltaChunk + t1) = make_float4(kt_[0], kt_[1], kt_[2], kt_[3]);
         }
     }
     __syncthreads();
@@ -149,39 +172,73 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
                 }
     }
     __syncthreads();
+    // (I + L_A)^-1 = [[T1, 0], [-T2 L21 T1, T2]]: the two 16 x 16 inverses by a column per thread, the third block by products
     const float* l_a = mats;
+    const float* l_k = mats + kDeltaChunk * kDeltaMat;
     const float* d_a = mats + 2 * kDeltaChunk * kDeltaMat;
-    for (int c = tid; c < dp + kDeltaChunk; c += kDecThreads) {    // columns of (U, L_K) solved, and of (R, D_K) less D_A times them
-        const bool wide = c < dp;
-        const float* y = wide ? us + c : mats + kDeltaChunk * kDeltaMat + (c - dp);
-        const float* z = wide ? rs + c : mats + 3 * kDeltaChunk * kDeltaMat + (c - dp);
-        const int step = wide ? stride : kDeltaMat, out_step = wide ? dp : kDeltaChunk;
-        float* solved_out = scratch + (wide ? at.m + c : at.n + c - dp);
-        float* rest_out = scratch + (wide ? at.x + c : at.y + c - dp);
-        float solved[kDeltaChunk];
+    const float* d_k = mats + 3 * kDeltaChunk * kDeltaMat;
+    if (tid < kDeltaChunk) {
+        const int b = tid & 16, c = tid & 15;
+        float solved[16];
 #pragma unroll
-        for (int t = 0; t < kDeltaChunk; ++t) {
-            float v = y[t * step], x = z[t * step];
+        for (int t = 0; t < 16; ++t) {
+            float v = t == c ? 1.0f : 0.0f;
 #pragma unroll
             for (int s = 0; s < t; s += 4) {
-                const float4 m = *reinterpret_cast<const float4*>(l_a + t * kDeltaMat + s);
+                const float4 m = *reinterpret_cast<const float4*>(l_a + (b + t) * kDeltaMat + b + s);
                 v = fmaf(-m.x, solved[s], v);
                 if (s + 1 < t) v = fmaf(-m.y, solved[s + 1], v);
                 if (s + 2 < t) v = fmaf(-m.z, solved[s + 2], v);
                 if (s + 3 < t) v = fmaf(-m.w, solved[s + 3], v);
             }
             solved[t] = v;
-#pragma unroll
-            for (int s = 0; s <= t; s += 4) {
-                const float4 m = *reinterpret_cast<const float4*>(d_a + t * kDeltaMat + s);
-                x = fmaf(-m.x, solved[s], x);
-                if (s + 1 <= t) x = fmaf(-m.y, solved[s + 1], x);
-                if (s + 2 <= t) x = fmaf(-m.z, solved[s + 2], x);
-                if (s + 3 <= t) x = fmaf(-m.w, solved[s + 3], x);
-            }
-            solved_out[t * out_step] = v;
-            rest_out[t * out_step] = x;
         }
+#pragma unroll
+        for (int t = 0; t < 16; ++t) inverted[(b + t) * kDeltaMat + b + c] = solved[t];
+    }
+    __syncthreads();
+    auto left_operand = [&](const float* m, int rows, int terms) { return *reinterpret_cast<const float4*>(m + (rows + l16) * kDeltaMat + terms + 4 * g); };
+    auto right_operand = [&](const float* m, int step, int terms, int columns) {
+        const float* p = m + (terms + 4 * g) * step + columns + l16;
+        return make_float4(p[0], p[step], p[2 * step], p[3 * step]);
+    };
+    auto as_operand = [](f32x4_t v) { return make_float4(v[0], v[1], v[2], v[3]); };
+    if (wave == 0) {
+        const f32x4_t none = {};
+        const f32x4_t lower = mfma32_block(left_operand(l_a, 16, 0), right_operand(inverted, kDeltaMat, 0, 0), none);      // L21 T1
+        const f32x4_t third = mfma32_block(left_operand(inverted, 16, 16), as_operand(lower), none);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) inverted[(16 + 4 * g + r) * kDeltaMat + l16] = -third[r];
+    }
+    __syncthreads();
+    // sixteen columns at a time of (U, L_K): times the inverse, and of (R, D_K) less D_A times that
+    for (int n = wave; n < dp / 16 + 2; n += 4) {
+        const bool wide = n < dp / 16;
+        const int c = wide ? 16 * n : 16 * (n - dp / 16), step = wide ? stride : kDeltaMat, out_step = wide ? dp : kDeltaChunk;
+        const float* y = wide ? us : l_k;
+        const float* z = wide ? rs : d_k;
+        float* solved_out = scratch + (wide ? at.m : at.n);
+        float* rest_out = scratch + (wide ? at.x : at.y);
+        const float4 y0 = right_operand(y, step, 0, c), y1 = right_operand(y, step, 16, c);
+        f32x4_t m[2] = {}, x[2];
+        m[0] = mfma32_block(left_operand(inverted, 0, 0), y0, m[0]);
+        m[1] = mfma32_block(left_operand(inverted, 16, 0), y0, m[1]);
+        m[1] = mfma32_block(left_operand(inverted, 16, 16), y1, m[1]);
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) x[b][r] = -z[(16 * b + 4 * g + r) * step + c + l16];
+            x[b] = mfma32_block(left_operand(d_a, 16 * b, 0), as_operand(m[0]), x[b]);
+        }
+        x[1] = mfma32_block(left_operand(d_a, 16, 16), as_operand(m[1]), x[1]);
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int t = 16 * b + 4 * g + r;
+                solved_out[t * out_step + c + l16] = m[b][r];
+                rest_out[t * out_step + c + l16] = -x[b][r];
+            }
     }
 }
 
@@ -190,7 +247,7 @@ template <int TW>
 struct DeltaStep {
     float4 m[2][TW], x[2][TW], at[TW][2], kt[TW][2], w[TW];
     float2 n[2], y[2];
-    float v[2][4];
+    float v[2][4], own[2];
 };
 
 // TW: 16-row tiles of the state per wave (tile = wave + 4 i)
@@ -213,6 +270,9 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
             s[i][r] = d < dim && column < dim ? state[static_cast<int64_t>(d) * dim + column] : 0.0f;
         }
     const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    auto value_at = [&](int token) {
+        return token < prm.rows && column < dim ? prm.proj[token * prm.ld_proj + prm.v_column + head * dim + column] : 0.0f;
+    };
     auto request = [&](int chunk, DeltaStep<TW>& f) __attribute__((always_inline)) {
         const float* from = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * at.floats;
 #pragma unroll
@@ -235,10 +295,8 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
             f.n[b] = *reinterpret_cast<const float2*>(from + at.n + row);
             f.y[b] = *reinterpret_cast<const float2*>(from + at.y + row);
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                const int token = chunk * kDeltaChunk + 16 * b + 4 * g + t;
-                f.v[b][t] = token < prm.rows && column < dim ? prm.proj[token * prm.ld_proj + prm.v_column + head * dim + column] : 0.0f;
-            }
+            for (int t = 0; t < 4; ++t) f.v[b][t] = value_at(chunk * kDeltaChunk + 16 * b + 4 * g + t);
+            f.own[b] = value_at(chunk * kDeltaChunk + 16 * part + 4 * g + pair + b);
         }
     };
     auto walk = [&](int chunk, DeltaStep<TW>& f, DeltaStep<TW>& next) __attribute__((always_inline)) {
@@ -253,13 +311,11 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
                 o[half] = mfma32_block(f.x[half][i], b, o[half]);
             }
         }
-        const float v0 = part ? (pair ? f.v[1][2] : f.v[1][0]) : (pair ? f.v[0][2] : f.v[0][0]);
-        const float v1 = part ? (pair ? f.v[1][3] : f.v[1][1]) : (pair ? f.v[0][3] : f.v[0][1]);
         float (*mine)[kDeltaChunk * kStride] = sh[chunk & 1][wave];
 #pragma unroll
         for (int half = 0; half < 2; ++half) {
-            p[half] = mfma32(f.n[half].y, v1, mfma32(f.n[half].x, v0, p[half]));
-            o[half] = mfma32(f.y[half].y, v1, mfma32(f.y[half].x, v0, o[half]));
+            p[half] = mfma32(f.n[half].y, f.own[1], mfma32(f.n[half].x, f.own[0], p[half]));
+            o[half] = mfma32(f.y[half].y, f.own[1], mfma32(f.y[half].x, f.own[0], o[half]));
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 mine[0][(16 * half + 4 * g + r) * kStride + l16] = p[half][r];

@@ -18,8 +18,10 @@ template <class T> __device__ __forceinline__ T from_f32(float v);
 template <> __device__ __forceinline__ uint16_t from_f32<uint16_t>(float v) { return f2bf(v); }
 template <> __device__ __forceinline__ float from_f32<float>(float v) { return v; }
 
-__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+// (v_exp_f32 and v_rcp_f32 are good to one unit in the last place)
+__device__ __forceinline__ float reciprocal(float x) { return __builtin_amdgcn_rcpf(x); }
+__device__ __forceinline__ float sigmoid_f32(float z) { return reciprocal(1.0f + fast_exp2(-z * kLog2e)); }
+__device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
 
 // Sum / maximum over the 64 lanes of a wave, in every lane.
 __device__ __forceinline__ float wave_sum(float v) {

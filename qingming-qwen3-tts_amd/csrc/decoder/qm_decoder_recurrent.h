@@ -176,4 +176,78 @@ __device__ __forceinline__ void general_delta_block(const DeltaParams& prm, int 
     store_state<RD>(s, state, prm.dim, prm.dim, sub, column);
 }
 
+// One token of the delta rule: everything from memory is requested before anything waits, a channel's decay is summed by
+// 256 / (4 RD) threads.
+__host__ __device__ inline int delta_step_lds_floats(int rd, int rank) { return 5 * rec_stride(rd) + rank + 256 + 8; }
+template <int RD>
+__device__ __forceinline__ void general_delta_step(const DeltaParams& prm, int head, int slice, float* lds) {
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = lane >> 4;
+    const int column = slice * kRecColumns + wave * 16 + (lane & 15);
+    constexpr int kStride = 4 * (RD + 4), kChannels = 4 * RD, kParts = kDecThreads / kChannels, kAhead = 16;
+    const int c = tid % kChannels, part = tid / kChannels;
+    float* sh_z = lds + 5 * kStride;                               // [rank]
+    float* sh_sum = sh_z + prm.rank;                               // [parts][channels]
+    float* sh_sq = sh_sum + kDecThreads;                           // [4]
+    const bool in = c < prm.dim;
+    const int at = head * prm.dim + (in ? c : 0), all = prm.heads * prm.dim;
+    const float* p = prm.proj + at;
+    const float k = in ? p[prm.k_column] : 0.0f, r = p[prm.r_column], a = p[prm.a_column];
+    const float bias = prm.a_bias[at], w0 = prm.w0[at];
+    const float v = column < prm.dim ? prm.proj[prm.v_column + head * prm.dim + column] : 0.0f;
+    const int ranks = (prm.rank + kParts - 1) / kParts, first = part * ranks, last = min(prm.rank, first + ranks);
+    const float* w2 = prm.w2 + at;
+    float piece[kAhead];
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i) piece[i] = first + i < last ? w2[static_cast<int64_t>(first + i) * all] : 0.0f;
+    const float z0 = tid < prm.rank ? prm.proj[prm.z_column + tid] : 0.0f;
+    float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.dim;
+    float s[RD];
+    load_state<RD>(s, state, prm.dim, prm.dim, sub, column);
+    if (tid < prm.rank) sh_z[tid] = tanhf(z0);
+    for (int i = tid + kDecThreads; i < prm.rank; i += kDecThreads) sh_z[i] = tanhf(prm.proj[prm.z_column + i]);
+    const float sq = wave_sum(part == 0 ? k * k : 0.0f);
+    if (lane == 0) sh_sq[wave] = sq;
+    __syncthreads();
+    float z = 0.0f;
+    for (int i0 = first; i0 < last; i0 += kAhead) {
+        float now[kAhead];
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i) {
+            now[i] = piece[i];
+            piece[i] = i0 + kAhead + i < last ? w2[static_cast<int64_t>(i0 + kAhead + i) * all] : 0.0f;
+        }
+#pragma unroll
+        for (int i = 0; i < kAhead; ++i)
+            if (i0 + i < last) z = fmaf(now[i], sh_z[i0 + i], z);
+    }
+    sh_sum[tid] = z;
+    __syncthreads();
+    if (part == 0) {
+        float sum = w0;
+#pragma unroll
+        for (int i = 0; i < kParts; ++i) sum += sh_sum[i * kChannels + c];
+        const float u = k * (1.0f / sqrtf((sh_sq[0] + sh_sq[1]) + (sh_sq[2] + sh_sq[3]) + prm.unit_eps));
+        float* put = lds + rec_at<RD>(c);
+        put[0] = in ? delta_decay_of(sum) : 0.0f;
+        put[kStride] = in ? sigmoid_f32(a + bias) * u : 0.0f;
+        put[2 * kStride] = u;
+        put[3 * kStride] = k;
+        put[4 * kStride] = in ? r : 0.0f;
+    }
+    __syncthreads();
+    const float* w = lds + sub * (RD + 4);
+    float seen = 0.0f, o = 0.0f;
+#pragma unroll
+    for (int i = 0; i < RD; ++i) seen = fmaf(w[2 * kStride + i], s[i], seen);
+    seen = quarter_sum(seen);
+#pragma unroll
+    for (int i = 0; i < RD; ++i) {
+        s[i] = fmaf(w[3 * kStride + i], v, fmaf(-w[kStride + i], seen, w[i] * s[i]));
+        o = fmaf(w[4 * kStride + i], s[i], o);
+    }
+    o = quarter_sum(o);
+    if (sub == 0 && column < prm.dim) prm.out[head * prm.dim + column] = o;
+    store_state<RD>(s, state, prm.dim, prm.dim, sub, column);
+}
+
 }  // namespace qm

@@ -18,6 +18,13 @@ __global__ __launch_bounds__(kDecThreads) void general_delta_kernel(DeltaParams 
 }
 
 template <int RD>
+__global__ __launch_bounds__(kDecThreads) void general_delta_step_kernel(DeltaParams prm) {
+    request_arguments(prm);
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    general_delta_step<RD>(prm, static_cast<int>(blockIdx.y), static_cast<int>(blockIdx.x), lds);
+}
+
+template <int RD>
 static int32_t decay_as(const DecayAttentionParams& prm, hipStream_t stream) {
     hipLaunchKernelGGL(decay_attention_kernel<RD>, dim3((prm.vdim + kRecColumns - 1) / kRecColumns, prm.heads), dim3(kDecThreads),
                        sizeof(float) * decay_lds_floats(RD), stream, prm);
@@ -43,12 +50,17 @@ int32_t launch_decay_attention(const DecayAttentionParams& prm, hipStream_t stre
 
 template <int RD>
 static int32_t delta_as(const DeltaParams& prm, hipStream_t stream) {
+    const dim3 grid((prm.dim + kRecColumns - 1) / kRecColumns, prm.heads);
+    if (prm.rows == 1) {
+        hipLaunchKernelGGL(general_delta_step_kernel<RD>, grid, dim3(kDecThreads), sizeof(float) * delta_step_lds_floats(RD, prm.rank), stream, prm);
+        return launch_status();
+    }
     const int bytes = static_cast<int>(sizeof(float)) * delta_lds_floats(RD, prm.rank);
     static std::atomic<bool> raised[kMaxDevices];
     const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(general_delta_kernel<RD>), kDotLdsMost, raised);
     if (rc != QM_OK) return rc;
     if (bytes > kDotLdsMost) return QM_ERR_GEOMETRY;
-    hipLaunchKernelGGL(general_delta_kernel<RD>, dim3((prm.dim + kRecColumns - 1) / kRecColumns, prm.heads), dim3(kDecThreads), bytes, stream, prm);
+    hipLaunchKernelGGL(general_delta_kernel<RD>, grid, dim3(kDecThreads), bytes, stream, prm);
     return launch_status();
 }
 
