@@ -18,6 +18,8 @@
 namespace qm {
 
 typedef float dec_f32x16 __attribute__((ext_vector_type(16)));
+typedef uint32_t dec_u32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t dec_u32x2 __attribute__((ext_vector_type(2)));
 
 constexpr int kFlashKeys = 128;                // keys per tile
 constexpr int kFlashParts = kFlashKeys / 32;   // waves that share 32 query rows
@@ -62,14 +64,14 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
     const int head = kv_head * group + min(query_row, total - 1) % group;
     const int position = prm.position + local;
     const int lo = chunk_start(position);
-    const int key_blocks = (prm.dim + 15) / 16, value_tiles = (prm.vdim + 31) / 32;
 
-    uint4 q[kKb];
+    dec_u32x4 q[kKb];
     const uint16_t* q_row = static_cast<const uint16_t*>(prm.q_rot) + (static_cast<int64_t>(local) * prm.heads + head) * prm.k_stride;
 #pragma unroll
     for (int kb = 0; kb < kKb; ++kb) {
         const int c = kb * 16 + 8 * half;
-        q[kb] = c < prm.k_stride ? *reinterpret_cast<const uint4*>(q_row + c) : make_uint4(0, 0, 0, 0);
+        const dec_u32x4 read = *reinterpret_cast<const dec_u32x4*>(q_row + min(c, prm.k_stride - 8));
+        q[kb] = c < prm.k_stride ? read : dec_u32x4{0, 0, 0, 0};
     }
     dec_f32x16 o[kVt];
 #pragma unroll
@@ -83,46 +85,47 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
     const uint16_t* v_head = static_cast<const uint16_t*>(prm.v_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.v_stride;
     constexpr int kKPieces = kFlashKeys * (C / 8) / kFlashThreads;                // 16-byte pieces of keys per thread
     constexpr int kVBlocks = (kFlashKeys / 4 * (C / 4) + kFlashThreads - 1) / kFlashThreads;    // blocks of 4 keys x 4 channels per thread
-    uint4 k_piece[kKPieces];
-    uint2 v_piece[kVBlocks][4];
-    // (keys past the last one that the block sees are not read: zeros, whose weights are zero as well)
-    auto request = [&](int tile) {
-        const int base = tile % prm.ring;
+    dec_u32x4 k_piece[kKPieces];
+    dec_u32x2 v_piece[kVBlocks][4];
+    // (keys past the last one that the block sees repeat it, channels past the head's repeat others: the first are masked,
+    // the second meet zeros of the query or are not stored; no branch around a load)
+    auto request = [&](int tile) __attribute__((always_inline)) {
+        const int base = tile % prm.ring, last = block_hi - tile;
         auto slot_of = [&](int key) {
-            const int s = base + key;
-            return static_cast<int64_t>(s >= prm.ring ? s - prm.ring : s);
+            const int s = base + min(key, last);
+            return s >= prm.ring ? s - prm.ring : s;
         };
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
             const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
-            k_piece[i] = tile + key <= block_hi && c < prm.k_stride ? *reinterpret_cast<const uint4*>(k_head + slot_of(key) * prm.k_stride + c)
-                                                                    : make_uint4(0, 0, 0, 0);
+            k_piece[i] = *reinterpret_cast<const dec_u32x4*>(k_head + slot_of(key) * prm.k_stride + min(c, prm.k_stride - 8));
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
             const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-                v_piece[i][j] = at < kFlashKeys / 4 * (C / 4) && tile + key + j <= block_hi && c < prm.v_stride
-                                    ? *reinterpret_cast<const uint2*>(v_head + slot_of(key + j) * prm.v_stride + c) : make_uint2(0, 0);
+                v_piece[i][j] = *reinterpret_cast<const dec_u32x2*>(v_head + slot_of(key + j) * prm.v_stride + min(c, prm.v_stride - 4));
         }
     };
-    auto deposit = [&]() {
+    auto deposit = [&]() __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
             const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
-            *reinterpret_cast<uint4*>(ks + key * Shape::kKStride + c) = k_piece[i];
+            *reinterpret_cast<dec_u32x4*>(ks + key * Shape::kKStride + c) = k_piece[i];
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
             const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
             if (at >= kFlashKeys / 4 * (C / 4)) break;
-            const uint2 *p = v_piece[i];
+            const dec_u32x2 p0 = v_piece[i][0], p1 = v_piece[i][1], p2 = v_piece[i][2], p3 = v_piece[i][3];
             uint16_t* to = vt + c * kFlashVStride + key;
-            *reinterpret_cast<uint2*>(to) = make_uint2(__builtin_amdgcn_perm(p[1].x, p[0].x, 0x05040100U), __builtin_amdgcn_perm(p[3].x, p[2].x, 0x05040100U));
-            *reinterpret_cast<uint2*>(to + kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].x, p[0].x, 0x07060302U), __builtin_amdgcn_perm(p[3].x, p[2].x, 0x07060302U));
-            *reinterpret_cast<uint2*>(to + 2 * kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].y, p[0].y, 0x05040100U), __builtin_amdgcn_perm(p[3].y, p[2].y, 0x05040100U));
-            *reinterpret_cast<uint2*>(to + 3 * kFlashVStride) = make_uint2(__builtin_amdgcn_perm(p[1].y, p[0].y, 0x07060302U), __builtin_amdgcn_perm(p[3].y, p[2].y, 0x07060302U));
+            auto pair_low = [](uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x05040100U); };
+            auto pair_high = [](uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x07060302U); };
+            *reinterpret_cast<dec_u32x2*>(to) = dec_u32x2{pair_low(p0[0], p1[0]), pair_low(p2[0], p3[0])};
+            *reinterpret_cast<dec_u32x2*>(to + kFlashVStride) = dec_u32x2{pair_high(p0[0], p1[0]), pair_high(p2[0], p3[0])};
+            *reinterpret_cast<dec_u32x2*>(to + 2 * kFlashVStride) = dec_u32x2{pair_low(p0[1], p1[1]), pair_low(p2[1], p3[1])};
+            *reinterpret_cast<dec_u32x2*>(to + 3 * kFlashVStride) = dec_u32x2{pair_high(p0[1], p1[1]), pair_high(p2[1], p3[1])};
         }
     };
 
@@ -140,23 +143,22 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
         const uint16_t* k_row = ks + (32 * part + (lane & 31)) * Shape::kKStride + 8 * half;
 #pragma unroll
         for (int kb = 0; kb < kKb; ++kb) {
-            if (kb >= key_blocks) break;
-            const uint4 a = *reinterpret_cast<const uint4*>(k_row + kb * 16);
+            const dec_u32x4 a = *reinterpret_cast<const dec_u32x4*>(k_row + kb * 16);
             s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, q[kb]), s, 0, 0, 0);
         }
         // register r is key k0 + 8 (r / 4) + 4 half + r % 4
         float p[16];
         const bool whole = k0 >= wave_lo_most && k0 + 31 <= wave_first;
-        float largest = -INFINITY;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) {
-            p[r] = s[r] * to_log2;
-            if (!whole) {
-                const int key = k0 + 8 * (r / 4) + 4 * half + r % 4;
-                if (key < lo || key > position) p[r] = -INFINITY;
-            }
-            largest = fmaxf(largest, p[r]);
+        for (int r = 0; r < 16; ++r) p[r] = s[r] * to_log2;
+        if (!whole) {
+            const int first = lo - k0 - 4 * half, last = position - k0 - 4 * half;
+#pragma unroll
+            for (int r = 0; r < 16; ++r) p[r] = 8 * (r / 4) + r % 4 >= first && 8 * (r / 4) + r % 4 <= last ? p[r] : -INFINITY;
         }
+        float largest = p[0];
+#pragma unroll
+        for (int r = 1; r < 16; ++r) largest = fmaxf(largest, p[r]);
         largest = fmaxf(largest, __shfl_xor(largest, 32, 64));
         const float before = m;
         m = fmaxf(m, largest);
@@ -175,27 +177,24 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
 #pragma unroll
                 for (int r = 0; r < 16; ++r) o[t][r] *= alpha;
         }
-        uint4 high[2], low[2];
+        dec_u32x4 high[2], low[2];
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
-            uint32_t h4[4], l4[4];
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const float x = p[8 * b + 2 * e], y = p[8 * b + 2 * e + 1];
-                h4[e] = pack_bf16_pair(x, y);
-                l4[e] = pack_bf16_pair(x - lo_bf16(h4[e]), y - hi_bf16(h4[e]));
+                const uint32_t pair_of = pack_bf16_pair(x, y);
+                high[b][e] = pair_of;
+                low[b][e] = pack_bf16_pair(x - lo_bf16(pair_of), y - hi_bf16(pair_of));
             }
-            high[b] = make_uint4(h4[0], h4[1], h4[2], h4[3]);
-            low[b] = make_uint4(l4[0], l4[1], l4[2], l4[3]);
         }
 #pragma unroll
         for (int t = 0; t < kVt; ++t) {
-            if (t >= value_tiles) break;
             const uint16_t* v_row = vt + (32 * t + (lane & 31)) * kFlashVStride + 32 * part + 4 * half;
 #pragma unroll
             for (int b = 0; b < 2; ++b) {
-                const uint2 first = *reinterpret_cast<const uint2*>(v_row + 16 * b), second = *reinterpret_cast<const uint2*>(v_row + 16 * b + 8);
-                const uint4 a = make_uint4(first.x, first.y, second.x, second.y);
+                const dec_u32x2 first = *reinterpret_cast<const dec_u32x2*>(v_row + 16 * b), second = *reinterpret_cast<const dec_u32x2*>(v_row + 16 * b + 8);
+                const dec_u32x4 a = {first[0], first[1], second[0], second[1]};
                 o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, high[b]), o[t], 0, 0, 0);
                 o[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, low[b]), o[t], 0, 0, 0);
             }

@@ -19,20 +19,22 @@ constexpr int kDecayVStride = kDecaySlice + 4;
 template <class F>
 __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, float* to, int stride, int t0, int column, int columns, int padded, F factor) {
     const int c4 = (threadIdx.x & 15) * 4, row = threadIdx.x >> 4;
+    const bool vectors = ((column | columns | prm.ld_proj) & 3) == 0;
     for (int c = c4; c < padded; c += 64) {
         float4 x[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int j = row + 16 * i;
-            const bool in = t0 + j < prm.rows;
-            const float* p = prm.proj + (t0 + j) * prm.ld_proj + column + c;
-            if (in && c + 3 < columns && ((column | prm.ld_proj) & 3) == 0) {
-                x[i] = *reinterpret_cast<const float4*>(p);
+        for (int i = 0; i < 4; ++i) {          // (rows past the last repeat it, with factor zero: no branch around a load)
+            const float* p = prm.proj + min(t0 + row + 16 * i, prm.rows - 1) * prm.ld_proj + column;
+            if (vectors) {
+                x[i] = load4_if(c < columns, p, c >> 2);
             } else {
-                x[i].x = in && c < columns ? p[0] : 0.0f;
-                x[i].y = in && c + 1 < columns ? p[1] : 0.0f;
-                x[i].z = in && c + 2 < columns ? p[2] : 0.0f;
-                x[i].w = in && c + 3 < columns ? p[3] : 0.0f;
+                float e[4];
+#pragma unroll
+                for (int n = 0; n < 4; ++n) {
+                    const float v = p[min(c + n, columns - 1)];
+                    e[n] = c + n < columns ? v : 0.0f;
+                }
+                x[i] = make_float4(e[0], e[1], e[2], e[3]);
             }
         }
 #pragma unroll
@@ -47,7 +49,7 @@ __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, floa
 __global__ __launch_bounds__(kDecThreads) void decay_chunk_state_kernel(DecayAttentionParams prm) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, l16 = lane & 15;
-    const int chunk = static_cast<int>(blockIdx.x), head = static_cast<int>(blockIdx.y), e0 = static_cast<int>(blockIdx.z) * kDecaySlice;
+    const int head = static_cast<int>(blockIdx.x), chunk = static_cast<int>(blockIdx.y), e0 = static_cast<int>(blockIdx.z) * kDecaySlice;
     const int t0 = chunk * kDecayChunk, tokens = min(kDecayChunk, prm.rows - t0);
     const int dp = mfma32_pad(prm.dim), stride = mfma32_stride(prm.dim);
     const float* powers = prm.powers + head * kDecayPowers;
@@ -103,7 +105,7 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_walk_kernel(DecayAtte
 __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAttentionParams prm) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, l16 = lane & 15;
-    const int chunk = static_cast<int>(blockIdx.x), head = static_cast<int>(blockIdx.y);
+    const int head = static_cast<int>(blockIdx.x), chunk = static_cast<int>(blockIdx.y);
     const int t0 = chunk * kDecayChunk, e0 = static_cast<int>(blockIdx.z) * kDecaySlice;
     const int dp = mfma32_pad(prm.dim), stride = mfma32_stride(prm.dim);
     const float* powers = prm.powers + head * kDecayPowers;
@@ -143,10 +145,7 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
     for (int d0 = 0; d0 < dp; d0 += 16) {
         float s[4];
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            const int d = d0 + 4 * g + t;
-            s[t] = d < prm.dim && column < prm.vdim ? before[static_cast<int64_t>(d) * prm.vdim + column] : 0.0f;
-        }
+        for (int t = 0; t < 4; ++t) s[t] = before[min(d0 + 4 * g + t, prm.dim - 1) * prm.vdim + min(column, prm.vdim - 1)];   // (q is zero past the head)
         const float4 b = make_float4(s[0], s[1], s[2], s[3]);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -187,11 +186,11 @@ int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream)
     if (rc == QM_OK) rc = ensure_dynamic_lds(reinterpret_cast<const void*>(decay_chunk_output_kernel), kDotLdsMost, raised[1]);
     if (rc != QM_OK) return rc;
     if (output_lds > kDotLdsMost || chunks > 65535 || prm.scratch_floats < decay_scratch_floats(prm.rows, prm.heads, prm.dim, prm.vdim)) return QM_ERR_WORKSPACE;
-    hipLaunchKernelGGL(decay_chunk_state_kernel, dim3(chunks, prm.heads, slices), dim3(kDecThreads), state_lds, stream, prm);
+    hipLaunchKernelGGL(decay_chunk_state_kernel, dim3(prm.heads, chunks, slices), dim3(kDecThreads), state_lds, stream, prm);
     const int64_t plane = static_cast<int64_t>(prm.heads) * prm.dim * prm.vdim;
     hipLaunchKernelGGL(decay_chunk_walk_kernel, dim3(static_cast<unsigned>((plane + kDecThreads - 1) / kDecThreads)), dim3(kDecThreads), 0, stream, prm,
                        chunks);
-    hipLaunchKernelGGL(decay_chunk_output_kernel, dim3(chunks, prm.heads, slices), dim3(kDecThreads), output_lds, stream, prm);
+    hipLaunchKernelGGL(decay_chunk_output_kernel, dim3(prm.heads, chunks, slices), dim3(kDecThreads), output_lds, stream, prm);
     return launch_status();
 }
 

@@ -21,36 +21,45 @@ namespace qm {
 constexpr int kDeltaChunk = 32;
 constexpr int kDeltaMat = kDeltaChunk + 4;     // row stride of a [32][32] matrix in LDS
 
-// Scratch of a (chunk, head), floats: M, X [32][dp], -A^T W, K^T W [dp][32], N, Y [32][32], W [dp].
+// Channels of a head as the prepared matrices have them: what lies behind the head's own is zero (decays: one).
+__host__ __device__ inline int delta_pad(int dim) { return (dim + 63) / 64 * 64; }
+
+// Scratch of a (chunk, head), floats: M, X (32 x dp), -A^T W, K^T W (dp x 32), N, Y [32][32], W [dp].  The first four are kept
+// as the walk's left operands: 16 x 16 blocks of 64 float4s, lane l's being row l % 16, columns 4 (l / 16) .. + 3 of the block.
 struct DeltaScratch {
     int m, x, at, kt, n, y, w, floats;
 };
 __host__ __device__ inline DeltaScratch delta_scratch(int dim) {
-    const int dp = mfma32_pad(dim), rows = kDeltaChunk * dp, square = kDeltaChunk * kDeltaChunk;
+    const int dp = delta_pad(dim), rows = kDeltaChunk * dp, square = kDeltaChunk * kDeltaChunk;
     DeltaScratch s;
     s.m = 0; s.x = rows; s.at = 2 * rows; s.kt = 3 * rows; s.n = 4 * rows; s.y = s.n + square; s.w = s.y + square;
-    s.floats = s.w + (dp + 63) / 64 * 64;
+    s.floats = s.w + dp;
     return s;
 }
 __host__ __device__ inline int delta_z_stride(int rank) { return (rank + 3) / 4 * 4; }
-inline int delta_prepare_lds(int dim) { return 4 * kDeltaChunk * mfma32_stride(dim) + 5 * kDeltaChunk * kDeltaMat + kDeltaChunk; }
+// the float4 of row r, columns c .. c + 3 of block `block` (16 x 16)
+__device__ __forceinline__ int operand_at(int block, int r, int c) { return (block * 64 + (c >> 2 & 3) * 16 + (r & 15)) * 4; }
+inline int delta_prepare_lds(int dim) {
+    const int half = 2 * kDeltaChunk * mfma32_stride(dim), squares = 5 * kDeltaChunk * kDeltaMat;
+    return kDeltaChunk + half + (half > squares ? half : squares);
+}
 
 __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaParams prm) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l16 = lane & 15;
     const int chunk = static_cast<int>(blockIdx.x), head = static_cast<int>(blockIdx.y);
     const int t0 = chunk * kDeltaChunk, tokens = min(kDeltaChunk, prm.rows - t0);
-    const int dim = prm.dim, dp = mfma32_pad(dim), stride = mfma32_stride(dim);
+    const int dim = prm.dim, dp = delta_pad(dim), stride = mfma32_stride(dim);
     const DeltaScratch at = delta_scratch(dim);
     float* scratch = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * at.floats;
-    float* us = lds;                           // [32][stride] each; us holds the decays first
-    float* as = us + kDeltaChunk * stride;
+    float* inverse = lds;                      // [32]
+    float* us = inverse + kDeltaChunk;         // [32][stride] each; us holds the decays first
+    float* rs = us + kDeltaChunk * stride;
+    float* as = rs + kDeltaChunk * stride;
     float* ks = as + kDeltaChunk * stride;
-    float* rs = ks + kDeltaChunk * stride;
-    float* mats = rs + kDeltaChunk * stride;   // L_A, L_K, D_A, D_K, each [32][kDeltaMat]
-    float* inverted = mats + 4 * kDeltaChunk * kDeltaMat;          // (I + L_A)^-1
-    float* inverse = inverted + kDeltaChunk * kDeltaMat;
-    float* zs = as;                            // tanh of the rank-sized projection, [32][z_stride], until the decays are there
+    float* mats = as;                          // once A and K are used up: L_A, L_K, D_A, D_K, each [32][kDeltaMat]
+    float* inverted = mats + 4 * kDeltaChunk * kDeltaMat;          // and (I + L_A)^-1
+    float* zs = rs;                            // tanh of the rank-sized projection, [32][z_stride], until the decays are there
     const int z_stride = delta_z_stride(prm.rank);
 
     for (int i = tid; i < kDeltaChunk * z_stride; i += kDecThreads) {
@@ -78,7 +87,7 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
             for (int r = 0; r < prm.rank; r += 4) {
                 float w[4];
 #pragma unroll
-                for (int e = 0; e < 4; ++e) w[e] = r + e < prm.rank ? w2[static_cast<int64_t>(r + e) * all] : 0.0f;
+                for (int e = 0; e < 4; ++e) w[e] = w2[static_cast<int64_t>(min(r + e, prm.rank - 1)) * all];      // (zs is zero past the rank)
 #pragma unroll
                 for (int t = 0; t < 16; ++t) {
                     const float4 x = *reinterpret_cast<const float4*>(zs + (first + t) * z_stride + r);
@@ -122,16 +131,17 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const bool in = t1 + e < tokens && c < dim;
-                const float* p = prm.proj + (t0 + t1 + e) * prm.ld_proj + head * dim + c;
-                k[e] = in ? p[prm.k_column] : 0.0f;
-                r[e] = in ? p[prm.r_column] : 0.0f;
-                a[e] = in ? p[prm.a_column] : 0.0f;
+                const float* p = prm.proj + min(t0 + t1 + e, prm.rows - 1) * prm.ld_proj + head * dim + min(c, dim - 1);
+                const float k_read = p[prm.k_column], r_read = p[prm.r_column];
+                a[e] = p[prm.a_column];
+                k[e] = in ? k_read : 0.0f;
+                r[e] = in ? r_read : 0.0f;
             }
 #pragma unroll
             for (int e = 3; e >= 0; --e) {
                 const int t = t1 + e;
                 const float after = rs[t * stride + c], before = t > first ? rs[(t - 1) * stride + c] : edge[n];
-                const float u = t < tokens ? k[e] * inverse[t] : 0.0f;
+                const float u = k[e] * inverse[min(t, tokens - 1)];
                 const float removal = sigmoid_f32(a[e] + bias) * u, over = reciprocal(after);
                 us[t * stride + c] = u * before;
                 as[t * stride + c] = removal * over;
@@ -140,8 +150,9 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
                 at_[e] = -whole[n] * removal * over;
                 kt_[e] = whole[n] * k[e] * over;
             }
-            *reinterpret_cast<float4*>(scratch + at.at + c * kDeltaChunk + t1) = make_float4(at_[0], at_[1], at_[2], at_[3]);
-            *reinterpret_cast<float4*>(scratch + at.kt + c * kDeltaChunk + t1) = make_float4(kt_[0], kt_[1], kt_[2], kt_[3]);
+            const int to = operand_at(c / 16 * 2 + t1 / 16, c, t1);
+            *reinterpret_cast<float4*>(scratch + at.at + to) = make_float4(at_[0], at_[1], at_[2], at_[3]);
+            *reinterpret_cast<float4*>(scratch + at.kt + to) = make_float4(kt_[0], kt_[1], kt_[2], kt_[3]);
         }
     }
     __syncthreads();
@@ -160,6 +171,7 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
             acc[1][0] = mfma32_block(a[1], b[0], acc[1][0]);
             acc[1][1] = mfma32_block(a[1], b[1], acc[1][1]);
         }
+        __syncthreads();
         float* mat = mats + wave * kDeltaChunk * kDeltaMat;
 #pragma unroll
         for (int i = 0; i < 2; ++i)
@@ -214,7 +226,7 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
     // sixteen columns at a time of (U, L_K): times the inverse, and of (R, D_K) less D_A times that
     for (int n = wave; n < dp / 16 + 2; n += 4) {
         const bool wide = n < dp / 16;
-        const int c = wide ? 16 * n : 16 * (n - dp / 16), step = wide ? stride : kDeltaMat, out_step = wide ? dp : kDeltaChunk;
+        const int c = wide ? 16 * n : 16 * (n - dp / 16), step = wide ? stride : kDeltaMat;
         const float* y = wide ? us : l_k;
         const float* z = wide ? rs : d_k;
         float* solved_out = scratch + (wide ? at.m : at.n);
@@ -236,8 +248,9 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_prepare_kernel(DeltaP
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int t = 16 * b + 4 * g + r;
-                solved_out[t * out_step + c + l16] = m[b][r];
-                rest_out[t * out_step + c + l16] = -x[b][r];
+                const int to = wide ? operand_at(2 * n + b, t, l16) + (l16 & 3) : t * kDeltaChunk + c + l16;
+                solved_out[to] = m[b][r];
+                rest_out[to] = -x[b][r];
             }
     }
 }
@@ -250,14 +263,18 @@ struct DeltaStep {
     float v[2][4], own[2];
 };
 
+// A barrier for what went into LDS: unlike __syncthreads it leaves the loads under way (the next chunk's) in flight.
+__device__ __forceinline__ void block_exchange() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // TW: 16-row tiles of the state per wave (tile = wave + 4 i)
 template <int TW>
 __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaParams prm, int chunks) {
     constexpr int kStride = 20;                                    // the four row groups of a store lie in different banks
     __shared__ float sh[2][4][2][kDeltaChunk * kStride];           // by turns: each wave's share of P and of O
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, l16 = lane & 15;
-    const int head = static_cast<int>(blockIdx.y), column = static_cast<int>(blockIdx.x) * 16 + l16;
-    const int dim = prm.dim, dp = mfma32_pad(dim);
+    // (block numbers go round the dies: the blocks of a head, which read the same matrices, share one's L2)
+    const int head = static_cast<int>(blockIdx.x), column = static_cast<int>(blockIdx.y) * 16 + l16;
+    const int dim = prm.dim;
     const DeltaScratch at = delta_scratch(dim);
     float* state = prm.state + static_cast<int64_t>(head) * dim * dim;
     const int part = wave >> 1, pair = 2 * (wave & 1);             // the wave's terms of N V and Y V: tokens 16 part + 4 g + pair, + 1
@@ -267,27 +284,26 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int d = 16 * (wave + 4 * i) + 4 * g + r;
-            s[i][r] = d < dim && column < dim ? state[static_cast<int64_t>(d) * dim + column] : 0.0f;
+            const float value = state[min(d, dim - 1) * dim + min(column, dim - 1)];
+            s[i][r] = d < dim ? value : 0.0f;
         }
-    const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-    auto value_at = [&](int token) {
-        return token < prm.rows && column < dim ? prm.proj[token * prm.ld_proj + prm.v_column + head * dim + column] : 0.0f;
-    };
+    // (a token past the last meets zeros, a column past the head is not stored: both repeat the last, no branch around a load)
+    const float* values = prm.proj + prm.v_column + head * dim + min(column, dim - 1);
+    auto value_at = [&](int token) { return values[min(token, prm.rows - 1) * prm.ld_proj]; };
     auto request = [&](int chunk, DeltaStep<TW>& f) __attribute__((always_inline)) {
         const float* from = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * at.floats;
 #pragma unroll
         for (int i = 0; i < TW; ++i) {
             const int tile = wave + 4 * i;
-            const bool in = 16 * tile < dp;
 #pragma unroll
             for (int b = 0; b < 2; ++b) {
-                const int row = (16 * b + l16) * dp + 16 * tile + 4 * g, channel = (16 * tile + l16) * kDeltaChunk + 16 * b + 4 * g;
-                f.m[b][i] = in ? *reinterpret_cast<const float4*>(from + at.m + row) : zero;
-                f.x[b][i] = in ? *reinterpret_cast<const float4*>(from + at.x + row) : zero;
-                f.at[i][b] = in ? *reinterpret_cast<const float4*>(from + at.at + channel) : zero;
-                f.kt[i][b] = in ? *reinterpret_cast<const float4*>(from + at.kt + channel) : zero;
+                const int operand = ((2 * tile + b) * 64 + lane) * 4;
+                f.m[b][i] = *reinterpret_cast<const float4*>(from + at.m + operand);
+                f.x[b][i] = *reinterpret_cast<const float4*>(from + at.x + operand);
+                f.at[i][b] = *reinterpret_cast<const float4*>(from + at.at + operand);
+                f.kt[i][b] = *reinterpret_cast<const float4*>(from + at.kt + operand);
             }
-            f.w[i] = in ? *reinterpret_cast<const float4*>(from + at.w + 16 * tile + 4 * g) : zero;
+            f.w[i] = *reinterpret_cast<const float4*>(from + at.w + 16 * tile + 4 * g);
         }
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
@@ -300,7 +316,11 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
         }
     };
     auto walk = [&](int chunk, DeltaStep<TW>& f, DeltaStep<TW>& next) __attribute__((always_inline)) {
-        if (chunk + 1 < chunks) request(chunk + 1, next);
+        // this chunk's loads, a whole step under way, have to be there; then the next one's go out
+        __builtin_amdgcn_s_waitcnt((7 << 4) | (15 << 8));          // vmcnt(0), nothing else
+        __builtin_amdgcn_sched_barrier(0);
+        request(min(chunk + 1, chunks - 1), next);
+        __builtin_amdgcn_sched_barrier(0);
         f32x4_t p[2] = {}, o[2] = {};
 #pragma unroll
         for (int i = 0; i < TW; ++i) {
@@ -329,15 +349,19 @@ __global__ __launch_bounds__(kDecThreads) void delta_chunk_walk_kernel(DeltaPara
 #pragma unroll
             for (int b = 0; b < 2; ++b) s[i] = mfma32_block(f.kt[i][b], make_float4(f.v[b][0], f.v[b][1], f.v[b][2], f.v[b][3]), s[i]);
         }
-        __syncthreads();
-        float read[2][4];
+        block_exchange();
+        float share[4][2][4], read[2][4];
+#pragma unroll
+        for (int w = 0; w < 4; ++w)
+#pragma unroll
+            for (int b = 0; b < 2; ++b)
+#pragma unroll
+                for (int t = 0; t < 4; ++t) share[w][b][t] = sh[chunk & 1][w][0][(16 * b + 4 * g + t) * kStride + l16];
+        __builtin_amdgcn_sched_barrier(0);                         // (all of them requested before the first is waited for)
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
-            for (int t = 0; t < 4; ++t) {
-                const int from = (16 * b + 4 * g + t) * kStride + l16;
-                read[b][t] = (sh[chunk & 1][0][0][from] + sh[chunk & 1][1][0][from]) + (sh[chunk & 1][2][0][from] + sh[chunk & 1][3][0][from]);
-            }
+            for (int t = 0; t < 4; ++t) read[b][t] = (share[0][b][t] + share[1][b][t]) + (share[2][b][t] + share[3][b][t]);
 #pragma unroll
         for (int i = 0; i < TW; ++i)
 #pragma unroll
@@ -380,9 +404,10 @@ int32_t launch_delta_chunks(const DeltaParams& prm, hipStream_t stream) {
     if (rc != QM_OK) return rc;
     if (lds > kDotLdsMost || prm.scratch_floats < delta_scratch_floats(prm.rows, prm.heads, prm.dim)) return QM_ERR_WORKSPACE;
     hipLaunchKernelGGL(delta_chunk_prepare_kernel, dim3(chunks, prm.heads), dim3(kDecThreads), lds, stream, prm);
-    const dim3 grid((prm.dim + 15) / 16, prm.heads);
+    const dim3 grid(prm.heads, (prm.dim + 15) / 16);
     if (prm.dim <= 64) hipLaunchKernelGGL(delta_chunk_walk_kernel<1>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
     else if (prm.dim <= 128) hipLaunchKernelGGL(delta_chunk_walk_kernel<2>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
+    else if (prm.dim <= 192) hipLaunchKernelGGL(delta_chunk_walk_kernel<3>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
     else hipLaunchKernelGGL(delta_chunk_walk_kernel<4>, grid, dim3(kDecThreads), 0, stream, prm, chunks);
     return launch_status();
 }

@@ -68,6 +68,13 @@ __device__ __forceinline__ void store4(uint16_t* p, int v, float a, float b, flo
     reinterpret_cast<uint2*>(p)[v] = make_uint2(pack_bf16_pair(a, b), pack_bf16_pair(c, d));
 }
 __device__ __forceinline__ float square_sum(float4 v, float sum) { return fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, sum)))); }
+// Element v, or zeros where it is not wanted: the load is made either way (from the first element), because a load under a
+// condition would wait its turn behind a branch.
+template <class P>
+__device__ __forceinline__ float4 load4_if(bool wanted, const P* p, int v) {
+    const float4 x = load4(p, wanted ? v : 0);
+    return make_float4(wanted ? x.x : 0.0f, wanted ? x.y : 0.0f, wanted ? x.z : 0.0f, wanted ? x.w : 0.0f);
+}
 // acc + f * y * w
 __device__ __forceinline__ float4 weighted(float4 acc, float f, float4 y, float4 w) {
     return make_float4(fmaf(f * y.x, w.x, acc.x), fmaf(f * y.y, w.y, acc.y), fmaf(f * y.z, w.z, acc.z), fmaf(f * y.w, w.w, acc.w));
@@ -93,9 +100,9 @@ __device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int
     for (int i = 0; i < NV; ++i) {
         const int v = tid + i * kDecThreads;
         const bool in = v < vectors;
-        x[i] = !in ? zero : embedding ? load4(embedding, v) : load4(prm.x_in + src * prm.ld_h, v);
+        x[i] = embedding ? load4_if(in, embedding, v) : load4_if(in, prm.x_in + src * prm.ld_h, v);
 #pragma unroll
-        for (int t = 0; t < 3; ++t) y[t][i] = in && y_row[t] ? load4(y_row[t], v) : zero;
+        for (int t = 0; t < 3; ++t) y[t][i] = y_row[t] ? load4_if(in, y_row[t], v) : zero;
     }
     const float inv_width = 1.0f / static_cast<float>(prm.width);
     float factor[3] = {0.0f, 0.0f, 0.0f};
@@ -152,9 +159,8 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
 #pragma unroll
         for (int i = 0; i < kHeld; ++i) {
             const int v = tid + i * kDecThreads;
-            if (v >= vectors) continue;
-            held[i] = load4(o, v);
-            g[i] = load4(gate, v);
+            held[i] = load4_if(v < vectors, o, v);
+            g[i] = load4_if(v < vectors, gate, v);
             sq[0] = square_sum(held[i], sq[0]);
         }
         block_sums<1>(sq, sh_red);
@@ -182,8 +188,10 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
             for (int i = 0; i < 4; ++i) {
                 const int c = lane + 64 * i;
                 const bool in = c < prm.size;
-                held[i] = in ? o[g * prm.size + c] : 0.0f;
-                gates[i] = in ? gate[g * prm.size + c] : 0.0f;
+                const int at = g * prm.size + (in ? c : 0);
+                const float value = o[at];
+                gates[i] = gate[at];
+                held[i] = in ? value : 0.0f;
                 sq = fmaf(held[i], held[i], sq);
             }
             for (int c = lane + 256; c < prm.size; c += 64) sq = fmaf(o[g * prm.size + c], o[g * prm.size + c], sq);

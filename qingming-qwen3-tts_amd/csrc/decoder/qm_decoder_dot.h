@@ -58,8 +58,9 @@ __device__ __forceinline__ DotRows<NR> dot_rows(const DecLinearGroup& g, int til
 
 template <int NR>
 __device__ __forceinline__ void dot_request_one(const DotRows<NR>& d, int k, int at, uint4 (&piece)[NR]) {
+    const int from = at < k ? at : 0;          // (past the end: not used; a load under a condition would stand behind a branch)
 #pragma unroll
-    for (int i = 0; i < NR; ++i) piece[i] = at < k ? *reinterpret_cast<const uint4*>(d.row[i] + at) : make_uint4(0, 0, 0, 0);
+    for (int i = 0; i < NR; ++i) piece[i] = *reinterpret_cast<const uint4*>(d.row[i] + from);
 }
 // Requests the first pieces of a wave's weight rows; they may be asked for before the input rows are known.
 template <int NR>

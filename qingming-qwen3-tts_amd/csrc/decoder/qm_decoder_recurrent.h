@@ -16,13 +16,13 @@ __host__ __device__ inline int rec_stride(int rd) { return 4 * (rd + 4); }
 template <int RD>
 __device__ __forceinline__ int rec_at(int channel) { return (channel / RD) * (RD + 4) + channel % RD; }
 
+// (Rows and columns past the state repeat its last ones: no branch around a load.  Their vectors are zeros, and they are
+// not stored.)
 template <int RD>
 __device__ __forceinline__ void load_state(float (&s)[RD], const float* state, int dim, int columns, int sub, int column) {
+    column = min(column, columns - 1);
 #pragma unroll
-    for (int i = 0; i < RD; ++i) {
-        const int d = sub * RD + i;
-        s[i] = d < dim && column < columns ? state[static_cast<int64_t>(d) * columns + column] : 0.0f;
-    }
+    for (int i = 0; i < RD; ++i) s[i] = state[min(sub * RD + i, dim - 1) * columns + column];
 }
 template <int RD>
 __device__ __forceinline__ void store_state(const float (&s)[RD], float* state, int dim, int columns, int sub, int column) {
@@ -191,14 +191,15 @@ __device__ __forceinline__ void general_delta_step(const DeltaParams& prm, int h
     const bool in = c < prm.dim;
     const int at = head * prm.dim + (in ? c : 0), all = prm.heads * prm.dim;
     const float* p = prm.proj + at;
-    const float k = in ? p[prm.k_column] : 0.0f, r = p[prm.r_column], a = p[prm.a_column];
+    const float k_read = p[prm.k_column], r = p[prm.r_column], a = p[prm.a_column];
+    const float k = in ? k_read : 0.0f;
     const float bias = prm.a_bias[at], w0 = prm.w0[at];
-    const float v = column < prm.dim ? prm.proj[prm.v_column + head * prm.dim + column] : 0.0f;
+    const float v = prm.proj[prm.v_column + head * prm.dim + min(column, prm.dim - 1)];
     const int ranks = (prm.rank + kParts - 1) / kParts, first = part * ranks, last = min(prm.rank, first + ranks);
     const float* w2 = prm.w2 + at;
     float piece[kAhead];
 #pragma unroll
-    for (int i = 0; i < kAhead; ++i) piece[i] = first + i < last ? w2[static_cast<int64_t>(first + i) * all] : 0.0f;
+    for (int i = 0; i < kAhead; ++i) piece[i] = w2[static_cast<int64_t>(min(first + i, prm.rank - 1)) * all];
     const float z0 = tid < prm.rank ? prm.proj[prm.z_column + tid] : 0.0f;
     float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.dim;
     float s[RD];
@@ -214,7 +215,7 @@ __device__ __forceinline__ void general_delta_step(const DeltaParams& prm, int h
 #pragma unroll
         for (int i = 0; i < kAhead; ++i) {
             now[i] = piece[i];
-            piece[i] = i0 + kAhead + i < last ? w2[static_cast<int64_t>(i0 + kAhead + i) * all] : 0.0f;
+            piece[i] = w2[static_cast<int64_t>(min(i0 + kAhead + i, prm.rank - 1)) * all];
         }
 #pragma unroll
         for (int i = 0; i < kAhead; ++i)

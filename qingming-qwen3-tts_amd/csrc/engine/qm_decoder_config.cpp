@@ -46,12 +46,14 @@ ChunkAttentionConfig chunk_attention(const Json& j) {
     c.vdim = count(j, "vdim");
     c.scale = number(j, "scale");
     c.chunk = count(member(j, "mask"), "size");
-    const Json& rot = member(j, "rot");
-    c.rot_dims = count(rot, "dims", 0);
-    c.rot_base = number(rot, "base");
+    if (!absent(j, "rot")) {
+        const Json& rot = member(j, "rot");
+        c.rot_dims = count(rot, "dims", 0);
+        c.rot_base = number(rot, "base");
+        if (!(c.rot_base > 0.0)) fail("'rot.base' is not positive");
+    }
     if (c.heads % c.kv_heads) fail("'heads' is not a multiple of 'kv_heads'");
     if (c.rot_dims % 2 || c.rot_dims > c.dim) fail("'rot.dims' does not fit the head");
-    if (!(c.rot_base > 0.0)) fail("'rot.base' is not positive");
     return c;
 }
 
@@ -63,7 +65,7 @@ DecayAttentionConfig decay_attention(const Json& j) {
     const Json& decay = member(j, "decay");
     if (decay.kind != Json::Array || static_cast<int>(decay.items.size()) != c.heads) fail("'decay' does not name one value per head");
     for (const Json& v : decay.items) {
-        if (v.kind != Json::Number || !(v.number >= 0.0) || v.number > 1.0) fail("a decay is not between 0 and 1");
+        if (v.kind != Json::Number || !std::isfinite(v.number)) fail("a decay is not a number");
         c.decay.push_back(v.number);
     }
     return c;

@@ -86,6 +86,22 @@ def lib():
     return _lib
 
 
+def build_if_missing():
+    """Builds the library (and nothing else) if it is not there; of several processes one builds."""
+    if os.path.exists(_LIB_PATH):
+        return
+    import fcntl
+    import importlib.util
+    spec = importlib.util.spec_from_file_location("qm_build", os.path.join(HERE, "build.py"))
+    build = importlib.util.module_from_spec(spec)
+    spec.loader.exec_module(build)
+    os.makedirs(build.LIB_DIR, exist_ok=True)
+    with open(os.path.join(build.LIB_DIR, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not os.path.exists(_LIB_PATH):
+            build.build_decoder(verbose=False)
+
+
 def _check(code):
     if code != 0:
         raise DecoderError(code, lib().qm_decoder_last_error().decode("utf-8", "replace"))
