@@ -1229,7 +1229,7 @@ def talker_throughput(dev, rows=1024, steps=64, layers=4):
 def decoder_report(which, dev):
     """Every size (or the one named), and the talker at the size they share."""
     report = {}
-    for size in DECODER_SIZES if which == "all" else [which.split(":")[0]]:
+    for size in DECODER_SIZES if which == "all" else [] if which == "talker" else [which.split(":")[0]]:
         kinds = which.split(":")[1].split(",") if ":" in which else None
         for name, r in decoder_throughput(size, dev, kinds=kinds).items():
             report[f"vabevik_{size}_{name}"] = r
@@ -1313,7 +1313,7 @@ def main():
                          "records counters for every dispatch is spared most of the input generation with a small number)")
     ap.add_argument("--decoder", nargs="?", const="all", default=None, metavar="SIZE[:KINDS]",
                     help="prefill and decode throughput of the decoder language models (" + ", ".join(DECODER_SIZES) + ", or all) beside the "
-                         "talker's, instead of the attention workloads; SIZE:KINDS times that size's layer kinds alone (mixed, parallel, "
+                         "talker's, instead of the attention workloads (talker: that alone); SIZE:KINDS times that size's layer kinds alone (mixed, parallel, "
                          "general_delta)")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run three plain 512 MiB device-to-device copies (for scaling rocprofv3's "

@@ -7,16 +7,26 @@ namespace qm {
 
 constexpr int kAttTile = 128;                  // keys per pass
 
-// eight consecutive values as fp32
-__device__ __forceinline__ void load8(const uint16_t* p, float (&v)[8]) {
-    const uint4 w = *reinterpret_cast<const uint4*>(p);
-    v[0] = lo_bf16(w.x); v[1] = hi_bf16(w.x); v[2] = lo_bf16(w.y); v[3] = hi_bf16(w.y);
-    v[4] = lo_bf16(w.z); v[5] = hi_bf16(w.z); v[6] = lo_bf16(w.w); v[7] = hi_bf16(w.w);
-}
-__device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
-    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
-    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
-}
+// Eight consecutive values as they lie in memory, and as fp32.
+template <class T> struct Raw8;
+template <> struct Raw8<uint16_t> {
+    uint4 w;
+    __device__ __forceinline__ void load(const uint16_t* p) { w = *reinterpret_cast<const uint4*>(p); }
+    __device__ __forceinline__ void widen(float (&v)[8]) const {
+        v[0] = lo_bf16(w.x); v[1] = hi_bf16(w.x); v[2] = lo_bf16(w.y); v[3] = hi_bf16(w.y);
+        v[4] = lo_bf16(w.z); v[5] = hi_bf16(w.z); v[6] = lo_bf16(w.w); v[7] = hi_bf16(w.w);
+    }
+};
+template <> struct Raw8<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float* p) {
+        a = reinterpret_cast<const float4*>(p)[0];
+        b = reinterpret_cast<const float4*>(p)[1];
+    }
+    __device__ __forceinline__ void widen(float (&v)[8]) const {
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+    }
+};
 
 // Channel c of a head as it enters the scores: channels i and i + rot_dims / 2 turn together, the rest pass, zeros behind.
 __device__ __forceinline__ float rotated_channel(const float* head, int c, int dim, int rot_dims, const double* frequency, int position) {
@@ -41,7 +51,9 @@ __host__ __device__ inline int attention_lds_floats(int gq, int k_stride, int v_
 }
 
 // FUSED: q comes from the projections and is rotated here, and the block that holds the row's own key rotates and stores
-// key and value first.  Otherwise q_rot and the cache are complete.  GQ query heads at a time.
+// key and value first.  Otherwise q_rot and the cache are complete.  GQ query heads at a time; VC: pieces of 128 channels of a
+// head.  Sixteen lanes hold a key (or a value) of 128 channels, a wave four of them, the block sixteen; a tile's eight keys
+// and values of a lane are requested at once, before the first is used.
 template <class T, int GQ, int VC, bool FUSED>
 __device__ __forceinline__ void chunk_attention_block(const ChunkAttentionParams& prm, int split, int kv_head, int row, float* lds) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -101,23 +113,46 @@ __device__ __forceinline__ void chunk_attention_block(const ChunkAttentionParams
 #pragma unroll
                 for (int e = 0; e < 8; ++e) acc[g][x][e] = 0.0f;
         __syncthreads();
+        float q[GQ][VC][8];                    // (channels past the head: zeros, against whatever the clamped loads bring)
+#pragma unroll
+        for (int g = 0; g < GQ; ++g)
+#pragma unroll
+            for (int x = 0; x < VC; ++x)
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const int c = x * 128 + l16 * 8 + e;
+                    q[g][x][e] = c < prm.k_stride ? qs[g * prm.k_stride + min(c, prm.k_stride - 1)] : 0.0f;
+                }
         for (int tile = begin; tile < end; tile += kAttTile) {
             const int keys = min(kAttTile, end - tile);
-            for (int j = wave * 4 + sub; j < keys; j += 16) {
-                const T* k = k_cache + slot_of(tile + j) * prm.k_stride;
+            constexpr int kEach = kAttTile / 16;
+            Raw8<T> k_raw[kEach][VC], v_raw[kEach][VC];
+#pragma unroll
+            for (int i = 0; i < kEach; ++i) {  // (keys past the last repeat it: not used)
+                const int64_t slot = slot_of(tile + min(wave * 4 + sub + 16 * i, keys - 1));
+#pragma unroll
+                for (int x = 0; x < VC; ++x) k_raw[i][x].load(k_cache + slot * prm.k_stride + min(x * 128 + l16 * 8, prm.k_stride - 8));
+            }
+#pragma unroll
+            for (int i = 0; i < kEach; ++i) {
+                const int64_t slot = slot_of(tile + min(wave * 4 + sub + 16 * i, keys - 1));
+#pragma unroll
+                for (int x = 0; x < VC; ++x) v_raw[i][x].load(v_cache + slot * prm.v_stride + min(x * 128 + l16 * 8, prm.v_stride - 8));
+            }
+#pragma unroll
+            for (int i = 0; i < kEach; ++i) {
+                const int j = wave * 4 + sub + 16 * i;
                 float s[GQ];
 #pragma unroll
                 for (int g = 0; g < GQ; ++g) s[g] = 0.0f;
-                for (int c = l16 * 8; c < prm.k_stride; c += 128) {
+#pragma unroll
+                for (int x = 0; x < VC; ++x) {
                     float kv[8];
-                    load8(k + c, kv);
+                    k_raw[i][x].widen(kv);
 #pragma unroll
-                    for (int g = 0; g < GQ; ++g) {
-                        float qv[8];
-                        load8(qs + g * prm.k_stride + c, qv);
+                    for (int g = 0; g < GQ; ++g)
 #pragma unroll
-                        for (int e = 0; e < 8; ++e) s[g] = fmaf(kv[e], qv[e], s[g]);
-                    }
+                        for (int e = 0; e < 8; ++e) s[g] = fmaf(kv[e], q[g][x][e], s[g]);
                 }
 #pragma unroll
                 for (int g = 0; g < GQ; ++g) {
@@ -152,20 +187,18 @@ __device__ __forceinline__ void chunk_attention_block(const ChunkAttentionParams
 #pragma unroll
                     for (int e = 0; e < 8; ++e) acc[g][x][e] *= f;
             }
-            for (int j = wave * 4 + sub; j < keys; j += 16) {
-                const T* v = v_cache + slot_of(tile + j) * prm.v_stride;
+#pragma unroll
+            for (int i = 0; i < kEach; ++i) {  // (weights past the last key are zero)
+                const int j = wave * 4 + sub + 16 * i;
 #pragma unroll
                 for (int x = 0; x < VC; ++x) {
-                    const int c = x * 128 + l16 * 8;
-                    if (c < prm.v_stride) {
-                        float vv[8];
-                        load8(v + c, vv);
+                    float vv[8];
+                    v_raw[i][x].widen(vv);
 #pragma unroll
-                        for (int g = 0; g < GQ; ++g) {
-                            const float p = sc[g * kAttTile + j];
+                    for (int g = 0; g < GQ; ++g) {
+                        const float p = sc[g * kAttTile + j];
 #pragma unroll
-                            for (int e = 0; e < 8; ++e) acc[g][x][e] = fmaf(p, vv[e], acc[g][x][e]);
-                        }
+                        for (int e = 0; e < 8; ++e) acc[g][x][e] = fmaf(p, vv[e], acc[g][x][e]);
                     }
                 }
             }

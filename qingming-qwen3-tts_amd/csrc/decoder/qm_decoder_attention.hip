@@ -75,9 +75,10 @@ __global__ __launch_bounds__(kDecThreads) void chunk_attention_kernel(ChunkAtten
 
 template <class T>
 __global__ __launch_bounds__(kDecThreads) void merge_attention_kernel(ChunkAttentionParams prm) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
     const int64_t row = blockIdx.x;
     const int position = position_of(prm.position_dev, prm.position) + static_cast<int>(row);
-    merge_attention_row<T>(prm.part, row, attention_active_splits(position, prm.chunk, prm.part.keys_per_split),
+    merge_attention_row<T>(prm.part, row, attention_active_splits(position, prm.chunk, prm.part.keys_per_split), lds,
                            static_cast<T*>(prm.out) + row * prm.ld_out, prm.ld_out);
 }
 
@@ -90,7 +91,8 @@ int32_t check_attention(const ChunkAttentionParams& p) {
     if (p.rot_dims < 0 || p.rot_dims > p.dim || p.rot_dims % 2 || p.chunk <= 0 || p.ring <= 0) return QM_ERR_GEOMETRY;
     if (p.part.heads != p.heads || p.part.vdim != p.vdim || p.part.splits < 1 || p.part.splits > kDecMaxSplits) return QM_ERR_GEOMETRY;
     if (p.part.keys_per_split <= 0 || static_cast<int64_t>(p.part.keys_per_split) * p.part.splits < p.chunk) return QM_ERR_GEOMETRY;
-    if (p.ld_out < static_cast<int64_t>(p.heads) * p.vdim || p.rows > 65535) return QM_ERR_GEOMETRY;
+    if (p.ld_out < static_cast<int64_t>(p.heads) * p.vdim || p.rows > 65535 || p.ld_out % 4) return QM_ERR_GEOMETRY;
+    if (static_cast<int64_t>(p.heads) * p.part.splits > kDecMaxMerge) return QM_ERR_GEOMETRY;
     return QM_OK;
 }
 
@@ -109,11 +111,11 @@ template <class T, int GQ>
 static int32_t launch_rows(const ChunkAttentionParams& prm, hipStream_t stream) {
     const dim3 grid(prm.part.splits, prm.kv_heads, prm.rows);
     const size_t lds = sizeof(float) * attention_lds_floats(GQ, prm.k_stride, prm.v_stride);
-    if (prm.v_stride <= 128) hipLaunchKernelGGL((chunk_attention_kernel<T, GQ, 1>), grid, dim3(kDecThreads), lds, stream, prm);
+    if (prm.v_stride <= 128 && prm.k_stride <= 128) hipLaunchKernelGGL((chunk_attention_kernel<T, GQ, 1>), grid, dim3(kDecThreads), lds, stream, prm);
     else hipLaunchKernelGGL((chunk_attention_kernel<T, GQ, 2>), grid, dim3(kDecThreads), lds, stream, prm);
     int32_t rc = launch_status();
     if (rc != QM_OK) return rc;
-    hipLaunchKernelGGL(merge_attention_kernel<T>, dim3(prm.rows), dim3(kDecThreads), 0, stream, prm);
+    hipLaunchKernelGGL(merge_attention_kernel<T>, dim3(prm.rows), dim3(kDecThreads), sizeof(float) * prm.heads * prm.part.splits, stream, prm);
     return launch_status();
 }
 

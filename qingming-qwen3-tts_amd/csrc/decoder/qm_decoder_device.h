@@ -210,28 +210,49 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
     for (int c = total + tid; c < prm.ld_out; c += kDecThreads) out[c] = from_f32<T>(0.0f);
 }
 
-// One row's heads, combined, by a block of 256 threads; `active` splits hold keys.
+// One row's heads, combined, by a block of 256 threads; `active` splits hold keys.  sh_w: heads * active floats of LDS.
 template <class T>
-__device__ __forceinline__ void merge_attention_row(const AttentionPartials& p, int64_t row, int active, T* out, int64_t ld_out) {
+__device__ __forceinline__ void merge_attention_row(const AttentionPartials& p, int64_t row, int active, float* sh_w, T* out, int64_t ld_out) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    for (int h = wave; h < p.heads; h += kDecThreads / 64) {
-        const int64_t base = (row * p.heads + h) * p.splits;
-        const float m = lane < active ? p.ml[(base + lane) * 2] : -INFINITY;
-        const float l = lane < active ? p.ml[(base + lane) * 2 + 1] : 0.0f;
-        const float largest = wave_max(m);
-        float w = lane < active ? expf(m - largest) : 0.0f;
-        w = w / wave_sum(w * l);
-        for (int e0 = 0; e0 < p.vdim; e0 += 64) {
-            const int e = e0 + lane;
-            float sum = 0.0f;
-            for (int s = 0; s < active; ++s) {
-                const float ws = __shfl(w, s, 64);
-                if (e < p.vdim) sum = fmaf(ws, p.acc[(base + s) * p.vdim + e], sum);
+    for (int h = wave; h < p.heads; h += kDecThreads / 64) {      // each split's factor: a wave per head, a lane per split
+        const int64_t at = ((row * p.heads + h) * p.splits + min(lane, active - 1)) * 2;
+        const float m_read = p.ml[at], l_read = p.ml[at + 1];
+        const float m = lane < active ? m_read : -INFINITY, l = lane < active ? l_read : 0.0f;
+        const float w = fast_exp2((m - wave_max(m)) * kLog2e);
+        const float total = wave_sum(w * l);
+        if (lane < active) sh_w[h * active + lane] = w / total;
+    }
+    __syncthreads();
+    const int n = p.heads * p.vdim;
+    const float* acc = p.acc + row * p.heads * p.splits * p.vdim;
+    if (p.vdim % 4 == 0) {
+        const int per_head = p.vdim >> 2;
+        for (int i = threadIdx.x; i < n >> 2; i += kDecThreads) {
+            const int h = i / per_head, e = i - h * per_head;
+            const float4* from = reinterpret_cast<const float4*>(acc + static_cast<int64_t>(h) * p.splits * p.vdim) + e;
+            float4 sum = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+            for (int s0 = 0; s0 < active; s0 += 8) {               // (splits past the last: the last one, with factor zero)
+                float4 v[8];
+#pragma unroll
+                for (int s = 0; s < 8; ++s) v[s] = from[min(s0 + s, active - 1) * per_head];
+#pragma unroll
+                for (int s = 0; s < 8; ++s) {
+                    const float w = s0 + s < active ? sh_w[h * active + min(s0 + s, active - 1)] : 0.0f;
+                    sum.x = fmaf(w, v[s].x, sum.x); sum.y = fmaf(w, v[s].y, sum.y);
+                    sum.z = fmaf(w, v[s].z, sum.z); sum.w = fmaf(w, v[s].w, sum.w);
+                }
             }
-            if (e < p.vdim) out[h * p.vdim + e] = from_f32<T>(sum);
+            store4(out, i, sum.x, sum.y, sum.z, sum.w);
+        }
+    } else {
+        for (int i = threadIdx.x; i < n; i += kDecThreads) {
+            const int h = i / p.vdim, e = i - h * p.vdim;
+            float sum = 0.0f;
+            for (int s = 0; s < active; ++s) sum = fmaf(sh_w[h * active + s], acc[(static_cast<int64_t>(h) * p.splits + s) * p.vdim + e], sum);
+            out[i] = from_f32<T>(sum);
         }
     }
-    for (int c = p.heads * p.vdim + threadIdx.x; c < ld_out; c += kDecThreads) out[c] = from_f32<T>(0.0f);
+    for (int c = n + threadIdx.x; c < ld_out; c += kDecThreads) out[c] = from_f32<T>(0.0f);
 }
 
 // Rotary factors of pair i at a position: the angle in double (position * frequency, reduced to one turn), its sine and

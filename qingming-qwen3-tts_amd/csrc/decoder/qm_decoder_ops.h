@@ -12,6 +12,7 @@ namespace qm {
 
 constexpr int kDecMaxWidth = 12288;       // columns of the residual stream (a block's threads hold a row)
 constexpr int kDecMaxSplits = 64;         // key splits of one attention (a wave's lanes combine them)
+constexpr int kDecMaxMerge = 4096;        // heads * key splits of one attention (their factors lie in LDS)
 constexpr int kDecMaxHead = 256;          // channels of a head
 constexpr int kAttentionMatrixRows = 16;  // rows from which bf16 attention goes to the matrix cores
 constexpr int kChunkedRows = 16;          // rows from which a recurrence is computed in chunks (given scratch)

@@ -39,7 +39,7 @@ __global__ __launch_bounds__(kDecThreads) void layer_in_kernel(LayerInParams prm
 }
 
 template <class T>
-__global__ __launch_bounds__(kDecThreads) void layer_out_kernel(LayerOutParams prm) {
+__global__ __launch_bounds__(kDecThreads) void layer_out_kernel(LayerOutParams prm, int most_k) {
     request_arguments(prm);
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     __shared__ float sh_red[4];
@@ -51,7 +51,8 @@ __global__ __launch_bounds__(kDecThreads) void layer_out_kernel(LayerOutParams p
     uint4 piece[kDotAhead][kOutRows];
     dot_request<kOutRows>(d, group.k, piece);
     if (prm.input[g] == 1) {
-        merge_attention_row<T>(prm.part, 0, attention_active_splits(*prm.position_dev, prm.chunk, prm.part.keys_per_split), xs, group.k);
+        merge_attention_row<T>(prm.part, 0, attention_active_splits(*prm.position_dev, prm.chunk, prm.part.keys_per_split),
+                               reinterpret_cast<float*>(xs + most_k), xs, group.k);
     } else if (prm.input[g] == 2) {
         gated_norm_row<T>(prm.gated, 0, sh_red, xs);
     } else {
@@ -162,12 +163,14 @@ int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream) {
 
 template <class T>
 static int32_t layer_out_as(const LayerOutParams& prm, hipStream_t stream) {
-    const size_t lds = static_cast<size_t>(most_k(prm.linears)) * sizeof(T);
+    const size_t merge = prm.part.ml ? static_cast<size_t>(prm.part.heads) * prm.part.splits * sizeof(float) : 0;
+    const int k = most_k(prm.linears);
+    const size_t lds = static_cast<size_t>(k) * sizeof(T) + merge;
     static std::atomic<bool> raised[kMaxDevices];
     const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(layer_out_kernel<T>), kDotLdsMost, raised);
     if (rc != QM_OK) return rc;
     if (lds > static_cast<size_t>(kDotLdsMost)) return QM_ERR_GEOMETRY;
-    hipLaunchKernelGGL(layer_out_kernel<T>, dim3(dot_tiles_of<kOutRows>(prm.linears)), dim3(kDecThreads), lds, stream, prm);
+    hipLaunchKernelGGL(layer_out_kernel<T>, dim3(dot_tiles_of<kOutRows>(prm.linears)), dim3(kDecThreads), lds, stream, prm, k);
     return launch_status();
 }
 
@@ -194,7 +197,7 @@ static int32_t mixer_step_as(const ChunkAttentionParams& a, const DecayAttention
 }
 template <class T, int GQ>
 static int32_t mixer_step_group(const ChunkAttentionParams& a, const DecayAttentionParams& d, hipStream_t stream) {
-    return a.v_stride <= 128 ? mixer_step_as<T, GQ, 1>(a, d, stream) : mixer_step_as<T, GQ, 2>(a, d, stream);
+    return a.v_stride <= 128 && a.k_stride <= 128 ? mixer_step_as<T, GQ, 1>(a, d, stream) : mixer_step_as<T, GQ, 2>(a, d, stream);
 }
 template <class T>
 static int32_t mixer_step(const ChunkAttentionParams& a, const DecayAttentionParams& d, hipStream_t stream) {
