@@ -176,7 +176,7 @@ int32_t qm_decoder_step(qm_decoder* decoder, int32_t sequence, const int32_t* to
 int32_t qm_decoder_generate(qm_decoder* decoder, int32_t sequence, const int32_t* prompt, int32_t count, int32_t maximum,
                             int32_t stop_token, int32_t top_k, float temperature, uint64_t seed, int32_t* tokens_out, int32_t* produced);
 /* Which kernels one-token steps use: 0 (default) fused launches replayed from a graph, 1 fused launches, 2 the operators of
- * the prompt pass; and prompt passes: bit 4 set keeps the recurrences token by token and the attention off the matrix cores. */
+ * the prompt pass.  4 added: prompt passes keep the recurrences token by token and the attention off the matrix cores. */
 int32_t qm_decoder_set_path(qm_decoder* decoder, int32_t path);
 /* Enqueues a step of `count` tokens (count 1: the one-token path) with no read-back, for measurement; then synchronise. */
 int32_t qm_decoder_enqueue(qm_decoder* decoder, int32_t sequence, const int32_t* tokens, int32_t count);
