@@ -20,7 +20,8 @@ extern "C" {
 #endif
 
 /* ---- residual sum and norm --------------------------------------------------------------------------------------- */
-/* x = x_in (or embed[token]) + sum_i scale_i * y_i + step_vec, where a y with a norm weight is first divided by its own
+/* x = x_in (or embed[token], plus with buckets > 0 a row of `bigram`: (token before * mul_prev + token * mul_cur) mod buckets,
+ * or row `buckets` where the token before, tokens[-1] for row 0, is negative) + sum_i scale_i * y_i + step_vec, where a y with a norm weight is first divided by its own
  * root mean square and weighted;  h = x / sqrt(mean(x^2) + eps) * norm_w.  Every row and vector here has ld_h columns (a
  * multiple of 4), zeros behind the first `width`; means are over `width`. */
 typedef struct {
@@ -34,6 +35,7 @@ typedef struct {
     const float* x_in;       /* [rows][ld_h]; NULL: the embedding of tokens[row] */
     const uint16_t* embed;   /* [vocab][ld_h] bf16 */
     const int32_t* tokens;
+    const uint16_t* bigram;  /* [buckets + 1][ld_h] bf16, with buckets > 0 */
     const int32_t* row_map;  /* NULL, or each row's source row in x_in, tokens and the terms */
     const float* step_vec;   /* [ld_h], or NULL */
     const float* norm_w;     /* [ld_h] */
@@ -42,21 +44,22 @@ typedef struct {
     int64_t ld_h;
     int32_t width, vocab, terms;
     float eps;
+    int32_t buckets, mul_prev, mul_cur, reserved;
     qm_residual_term term[3];
 } qm_residual_norm;
 int32_t qm_residual_norm_rows(const qm_residual_norm* op, int32_t rows, int32_t f32, void* hip_stream);
 
 /* ---- gated norm -------------------------------------------------------------------------------------------------- */
-/* `groups` slices of `size` values, each divided by its own root mean square, times weight, times sigmoid(gate). */
+/* `groups` slices of `size` values, each divided by its own root mean square, times weight, times sigmoid(gate) or silu(gate). */
 typedef struct {
     const float* o;          /* [rows][ld_o] */
-    const float* weight;     /* [groups * size] */
+    const float* weight;     /* [groups * size], or NULL: ones */
     const float* gate;       /* [rows][ld_gate] */
     void* out;               /* [rows][ld_out] bf16 or fp32; columns past groups * size become zero */
     int64_t ld_o, ld_gate, ld_out;
     int32_t groups, size;
     float eps;
-    int32_t reserved;
+    int32_t silu;            /* the gate's function: 0 sigmoid, 1 silu */
 } qm_gated_norm;
 int32_t qm_gated_norm_rows(const qm_gated_norm* op, int32_t rows, int32_t f32, void* hip_stream);
 
@@ -105,17 +108,23 @@ typedef struct {
 int32_t qm_chunk_attention_rows(const qm_chunk_attention* op, int32_t f32, void* hip_stream);
 
 /* ---- linear attention with a per-head decay ------------------------------------------------------------------------ */
-/* q, k, v = silu of their projections; S <- decay_h S + k v^T; out = S^T q. */
+/* S <- decay_h S + k v^T; out = S^T q.  q, k, v are silu of their projections; with QM_DECAY_ROTARY v is as projected, channels
+ * i and i + rot_dims / 2 of q and k turn by position * frequency[i], and k is multiplied by k_scale. */
 #define QM_DECAY_CHUNK 64
 #define QM_DECAY_POWERS (QM_DECAY_CHUNK + 1)
+#define QM_DECAY_ROTARY 1
 typedef struct {
-    const float* proj;       /* [rows][ld_proj]: q, k (heads x dim), v (heads x vdim) at their columns */
+    float* proj;             /* [rows][ld_proj]: q, k (heads x dim), v (heads x vdim) at their columns (rotated in place) */
     const float* powers;     /* [heads][QM_DECAY_POWERS]: decay^0, decay^1, ... */
     float* state;            /* [heads][dim][vdim], read and left for the next rows */
     float* out;              /* [rows][heads * vdim] */
     float* scratch;          /* qm_decay_attention_scratch_floats, or NULL: token by token */
+    const double* frequency; /* [rot_dims / 2] */
+    const int32_t* position_dev;    /* as in qm_chunk_attention */
     int64_t ld_proj, scratch_floats;
     int32_t rows, heads, dim, vdim, q_column, k_column, v_column;
+    int32_t options, rot_dims, position;
+    float k_scale;
     int32_t reserved;
 } qm_decay_attention;
 int64_t qm_decay_attention_scratch_floats(int32_t rows, int32_t heads, int32_t dim, int32_t vdim);
@@ -139,6 +148,70 @@ typedef struct {
 } qm_general_delta;
 int64_t qm_general_delta_scratch_floats(int32_t rows, int32_t heads, int32_t dim);
 int32_t qm_general_delta_rows(const qm_general_delta* op, void* hip_stream);
+
+/* ---- softmax attention over latents -------------------------------------------------------------------------------- */
+/* What a latent layer makes of its projections: the query latent and the key/value latent divided by their root mean square
+ * and weighted, the key part with channels 2i and 2i + 1 turned by position * frequency[i], times magnitude. */
+typedef struct {
+    const float* proj;       /* [rows][ld_proj]: query latent at q_column, key/value latent and key part at kv_column */
+    const float* q_norm;     /* [q_rank] */
+    const float* kv_norm;    /* [kv_rank] */
+    const double* frequency; /* [rot_dim / 2] */
+    const int32_t* position_dev;
+    void* q_latent;          /* [rows][ld_q] bf16 or fp32, zeros behind q_rank; NULL: not wanted */
+    void* latent_cache;      /* [positions][ld_latent] bf16 or fp32, zeros behind kv_rank; NULL: another layer's is used */
+    void* key_cache;         /* [positions][key_stride] */
+    int64_t ld_proj, ld_q, ld_latent;
+    int32_t position, rows, q_rank, kv_rank, rot_dim, key_stride, q_column, kv_column;
+    float eps, magnitude;
+} qm_latent_rows;
+int32_t qm_latent_rows_norm(const qm_latent_rows* op, int32_t f32, void* hip_stream);
+
+/* Position i sees every j <= i.  Head h's key is up_k[h] latent beside the key part, its value up_v[h] latent; scores are
+ * (q . k) * scale, the query's part behind `dim` turned like the key part.  Many bf16 rows make keys and values of every
+ * position (given `expanded`); otherwise the query goes through up_k, the softmax weighs latents, the result goes through up_v. */
+typedef struct {
+    const float* q;          /* [rows][ld_query]: heads x (dim + rot_dim), as projected */
+    const double* frequency; /* [rot_dim / 2] */
+    const uint16_t* up_k;    /* [heads * dim][ld_latent] bf16 */
+    const uint16_t* up_v;    /* [heads * vdim][ld_latent] bf16 */
+    const void* latent_cache;
+    const void* key_cache;
+    void* out;               /* [rows][ld_out] bf16 or fp32; columns past heads * vdim become zero */
+    void* q_scratch;         /* [rows][heads][qm_latent_query_stride] bf16 or fp32 */
+    float* ml;               /* [rows][heads][splits][2] */
+    float* acc;              /* [rows][heads][splits][kv_rank] */
+    float* expanded;         /* qm_latent_expanded_bytes(positions = position + rows at least), or NULL */
+    const int32_t* position_dev;
+    int64_t ld_query, ld_latent, ld_out, expanded_bytes;
+    int32_t position, rows, heads, dim, rot_dim, vdim, kv_rank, key_stride, splits;
+    int32_t up_rows;         /* rows of the matrix that begins at up_k and holds up_v up_v_row rows further on (multiple of 128) */
+    int32_t up_v_row;
+    int32_t options;         /* QM_ATTENTION_ROWS: off the matrix cores */
+    float scale, magnitude;
+} qm_latent_attention;
+int32_t qm_latent_query_stride(int32_t kv_rank, int32_t rot_dim);
+int64_t qm_latent_expanded_bytes(int32_t positions, int32_t heads, int32_t dim, int32_t rot_dim, int32_t vdim, int32_t up_rows);
+int32_t qm_latent_attention_rows(const qm_latent_attention* op, int32_t f32, void* hip_stream);
+
+/* ---- mixture of experts ---------------------------------------------------------------------------------------------- */
+/* The `top` experts of a row's highest logits (the lower number among equals), each weighted with sigmoid(logit):
+ * out32[row] = sum of weight * down_e (silu(gate_e x) * (up_e x)).  The experts' matrices lie one behind the other. */
+typedef struct {
+    const void* x;           /* [rows][width_p] bf16 or fp32 */
+    const float* logits;     /* [rows][ld_logits] */
+    const uint16_t* gate;    /* [experts][ff_p][width_p] */
+    const uint16_t* up;      /* [experts][ff_p][width_p] */
+    const uint16_t* down;    /* [experts][width_p][ff_p] */
+    float* out32;            /* [rows][width_p] */
+    void* scratch;           /* qm_expert_scratch_bytes */
+    int64_t ld_logits, scratch_bytes;
+    int32_t rows, experts, top, width_p, ff_p;      /* width_p, ff_p multiples of 128; at most 1024 experts */
+    int32_t options;         /* QM_EXPERTS_ROWS: many rows off the matrix cores */
+} qm_experts;
+#define QM_EXPERTS_ROWS 1
+int64_t qm_expert_scratch_bytes(int32_t rows, int32_t experts, int32_t top, int32_t width_p, int32_t ff_p, int32_t f32);
+int32_t qm_expert_rows(const qm_experts* op, int32_t f32, void* hip_stream);
 
 /* ---- engine ------------------------------------------------------------------------------------------------------------ */
 const char* qm_decoder_last_error(void);

@@ -41,6 +41,7 @@ def build(verbose=True, jobs=4):
 DECODER_SOURCES = ["decoder/qm_decoder_ops.hip", "decoder/qm_decoder_norm.hip", "decoder/qm_decoder_linear.hip",
                    "decoder/qm_decoder_attention.hip", "decoder/qm_decoder_attention_mfma.hip",
                    "decoder/qm_decoder_recurrent.hip", "decoder/qm_decoder_decay_chunks.hip", "decoder/qm_decoder_delta_chunks.hip",
+                   "decoder/qm_decoder_latent.hip", "decoder/qm_decoder_latent_mfma.hip", "decoder/qm_decoder_experts.hip",
                    "decoder/qm_decoder_step.hip"]
 DECODER_SHARED = ["qm_lib.hip", "qm_sampler.hip", "qm_linear_rows_mfma.hip"]
 DECODER_ENGINE_SOURCES = ["engine/qm_safetensors.cpp", "engine/qm_decoder_config.cpp", "engine/qm_decoder.cpp"]

@@ -27,25 +27,25 @@ constexpr int kFlashThreads = 2 * kFlashParts * 64;
 constexpr int kFlashRows = 64;                 // query rows per block
 constexpr int kFlashVStride = kFlashKeys + 4;  // bf16 per value channel in LDS: the 32 rows of a fragment lie in different banks
 
-// C: channels of a head, rounded up to 32, 64, 128 or 256 (the larger of the key and the value size)
-template <int C>
+// CK, CV: channels of a key and of a value, rounded up to multiples of 32
+template <int CK, int CV>
 struct FlashShape {
-    static constexpr int kKStride = C + 8;
+    static constexpr int kKStride = CK + 8;
     static constexpr int kKBytes = kFlashKeys * kKStride * 2;
-    static constexpr int kVBytes = C * kFlashVStride * 2;
+    static constexpr int kVBytes = CV * kFlashVStride * 2;
     // (the other parts' sums arrive two channel tiles at a time)
-    static constexpr int kCombineTiles = C / 32 < 2 ? 1 : 2;
+    static constexpr int kCombineTiles = CV / 32 < 2 ? 1 : 2;
     static constexpr int kCombineBytes = 2 * (kFlashParts - 1) * (kCombineTiles * 16 * 64 + 2 * 32) * 4;
     static constexpr int kLds = kKBytes + kVBytes > kCombineBytes ? kKBytes + kVBytes : kCombineBytes;
 };
 
-template <int C>
+template <int CK, int CV>
 __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(ChunkAttentionParams prm) {
-    using Shape = FlashShape<C>;
+    using Shape = FlashShape<CK, CV>;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     uint16_t* ks = reinterpret_cast<uint16_t*>(smem);                          // [keys][kKStride]
-    uint16_t* vt = reinterpret_cast<uint16_t*>(smem + Shape::kKBytes);         // [C][kFlashVStride]
-    constexpr int kKb = C / 16, kVt = C / 32;
+    uint16_t* vt = reinterpret_cast<uint16_t*>(smem + Shape::kKBytes);         // [CV][kFlashVStride]
+    constexpr int kKb = CK / 16, kVt = CV / 32;
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int pair = wave / kFlashParts, part = wave % kFlashParts, half = lane >> 5;
@@ -83,8 +83,8 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
 
     const uint16_t* k_head = static_cast<const uint16_t*>(prm.k_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.k_stride;
     const uint16_t* v_head = static_cast<const uint16_t*>(prm.v_cache) + static_cast<int64_t>(kv_head) * prm.ring * prm.v_stride;
-    constexpr int kKPieces = kFlashKeys * (C / 8) / kFlashThreads;                // 16-byte pieces of keys per thread
-    constexpr int kVBlocks = (kFlashKeys / 4 * (C / 4) + kFlashThreads - 1) / kFlashThreads;    // blocks of 4 keys x 4 channels per thread
+    constexpr int kKPieces = kFlashKeys * (CK / 8) / kFlashThreads;                // 16-byte pieces of keys per thread
+    constexpr int kVBlocks = (kFlashKeys / 4 * (CV / 4) + kFlashThreads - 1) / kFlashThreads;    // blocks of 4 keys x 4 channels per thread
     dec_u32x4 k_piece[kKPieces];
     dec_u32x2 v_piece[kVBlocks][4];
     // (keys past the last one that the block sees repeat it, channels past the head's repeat others: the first are masked,
@@ -97,12 +97,12 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
         };
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
-            const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            const int at = tid + i * kFlashThreads, key = at / (CK / 8), c = at % (CK / 8) * 8;
             k_piece[i] = *reinterpret_cast<const dec_u32x4*>(k_head + slot_of(key) * prm.k_stride + min(c, prm.k_stride - 8));
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
-            const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
+            const int at = tid + i * kFlashThreads, key = at / (CV / 4) * 4, c = at % (CV / 4) * 4;
 #pragma unroll
             for (int j = 0; j < 4; ++j)
                 v_piece[i][j] = *reinterpret_cast<const dec_u32x2*>(v_head + slot_of(key + j) * prm.v_stride + min(c, prm.v_stride - 4));
@@ -111,13 +111,13 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
     auto deposit = [&]() __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < kKPieces; ++i) {
-            const int at = tid + i * kFlashThreads, key = at / (C / 8), c = at % (C / 8) * 8;
+            const int at = tid + i * kFlashThreads, key = at / (CK / 8), c = at % (CK / 8) * 8;
             *reinterpret_cast<dec_u32x4*>(ks + key * Shape::kKStride + c) = k_piece[i];
         }
 #pragma unroll
         for (int i = 0; i < kVBlocks; ++i) {
-            const int at = tid + i * kFlashThreads, key = at / (C / 4) * 4, c = at % (C / 4) * 4;
-            if (at >= kFlashKeys / 4 * (C / 4)) break;
+            const int at = tid + i * kFlashThreads, key = at / (CV / 4) * 4, c = at % (CV / 4) * 4;
+            if (at >= kFlashKeys / 4 * (CV / 4)) break;
             const dec_u32x2 p0 = v_piece[i][0], p1 = v_piece[i][1], p2 = v_piece[i][2], p3 = v_piece[i][3];
             uint16_t* to = vt + c * kFlashVStride + key;
             auto pair_low = [](uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x05040100U); };
@@ -271,25 +271,27 @@ __global__ __launch_bounds__(kFlashThreads) void chunk_attention_mfma_kernel(Chu
     }
 }
 
-template <int C>
+template <int CK, int CV>
 static int32_t flash_as(const ChunkAttentionParams& prm, hipStream_t stream) {
+    constexpr int kLds = FlashShape<CK, CV>::kLds;
     static std::atomic<bool> raised[kMaxDevices];
-    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(chunk_attention_mfma_kernel<C>), FlashShape<C>::kLds, raised);
+    const int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(chunk_attention_mfma_kernel<CK, CV>), kLds, raised);
     if (rc != QM_OK) return rc;
     const int64_t total = static_cast<int64_t>(prm.rows) * (prm.heads / prm.kv_heads);
     if ((total + kFlashRows - 1) / kFlashRows > 65535) return QM_ERR_GEOMETRY;
-    hipLaunchKernelGGL((chunk_attention_mfma_kernel<C>), dim3(prm.kv_heads, static_cast<unsigned>((total + kFlashRows - 1) / kFlashRows)),
-                       dim3(kFlashThreads), FlashShape<C>::kLds, stream, prm);
+    hipLaunchKernelGGL((chunk_attention_mfma_kernel<CK, CV>), dim3(prm.kv_heads, static_cast<unsigned>((total + kFlashRows - 1) / kFlashRows)),
+                       dim3(kFlashThreads), kLds, stream, prm);
     return launch_status();
 }
 
 int32_t launch_chunk_attention_mfma(const ChunkAttentionParams& prm, hipStream_t stream) {
     if (prm.ld_out % 4 || (reinterpret_cast<uintptr_t>(prm.out) & 7)) return QM_ERR_GEOMETRY;
     const int c = prm.dim > prm.vdim ? prm.dim : prm.vdim;
-    if (c <= 32) return flash_as<32>(prm, stream);
-    if (c <= 64) return flash_as<64>(prm, stream);
-    if (c <= 128) return flash_as<128>(prm, stream);
-    return flash_as<256>(prm, stream);
+    if (c <= 32) return flash_as<32, 32>(prm, stream);
+    if (c <= 64) return flash_as<64, 64>(prm, stream);
+    if (c <= 128) return flash_as<128, 128>(prm, stream);
+    if (prm.dim <= 192 && prm.vdim <= 128) return flash_as<192, 128>(prm, stream);
+    return flash_as<256, 256>(prm, stream);
 }
 
 }  // namespace qm

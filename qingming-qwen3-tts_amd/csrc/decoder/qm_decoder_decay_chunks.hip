@@ -14,12 +14,39 @@ namespace qm {
 constexpr int kDecaySlice = 64;                // value channels staged at once
 constexpr int kDecayVStride = kDecaySlice + 4;
 
-// Rows [t0, t0 + 64) of a head's q, k or v columns into LDS as silu(x) (zeros past the rows or the head), times factor(j):
-// sixteen threads take 64 columns of a row, four each.  `padded`: a multiple of 16.
+// Rotation of every row's q and k in place, k scaled: a block per row, a pair's angle once for all heads.
+__global__ __launch_bounds__(kDecThreads) void decay_rotate_kernel(DecayAttentionParams prm) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int row = static_cast<int>(blockIdx.x), half = prm.rot_dims >> 1;
+    const int position = position_of(prm.position_dev, prm.position) + row;
+    float* sh_cos = lds;
+    float* sh_sin = lds + half;
+    for (int i = threadIdx.x; i < half; i += kDecThreads) rotary(position, prm.frequency[i], sh_cos[i], sh_sin[i]);
+    __syncthreads();
+    float* q = prm.proj + row * prm.ld_proj + prm.q_column;
+    float* k = prm.proj + row * prm.ld_proj + prm.k_column;
+#pragma unroll 2
+    for (int i = threadIdx.x; i < prm.heads * prm.dim; i += kDecThreads) {
+        const int c = i % prm.dim;
+        if (c < half) {
+            const float cosine = sh_cos[c], sine = sh_sin[c];
+            const float qu = q[i], qv = q[i + half], ku = k[i] * prm.k_scale, kv = k[i + half] * prm.k_scale;
+            q[i] = qu * cosine - qv * sine;
+            q[i + half] = qv * cosine + qu * sine;
+            k[i] = ku * cosine - kv * sine;
+            k[i + half] = kv * cosine + ku * sine;
+        } else if (c >= prm.rot_dims) {
+            k[i] *= prm.k_scale;
+        }
+    }
+}
+
+// Rows [t0, t0 + 64) of a head's q, k or v columns into LDS, through silu unless they were rotated (zeros past the rows or
+// the head), times factor(j): sixteen threads take 64 columns of a row, four each.  `padded`: a multiple of 16.
 template <class F>
 __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, float* to, int stride, int t0, int column, int columns, int padded, F factor) {
     const int c4 = (threadIdx.x & 15) * 4, row = threadIdx.x >> 4;
-    const bool vectors = ((column | columns | prm.ld_proj) & 3) == 0;
+    const bool vectors = ((column | columns | prm.ld_proj) & 3) == 0, silu = !(prm.options & QM_DECAY_ROTARY);
     for (int c = c4; c < padded; c += 64) {
         float4 x[4];
 #pragma unroll
@@ -41,7 +68,8 @@ __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, floa
         for (int i = 0; i < 4; ++i) {
             const int j = row + 16 * i;
             const float f = t0 + j < prm.rows ? factor(j) : 0.0f;
-            *reinterpret_cast<float4*>(to + j * stride + c) = make_float4(silu_f32(x[i].x) * f, silu_f32(x[i].y) * f, silu_f32(x[i].z) * f, silu_f32(x[i].w) * f);
+            if (silu) x[i] = make_float4(silu_f32(x[i].x), silu_f32(x[i].y), silu_f32(x[i].z), silu_f32(x[i].w));
+            *reinterpret_cast<float4*>(to + j * stride + c) = make_float4(x[i].x * f, x[i].y * f, x[i].z * f, x[i].w * f);
         }
     }
 }
@@ -186,6 +214,8 @@ int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream)
     if (rc == QM_OK) rc = ensure_dynamic_lds(reinterpret_cast<const void*>(decay_chunk_output_kernel), kDotLdsMost, raised[1]);
     if (rc != QM_OK) return rc;
     if (output_lds > kDotLdsMost || chunks > 65535 || prm.scratch_floats < decay_scratch_floats(prm.rows, prm.heads, prm.dim, prm.vdim)) return QM_ERR_WORKSPACE;
+    if (prm.options & QM_DECAY_ROTARY)
+        hipLaunchKernelGGL(decay_rotate_kernel, dim3(prm.rows), dim3(kDecThreads), sizeof(float) * (prm.rot_dims + 1), stream, prm);
     hipLaunchKernelGGL(decay_chunk_state_kernel, dim3(prm.heads, chunks, slices), dim3(kDecThreads), state_lds, stream, prm);
     const int64_t plane = static_cast<int64_t>(prm.heads) * prm.dim * prm.vdim;
     hipLaunchKernelGGL(decay_chunk_walk_kernel, dim3(static_cast<unsigned>((plane + kDecThreads - 1) / kDecThreads)), dim3(kDecThreads), 0, stream, prm,

@@ -92,8 +92,15 @@ __device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int
         y_row[i] = i < prm.terms ? prm.term[i].y + src * prm.term[i].ld : nullptr;
         normed[i] = i < prm.terms && prm.term[i].norm_w;
     }
-    const uint16_t* embedding = nullptr;
-    if (!prm.x_in) embedding = prm.embed + min(max(prm.tokens[src], 0), prm.vocab - 1) * prm.ld_h;
+    const uint16_t *embedding = nullptr, *bigram = nullptr;
+    if (!prm.x_in) {
+        const int64_t token = min(max(prm.tokens[src], 0), prm.vocab - 1);
+        embedding = prm.embed + token * prm.ld_h;
+        if (prm.buckets > 0) {
+            const int64_t before = prm.tokens[src - 1];
+            bigram = prm.bigram + (before < 0 ? prm.buckets : (before * prm.mul_prev + token * prm.mul_cur) % prm.buckets) * prm.ld_h;
+        }
+    }
     const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f), one = make_float4(1.0f, 1.0f, 1.0f, 1.0f);
     float4 x[NV], y[3][NV];
 #pragma unroll
@@ -101,6 +108,7 @@ __device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int
         const int v = tid + i * kDecThreads;
         const bool in = v < vectors;
         x[i] = embedding ? load4_if(in, embedding, v) : load4_if(in, prm.x_in + src * prm.ld_h, v);
+        if (bigram) x[i] = weighted(x[i], 1.0f, load4_if(in, bigram, v), one);
 #pragma unroll
         for (int t = 0; t < 3; ++t) y[t][i] = y_row[t] ? load4_if(in, y_row[t], v) : zero;
     }
@@ -143,14 +151,19 @@ __device__ __forceinline__ void residual_norm_row(const ResidualParams& prm, int
     }
 }
 
+// The factor that a gate's projection g becomes.
+__device__ __forceinline__ float gate_f32(float g, bool silu) { return silu ? silu_f32(g) : sigmoid_f32(g); }
+
 // One row of the gated norm by a block of 256 threads; sh_red: 4 floats of LDS.
 template <class T>
 __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64_t row, float* sh_red, T* out) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const float* o = prm.o + row * prm.ld_o;
     const float* gate = prm.gate + row * prm.ld_gate;
+    const bool silu = prm.silu != 0;
     const int total = prm.groups * prm.size;
     const float inv_size = 1.0f / static_cast<float>(prm.size);
+    auto weight_at = [&](int at) { return prm.weight ? prm.weight[at] : 1.0f; };
     constexpr int kHeld = 4;                   // float4s a thread holds between its two uses of a value
     if (prm.groups == 1 && total % 4 == 0 && prm.ld_o % 4 == 0 && total <= kHeld * 4 * kDecThreads) {
         const int vectors = total >> 2;
@@ -169,9 +182,9 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
         for (int i = 0; i < kHeld; ++i) {
             const int v = tid + i * kDecThreads;
             if (v >= vectors) continue;
-            const float4 w = load4(prm.weight, v);
-            store4(out, v, held[i].x * inverse * w.x * sigmoid_f32(g[i].x), held[i].y * inverse * w.y * sigmoid_f32(g[i].y),
-                   held[i].z * inverse * w.z * sigmoid_f32(g[i].z), held[i].w * inverse * w.w * sigmoid_f32(g[i].w));
+            const float4 w = prm.weight ? load4(prm.weight, v) : make_float4(1.0f, 1.0f, 1.0f, 1.0f);
+            store4(out, v, held[i].x * inverse * w.x * gate_f32(g[i].x, silu), held[i].y * inverse * w.y * gate_f32(g[i].y, silu),
+                   held[i].z * inverse * w.z * gate_f32(g[i].z, silu), held[i].w * inverse * w.w * gate_f32(g[i].w, silu));
         }
     } else if (prm.groups == 1) {
         float sq[1] = {0.0f};
@@ -179,7 +192,7 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
         block_sums<1>(sq, sh_red);
         const float inverse = 1.0f / sqrtf(sq[0] * inv_size + prm.eps);
         for (int c = tid; c < total; c += kDecThreads)
-            out[c] = from_f32<T>(o[c] * inverse * prm.weight[c] * sigmoid_f32(gate[c]));
+            out[c] = from_f32<T>(o[c] * inverse * weight_at(c) * gate_f32(gate[c], silu));
     } else {
         // a wave per slice, a slice of up to 256 values held by its lanes
         for (int g = wave; g < prm.groups; g += kDecThreads / 64) {
@@ -199,11 +212,11 @@ __device__ __forceinline__ void gated_norm_row(const GatedNormParams& prm, int64
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int c = lane + 64 * i, at = g * prm.size + c;
-                if (c < prm.size) out[at] = from_f32<T>(held[i] * inverse * prm.weight[at] * sigmoid_f32(gates[i]));
+                if (c < prm.size) out[at] = from_f32<T>(held[i] * inverse * weight_at(at) * gate_f32(gates[i], silu));
             }
             for (int c = lane + 256; c < prm.size; c += 64) {
                 const int at = g * prm.size + c;
-                out[at] = from_f32<T>(o[at] * inverse * prm.weight[at] * sigmoid_f32(gate[at]));
+                out[at] = from_f32<T>(o[at] * inverse * weight_at(at) * gate_f32(gate[at], silu));
             }
         }
     }
@@ -262,6 +275,32 @@ __device__ __forceinline__ void rotary(int position, double frequency, float& co
     const double turns = rint(angle * 0.15915494309189535);
     const float reduced = static_cast<float>(fma(-turns, 6.283185307179586, angle));
     sincosf(reduced, &sine, &cosine);
+}
+
+// n values divided by their root mean square and weighted, by a block of 256 threads, zeros behind them up to `padded`;
+// sh_red: 4 floats of LDS.
+template <class T>
+__device__ __forceinline__ void slice_norm_row(const float* x, const float* weight, int n, int64_t padded, float eps, float* sh_red, T* out) {
+    const int tid = threadIdx.x;
+    constexpr int kHeld = 4;
+    float held[kHeld], sq[1] = {0.0f};
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+        const int c = tid + i * kDecThreads;
+        const float value = x[min(c, n - 1)];
+        held[i] = c < n ? value : 0.0f;
+        sq[0] = fmaf(held[i], held[i], sq[0]);
+    }
+    for (int c = tid + kHeld * kDecThreads; c < n; c += kDecThreads) sq[0] = fmaf(x[c], x[c], sq[0]);
+    block_sums<1>(sq, sh_red);
+    const float inverse = 1.0f / sqrtf(sq[0] / static_cast<float>(n) + eps);
+#pragma unroll
+    for (int i = 0; i < kHeld; ++i) {
+        const int c = tid + i * kDecThreads;
+        if (c < n) out[c] = from_f32<T>(held[i] * inverse * weight[c]);
+    }
+    for (int c = tid + kHeld * kDecThreads; c < n; c += kDecThreads) out[c] = from_f32<T>(x[c] * inverse * weight[c]);
+    for (int64_t c = n + tid; c < padded; c += kDecThreads) out[c] = from_f32<T>(0.0f);
 }
 
 }  // namespace qm

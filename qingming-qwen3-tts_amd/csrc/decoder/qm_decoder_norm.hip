@@ -24,6 +24,8 @@ int32_t check_residual(const ResidualParams& prm) {
     if (prm.width <= 0 || prm.ld_h < prm.width || prm.terms < 0 || prm.terms > 3) return QM_ERR_ARGUMENT;
     if (!prm.norm_w || (!prm.x_in && (!prm.embed || !prm.tokens))) return QM_ERR_NULL;
     if (prm.ld_h % 4 || prm.ld_h > kDecMaxWidth) return QM_ERR_GEOMETRY;
+    if (!prm.x_in && prm.buckets > 0 && !prm.bigram) return QM_ERR_NULL;
+    if (prm.buckets < 0 || (prm.buckets > 0 && (prm.mul_prev < 0 || prm.mul_cur < 0))) return QM_ERR_ARGUMENT;
     for (int i = 0; i < prm.terms; ++i) {
         if (!prm.term[i].y) return QM_ERR_NULL;
         if (prm.term[i].ld < prm.ld_h || prm.term[i].ld % 4) return QM_ERR_GEOMETRY;
@@ -53,7 +55,7 @@ int32_t launch_residual_norm(const ResidualParams& prm, int rows, int f32, hipSt
 
 int32_t launch_gated_norm(const GatedNormParams& prm, int rows, int f32, hipStream_t stream) {
     if (rows < 0 || prm.groups <= 0 || prm.size <= 0 || prm.ld_out < static_cast<int64_t>(prm.groups) * prm.size) return QM_ERR_ARGUMENT;
-    if (!prm.o || !prm.weight || !prm.gate || !prm.out) return QM_ERR_NULL;
+    if (!prm.o || !prm.gate || !prm.out) return QM_ERR_NULL;
     if (rows == 0) return QM_OK;
     if (f32) hipLaunchKernelGGL(gated_norm_kernel<float>, dim3(rows), dim3(kDecThreads), 0, stream, prm);
     else hipLaunchKernelGGL(gated_norm_kernel<uint16_t>, dim3(rows), dim3(kDecThreads), 0, stream, prm);

@@ -31,6 +31,13 @@ using DecLinearGroup = qm_decoder_linear;
 using ChunkAttentionParams = qm_chunk_attention;
 using DecayAttentionParams = qm_decay_attention;
 using DeltaParams = qm_general_delta;
+using LatentRowsParams = qm_latent_rows;
+using LatentAttentionParams = qm_latent_attention;
+using ExpertParams = qm_experts;
+constexpr int kLatentKeys = 64;           // keys per pass of the attention over latents; its splits are whole passes
+constexpr int kLatentMaxRank = 1024;      // channels of a latent
+constexpr int kLatentMaxRotary = 256;     // channels of the key part that heads share
+constexpr int kExpertsMost = 1024;
 constexpr int kDecayChunk = QM_DECAY_CHUNK;
 constexpr int kDecayPowers = QM_DECAY_POWERS;
 
@@ -57,15 +64,30 @@ bool delta_chunks_fit(const DeltaParams& prm);
 int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream);
 int32_t launch_delta_chunks(const DeltaParams& prm, hipStream_t stream);
 int32_t launch_general_delta(const DeltaParams& prm, hipStream_t stream);
+int32_t launch_latent_rows(const LatentRowsParams& prm, int f32, hipStream_t stream);
+// keep: what the step's token leaves in the cache, written by the launch that prepares the queries (NULL: it is there).
+int32_t launch_latent_attention(const LatentAttentionParams& prm, const LatentRowsParams* keep, int f32, hipStream_t stream);
+int32_t launch_latent_partials_mfma(const LatentAttentionParams& prm, hipStream_t stream);
+bool latent_partials_fit_mfma(const LatentAttentionParams& prm);
+int latent_q_stride(int kv_rank, int rot_dim);
+int64_t expert_scratch_bytes(int rows, int experts, int top, int width_p, int ff_p, int f32);
+int32_t launch_experts(const ExpertParams& prm, int f32, hipStream_t stream);
 
 // ---- one token: a layer run in three launches -----------------------------------------------------------------------
-// Residual sum and norm by every block for itself, then the linears that read it (row 0 of everything).
+// Residual sum and norm by every block for itself, then the linears that read it (row 0 of everything); the norm's output
+// also goes to residual.h if that is given.
 struct LayerInParams {
     ResidualParams residual;
     DecLinearParams linears;
 };
 // The output linears, each block preparing the input of its own: 0 as it is in memory, 1 the attention's key splits
-// combined, 2 the gated norm.
+// combined, 2 the gated norm, 3 a slice of fp32 values divided by its root mean square and weighted.
+struct SliceNorm {
+    const float* x;
+    const float* weight;
+    int n;
+    float eps;
+};
 struct LayerOutParams {
     DecLinearParams linears;
     int input[kDecGroups];
@@ -73,14 +95,17 @@ struct LayerOutParams {
     AttentionPartials part;
     const int32_t* position_dev;
     GatedNormParams gated;           // (input 2)
+    SliceNorm slice;                 // (input 3)
 };
 int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream);
 // The attention (rotation and cache write included) beside the decayed linear attention, one token each.
 int32_t launch_mixer_step(const ChunkAttentionParams& attention, const DecayAttentionParams& decay, int f32, hipStream_t stream);
 int32_t launch_layer_out(const LayerOutParams& prm, int f32, hipStream_t stream);
-// step = {position, token, emitted}: the token of the highest of `vocab` scores (lowest id among equals) into step[1]
-int32_t launch_argmax(const float* scores, int vocab, int32_t* step, hipStream_t stream);
-// out[step[2]++] = step[1], and the position moves on by `advance`
+// the id of the highest of `vocab` scores (lowest among equals)
+int32_t launch_argmax(const float* scores, int vocab, int32_t* token, hipStream_t stream);
+// step = the words below: the chosen token is put out and becomes the one to feed, the token that was fed the one before it,
+// and the position moves on by `advance`
+enum StepWord { kStepPosition, kStepBefore, kStepToken, kStepEmitted, kStepChosen, kStepWords };
 int32_t launch_emit(int32_t* step, int32_t* out, int advance, hipStream_t stream);
 
 }  // namespace qm

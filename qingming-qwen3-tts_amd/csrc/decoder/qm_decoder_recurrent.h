@@ -40,6 +40,29 @@ __device__ __forceinline__ float quarter_sum(float v) {
 
 __host__ __device__ inline int decay_lds_floats(int rd) { return kRecTokens * 2 * rec_stride(rd); }
 
+// Channel c of a head's q and k as they enter the recurrence: silu of the projections, or rotated (channels i and
+// i + rot_dims / 2 together) and k scaled.
+__device__ __forceinline__ void decay_channel(const DecayAttentionParams& prm, const float* q_head, const float* k_head, int c, int position, float& q,
+                                              float& k) {
+    q = q_head[c];
+    k = k_head[c];
+    if (!(prm.options & QM_DECAY_ROTARY)) {
+        q = silu_f32(q);
+        k = silu_f32(k);
+        return;
+    }
+    if (c < prm.rot_dims) {
+        const int half = prm.rot_dims >> 1, pair = c < half ? c : c - half, other = c < half ? c + half : pair;
+        float cosine, sine;
+        rotary(position, prm.frequency[pair], cosine, sine);
+        if (c < half) sine = -sine;
+        q = q * cosine + q_head[other] * sine;
+        k = k * cosine + k_head[other] * sine;
+    }
+    k *= prm.k_scale;
+}
+__device__ __forceinline__ float decay_value(const DecayAttentionParams& prm, float v) { return prm.options & QM_DECAY_ROTARY ? v : silu_f32(v); }
+
 // Linear attention with decay: head `head`, state columns [64 slice, 64 slice + 64).
 template <int RD>
 __device__ __forceinline__ void decay_attention_block(const DecayAttentionParams& prm, int head, int slice, float* lds) {
@@ -48,6 +71,7 @@ __device__ __forceinline__ void decay_attention_block(const DecayAttentionParams
     constexpr int kStride = 4 * (RD + 4);
     float* state = prm.state + static_cast<int64_t>(head) * prm.dim * prm.vdim;
     const float decay = prm.powers[head * kDecayPowers + 1];
+    const int position = position_of(prm.position_dev, prm.position);
     float s[RD];
     load_state<RD>(s, state, prm.dim, prm.vdim, sub, column);
     for (int t0 = 0; t0 < prm.rows; t0 += kRecTokens) {
@@ -55,15 +79,17 @@ __device__ __forceinline__ void decay_attention_block(const DecayAttentionParams
         __syncthreads();
         for (int i = tid; i < tokens * 4 * RD; i += kDecThreads) {
             const int t = i / (4 * RD), c = i % (4 * RD);
-            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim + c;
+            const float* p = prm.proj + (t0 + t) * prm.ld_proj + head * prm.dim;
             float* to = lds + t * 2 * kStride + rec_at<RD>(c);
-            to[0] = c < prm.dim ? silu_f32(p[prm.q_column]) : 0.0f;
-            to[kStride] = c < prm.dim ? silu_f32(p[prm.k_column]) : 0.0f;
+            float q = 0.0f, k = 0.0f;
+            if (c < prm.dim) decay_channel(prm, p + prm.q_column, p + prm.k_column, c, position + t0 + t, q, k);
+            to[0] = q;
+            to[kStride] = k;
         }
         float v[kRecTokens];
 #pragma unroll
         for (int t = 0; t < kRecTokens; ++t)
-            v[t] = t < tokens && column < prm.vdim ? silu_f32(prm.proj[(t0 + t) * prm.ld_proj + prm.v_column + head * prm.vdim + column]) : 0.0f;
+            v[t] = t < tokens && column < prm.vdim ? decay_value(prm, prm.proj[(t0 + t) * prm.ld_proj + prm.v_column + head * prm.vdim + column]) : 0.0f;
         __syncthreads();
 #pragma unroll
         for (int t = 0; t < kRecTokens; ++t) {

@@ -35,6 +35,11 @@ int32_t check_decay_attention(const DecayAttentionParams& prm) {
     if (!prm.proj || !prm.powers || !prm.state || !prm.out) return QM_ERR_NULL;
     if (prm.rows < 0) return QM_ERR_ARGUMENT;
     if (prm.heads <= 0 || prm.heads > 65535 || prm.dim <= 0 || prm.vdim <= 0 || prm.dim > kDecMaxHead || prm.vdim > kDecMaxHead) return QM_ERR_GEOMETRY;
+    if (prm.options & QM_DECAY_ROTARY) {
+        if (prm.rot_dims < 0 || prm.rot_dims > prm.dim || prm.rot_dims % 2) return QM_ERR_GEOMETRY;
+        if (prm.rot_dims > 0 && !prm.frequency) return QM_ERR_NULL;
+        if (prm.position < 0) return QM_ERR_ARGUMENT;
+    }
     return QM_OK;
 }
 

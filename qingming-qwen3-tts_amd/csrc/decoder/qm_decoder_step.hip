@@ -28,6 +28,10 @@ __global__ __launch_bounds__(kDecThreads) void layer_in_kernel(LayerInParams prm
     dot_request<kInRows>(d, prm.linears.group[g].k, piece);
     residual_norm_row<T, NV>(prm.residual, 0, sh_red, hs, blockIdx.x == 0);
     __syncthreads();
+    if (prm.residual.h && blockIdx.x == 0) {
+        T* out = static_cast<T*>(prm.residual.h);
+        for (int c = threadIdx.x; c < prm.residual.ld_h; c += kDecThreads) out[c] = hs[c];
+    }
     for (int next = static_cast<int>(blockIdx.x) + static_cast<int>(gridDim.x);; next += static_cast<int>(gridDim.x)) {
         dot_finish<T, 1, kInRows>(prm.linears.group[g], d, piece, hs, 0, 1);
         if (next >= tiles) break;
@@ -55,6 +59,8 @@ __global__ __launch_bounds__(kDecThreads) void layer_out_kernel(LayerOutParams p
                                reinterpret_cast<float*>(xs + most_k), xs, group.k);
     } else if (prm.input[g] == 2) {
         gated_norm_row<T>(prm.gated, 0, sh_red, xs);
+    } else if (prm.input[g] == 3) {
+        slice_norm_row<T>(prm.slice.x, prm.slice.weight, prm.slice.n, group.k, prm.slice.eps, sh_red, xs);
     } else {
         constexpr int kVec = 16 / sizeof(T);
         const T* x = static_cast<const T*>(group.x);
@@ -85,7 +91,7 @@ __global__ __launch_bounds__(kDecThreads) void mixer_step_kernel(ChunkAttentionP
 }
 
 constexpr int kArgmaxThreads = 1024;
-__global__ __launch_bounds__(kArgmaxThreads) void argmax_kernel(const float* scores, int vocab, int32_t* step) {
+__global__ __launch_bounds__(kArgmaxThreads) void argmax_kernel(const float* scores, int vocab, int32_t* token) {
     __shared__ float sh_best[kArgmaxThreads / 64];
     __shared__ int sh_id[kArgmaxThreads / 64];
     float best = -INFINITY;
@@ -116,14 +122,15 @@ __global__ __launch_bounds__(kArgmaxThreads) void argmax_kernel(const float* sco
     __syncthreads();
     if (threadIdx.x == 0) {
         for (int w = 1; w < kArgmaxThreads / 64; ++w) take(sh_best[w], sh_id[w]);
-        step[1] = id < vocab ? id : 0;
+        *token = id < vocab ? id : 0;
     }
 }
 
 __global__ void emit_kernel(int32_t* step, int32_t* out, int advance) {
-    out[step[2]] = step[1];
-    ++step[2];
-    step[0] += advance;
+    out[step[kStepEmitted]++] = step[kStepChosen];
+    step[kStepBefore] = step[kStepToken];
+    step[kStepToken] = step[kStepChosen];
+    step[kStepPosition] += advance;
 }
 
 static int most_k(const DecLinearParams& prm) {
@@ -182,6 +189,7 @@ int32_t launch_layer_out(const LayerOutParams& prm, int f32, hipStream_t stream)
         if (d.n <= 0 || d.n % 128 || d.k % 128) return QM_ERR_GEOMETRY;
         if (prm.input[g] == 1 && d.k < prm.part.heads * prm.part.vdim) return QM_ERR_GEOMETRY;
         if (prm.input[g] == 2 && (d.k < prm.gated.groups * prm.gated.size || prm.gated.ld_out != d.k)) return QM_ERR_GEOMETRY;
+        if (prm.input[g] == 3 && (!prm.slice.x || !prm.slice.weight || prm.slice.n <= 0 || prm.slice.n > d.k)) return QM_ERR_GEOMETRY;
     }
     return f32 ? layer_out_as<float>(prm, stream) : layer_out_as<uint16_t>(prm, stream);
 }
@@ -213,10 +221,10 @@ int32_t launch_mixer_step(const ChunkAttentionParams& attention, const DecayAtte
     return f32 ? mixer_step<float>(attention, decay, stream) : mixer_step<uint16_t>(attention, decay, stream);
 }
 
-int32_t launch_argmax(const float* scores, int vocab, int32_t* step, hipStream_t stream) {
-    if (!scores || !step) return QM_ERR_NULL;
+int32_t launch_argmax(const float* scores, int vocab, int32_t* token, hipStream_t stream) {
+    if (!scores || !token) return QM_ERR_NULL;
     if (vocab <= 0) return QM_ERR_ARGUMENT;
-    hipLaunchKernelGGL(argmax_kernel, dim3(1), dim3(kArgmaxThreads), 0, stream, scores, vocab, step);
+    hipLaunchKernelGGL(argmax_kernel, dim3(1), dim3(kArgmaxThreads), 0, stream, scores, vocab, token);
     return launch_status();
 }
 

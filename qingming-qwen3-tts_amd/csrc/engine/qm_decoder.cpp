@@ -8,10 +8,12 @@
 // A pass of many rows, per layer run:
 //   qm_residual_norm_rows   the last layer's sublayers onto the stream, the vector of a loop's pass, norm1
 //   linears                 every projection of the mixer as one matrix (fp32 out), gate/up with SwiGLU
-//   mixer                   rotation + cache write + attention and decayed linear attention, or the delta rule; gated norm
+//   mixer                   rotation + cache write + attention and decayed linear attention, or the delta rule, or retention,
+//                           or attention over latents; gated norm
 //   linears                 the output projections and the feed-forward's down projection in one launch
-// One token: three fused launches per layer run (qm_decoder_step_ops.h), replayed from a graph that reads token and
-// position from device memory.
+// Where a layer's feed-forward has norms of its own it follows in the same way: residual + norm, gate/up, down, or the experts.
+// One token: the same in few fused launches per layer run, replayed from a graph that reads tokens and position from device
+// memory.
 #include "../../../include/qm_decoder.h"
 
 #include <hip/hip_runtime.h>
@@ -38,7 +40,7 @@ namespace {
 
 constexpr float kUnitEps = 1.0e-6f;       // inside the root of the delta rule's unit key
 constexpr int kLogitRows = 256;           // rows of the head at once
-constexpr int kStepWords = 4;             // device words of a one-token step: position, token, tokens emitted
+using qm::kStepWords;                      // device words of a one-token step
 
 int padded(int n, int to) { return (n + to - 1) / to * to; }
 
@@ -69,10 +71,15 @@ struct DecoderLayer {
     Section r, kk, vv, a, g, z;                     // delta rule's
     DeviceBuffer out_left, out_right, mix_norm, powers, frequency, w2, w0, a_bias;
     int rank = 0;
+    DeviceBuffer norm2, after_mixer, after_ff;      // a sandwich layer's other norms
+    Section q_latent, kv_latent, up_v;              // latent attention's: in `in`, and the values in `up_latent` (keys at 0)
+    Matrix q_up, up_latent, router;
+    DeviceBuffer q_norm, kv_norm;
+    double magnitude = 1.0;
 };
 
 struct RunState {                                   // byte offsets inside a sequence's memory
-    size_t k = 0, v = 0, decay = 0, delta = 0;
+    size_t k = 0, v = 0, decay = 0, delta = 0, latent = 0, key = 0;
 };
 
 }  // namespace
@@ -85,16 +92,17 @@ struct qm_decoder {
     std::vector<qm_engine::RunState> states;
     std::vector<qm_engine::DeviceBuffer> memory;    // one per sequence
     std::vector<int> length;                        // tokens of each live sequence, -1: free
+    std::vector<int32_t> before;                    // its last token, -1: none
     size_t sequence_bytes = 0;
     qm_engine::DeviceBuffer final_norm, loop_step;
-    qm_engine::Matrix embed, head;
+    qm_engine::Matrix embed, bigram, head;
     int capacity = 0, max_rows = 0, f32 = 0, path = 0;
     bool warm = false;
     int width_p = 0, vocab_p = 0;
     hipStream_t stream = nullptr;
     bool own_stream = false;
     qm_engine::DeviceBuffer x[2], h, proj, mlp, attended, gated, y[3], q_rot, raw, ml, acc, scratch, tokens, wanted, head_h, logits, tap, tap_h,
-        step_words;
+        step_words, q_latent, queries, q_scratch, expanded, expert_logits, expert_scratch;
     std::vector<hipGraphExec_t> graphs;             // one-token step of each sequence
 
     ~qm_decoder() {
@@ -136,6 +144,14 @@ public:
         std::vector<float> host(rows * columns, 0.0f);
         for (size_t r = 0; r < rows; ++r)
             for (size_t c = 0; c < from; ++c) host[r * columns + c] = element(t, r * from + c);
+        return upload(host.data(), host.size() * sizeof(float));
+    }
+    // a norm's weight, stored less one or as it is, times `scale`
+    DeviceBuffer norm(const std::string& name, int width, bool around_zero, double scale = 1.0) const {
+        const TensorView& t = get(name, {width});
+        std::vector<float> host(static_cast<size_t>(padded(width, 128)), 0.0f);
+        for (int c = 0; c < width; ++c)
+            host[static_cast<size_t>(c)] = static_cast<float>(((around_zero ? 1.0 : 0.0) + element(t, static_cast<size_t>(c))) * scale);
         return upload(host.data(), host.size() * sizeof(float));
     }
     DeviceBuffer transposed_floats(const std::string& name, int64_t rows, int64_t columns) const {
@@ -182,16 +198,51 @@ public:
         return m;
     }
     Matrix matrix(const std::string& name, int n, int k) const { return stacked({{name, n, nullptr}}, k); }
+    // `count` matrices of one shape one behind the other, each padded for itself (n: rows of one)
+    template <class Name>
+    Matrix each(int count, Name name, int n, int k) const {
+        Matrix m;
+        m.n = padded(n, 128);
+        m.k = padded(k, 128);
+        m.data = DeviceBuffer(static_cast<size_t>(count) * m.n * m.k * 2);
+        std::vector<uint16_t> host(static_cast<size_t>(m.n) * m.k, 0);
+        for (int i = 0; i < count; ++i) {
+            const TensorView& t = get(name(i), {n, k});
+            for (int r = 0; r < n; ++r)
+                std::memcpy(host.data() + static_cast<size_t>(r) * m.k, t.data + static_cast<size_t>(r) * k * 2, static_cast<size_t>(k) * 2);
+            hip_check(hipMemcpy(m.data.u16() + static_cast<size_t>(i) * m.n * m.k, host.data(), host.size() * 2, hipMemcpyHostToDevice), "weight upload");
+        }
+        return m;
+    }
 
 private:
     ModelDirectory files_;
 };
 
-DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, int index, int width) {
+DeviceBuffer upload_doubles(std::vector<double> values) {
+    if (values.empty()) values.push_back(0.0);
+    return Loader::upload(values.data(), values.size() * sizeof(double));
+}
+DeviceBuffer decay_powers(const std::vector<double>& decays) {
+    std::vector<float> powers;
+    for (double decay : decays)
+        for (int i = 0; i < QM_DECAY_POWERS; ++i) powers.push_back(static_cast<float>(i == 0 ? 1.0 : std::pow(decay, i)));
+    return Loader::upload(powers.data(), powers.size() * sizeof(float));
+}
+
+DecoderLayer load_layer(const Loader& from, const DecoderConfig& model, int index) {
     DecoderLayer w;
-    w.config = config;
+    const DecoderLayerConfig& config = w.config = model.layers[static_cast<size_t>(index)];
+    const int width = model.width;
     const std::string base = "l" + std::to_string(index) + ".", mix = base + "mix.";
-    w.norm1 = from.padded_floats(base + "norm1", {width}, padded(width, 128));
+    w.norm1 = from.norm(base + "norm1", width, model.norms_around_zero);
+    if (config.form == LayerForm::Sandwich) {
+        w.after_mixer = from.norm(base + "norm1b", width, model.norms_around_zero);
+        if (config.ff) {
+            w.norm2 = from.norm(base + "norm2", width, model.norms_around_zero);
+            w.after_ff = from.norm(base + "norm2b", width, model.norms_around_zero);
+        }
+    }
     if (config.mixer == MixerKind::AttentionBesideDecay) {
         const ChunkAttentionConfig& a = config.attention;
         const DecayAttentionConfig& d = config.decay;
@@ -204,13 +255,28 @@ DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, in
         w.mix_norm = from.floats(mix + "right.norm", {d.heads * d.vdim});
         w.out_left = from.padded_floats(mix + "left.out", {width}, padded(width, 128));
         w.out_right = from.padded_floats(mix + "right.out", {width}, padded(width, 128));
-        std::vector<double> frequency(static_cast<size_t>(std::max(1, a.rot_dims / 2)), 0.0);
-        for (int i = 0; i < a.rot_dims / 2; ++i) frequency[static_cast<size_t>(i)] = std::pow(a.rot_base, -2.0 * i / a.rot_dims);
-        w.frequency = Loader::upload(frequency.data(), frequency.size() * sizeof(double));
-        std::vector<float> powers;
-        for (double decay : d.decay)
-            for (int i = 0; i < QM_DECAY_POWERS; ++i) powers.push_back(static_cast<float>(i == 0 ? 1.0 : std::pow(decay, i)));
-        w.powers = Loader::upload(powers.data(), powers.size() * sizeof(float));
+        w.frequency = upload_doubles(rotary_frequencies(a.rot_dims, a.rot_base, {}, nullptr));
+        w.powers = decay_powers(d.decay);
+    } else if (config.mixer == MixerKind::Retention) {
+        const RetentionConfig& c = config.retention;
+        w.in = from.stacked({{mix + "q", c.heads * c.dim, &w.dq}, {mix + "k", c.heads * c.dim, &w.dk}, {mix + "v", c.heads * c.vdim, &w.dv},
+                             {mix + "g", c.heads * c.vdim, &w.dg}}, width);
+        w.o_right = from.matrix(mix + "o", width, c.heads * c.vdim);
+        w.frequency = upload_doubles(rotary_frequencies(c.rot_dims, c.rot_base, {}, nullptr));
+        w.powers = decay_powers(c.decay);
+    } else if (config.mixer == MixerKind::LatentAttention) {
+        const LatentAttentionConfig& c = config.latent;
+        std::vector<Loader::Part> in = {{mix + "dq", c.q_rank, &w.q_latent}};
+        if (c.kv_from < 0) {
+            in.push_back({mix + "dkv", c.kv_rank + c.rot_dim, &w.kv_latent});
+            w.kv_norm = from.floats(mix + "dkv.norm", {c.kv_rank});
+        }
+        w.in = from.stacked(in, width);
+        w.q_norm = from.floats(mix + "dq.norm", {c.q_rank});
+        w.q_up = from.matrix(mix + "uq", c.heads * (c.dim + c.rot_dim), c.q_rank);
+        w.up_latent = from.stacked({{mix + "uk", c.heads * c.dim, nullptr}, {mix + "uv", c.heads * c.vdim, &w.up_v}}, c.kv_rank);
+        w.o_left = from.matrix(mix + "o", width, c.heads * c.vdim);
+        w.frequency = upload_doubles(rotary_frequencies(c.rot_dim, c.rot_base, c.scaling, &w.magnitude));
     } else {
         const int all = config.delta.heads * config.delta.dim;
         w.rank = static_cast<int>(from.extent(mix + "w1", 0));
@@ -222,7 +288,13 @@ DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, in
         w.mix_norm = from.floats(mix + "norm", {all});
         w.o_right = from.matrix(mix + "o", width, all);
     }
-    if (config.ff) {
+    if (config.experts) {
+        auto named = [&](const char* which) { return [&base, which](int e) { return base + "mlp.e" + std::to_string(e) + "." + which; }; };
+        w.gate = from.each(config.experts, named("gate"), config.ff, width);
+        w.up = from.each(config.experts, named("up"), config.ff, width);
+        w.down = from.each(config.experts, named("down"), width, config.ff);
+        w.router = from.matrix(base + "mlp.router", config.experts, width);
+    } else if (config.ff) {
         w.gate = from.matrix(base + "mlp.gate", config.ff, width);
         w.up = from.matrix(base + "mlp.up", config.ff, width);
         w.down = from.matrix(base + "mlp.down", width, config.ff);
@@ -232,6 +304,10 @@ DecoderLayer load_layer(const Loader& from, const DecoderLayerConfig& config, in
 
 int ring_of(const qm_decoder& d, const ChunkAttentionConfig& a) { return std::min<int64_t>(d.capacity, static_cast<int64_t>(a.chunk) + d.max_rows); }
 int chunk_of(const qm_decoder& d, const ChunkAttentionConfig& a) { return std::min(a.chunk, d.capacity); }
+
+// Key splits of one token's attention over latents: passes of 64 keys, at most 32 splits (their sums are combined by every
+// block behind them).
+int latent_splits(int capacity) { return std::clamp((capacity + 63) / 64, 1, 32); }
 
 // A chunk's keys in at most 16 splits of whole passes of 128 keys.
 int keys_per_split(int chunk) { return padded(std::max(128, (chunk + 15) / 16), 128); }
@@ -257,11 +333,12 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
     d->width_p = padded(width, 128);
     d->vocab_p = padded(d->config.vocab, 128);
     d->embed = from.matrix("embed", d->config.vocab, width);
-    d->final_norm = from.padded_floats("final.norm", {width}, d->width_p);
+    if (d->config.bigram_buckets) d->bigram = from.matrix("bigram", d->config.bigram_buckets + 1, width);
+    d->final_norm = from.norm("final.norm", width, d->config.norms_around_zero, d->config.logit_scale);    // (the scores' scale is linear in it)
     d->head = from.matrix("head", d->config.vocab, width);
     if (d->config.loop_times) d->loop_step = from.padded_floats("loop.step", {d->config.loop_times, width}, d->width_p);
     for (size_t i = 0; i < d->config.layers.size(); ++i)
-        d->layers.push_back(load_layer(from, d->config.layers[i], static_cast<int>(i), width));
+        d->layers.push_back(load_layer(from, d->config, static_cast<int>(i)));
 
     // one sequence's memory
     const size_t item = f32 ? 4 : 2;
@@ -279,6 +356,15 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
             s.k = take(ring * padded(c.attention.dim, 8));
             s.v = take(ring * padded(c.attention.vdim, 8));
             s.decay = take(static_cast<size_t>(c.decay.heads) * c.decay.dim * c.decay.vdim * 4);
+        } else if (c.mixer == MixerKind::Retention) {
+            s.decay = take(static_cast<size_t>(c.retention.heads) * c.retention.dim * c.retention.vdim * 4);
+        } else if (c.mixer == MixerKind::LatentAttention) {
+            if (c.latent.kv_from >= 0) {
+                s = d->states[static_cast<size_t>(c.latent.kv_from)];          // (such models have no loop: run i is layer i)
+            } else {
+                s.latent = take(static_cast<size_t>(capacity) * padded(c.latent.kv_rank, 128) * item);
+                s.key = take(static_cast<size_t>(capacity) * padded(c.latent.rot_dim, 8) * item);
+            }
         } else {
             s.delta = take(static_cast<size_t>(c.delta.heads) * c.delta.dim * c.delta.dim * 4);
         }
@@ -288,16 +374,22 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
     for (int i = 0; i < sequences; ++i) {
         d->memory.emplace_back(at);
         d->length.push_back(-1);
+        d->before.push_back(-1);
     }
     d->graphs.assign(static_cast<size_t>(sequences), nullptr);
 
     // activations of a pass
     const size_t rows = static_cast<size_t>(d->max_rows);
     size_t proj = 0, mlp = 0, attended = 0, gated = 0, q_rot = 0, raw = 0, ml = 0, acc = 0, scratch = 0;
+    size_t q_latent = 0, queries = 0, q_scratch = 0, expanded = 0, expert_logits = 0, expert_scratch = 0;
     for (const DecoderLayer& w : d->layers) {
         const DecoderLayerConfig& c = w.config;
         proj = std::max(proj, static_cast<size_t>(w.in.n));
-        mlp = std::max(mlp, static_cast<size_t>(w.down.k));
+        if (!c.experts) mlp = std::max(mlp, static_cast<size_t>(w.down.k));
+        if (c.experts) {
+            expert_logits = std::max(expert_logits, static_cast<size_t>(w.router.n));
+            expert_scratch = std::max(expert_scratch, static_cast<size_t>(qm::expert_scratch_bytes(d->max_rows, c.experts, c.top, d->width_p, w.gate.n, f32)));
+        }
         gated = std::max(gated, static_cast<size_t>(w.o_right.k));
         if (c.mixer == MixerKind::AttentionBesideDecay) {
             const int splits = key_splits(chunk_of(*d, c.attention));
@@ -309,6 +401,21 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
             acc = std::max(acc, records * c.attention.vdim);
             raw = std::max(raw, static_cast<size_t>(c.decay.heads) * c.decay.vdim);
             scratch = std::max(scratch, static_cast<size_t>(qm::decay_scratch_floats(d->max_rows, c.decay.heads, c.decay.dim, c.decay.vdim)));
+        } else if (c.mixer == MixerKind::Retention) {
+            const RetentionConfig& r = c.retention;
+            raw = std::max(raw, static_cast<size_t>(r.heads) * r.vdim);
+            scratch = std::max(scratch, static_cast<size_t>(qm::decay_scratch_floats(d->max_rows, r.heads, r.dim, r.vdim)));
+        } else if (c.mixer == MixerKind::LatentAttention) {
+            const LatentAttentionConfig& l = c.latent;
+            attended = std::max(attended, static_cast<size_t>(w.o_left.k));
+            q_latent = std::max(q_latent, static_cast<size_t>(w.q_up.k));
+            queries = std::max(queries, static_cast<size_t>(w.q_up.n));
+            q_scratch = std::max(q_scratch, rows * l.heads * qm::latent_q_stride(l.kv_rank, l.rot_dim));
+            const size_t records = std::max(rows, static_cast<size_t>(qm::kAttentionMatrixRows) * latent_splits(capacity)) * l.heads;
+            ml = std::max(ml, records * 2);
+            acc = std::max(acc, records * l.kv_rank);
+            if (!f32)
+                expanded = std::max(expanded, static_cast<size_t>(qm_latent_expanded_bytes(capacity, l.heads, l.dim, l.rot_dim, l.vdim, w.up_latent.n)));
         } else {
             raw = std::max(raw, static_cast<size_t>(c.delta.heads) * c.delta.dim);
             scratch = std::max(scratch, static_cast<size_t>(qm::delta_scratch_floats(d->max_rows, c.delta.heads, c.delta.dim)));
@@ -334,7 +441,13 @@ std::unique_ptr<qm_decoder> create_decoder(const std::string& dir, int f32, int 
     d->ml = zeros(ml * 4);
     d->acc = zeros(acc * 4);
     d->scratch = zeros(scratch * 4);
-    d->tokens = zeros(rows * 4);
+    d->tokens = zeros((rows + 1) * 4);                                         // the token before, then the pass's
+    d->q_latent = zeros(rows * q_latent * item);
+    d->queries = zeros(rows * queries * 4);
+    d->q_scratch = zeros(q_scratch * item);
+    d->expanded = zeros(expanded);
+    d->expert_logits = zeros(rows * expert_logits * 4);
+    d->expert_scratch = zeros(expert_scratch);
     d->wanted = zeros(kLogitRows * 4);
     d->head_h = zeros(static_cast<size_t>(kLogitRows) * d->width_p * item);
     d->logits = zeros(static_cast<size_t>(kLogitRows) * d->vocab_p * 4);
@@ -356,7 +469,9 @@ qm_residual_norm residual_of(const qm_decoder& d, const Pending& pending, const 
     qm_residual_norm p = {};
     p.x_in = x_in;
     p.embed = d.embed.u16();
-    p.tokens = static_cast<const int32_t*>(d.tokens.raw());
+    p.tokens = static_cast<const int32_t*>(d.tokens.raw()) + 1;
+    p.bigram = d.bigram.u16();
+    p.buckets = d.config.bigram_buckets; p.mul_prev = d.config.bigram_mul_prev; p.mul_cur = d.config.bigram_mul_cur;
     p.step_vec = step_vec;
     p.norm_w = norm;
     p.x_out = x_out;
@@ -408,8 +523,10 @@ qm_chunk_attention attention_of(const qm_decoder& d, const DecoderLayer& w, cons
     return p;
 }
 
-qm_decay_attention decay_of(const qm_decoder& d, const DecoderLayer& w, const RunState& s, int sequence, int rows) {
+qm_decay_attention decay_of(const qm_decoder& d, const DecoderLayer& w, const RunState& s, int sequence, int rows, int position) {
     const DecayAttentionConfig& c = w.config.decay;
+    const RetentionConfig& retention = w.config.retention;
+    const bool rotary = w.config.mixer == MixerKind::Retention;
     qm_decay_attention p = {};
     p.proj = f32_of(d.proj);
     p.powers = f32_of(w.powers);
@@ -420,8 +537,83 @@ qm_decay_attention decay_of(const qm_decoder& d, const DecoderLayer& w, const Ru
         p.scratch = f32_of(d.scratch);
         p.scratch_floats = static_cast<int64_t>(d.scratch.bytes() / 4);
     }
-    p.rows = rows; p.heads = c.heads; p.dim = c.dim; p.vdim = c.vdim;
+    p.rows = rows;
+    p.heads = rotary ? retention.heads : c.heads;
+    p.dim = rotary ? retention.dim : c.dim;
+    p.vdim = rotary ? retention.vdim : c.vdim;
     p.q_column = w.dq.at; p.k_column = w.dk.at; p.v_column = w.dv.at;
+    if (rotary) {
+        p.options = QM_DECAY_ROTARY;
+        p.frequency = static_cast<const double*>(w.frequency.raw());
+        p.rot_dims = retention.rot_dims;
+        p.position = position;
+        p.k_scale = static_cast<float>(1.0 / std::sqrt(static_cast<double>(retention.dim)));
+    }
+    return p;
+}
+
+qm_latent_rows latent_rows_of(const qm_decoder& d, const DecoderLayer& w, const RunState& s, int sequence, int rows, int position) {
+    const LatentAttentionConfig& c = w.config.latent;
+    const DeviceBuffer& memory = d.memory[static_cast<size_t>(sequence)];
+    qm_latent_rows p = {};
+    p.proj = f32_of(d.proj);
+    p.q_norm = f32_of(w.q_norm); p.kv_norm = f32_of(w.kv_norm);
+    p.frequency = static_cast<const double*>(w.frequency.raw());
+    p.q_latent = d.q_latent.raw();
+    if (c.kv_from < 0) {
+        p.latent_cache = at_of(memory, s.latent);
+        p.key_cache = at_of(memory, s.key);
+    }
+    p.ld_proj = w.in.n; p.ld_q = w.q_up.k; p.ld_latent = w.up_latent.k;
+    p.position = position; p.rows = rows;
+    p.q_rank = c.q_rank; p.kv_rank = c.kv_rank; p.rot_dim = c.rot_dim;
+    p.key_stride = padded(c.rot_dim, 8);
+    p.q_column = w.q_latent.at; p.kv_column = w.kv_latent.at;
+    p.eps = static_cast<float>(d.config.eps);
+    p.magnitude = static_cast<float>(w.magnitude);
+    return p;
+}
+
+qm_latent_attention latent_attention_of(const qm_decoder& d, const DecoderLayer& w, const RunState& s, int sequence, int rows, int position) {
+    const LatentAttentionConfig& c = w.config.latent;
+    const DeviceBuffer& memory = d.memory[static_cast<size_t>(sequence)];
+    qm_latent_attention p = {};
+    p.q = f32_of(d.queries);
+    p.frequency = static_cast<const double*>(w.frequency.raw());
+    p.up_k = w.up_latent.u16();
+    p.up_v = w.up_latent.u16() + static_cast<size_t>(w.up_v.at) * w.up_latent.k;
+    p.latent_cache = at_of(memory, s.latent);
+    p.key_cache = at_of(memory, s.key);
+    p.out = d.attended.raw();
+    p.q_scratch = d.q_scratch.raw();
+    p.ml = f32_of(d.ml); p.acc = f32_of(d.acc);
+    if (!d.f32) {
+        p.expanded = f32_of(d.expanded);
+        p.expanded_bytes = static_cast<int64_t>(d.expanded.bytes());
+    }
+    p.ld_query = w.q_up.n; p.ld_latent = w.up_latent.k; p.ld_out = w.o_left.k;
+    p.position = position; p.rows = rows;
+    p.heads = c.heads; p.dim = c.dim; p.rot_dim = c.rot_dim; p.vdim = c.vdim; p.kv_rank = c.kv_rank;
+    p.key_stride = padded(c.rot_dim, 8);
+    p.splits = rows < qm::kAttentionMatrixRows ? latent_splits(d.capacity) : 1;
+    p.up_rows = w.up_latent.n; p.up_v_row = w.up_v.at;
+    p.options = d.path & 4 ? QM_ATTENTION_ROWS : 0;
+    p.scale = static_cast<float>(c.scale);
+    p.magnitude = static_cast<float>(w.magnitude);
+    return p;
+}
+
+qm_experts experts_of(const qm_decoder& d, const DecoderLayer& w, int rows, float* y) {
+    qm_experts p = {};
+    p.x = d.h.raw();
+    p.logits = f32_of(d.expert_logits);
+    p.gate = w.gate.u16(); p.up = w.up.u16(); p.down = w.down.u16();
+    p.out32 = y;
+    p.scratch = d.expert_scratch.raw();
+    p.ld_logits = w.router.n;
+    p.scratch_bytes = static_cast<int64_t>(d.expert_scratch.bytes());
+    p.rows = rows; p.experts = w.config.experts; p.top = w.config.top; p.width_p = w.gate.k; p.ff_p = w.gate.n;
+    p.options = d.path & 4 ? QM_EXPERTS_ROWS : 0;
     return p;
 }
 
@@ -444,14 +636,27 @@ qm_general_delta delta_of(const qm_decoder& d, const DecoderLayer& w, const RunS
 }
 
 qm_gated_norm gated_of(const qm_decoder& d, const DecoderLayer& w) {
-    const bool delta = w.config.mixer == MixerKind::GeneralDelta;
     qm_gated_norm p = {};
     p.o = f32_of(d.raw);
     p.weight = f32_of(w.mix_norm);
-    p.gate = f32_of(d.proj) + (delta ? w.g.at : w.dg.at);
     p.out = d.gated.raw();
-    p.groups = delta ? w.config.delta.heads : 1;      // a norm per head, or one over all of them
-    p.size = delta ? w.config.delta.dim : w.config.decay.heads * w.config.decay.vdim;
+    int gate = w.dg.at;
+    switch (w.config.mixer) {
+        case MixerKind::GeneralDelta:                 // a norm per head
+            gate = w.g.at;
+            p.groups = w.config.delta.heads;
+            p.size = w.config.delta.dim;
+            break;
+        case MixerKind::Retention:                    // the same, without a weight
+            p.groups = w.config.retention.heads;
+            p.size = w.config.retention.vdim;
+            p.silu = 1;
+            break;
+        default:                                      // one over all heads
+            p.groups = 1;
+            p.size = w.config.decay.heads * w.config.decay.vdim;
+    }
+    p.gate = f32_of(d.proj) + gate;
     p.ld_o = static_cast<int64_t>(p.groups) * p.size;
     p.ld_gate = w.in.n;
     p.ld_out = w.o_right.k;
@@ -472,13 +677,19 @@ qm_decoder_linear gate_up_of(const DecoderLayer& w, const void* x, void* out) {
     return l;
 }
 
+bool sandwich(const DecoderLayer& w) { return w.config.form == LayerForm::Sandwich; }
+
 // The linears that read a layer's norm, and those that leave its sublayers' outputs in y[0 ..]; the terms they become.
 qm::DecLinearParams linears_in(const qm_decoder& d, const DecoderLayer& w, int rows) {
     qm::DecLinearParams p = {};
     p.rows = rows;
     p.group[p.groups++] = linear_of(w.in, d.h.raw(), f32_of(d.proj));
-    if (w.config.ff) p.group[p.groups++] = gate_up_of(w, d.h.raw(), d.mlp.raw());
+    if (w.config.ff && !sandwich(w)) p.group[p.groups++] = gate_up_of(w, d.h.raw(), d.mlp.raw());
     return p;
+}
+void add_term(const qm_decoder& d, Pending& pending, const float* y, const float* norm, float scale) {
+    qm_residual_term& t = pending.term[pending.count++];
+    t.y = y; t.norm_w = norm; t.ld = d.width_p; t.scale = scale;
 }
 qm::DecLinearParams linears_out(const qm_decoder& d, const DecoderLayer& w, int rows, Pending& pending) {
     qm::DecLinearParams p = {};
@@ -487,17 +698,39 @@ qm::DecLinearParams linears_out(const qm_decoder& d, const DecoderLayer& w, int 
     auto add = [&](const Matrix& m, const void* x, const float* norm, float scale) {
         float* y = f32_of(d.y[p.groups]);
         p.group[p.groups++] = linear_of(m, x, y);
-        qm_residual_term& t = pending.term[pending.count++];
-        t.y = y; t.norm_w = norm; t.ld = d.width_p; t.scale = scale;
+        add_term(d, pending, y, norm, scale);
     };
-    if (w.config.mixer == MixerKind::AttentionBesideDecay) {
-        add(w.o_left, d.attended.raw(), f32_of(w.out_left), 0.5f);
-        add(w.o_right, d.gated.raw(), f32_of(w.out_right), 0.5f);
-    } else {
-        add(w.o_right, d.gated.raw(), nullptr, 1.0f);
+    const float mult = static_cast<float>(d.config.residual_mult);
+    switch (w.config.mixer) {
+        case MixerKind::AttentionBesideDecay:
+            add(w.o_left, d.attended.raw(), f32_of(w.out_left), 0.5f);
+            add(w.o_right, d.gated.raw(), f32_of(w.out_right), 0.5f);
+            break;
+        case MixerKind::GeneralDelta: add(w.o_right, d.gated.raw(), nullptr, 1.0f); break;
+        case MixerKind::Retention: add(w.o_right, d.gated.raw(), f32_of(w.after_mixer), mult); break;
+        case MixerKind::LatentAttention: add(w.o_left, d.attended.raw(), f32_of(w.after_mixer), mult); break;
     }
-    if (w.config.ff) add(w.down, d.mlp.raw(), nullptr, 1.0f);
+    if (w.config.ff && !sandwich(w)) add(w.down, d.mlp.raw(), nullptr, 1.0f);
     return p;
+}
+
+// A sandwich layer's feed-forward: what reads norm2, and (dense) the linear behind it.
+qm::DecLinearParams feed_in(const qm_decoder& d, const DecoderLayer& w, int rows) {
+    qm::DecLinearParams p = {};
+    p.rows = rows;
+    p.group[p.groups++] = w.config.experts ? linear_of(w.router, d.h.raw(), f32_of(d.expert_logits)) : gate_up_of(w, d.h.raw(), d.mlp.raw());
+    return p;
+}
+qm::DecLinearParams feed_out(const qm_decoder& d, const DecoderLayer& w, int rows) {
+    qm::DecLinearParams p = {};
+    p.rows = rows;
+    p.group[p.groups++] = linear_of(w.down, d.mlp.raw(), f32_of(d.y[0]));
+    return p;
+}
+Pending feed_term(const qm_decoder& d, const DecoderLayer& w) {
+    Pending pending;
+    add_term(d, pending, f32_of(d.y[0]), f32_of(w.after_ff), static_cast<float>(d.config.residual_mult));
+    return pending;
 }
 
 // Every layer run over `rows` tokens of d.tokens at `position`; leaves the stream and what is pending for the head.
@@ -517,12 +750,32 @@ void run_layers(qm_decoder& d, int sequence, int rows, int position, const float
         op_check(qm::launch_decoder_linears(linears_in(d, w, rows), d.f32, s), "input projections");
         if (w.config.mixer == MixerKind::AttentionBesideDecay) {
             op_check(qm::launch_chunk_attention(attention_of(d, w, d.states[i], sequence, rows, position), d.f32, s), "chunked attention");
-            op_check(qm::launch_decay_attention(decay_of(d, w, d.states[i], sequence, rows), s), "decayed linear attention");
+            op_check(qm::launch_decay_attention(decay_of(d, w, d.states[i], sequence, rows, position), s), "decayed linear attention");
+        } else if (w.config.mixer == MixerKind::Retention) {
+            op_check(qm::launch_decay_attention(decay_of(d, w, d.states[i], sequence, rows, position), s), "retention");
+        } else if (w.config.mixer == MixerKind::LatentAttention) {
+            op_check(qm::launch_latent_rows(latent_rows_of(d, w, d.states[i], sequence, rows, position), d.f32, s), "latents");
+            qm::DecLinearParams up = {};
+            up.rows = rows;
+            up.group[up.groups++] = linear_of(w.q_up, d.q_latent.raw(), f32_of(d.queries));
+            op_check(qm::launch_decoder_linears(up, d.f32, s), "queries");
+            op_check(qm::launch_latent_attention(latent_attention_of(d, w, d.states[i], sequence, rows, position), nullptr, d.f32, s),
+                     "attention over latents");
         } else {
             op_check(qm::launch_general_delta(delta_of(d, w, d.states[i], sequence, rows), s), "generalized delta rule");
         }
-        op_check(qm::launch_gated_norm(gated_of(d, w), rows, d.f32, s), "gated norm");
+        if (w.config.mixer != MixerKind::LatentAttention) op_check(qm::launch_gated_norm(gated_of(d, w), rows, d.f32, s), "gated norm");
         op_check(qm::launch_decoder_linears(linears_out(d, w, rows, pending), d.f32, s), "output projections");
+        if (sandwich(w) && w.config.ff) {
+            x_new = f32_of(d.x[next]);
+            op_check(qm::launch_residual_norm(residual_of(d, pending, x, x_new, nullptr, f32_of(w.norm2), d.h.raw()), rows, d.f32, s), "residual + norm");
+            x = x_new;
+            next ^= 1;
+            op_check(qm::launch_decoder_linears(feed_in(d, w, rows), d.f32, s), "feed-forward");
+            if (w.config.experts) op_check(qm::launch_experts(experts_of(d, w, rows, f32_of(d.y[0])), d.f32, s), "experts");
+            else op_check(qm::launch_decoder_linears(feed_out(d, w, rows), d.f32, s), "feed-forward");
+            pending = feed_term(d, w);
+        }
         if (taps) {
             // the stream behind this run, before anything is added ahead of the next one
             op_check(qm::launch_residual_norm(residual_of(d, pending, x, f32_of(d.tap), nullptr, f32_of(d.final_norm), d.tap_h.raw()), rows, d.f32, s),
@@ -570,7 +823,7 @@ void enqueue_one(qm_decoder& d, int sequence) {
     Pending pending;
     auto residual = [&](float* x_new, const float* step_vec, const float* norm) {
         qm_residual_norm p = residual_of(d, pending, x, x_new, step_vec, norm, nullptr);
-        p.tokens = step_words(d) + 1;
+        p.tokens = step_words(d) + qm::kStepToken;
         return p;
     };
     for (size_t i = 0; i < d.runs.size(); ++i) {
@@ -584,22 +837,65 @@ void enqueue_one(qm_decoder& d, int sequence) {
         x = x_new;
         next ^= 1;
         qm::LayerOutParams out = {};
-        out.linears = linears_out(d, w, 1, pending);
-        out.gated = gated_of(d, w);
         out.position_dev = step_words(d);
-        if (w.config.mixer == MixerKind::AttentionBesideDecay) {
-            qm_chunk_attention a = attention_of(d, w, d.states[i], sequence, 1, 0);
-            a.position_dev = step_words(d);
-            op_check(qm::launch_mixer_step(a, decay_of(d, w, d.states[i], sequence, 1), d.f32, s), "attention beside decayed attention");
-            out.part = a.part;
-            out.chunk = a.chunk;
-            out.input[0] = 1;
-            out.input[1] = 2;
-        } else {
-            op_check(qm::launch_general_delta(delta_of(d, w, d.states[i], sequence, 1), s), "generalized delta rule");
-            out.input[0] = 2;
+        switch (w.config.mixer) {
+            case MixerKind::AttentionBesideDecay: {
+                qm_chunk_attention a = attention_of(d, w, d.states[i], sequence, 1, 0);
+                a.position_dev = step_words(d);
+                op_check(qm::launch_mixer_step(a, decay_of(d, w, d.states[i], sequence, 1, 0), d.f32, s), "attention beside decayed attention");
+                out.part = a.part;
+                out.chunk = a.chunk;
+                out.input[0] = 1;
+                out.input[1] = 2;
+                break;
+            }
+            case MixerKind::GeneralDelta:
+                op_check(qm::launch_general_delta(delta_of(d, w, d.states[i], sequence, 1), s), "generalized delta rule");
+                out.input[0] = 2;
+                break;
+            case MixerKind::Retention: {
+                qm_decay_attention r = decay_of(d, w, d.states[i], sequence, 1, 0);
+                r.position_dev = step_words(d);
+                op_check(qm::launch_decay_attention(r, s), "retention");
+                out.input[0] = 2;
+                break;
+            }
+            case MixerKind::LatentAttention: {
+                qm_latent_rows rows = latent_rows_of(d, w, d.states[i], sequence, 1, 0);
+                qm_latent_attention a = latent_attention_of(d, w, d.states[i], sequence, 1, 0);
+                rows.position_dev = a.position_dev = step_words(d);
+                qm::LayerOutParams up = {};
+                up.linears.rows = 1;
+                up.linears.group[up.linears.groups++] = linear_of(w.q_up, nullptr, f32_of(d.queries));
+                up.input[0] = 3;
+                up.slice = {rows.proj + rows.q_column, rows.q_norm, rows.q_rank, rows.eps};
+                op_check(qm::launch_layer_out(up, d.f32, s), "queries");
+                rows.q_latent = nullptr;
+                op_check(qm::launch_latent_attention(a, rows.latent_cache ? &rows : nullptr, d.f32, s), "attention over latents");
+                break;
+            }
         }
+        out.linears = linears_out(d, w, 1, pending);
+        if (w.config.mixer != MixerKind::LatentAttention) out.gated = gated_of(d, w);
         op_check(qm::launch_layer_out(out, d.f32, s), "output projections");
+        if (sandwich(w) && w.config.ff) {
+            x_new = f32_of(d.x[next]);
+            qm::LayerInParams feed = {};
+            feed.residual = residual(x_new, nullptr, f32_of(w.norm2));
+            if (w.config.experts) feed.residual.h = d.h.raw();
+            feed.linears = feed_in(d, w, 1);
+            op_check(qm::launch_layer_in(feed, d.f32, s), "residual + norm + feed-forward");
+            x = x_new;
+            next ^= 1;
+            if (w.config.experts) {
+                op_check(qm::launch_experts(experts_of(d, w, 1, f32_of(d.y[0])), d.f32, s), "experts");
+            } else {
+                qm::LayerOutParams down = {};
+                down.linears = feed_out(d, w, 1);
+                op_check(qm::launch_layer_out(down, d.f32, s), "feed-forward");
+            }
+            pending = feed_term(d, w);
+        }
     }
     qm::LayerInParams head = {};
     head.residual = residual(nullptr, nullptr, f32_of(d.final_norm));
@@ -610,7 +906,7 @@ void enqueue_one(qm_decoder& d, int sequence) {
 
 // The same by the operators of the prompt pass.
 void enqueue_one_by_operators(qm_decoder& d, int sequence, int position) {
-    hip_check(hipMemcpyAsync(d.tokens.raw(), step_words(d) + 1, 4, hipMemcpyDeviceToDevice, d.stream), "token");
+    hip_check(hipMemcpyAsync(d.tokens.raw(), step_words(d) + qm::kStepBefore, 8, hipMemcpyDeviceToDevice, d.stream), "token");
     const float* x = nullptr;
     Pending pending;
     run_layers(d, sequence, 1, position, &x, pending, nullptr);
@@ -652,8 +948,8 @@ void run_one(qm_decoder& d, int sequence) {
     ++length;
 }
 
-void put_step_words(qm_decoder& d, int position, int token) {
-    const int32_t words[3] = {position, token, 0};
+void put_step_words(qm_decoder& d, int position, int before, int token) {
+    const int32_t words[kStepWords] = {position, before, token, 0, 0};
     hip_check(hipMemcpyAsync(d.step_words.raw(), words, sizeof words, hipMemcpyHostToDevice, d.stream), "step words");
 }
 
@@ -672,6 +968,7 @@ int& length_of(qm_decoder& d, int sequence) {
 void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const int32_t* want, int wanted, float* logits, float* streams,
           bool read_back = true) {
     int& length = length_of(d, sequence);
+    int32_t& before = d.before[static_cast<size_t>(sequence)];
     if (count <= 0) throw ApiError(QM_ERR_ARGUMENT, "a step has at least one token");
     check_tokens(d, tokens, count);
     if (count > d.capacity - length) throw ApiError(QM_ERR_SLOT_RANGE, "the sequence exceeds its capacity");
@@ -684,8 +981,9 @@ void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const i
         d.tap_h = DeviceBuffer(static_cast<size_t>(d.max_rows) * d.width_p * 4);
     }
     if (count == 1 && !streams) {
-        put_step_words(d, length, tokens[0]);
+        put_step_words(d, length, before, tokens[0]);
         run_one(d, sequence);
+        before = tokens[0];
         for (int i = 0; i < wanted; ++i)
             hip_check(hipMemcpyAsync(logits + static_cast<size_t>(i) * d.config.vocab, d.logits.raw(), static_cast<size_t>(d.config.vocab) * 4,
                                      hipMemcpyDeviceToHost, d.stream), "logits read");
@@ -701,11 +999,14 @@ void step(qm_decoder& d, int sequence, const int32_t* tokens, int count, const i
                 places.push_back(want[i] - first);
                 order.push_back(i);
             }
-        hip_check(hipMemcpyAsync(d.tokens.raw(), tokens + first, static_cast<size_t>(rows) * 4, hipMemcpyHostToDevice, d.stream), "token upload");
+        std::vector<int32_t> fed(static_cast<size_t>(rows) + 1, before);
+        std::copy(tokens + first, tokens + first + rows, fed.begin() + 1);
+        hip_check(hipMemcpyAsync(d.tokens.raw(), fed.data(), fed.size() * 4, hipMemcpyHostToDevice, d.stream), "token upload");
         const float* x = nullptr;
         Pending pending;
         run_layers(d, sequence, rows, length, &x, pending, streams);
         length += rows;
+        before = tokens[first + rows - 1];
         if (!places.empty()) {
             std::vector<float> some(places.size() * static_cast<size_t>(d.config.vocab));
             run_head(d, x, pending, places.data(), static_cast<int>(places.size()), some.data());
@@ -732,20 +1033,21 @@ int generate(qm_decoder& d, int sequence, const int32_t* prompt, int count, int 
     step(d, sequence, prompt, count, &want, 1, last.data(), nullptr);    // leaves the scores in row 0 of d.logits
     DeviceBuffer emitted(static_cast<size_t>(maximum) * 4), generator(8);
     hip_check(hipMemcpyAsync(generator.raw(), &seed, 8, hipMemcpyHostToDevice, d.stream), "generator state");
-    put_step_words(d, length, 0);
+    int32_t& before = d.before[static_cast<size_t>(sequence)];
+    put_step_words(d, length, 0, before);
     StreamDrain drain(d.stream);          // (the two buffers outlive what reads them, also on an error)
     int produced = 0;
     for (;;) {
         if (top_k > 0)
             op_check(qm_sample_topk(d.logits.raw(), 0, 0, d.config.vocab, top_k, temperature, static_cast<uint64_t*>(generator.raw()),
-                                    step_words(d) + 1, d.stream), "sampler");
+                                    step_words(d) + qm::kStepChosen, d.stream), "sampler");
         else
-            op_check(qm::launch_argmax(f32_of(d.logits), d.config.vocab, step_words(d), d.stream), "arg-max");
+            op_check(qm::launch_argmax(f32_of(d.logits), d.config.vocab, step_words(d) + qm::kStepChosen, d.stream), "arg-max");
         op_check(qm::launch_emit(step_words(d), static_cast<int32_t*>(emitted.raw()), produced > 0, d.stream), "emit");
         ++produced;
         if (stop_token >= 0) {
             int32_t token = 0;
-            hip_check(hipMemcpyAsync(&token, step_words(d) + 1, 4, hipMemcpyDeviceToHost, d.stream), "token read");
+            hip_check(hipMemcpyAsync(&token, step_words(d) + qm::kStepToken, 4, hipMemcpyDeviceToHost, d.stream), "token read");
             hip_check(hipStreamSynchronize(d.stream), "token read");
             if (token == stop_token) break;
         }
@@ -754,6 +1056,7 @@ int generate(qm_decoder& d, int sequence, const int32_t* prompt, int count, int 
     }
     hip_check(hipMemcpyAsync(out, emitted.raw(), static_cast<size_t>(produced) * 4, hipMemcpyDeviceToHost, d.stream), "tokens read");
     hip_check(hipStreamSynchronize(d.stream), "tokens read");
+    if (produced > 1) before = out[produced - 2];             // (the last token emitted was not fed)
     return produced;
 }
 
@@ -802,6 +1105,7 @@ extern "C" int32_t qm_decoder_open(qm_decoder* d, int32_t* sequence) {
         const size_t at = static_cast<size_t>(free - d->length.begin());
         hip_check(hipMemsetAsync(d->memory[at].raw(), 0, d->memory[at].bytes(), d->stream), "sequence reset");
         *free = 0;
+        d->before[at] = -1;
         *sequence = static_cast<int32_t>(at);
     });
 }

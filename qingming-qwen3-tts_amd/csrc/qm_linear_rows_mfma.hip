@@ -193,6 +193,12 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
         }
     }
     const int n0 = tile * BN;
+    int64_t matrix_at = 0;
+    if (prm.tile_matrix) {
+        const int matrix = prm.tile_matrix[blockIdx.y];
+        if (matrix < 0) return;
+        matrix_at = static_cast<int64_t>(matrix) * columns * K;
+    }
 
     // ---- this wave's pieces of a stage: instruction q = wave + 4 i covers LDS bytes [1024 q, 1024 q + 1024) of the
     // stage (x tile, then w, then up); its lane l fills slot l % kSlots of tile row kRowsPerPiece (q within the tile) +
@@ -205,9 +211,9 @@ __global__ __launch_bounds__(kGmThreads) void linear_rows_mfma_kernel(LinearRows
     const __amdgpu_buffer_rsrc_t x_rsrc = __builtin_amdgcn_make_buffer_rsrc(
         const_cast<uint16_t*>(input + static_cast<int64_t>(m0) * K), 0, static_cast<int>(x_rows * row_bytes), 0x00020000);
     const __amdgpu_buffer_rsrc_t w_rsrc = __builtin_amdgcn_make_buffer_rsrc(
-        const_cast<uint16_t*>(weight0 + static_cast<int64_t>(n0) * K), 0, static_cast<int>(BN * row_bytes), 0x00020000);
+        const_cast<uint16_t*>(weight0 + matrix_at + static_cast<int64_t>(n0) * K), 0, static_cast<int>(BN * row_bytes), 0x00020000);
     const __amdgpu_buffer_rsrc_t u_rsrc = __builtin_amdgcn_make_buffer_rsrc(
-        const_cast<uint16_t*>((DUAL ? prm.weight[1] : weight0) + static_cast<int64_t>(n0) * K), 0, static_cast<int>(BN * row_bytes), 0x00020000);
+        const_cast<uint16_t*>((DUAL ? prm.weight[1] : weight0) + matrix_at + static_cast<int64_t>(n0) * K), 0, static_cast<int>(BN * row_bytes), 0x00020000);
     const int lane_row = kRowsPerPiece * wave + lane / kSlots;
     const uint32_t lane_off = static_cast<uint32_t>(lane_row) * row_bytes
                             + 16u * static_cast<uint32_t>((lane % kSlots) ^ slot_key<kRowBytes>(lane_row));
@@ -581,6 +587,11 @@ size_t rows_mfma_workspace_bytes(int rows, int columns, int reduction, bool dual
 
 int32_t launch_rows_mfma(const LinearRowsParams& prm, bool dual, hipStream_t stream) {
     if (prm.rows == 0 || prm.columns == 0) return QM_OK;
+    if (prm.tile_matrix) {
+        if (prm.groups > 1 || prm.reduction_parts != 1 || (prm.tile_rows != 64 && prm.tile_rows != 128) || prm.rows % prm.tile_rows) return QM_ERR_ARGUMENT;
+        if (prm.tile_rows == 64) return dual ? launch_rows_mfma_as<true, 64, 128, 64>(prm, stream) : launch_rows_mfma_as<false, 64, 128, 64>(prm, stream);
+        return dual ? launch_rows_mfma_as<true, 128, 128, 64>(prm, stream) : launch_rows_mfma_as<false, 128, 128, 64>(prm, stream);
+    }
     // blocks of 64 token rows where blocks of 128 would leave CUs without one (one block per CU either way)
     const int64_t row_tiles = (prm.rows + 127) / 128;
     int64_t columns = prm.columns;

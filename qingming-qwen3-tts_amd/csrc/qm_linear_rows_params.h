@@ -38,6 +38,10 @@ struct LinearRowsParams {
     // blocks in the order linear by linear (all row tiles of the first, then of the next) instead of row tile by row
     // tile: the linears with the long reductions first, so that none of them starts late
     int linear_by_linear;
+    // (matrix cores, reduction uncut, one linear or pair) several matrices of one shape, one behind the other: row tile t of
+    // tile_rows rows (64 or 128) takes matrix tile_matrix[t], or is left out where that is negative
+    const int32_t* tile_matrix;
+    int tile_rows;
 };
 
 // The row linears on the matrix cores (qm_linear_rows_mfma.hip).  `dual`: weight[0] / weight[1] are the gate and up

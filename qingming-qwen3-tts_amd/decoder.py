@@ -21,20 +21,32 @@ def _same(kind, names):
 
 
 ResidualTerm = _structure("ResidualTerm", *_same(_P, "y norm_w"), ("ld", _I64), ("scale", _F), ("reserved", _I32))
-ResidualNorm = _structure("ResidualNorm", *_same(_P, "x_in embed tokens row_map step_vec norm_w x_out h"), ("ld_h", _I64),
-                          *_same(_I32, "width vocab terms"), ("eps", _F), ("term", ResidualTerm * 3))
+ResidualNorm = _structure("ResidualNorm", *_same(_P, "x_in embed tokens bigram row_map step_vec norm_w x_out h"), ("ld_h", _I64),
+                          *_same(_I32, "width vocab terms"), ("eps", _F), *_same(_I32, "buckets mul_prev mul_cur reserved"),
+                          ("term", ResidualTerm * 3))
 GatedNorm = _structure("GatedNorm", *_same(_P, "o weight gate out"), *_same(_I64, "ld_o ld_gate ld_out"), *_same(_I32, "groups size"),
-                       ("eps", _F), ("reserved", _I32))
+                       ("eps", _F), ("silu", _I32))
 DecoderLinear = _structure("DecoderLinear", *_same(_P, "x w w_up out32 out"), *_same(_I64, "ldx ldo"), *_same(_I32, "n k"))
 AttentionPartials = _structure("AttentionPartials", *_same(_P, "ml acc"), *_same(_I32, "heads vdim splits keys_per_split"))
 ChunkAttention = _structure("ChunkAttention", *_same(_P, "proj frequency q_rot k_cache v_cache out"), ("part", AttentionPartials),
                             ("position_dev", _P), *_same(_I64, "ld_proj ld_out"), *_same(_I32, "position rows"),
                             *_same(_I32, "heads kv_heads dim vdim k_stride v_stride ring chunk rot_dims k_column v_column"), ("scale", _F), ("options", _I32), ("reserved", _I32))
-DecayAttention = _structure("DecayAttention", *_same(_P, "proj powers state out scratch"), *_same(_I64, "ld_proj scratch_floats"),
-                            *_same(_I32, "rows heads dim vdim q_column k_column v_column reserved"))
+DecayAttention = _structure("DecayAttention", *_same(_P, "proj powers state out scratch frequency position_dev"),
+                            *_same(_I64, "ld_proj scratch_floats"), *_same(_I32, "rows heads dim vdim q_column k_column v_column options rot_dims position"),
+                            ("k_scale", _F), ("reserved", _I32))
 GeneralDelta = _structure("GeneralDelta", *_same(_P, "proj w2 w0 a_bias state out scratch"), *_same(_I64, "ld_proj scratch_floats"),
                           *_same(_I32, "rows heads dim rank r_column k_column v_column a_column z_column"), ("unit_eps", _F))
+LatentRows = _structure("LatentRows", *_same(_P, "proj q_norm kv_norm frequency position_dev q_latent latent_cache key_cache"),
+                        *_same(_I64, "ld_proj ld_q ld_latent"), *_same(_I32, "position rows q_rank kv_rank rot_dim key_stride q_column kv_column"),
+                        *_same(_F, "eps magnitude"))
+LatentAttention = _structure("LatentAttention", *_same(_P, "q frequency up_k up_v latent_cache key_cache out q_scratch ml acc expanded position_dev"),
+                             *_same(_I64, "ld_query ld_latent ld_out expanded_bytes"),
+                             *_same(_I32, "position rows heads dim rot_dim vdim kv_rank key_stride splits up_rows up_v_row options"),
+                             *_same(_F, "scale magnitude"))
+Experts = _structure("Experts", *_same(_P, "x logits gate up down out32 scratch"), *_same(_I64, "ld_logits scratch_bytes"),
+                     *_same(_I32, "rows experts top width_p ff_p options"))
 DECAY_POWERS = 65
+DECAY_ROTARY = ATTENTION_ROWS = EXPERTS_ROWS = 1
 
 _SIGNATURES = {
     "qm_residual_norm_rows": (_I32, [C.POINTER(ResidualNorm), _I32, _I32, _P]),
@@ -45,6 +57,12 @@ _SIGNATURES = {
     "qm_decay_attention_rows": (_I32, [C.POINTER(DecayAttention), _P]),
     "qm_general_delta_scratch_floats": (_I64, [_I32, _I32, _I32]),
     "qm_general_delta_rows": (_I32, [C.POINTER(GeneralDelta), _P]),
+    "qm_latent_rows_norm": (_I32, [C.POINTER(LatentRows), _I32, _P]),
+    "qm_latent_query_stride": (_I32, [_I32, _I32]),
+    "qm_latent_expanded_bytes": (_I64, [_I32] * 6),
+    "qm_latent_attention_rows": (_I32, [C.POINTER(LatentAttention), _I32, _P]),
+    "qm_expert_scratch_bytes": (_I64, [_I32] * 6),
+    "qm_expert_rows": (_I32, [C.POINTER(Experts), _I32, _P]),
     "qm_decoder_last_error": (C.c_char_p, []),
     "qm_decoder_architecture": (C.c_char_p, [_I32]),
     "qm_decoder_check_config": (_I32, [C.c_char_p]),

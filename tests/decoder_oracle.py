@@ -135,12 +135,130 @@ def layer_runs(config):
     return runs + [(i, None, False) for i in range(loop["stop"], count)]
 
 
+def rotate_neighbours(x, first_position, frequencies, magnitude=1.0):
+    """x [tokens][heads][dim]: channels 2i and 2i + 1 turn by position * frequencies[i], times `magnitude`."""
+    n = 2 * len(frequencies)
+    p = first_position + np.arange(x.shape[0], dtype=F)
+    angle = (p[:, None] * np.asarray(frequencies, F)[None, :])[:, None, :]
+    c, s = np.cos(angle) * magnitude, np.sin(angle) * magnitude
+    out = x.copy()
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    out[..., 0:n:2], out[..., 1:n:2] = u * c - v * s, v * c + u * s
+    return out
+
+
+def yarn(dims, base, scaling):
+    """(frequencies, magnitude): slow pairs are stretched by `factor`, fast ones stay, a ramp between."""
+    f = np.power(F(base), -2.0 * np.arange(dims // 2, dtype=F) / dims)
+    if scaling is None:
+        return f, 1.0
+
+    def pair_that_turns(times):
+        return dims * np.log(scaling["original"] / (2 * np.pi * times)) / (2 * np.log(base))
+
+    lo = max(np.floor(pair_that_turns(scaling["fast"])), 0)
+    hi = min(np.ceil(pair_that_turns(scaling["slow"])), dims - 1)
+    ramp = np.clip((np.arange(dims // 2) - lo) / max(hi - lo, 0.001), 0, 1)
+    return f / scaling["factor"] * ramp + f * (1 - ramp), 0.1 * np.log(scaling["factor"]) + 1
+
+
+def retention(q, k, v, decay, rot):
+    """q, k [n][H][d] turned in halves, k scaled by d^(-1/2), then linear attention with a decay per head."""
+    dims, base = (rot["dims"], rot["base"]) if rot else (0, 1.0)
+    q, k = rotate(q, 0, dims, base), rotate(k, 0, dims, base) * q.shape[2] ** -0.5
+    return decayed_linear_attention(q, k, v, decay)[0]
+
+
+def mix_retention(h, spec, weight, eps, shared, index):
+    n, heads = h.shape[0], spec["heads"]
+    split = lambda name: (h @ weight(name).T).reshape(n, heads, -1)
+    o = retention(split("q"), split("k"), split("v"), spec["decay"], spec.get("rot"))
+    o = rms_norm(o, 1.0, eps).reshape(n, -1) * silu(h @ weight("g").T)
+    return o @ weight("o").T
+
+
+def latent_of(h, spec, down, norm, eps):
+    """What a latent layer keeps of each token: the normed latent and the turned key part that all heads share."""
+    kept = h @ down.T
+    rank = spec["kv_rank"]
+    frequencies, magnitude = yarn(spec["rot_dim"], spec["rot"]["base"], spec["rot"].get("scaling"))
+    return rms_norm(kept[:, :rank], norm, eps), rotate_neighbours(kept[:, None, rank:], 0, frequencies, magnitude)[:, 0]
+
+
+def latent_attention(q, latent, key_part, up_k, up_v, spec):
+    """q [n][H][dim + rot_dim] as projected; each head's keys and values are made from the latent -> [n][H][vdim]."""
+    n, heads, dim = q.shape[0], spec["heads"], spec["dim"]
+    frequencies, magnitude = yarn(spec["rot_dim"], spec["rot"]["base"], spec["rot"].get("scaling"))
+    q = np.concatenate([q[..., :dim], rotate_neighbours(q[..., dim:], 0, frequencies, magnitude)], axis=-1)
+    k = (latent @ up_k.T).reshape(n, heads, dim)
+    k = np.concatenate([k, np.broadcast_to(key_part[:, None, :], (n, heads, key_part.shape[1]))], axis=-1)
+    v = (latent @ up_v.T).reshape(n, heads, spec["vdim"])
+    return softmax_attention(q, k, v, spec["scale"], np.tril(np.ones((n, n), bool)))
+
+
+def mix_latent(h, spec, weight, eps, shared, index):
+    """`shared` maps a layer to what it keeps; a layer with 'kv_from' reads another's."""
+    n = h.shape[0]
+    source = spec.get("kv_from")
+    if source is None:
+        source = index
+        shared[index] = latent_of(h, spec, weight("dkv"), weight("dkv.norm"), eps)
+    q = rms_norm(h @ weight("dq").T, weight("dq.norm"), eps) @ weight("uq").T
+    o = latent_attention(q.reshape(n, spec["heads"], -1), *shared[source], weight("uk"), weight("uv"), spec)
+    return o.reshape(n, -1) @ weight("o").T
+
+
+def sigmoid_experts(h, router, experts, top):
+    """Each token's `top` experts of the highest sigmoid(router), weighted with it; `experts` is a list of functions."""
+    score = sigmoid(h @ router.T)
+    out = np.zeros((h.shape[0], experts[0](h[:1]).shape[1]), F)
+    for t in range(h.shape[0]):
+        for e in np.argsort(-score[t], kind="stable")[:top]:
+            out[t] += score[t, e] * experts[e](h[t:t + 1])[0]
+    return out
+
+
+def feed_forward(h, spec, weight):
+    if spec["kind"] == "dense":
+        return gated_mlp(h, weight("gate"), weight("up"), weight("down"))
+    experts = [lambda x, e=e: gated_mlp(x, *(weight(f"e{e}.{name}") for name in ("gate", "up", "down"))) for e in range(spec["router"]["experts"])]
+    return sigmoid_experts(h, weight("router"), experts, spec["router"]["top"])
+
+
+def bigram_rows(tokens, spec):
+    rows = [spec["buckets"]]
+    for before, token in zip(tokens[:-1], tokens[1:]):
+        rows.append((int(before) * spec["mul_prev"] + int(token) * spec["mul_cur"]) % spec["buckets"])
+    return np.array(rows)
+
+
+def forward_tuzavik(config, weights, tokens, streams=None):
+    eps, m = config["norm"]["eps"], config["residual_mult"]
+    tokens = np.asarray(tokens)
+    norm = lambda x, name: rms_norm(x, 1.0 + weights[name], eps)
+    x = weights["embed"][tokens] + weights["bigram"][bigram_rows(tokens, config["embedding"]["bigram"])]
+    shared = {}
+    for index, layer in enumerate(config["layers"]):
+        base = f"l{index}."
+        mix = {"retention": mix_retention, "latent_attention": mix_latent}[layer["type"]]
+        y = mix(norm(x, base + "norm1"), layer["mixer"], lambda name: weights[f"{base}mix.{name}"], eps, shared, index)
+        x = x + m * norm(y, base + "norm1b")
+        if layer["mlp"] is not None:
+            y = feed_forward(norm(x, base + "norm2"), layer["mlp"], lambda name: weights[f"{base}mlp.{name}"])
+            x = x + m * norm(y, base + "norm2b")
+        if streams is not None:
+            streams.append(x)
+    return norm(x, "final.norm") @ weights["head"].T * config["logit_scale"]
+
+
 MIXERS = {"parallel": mix_parallel, "general_delta": mix_general_delta}
 
 
 def forward(config, weights, tokens, streams=None):
     """Logits [tokens][vocab]; `streams` (a list) receives the residual stream behind every layer run."""
     weights = {name: np.asarray(t, dtype=F) for name, t in weights.items()}
+    if config["architecture"] == "Tuzavik":
+        return forward_tuzavik(config, weights, tokens, streams)
     eps = config["norm"]["eps"]
     x = weights["embed"][np.asarray(tokens)]
     for index, turn, opens in layer_runs(config):
