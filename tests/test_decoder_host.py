@@ -33,7 +33,8 @@ def test_header_symbols_are_exported(decoder):
 def test_structures_have_the_headers_layout(decoder, tmp_path):
     structures = {"qm_residual_term": decoder.ResidualTerm, "qm_residual_norm": decoder.ResidualNorm, "qm_gated_norm": decoder.GatedNorm,
                   "qm_decoder_linear": decoder.DecoderLinear, "qm_attention_partials": decoder.AttentionPartials,
-                  "qm_chunk_attention": decoder.ChunkAttention, "qm_decay_attention": decoder.DecayAttention, "qm_general_delta": decoder.GeneralDelta}
+                  "qm_chunk_attention": decoder.ChunkAttention, "qm_decay_attention": decoder.DecayAttention, "qm_general_delta": decoder.GeneralDelta,
+                  "qm_latent_rows": decoder.LatentRows, "qm_latent_attention": decoder.LatentAttention, "qm_experts": decoder.Experts}
     lines = [f'printf("{c} %zu\\n", sizeof({c}));' for c in structures]
     fields = [(c, name) for c, s in structures.items() for name, _ in s._fields_]
     lines += [f'printf("{c}.{name} %zu\\n", offsetof({c}, {name}));' for c, name in fields]
@@ -50,7 +51,7 @@ def test_structures_have_the_headers_layout(decoder, tmp_path):
 
 
 def test_registry_and_configurations(decoder, tmp_path):
-    assert decoder.architectures() == ["Vabevik"]
+    assert decoder.architectures() == ["Vabevik", "Tuzavik"]
     path = os.path.join(str(tmp_path), "config.json")
 
     def check(cfg):
@@ -87,6 +88,31 @@ def test_registry_and_configurations(decoder, tmp_path):
     broken(lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=64))
     broken(lambda c: c["layers"][1]["mixer"]["left"].pop("mask"))
     broken(lambda c: c["layers"][1]["mixer"]["right"].update(decay=[0.5]))
+    base = cases.CONFIGS["mixed"]
+    unscaled = copy.deepcopy(base)
+    unscaled["layers"][0]["mixer"]["rot"]["scaling"] = None
+    check(unscaled)
+    no_rotation = copy.deepcopy(base)
+    no_rotation["layers"][1]["mixer"]["rot"] = None
+    check(no_rotation)
+    broken(lambda c: c.pop("embedding"))
+    broken(lambda c: c["embedding"]["bigram"].update(buckets=0))
+    broken(lambda c: c["embedding"]["bigram"].update(mul_cur=1.5))
+    broken(lambda c: c.pop("residual_mult"))
+    broken(lambda c: c.pop("logit_scale"))
+    broken(lambda c: c["layers"][0].update(type="parallel"))
+    broken(lambda c: c["layers"][0]["mixer"].pop("scale"))
+    broken(lambda c: c["layers"][0]["mixer"]["rot"].update(dims=6))
+    broken(lambda c: c["layers"][0]["mixer"].update(rot_dim=7))
+    broken(lambda c: c["layers"][0]["mixer"]["rot"].update(scaling={"factor": 2.0}))
+    broken(lambda c: c["layers"][2]["mixer"].update(kv_from=1))       # not a latent layer
+    broken(lambda c: c["layers"][2]["mixer"].update(kv_from=2))       # not an earlier one
+    broken(lambda c: c["layers"][2]["mixer"].update(kv_rank=48))
+    broken(lambda c: c["layers"][2]["mixer"]["rot"].update(base=3.0))
+    broken(lambda c: c["layers"][1]["mixer"].update(decay=[0.5]))
+    broken(lambda c: c["layers"][1]["mixer"]["rot"].update(dims=18))
+    broken(lambda c: c["layers"][0]["mlp"]["router"].update(top=7))
+    broken(lambda c: c["layers"][0]["mlp"].update(kind="other"))
     with pytest.raises(decoder.DecoderError):
         check("{")
     with pytest.raises(decoder.DecoderError):
@@ -126,6 +152,24 @@ def test_operators_check_their_arguments(decoder):
     assert lib.qm_general_delta_rows(C.byref(decoder.GeneralDelta(**delta)), None) == 0
     for change in (dict(dim=257), dict(rank=0), dict(heads=0), dict(rows=-1), dict(w2=None)):
         assert lib.qm_general_delta_rows(C.byref(decoder.GeneralDelta(**{**delta, **change})), None) < 0, change
+    for change in (dict(rot_dims=18), dict(rot_dims=3, frequency=at), dict(rot_dims=8), dict(position=-1)):
+        assert lib.qm_decay_attention_rows(C.byref(decoder.DecayAttention(**{**decay, "options": decoder.DECAY_ROTARY, **change})), None) < 0, change
+    rows = dict(proj=at, q_norm=at, kv_norm=at, frequency=at, q_latent=at, latent_cache=at, key_cache=at, ld_proj=200, ld_q=128, ld_latent=128, rows=0,
+                q_rank=40, kv_rank=64, rot_dim=16, key_stride=16)
+    assert lib.qm_latent_rows_norm(C.byref(decoder.LatentRows(**rows)), 0, None) == 0
+    for change in (dict(kv_rank=129), dict(kv_rank=0), dict(rot_dim=15), dict(key_stride=8), dict(ld_q=30), dict(position=-1), dict(key_cache=None)):
+        assert lib.qm_latent_rows_norm(C.byref(decoder.LatentRows(**{**rows, **change})), 0, None) < 0, change
+    latent = dict(q=at, frequency=at, up_k=at, up_v=at, latent_cache=at, key_cache=at, out=at, q_scratch=at, ml=at, acc=at, ld_query=200, ld_latent=128,
+                  ld_out=128, rows=0, heads=4, dim=32, rot_dim=16, vdim=32, kv_rank=64, key_stride=16, splits=4)
+    assert lib.qm_latent_attention_rows(C.byref(decoder.LatentAttention(**latent)), 0, None) == 0
+    for change in (dict(heads=0), dict(kv_rank=2000), dict(ld_latent=60), dict(ld_query=100), dict(ld_out=100), dict(splits=65), dict(splits=0),
+                   dict(key_stride=8), dict(rot_dim=3), dict(position=-1), dict(acc=None)):
+        assert lib.qm_latent_attention_rows(C.byref(decoder.LatentAttention(**{**latent, **change})), 0, None) < 0, change
+    experts = dict(x=at, logits=at, gate=at, up=at, down=at, out32=at, scratch=at, ld_logits=8, rows=0, experts=8, top=2, width_p=128, ff_p=128)
+    assert lib.qm_expert_rows(C.byref(decoder.Experts(**experts)), 0, None) == 0
+    for change in (dict(top=9), dict(top=0), dict(experts=2000, ld_logits=2000), dict(ld_logits=7), dict(width_p=100), dict(ff_p=64), dict(down=None),
+                   dict(rows=4)):                                                  # (rows=4: no scratch)
+        assert lib.qm_expert_rows(C.byref(decoder.Experts(**{**experts, **change})), 0, None) < 0, change
     handle = C.c_void_p()
     assert lib.qm_decoder_create(None, 0, 1, 1, 0, None, C.byref(handle)) == null
     assert lib.qm_decoder_step(None, 0, None, 0, None, 0, None, None) == null
@@ -188,13 +232,114 @@ def test_delta_rule_writes_and_removes():
     assert np.allclose(o[2, 0], 0.25 * v[0, 0] + v[2, 0])
 
 
+def test_neighbours_turn_together():
+    x = np.zeros((3, 1, 6))
+    x[:, 0, 0], x[:, 0, 5] = 1.0, 7.0
+    y = plain.rotate_neighbours(x, 5, [1.0, 0.1], 2.0)
+    for t in range(3):
+        assert np.allclose(y[t, 0], [2 * np.cos(5 + t), 2 * np.sin(5 + t), 0, 0, 0, 7])
+
+
+def test_stretched_frequencies():
+    f, magnitude = plain.yarn(16, 10000.0, dict(factor=8.0, original=512, fast=32.0, slow=1.0))
+    unstretched, one = plain.yarn(16, 10000.0, None)
+    assert one == 1 and np.isclose(magnitude, 0.1 * np.log(8) + 1)
+    # pairs that turn often keep their frequency, those that turn less than once are stretched whole
+    turns = 512 * unstretched / (2 * np.pi)
+    assert np.allclose(f[turns > 32], unstretched[turns > 32]) and np.allclose(f[-1], unstretched[-1] / 8)
+    assert np.all(f <= unstretched + 1e-15) and np.all(f >= unstretched / 8 - 1e-15)
+    f, magnitude = plain.yarn(16, 10000.0, dict(factor=1.0, original=512, fast=32.0, slow=1.0))
+    assert np.allclose(f, unstretched) and magnitude == 1
+
+
+def test_retention_is_a_weighted_sum_of_turned_keys():
+    rng = np.random.default_rng(0)
+    q, k, v = rng.standard_normal((9, 2, 4)), rng.standard_normal((9, 2, 4)), rng.standard_normal((9, 2, 3))
+    decay = [0.5, 1.0]
+    o = plain.retention(q, k, v, decay, {"dims": 2, "base": 50.0})
+    for h in range(2):
+        for t in range(9):
+            want = np.zeros(3)
+            for j in range(t + 1):                              # one pair of frequency 1: only the distance counts
+                c, s = np.cos(t - j), np.sin(t - j)
+                turned = q[t, h, 0] * (c * k[j, h, 0] + s * k[j, h, 1]) + q[t, h, 1] * (c * k[j, h, 1] - s * k[j, h, 0])
+                want += decay[h] ** (t - j) * 0.5 * (turned + q[t, h, 2:] @ k[j, h, 2:]) * v[j, h]
+            assert np.allclose(o[t, h], want)
+
+
+def test_latent_attention_in_the_latents_space():
+    """Keys and values made from latents give what queries sent through up_k and results sent through up_v give."""
+    spec = dict(heads=3, dim=5, rot_dim=4, vdim=6, kv_rank=7, scale=0.4, rot={"base": 30.0, "dims": 4})
+    rng = np.random.default_rng(1)
+    q, c, k = rng.standard_normal((8, 3, 9)), rng.standard_normal((8, 7)), rng.standard_normal((8, 4))
+    up_k, up_v = rng.standard_normal((15, 7)), rng.standard_normal((18, 7))
+    o = plain.latent_attention(q, c, k, up_k, up_v, spec)
+    turned = plain.rotate_neighbours(q[..., 5:], 0, plain.yarn(4, 30.0, None)[0])
+    for h in range(3):
+        for t in range(8):
+            score = (c[:t + 1] @ (up_k[5 * h:5 * h + 5].T @ q[t, h, :5]) + k[:t + 1] @ turned[t, h]) * 0.4
+            p = np.exp(score - score.max())
+            assert np.allclose(o[t, h], up_v[6 * h:6 * h + 6] @ ((p / p.sum()) @ c[:t + 1]))
+
+
+def test_experts_of_the_highest_scores_are_weighted_with_them():
+    h = np.array([[1.0, -2.0], [0.5, 3.0]])
+    router = np.array([[1.0, 0.0], [0.0, 1.0], [-1.0, 0.0]])
+    experts = [lambda x, e=e: np.full((1, 2), float(10 ** e)) for e in range(3)]
+    s = plain.sigmoid(h @ router.T)
+    out = plain.sigmoid_experts(h, router, experts, 2)
+    assert np.allclose(out[0], s[0, 0] * 1 + s[0, 2] * 100) and np.allclose(out[1], s[1, 1] * 10 + s[1, 0] * 1)
+
+
+def test_bigram_rows():
+    assert list(plain.bigram_rows([4, 9, 2], dict(buckets=7, mul_prev=3, mul_cur=5))) == [7, (12 + 45) % 7, (27 + 10) % 7]
+
+
 def test_layer_runs_of_a_loop():
     assert plain.layer_runs(cases.CONFIGS["looped"]) == [(0, None, False)] + [(1, 0, True), (2, 0, False), (1, 1, True), (2, 1, False),
                                                                                (1, 2, True), (2, 2, False)] + [(3, None, False)]
     assert [r[0] for r in plain.layer_runs(cases.CONFIGS["plain"])] == [0, 1, 2]
 
 
-@pytest.mark.parametrize("name", sorted(cases.CONFIGS))
+@pytest.mark.parametrize("name", cases.SANDWICH)
+def test_plain_model_sees_a_planted_mistake_in_a_sandwich_layer(name):
+    """Each mechanism of the tests' models moves the logits by far more than the product's tolerance when it is wrong."""
+    cfg, w = cases.CONFIGS[name], cases.weights(cases.CONFIGS[name])
+    tokens = cases.tokens_of(cfg, 90)
+    want = plain.forward(cfg, w, tokens)
+
+    def moved(change):
+        c = copy.deepcopy(cfg)
+        change(c)
+        return cases.error(plain.forward(c, w, tokens), want)
+
+    def every(kind, change):
+        def apply(c):
+            for layer in c["layers"]:
+                if layer["type"] == kind:
+                    change(layer["mixer"])
+        return apply
+
+    kinds = {layer["type"] for layer in cfg["layers"]}
+    assert moved(lambda c: c.update(residual_mult=c["residual_mult"] * 1.2)) > 0.05
+    assert moved(lambda c: c["embedding"]["bigram"].update(mul_cur=c["embedding"]["bigram"]["mul_cur"] + 1)) > 0.2
+    if "retention" in kinds:
+        assert moved(every("retention", lambda m: m.update(decay=[d * 0.97 for d in m["decay"]]))) > 0.004
+        assert moved(every("retention", lambda m: m["rot"].update(base=m["rot"]["base"] * 2))) > 0.02
+    if "latent_attention" in kinds:
+        assert moved(every("latent_attention", lambda m: m.update(scale=m["scale"] * 1.1))) > 0.01
+        assert moved(every("latent_attention", lambda m: m["rot"].update(base=m["rot"]["base"] * 2))) > 0.02
+        if any("scaling" in layer["mixer"]["rot"] for layer in cfg["layers"]):
+            assert moved(every("latent_attention", lambda m: m["rot"].pop("scaling", None))) > 0.05
+    if any(layer["mlp"] and layer["mlp"]["kind"] == "moe" and layer["mlp"]["router"]["top"] > 1 for layer in cfg["layers"]):
+        def fewer(c):
+            for layer in c["layers"]:
+                if layer["mlp"] and layer["mlp"]["kind"] == "moe":
+                    layer["mlp"]["router"]["top"] -= 1
+        assert moved(fewer) > 0.05
+
+
+@pytest.mark.parametrize("name", cases.PARALLEL)
 def test_plain_model_sees_a_planted_mistake(name):
     """The tests' weights make faults visible: a chunk that is one longer, a lost state, a missing loop vector, a key/value head
     taken for another all move some logits by far more than the product's tolerance."""

@@ -114,15 +114,16 @@ def test_sequences_side_by_side(decoder, models, name, f32):
 @pytest.mark.parametrize("f32", [True, False])
 def test_passes_of_few_rows_and_small_rings(decoder, models, f32):
     """A prompt longer than a pass, in an engine whose rings are a few positions longer than the chunks."""
-    m = models("short_chunks")
-    for max_rows in (3, 20, 64):
-        engine = decoder.Decoder(m.directory, 100000, float32=f32, max_rows=max_rows)
-        assert engine.sequence_bytes < 2 ** 20
-        s = engine.open()
-        assert cases.error(feed(engine, s, m.tokens, [120] + [1] * 20 + [30]), m.want) < LIMIT[f32]
+    for name, capacity in (("short_chunks", 100000), ("mixed", 300), ("retention", 100000)):
+        m = models(name)
+        for max_rows in (3, 20, 64):
+            engine = decoder.Decoder(m.directory, capacity, float32=f32, max_rows=max_rows)
+            assert engine.sequence_bytes < 2 ** 20
+            s = engine.open()
+            assert cases.error(feed(engine, s, m.tokens, [120] + [1] * 20 + [30]), m.want) < LIMIT[f32]
 
 
-@pytest.mark.parametrize("name", ["short_chunks", "looped"])
+@pytest.mark.parametrize("name", ["short_chunks", "looped", "mixed", "latents"])
 def test_long_decoding(decoder, models, name):
     m = models(name)
     tokens = cases.tokens_of(m.cfg, 420, seed=3)
@@ -208,15 +209,15 @@ def test_errors_leave_the_engine_usable(decoder, models):
         engine.step(s, [1])
 
 
+@pytest.mark.parametrize("model,name", [("plain", "l1.mix.w2"), ("mixed", "l2.mlp.e11.up"), ("mixed", "l0.mix.dkv"), ("retention", "bigram")])
 @pytest.mark.parametrize("change,code", [("missing", -8), ("shape", -8), ("dtype", -8)])
-def test_wrong_weights_are_refused(decoder, tmp_path, change, code):
+def test_wrong_weights_are_refused(decoder, tmp_path, change, code, model, name):
     import torch
     from safetensors.torch import load_file, save_file
-    cfg = cases.CONFIGS["plain"]
+    cfg = cases.CONFIGS[model]
     cases.write_model(str(tmp_path), cfg, cases.weights(cfg))
     path = os.path.join(str(tmp_path), "model.safetensors")
     tensors = load_file(path)
-    name = "l1.mix.w2"
     if change == "missing":
         del tensors[name]
     elif change == "shape":
@@ -227,6 +228,54 @@ def test_wrong_weights_are_refused(decoder, tmp_path, change, code):
     with pytest.raises(decoder.DecoderError) as e:
         decoder.Decoder(str(tmp_path), 16)
     assert e.value.code == code and name in str(e.value)
+
+
+def test_first_tokens_and_the_token_before(decoder, models):
+    """A sequence's first token has none before it, also in memory that was used; the next step's first token has the last one's."""
+    m = models("retention")
+    engine = decoder.Decoder(m.directory, 64, float32=True)
+    for portions in ([1, 1, 1, 1], [2, 2], [1, 3], [3, 1], [4]):
+        s = engine.open()
+        assert cases.error(feed(engine, s, m.tokens[:4], portions), m.want[:4]) < LIMIT[True]
+        engine.generate(s, m.tokens[4:9], 3)
+        engine.close(s)
+    engine.set_path(2)
+    s = engine.open()
+    assert cases.error(feed(engine, s, m.tokens[:6], [1, 1, 3, 1]), m.want[:6]) < LIMIT[True]
+
+
+@pytest.mark.parametrize("f32", [True, False])
+def test_a_far_key_decides(decoder, tmp_path, f32):
+    """Latent attention whose query looks for one token: its only occurrence is hundreds of positions back, at a pass's edge or in the
+    middle, and the logits tell it from a sequence without it."""
+    cfg = cases.sandwich(48, 96, [cases.latent(4, 24, 8, 32, 40, 64, cases.dense(64))], (13, 3, 1), residual_mult=2.0)
+    w = cases.weights(cfg, seed=3)
+    # token 7's latent stands out: a direction of its own through dkv and up_k, which every query carries through dq and up_q
+    rng = np.random.default_rng(4)
+    mark, mark_c, mark_q = (cases.bf16(v / np.linalg.norm(v)) for v in (rng.standard_normal(96), rng.standard_normal(64), rng.standard_normal(40)))
+    w["embed"][7] = cases.bf16(60 * mark)
+    w["l0.mix.dkv"][:64] = cases.bf16(0.3 * w["l0.mix.dkv"][:64] + 2.0 * np.outer(mark_c, mark))
+    head = cases.bf16(np.ones(24) * 0.4)
+    for h in range(4):
+        w["l0.mix.uk"][24 * h:24 * h + 24] = cases.bf16(0.1 * w["l0.mix.uk"][24 * h:24 * h + 24] + 4.0 * np.outer(head, mark_c))
+        w["l0.mix.uq"][32 * h:32 * h + 24] = cases.bf16(0.1 * w["l0.mix.uq"][32 * h:32 * h + 24] + 6.0 * np.outer(head, mark_q))
+    cases.write_model(str(tmp_path), cfg, w)
+    tokens = cases.tokens_of(cfg, 700, seed=2)
+    tokens[tokens == 7] = 8
+    for at in (0, 63, 64, 65, 127, 300, 511, 639):
+        marked = tokens.copy()
+        marked[at] = 7
+        want = plain.forward(cfg, w, marked)
+        if at == 0:
+            # (half of the queries look for the mark, the others away from it)
+            moved = np.abs(want - plain.forward(cfg, w, tokens)).max(axis=1)[650:] / np.abs(want).max()
+            assert np.quantile(moved, 0.75) > 0.1
+        engine = decoder.Decoder(str(tmp_path), 700, float32=f32)
+        for portions in ([660] + [1] * 40, [at + 1, 699 - at], [64, 2, 62, 572]):
+            s = engine.open()
+            got = feed(engine, s, marked, portions)
+            engine.close(s)
+            assert cases.error(got[640:], want[640:]) < LIMIT[f32], (at, portions)
 
 
 def test_trace_replay_program(models, tmp_path):

@@ -57,12 +57,19 @@ def test_residual_norm(decoder, dev, f32, width, ld, rows):
     table = put(embed, dev, torch.bfloat16)
     eps, w = 0.01, slice(0, width)
 
+    bigram = cases.bf16(padded(6))
+    d["fed"], bigrams = put(np.concatenate([[-1], tokens]).astype(np.int32), dev), put(bigram, dev, torch.bfloat16)      # (no token before row 0's)
+
     def terms(src):
         return (0.5 * plain.rms_norm(y[0][src, w], norms[0, w], eps) - 0.25 * plain.rms_norm(y[1][src, w], norms[1, w], eps) + y[2][src, w])
 
-    for mapped, embedded, count, stepped in ((False, False, 3, True), (True, False, 3, False), (True, True, 0, True), (False, True, 2, False)):
+    for mapped, embedded, count, stepped, pairs in ((False, False, 3, True, False), (True, False, 3, False, False), (True, True, 0, True, False),
+                                                    (False, True, 2, False, False), (False, True, 0, False, True), (True, True, 2, False, True)):
         src = row_map if mapped else np.arange(rows)
         want = (embed[tokens[src]][:, w] if embedded else x[src, w]).astype(np.float64)
+        if pairs:
+            rows_of = [5 if i == 0 else (3 * int(tokens[i - 1]) + 4 * int(tokens[i])) % 5 for i in src]
+            want = want + bigram[rows_of][:, w]
         if count == 3:
             want = want + terms(src)
         elif count == 2:
@@ -75,6 +82,9 @@ def test_residual_norm(decoder, dev, f32, width, ld, rows):
                                   row_map=d["map"].data_ptr() if mapped else None, step_vec=d["step"].data_ptr() if stepped else None,
                                   norm_w=d["norms"].data_ptr() + 8 * ld, x_out=x_out.data_ptr(), h=h.data_ptr(), ld_h=ld, width=width, vocab=11,
                                   terms=count, eps=eps)
+        if pairs:
+            op.tokens, op.bigram = d["fed"].data_ptr() + 4, bigrams.data_ptr()
+            op.buckets, op.mul_prev, op.mul_cur = 5, 3, 4
         chosen = [("y0", 0, 0.5), ("y1", 1, -0.25), ("y2", None, 1.0)] if count == 3 else [("y0", 0, 0.5), ("y2", None, 1.0)][:count]
         for i, (name, norm, scale) in enumerate(chosen):
             op.term[i] = decoder.ResidualTerm(d[name].data_ptr(), None if norm is None else d["norms"].data_ptr() + 4 * norm * ld, ld, scale, 0)
@@ -87,17 +97,19 @@ def test_residual_norm(decoder, dev, f32, width, ld, rows):
 
 @pytest.mark.parametrize("f32", [True, False])
 @pytest.mark.parametrize("groups,size,ld", [(1, 96, 128), (1, 2048, 2048), (1, 5000, 5120), (1, 70, 128), (3, 20, 128), (16, 128, 2048), (2, 160, 384), (1, 1, 128)])
-def test_gated_norm(decoder, dev, f32, groups, size, ld):
+@pytest.mark.parametrize("silu", [0, 1])
+def test_gated_norm(decoder, dev, f32, groups, size, ld, silu):
     import torch
     rng = np.random.default_rng(size)
     n, rows = groups * size, 3
     o, gate, weight = rng.standard_normal((rows, n)).astype(np.float32), rng.standard_normal((rows, n + 12)).astype(np.float32), rng.standard_normal(n).astype(np.float32)
     out = torch.full((rows, ld), 7.0, device=dev, dtype=activation(f32))
     d = [put(v, dev) for v in (o, weight, gate)]
-    op = decoder.GatedNorm(o=d[0].data_ptr(), weight=d[1].data_ptr(), gate=d[2].data_ptr(), out=out.data_ptr(), ld_o=n, ld_gate=n + 12, ld_out=ld,
+    op = decoder.GatedNorm(o=d[0].data_ptr(), weight=None if silu else d[1].data_ptr(), silu=silu, gate=d[2].data_ptr(), out=out.data_ptr(), ld_o=n, ld_gate=n + 12, ld_out=ld,
                            groups=groups, size=size, eps=0.02)
     assert decoder.lib().qm_gated_norm_rows(C.byref(op), rows, int(f32), torch.cuda.current_stream().cuda_stream) == 0
-    want = plain.rms_norm(o.astype(np.float64).reshape(rows, groups, size), 1.0, 0.02).reshape(rows, n) * weight * plain.sigmoid(gate[:, :n].astype(np.float64))
+    g = gate[:, :n].astype(np.float64)
+    want = plain.rms_norm(o.astype(np.float64).reshape(rows, groups, size), 1.0, 0.02).reshape(rows, n) * (plain.silu(g) if silu else weight * plain.sigmoid(g))
     got = get(out)
     close(got[:, :n], want, f32)
     assert np.all(got[:, n:] == 0)
@@ -290,3 +302,207 @@ def test_general_delta(decoder, dev, chunked, heads, dim, rank):
             at += rows
         close(np.concatenate(got), want.reshape(n, -1), True, tol32=2e-5)
         close(get(s), state, True, tol32=2e-5)
+
+
+@pytest.mark.parametrize("chunked", [False, True])
+@pytest.mark.parametrize("heads,dim,vdim,rot_dims", [(3, 16, 24, 16), (2, 20, 36, 6), (1, 48, 16, 0), (4, 64, 128, 64), (2, 132, 200, 130), (2, 256, 64, 256)])
+def test_retention(decoder, dev, chunked, heads, dim, vdim, rot_dims):
+    """The decayed attention with rotated queries and keys, scaled keys and plain values."""
+    import torch
+    rng = np.random.default_rng(dim)
+    n, base = 230, 700.0
+    decay = np.array([0.999, 1.0, 0.3, 0.0][:heads])
+    ld = heads * (2 * dim + vdim) + 12
+    proj = rng.standard_normal((n, ld)).astype(np.float32)
+    k_at, v_at = heads * dim + 4, 2 * heads * dim + 8
+    proj[3, k_at:k_at + heads * dim] *= 30.0                          # an early key that later queries see through the decay
+    part = lambda at, count, size: proj[:, at:at + count * size].astype(np.float64).reshape(n, count, size)
+    q, k, v = part(0, heads, dim), part(k_at, heads, dim), part(v_at, heads, vdim)
+    want = plain.retention(q, k, v, decay, {"dims": rot_dims, "base": base}).reshape(n, -1)
+    powers = put(np.power(decay[:, None], np.arange(decoder.DECAY_POWERS)[None]).astype(np.float32), dev)
+    frequency = put(base ** (-2.0 * np.arange(max(1, rot_dims // 2)) / max(1, rot_dims)), dev)
+    for portions in ([n], [100, 2, 28, 1, 17, 64, 16, 2], [1] * 20 + [65, 145]):
+        pd = put(proj, dev)                                           # (rotated in place)
+        s = torch.zeros((heads, dim, vdim), device=dev)
+        got, at = [], 0
+        for rows in portions:
+            out = torch.full((rows, heads * vdim), 7.0, device=dev)
+            floats = decoder.lib().qm_decay_attention_scratch_floats(rows, heads, dim, vdim)
+            scratch = torch.full((max(1, floats),), float("nan"), device=dev)
+            where = torch.tensor([at], dtype=torch.int32, device=dev)
+            op = decoder.DecayAttention(proj=pd.data_ptr() + 4 * ld * at, powers=powers.data_ptr(), state=s.data_ptr(), out=out.data_ptr(),
+                                        scratch=scratch.data_ptr() if chunked else None, frequency=frequency.data_ptr(), ld_proj=ld, scratch_floats=floats,
+                                        rows=rows, heads=heads, dim=dim, vdim=vdim, q_column=0, k_column=k_at, v_column=v_at, options=decoder.DECAY_ROTARY,
+                                        rot_dims=rot_dims, position=at, k_scale=dim ** -0.5)
+            if rows == 1:
+                op.position, op.position_dev = 0, where.data_ptr()
+            assert decoder.lib().qm_decay_attention_rows(C.byref(op), torch.cuda.current_stream().cuda_stream) == 0
+            got.append(get(out))
+            at += rows
+        close(np.concatenate(got), want, True, tol32=5e-6)
+
+
+LATENT = [
+    # heads, dim, rot_dim, vdim, kv_rank, scaling
+    (3, 16, 8, 24, 40, None), (8, 32, 16, 32, 64, (8.0, 100, 32.0, 1.0)), (5, 20, 6, 28, 100, None), (16, 64, 32, 64, 256, None), (17, 128, 64, 128, 512, None),
+    (1, 33, 10, 17, 300, (4.0, 50, 8.0, 0.5)), (2, 40, 64, 72, 128, None), (2, 200, 80, 24, 560, None), (2, 16, 70, 300, 96, None), (40, 8, 2, 8, 24, None),
+]
+
+
+class LatentCase:
+    """Projections of a sequence; some latents stand out so that single keys far away, at the edges of passes and tiles, decide."""
+
+    def __init__(self, shape, tokens, seed=0):
+        self.heads, self.dim, self.rot, self.vdim, self.rank, scaling = shape
+        rng = np.random.default_rng(seed)
+        self.n, self.base = tokens, 900.0
+        self.scaling = dict(zip(("factor", "original", "fast", "slow"), scaling)) if scaling else None
+        self.per_head = self.dim + self.rot
+        self.proj = rng.standard_normal((tokens, 20 + self.rank + self.rot + 8)).astype(np.float32)          # 20 columns of a query latent
+        self.kv_at = 20 + 4
+        self.q = (2.0 * rng.standard_normal((tokens, self.heads * self.per_head + 4))).astype(np.float32)
+        self.kv_norm = (1 + 0.2 * rng.standard_normal(self.rank)).astype(np.float32)
+        self.q_norm = (1 + 0.2 * rng.standard_normal(20)).astype(np.float32)
+        for at in (0, 1, 63, 64, 127, 128, tokens - 40):
+            self.proj[at, self.kv_at + self.rank:self.kv_at + self.rank + self.rot] *= 4.0                   # (the latent itself is normed)
+        self.up_k = cases.bf16(rng.standard_normal((self.heads * self.dim, self.rank)) * self.rank ** -0.5)
+        self.up_v = cases.bf16(rng.standard_normal((self.heads * self.vdim, self.rank)) * self.rank ** -0.5)
+        self.scale, self.eps = self.per_head ** -0.5, 0.01
+        self.spec = {"heads": self.heads, "dim": self.dim, "rot_dim": self.rot, "vdim": self.vdim, "kv_rank": self.rank, "scale": self.scale,
+                     "rot": {"base": self.base, "dims": self.rot, "scaling": self.scaling}}
+
+    def kept(self):
+        p = self.proj[:, self.kv_at:self.kv_at + self.rank + self.rot].astype(np.float64)
+        return plain.latent_of(p, self.spec, np.eye(self.rank + self.rot), self.kv_norm.astype(np.float64), self.eps)
+
+    def want(self):
+        q = self.q[:, :self.heads * self.per_head].astype(np.float64).reshape(self.n, self.heads, self.per_head)
+        return plain.latent_attention(q, *self.kept(), self.up_k.astype(np.float64), self.up_v.astype(np.float64), self.spec).reshape(self.n, -1)
+
+    def run(self, decoder, dev, f32, portions, rows_only=False, splits=5):
+        import torch
+        lib, dtype = decoder.lib(), activation(f32)
+        stream = torch.cuda.current_stream().cuda_stream
+        up128 = lambda n: (n + 127) // 128 * 128
+        ld, key_stride, n_out = up128(self.rank), (self.rot + 7) // 8 * 8, self.heads * self.vdim
+        ld_out = up128(n_out)
+        v_row = (self.heads * self.dim + 7) // 8 * 8
+        up_rows = up128(v_row + n_out)
+        up = np.zeros((up_rows, ld), np.float32)
+        up[:self.heads * self.dim, :self.rank] = self.up_k
+        up[v_row:v_row + n_out, :self.rank] = self.up_v
+        up = put(up, dev, torch.bfloat16)
+        frequencies, magnitude = plain.yarn(self.rot, self.base, self.scaling)
+        freq, proj, q = put(frequencies, dev), put(self.proj, dev), put(self.q, dev)
+        kv_norm, q_norm = put(self.kv_norm, dev), put(self.q_norm, dev)
+        latent = torch.full((self.n, ld), float("nan"), device=dev, dtype=dtype)
+        keys = torch.full((self.n, key_stride), float("nan"), device=dev, dtype=dtype)
+        most, stride = max(portions), lib.qm_latent_query_stride(self.rank, self.rot)
+        q_scratch = torch.full((most * self.heads * stride,), float("nan"), device=dev, dtype=dtype)
+        ml = torch.full((most * self.heads * splits * 2,), float("nan"), device=dev)
+        acc = torch.full((most * self.heads * splits * self.rank,), float("nan"), device=dev)
+        nbytes = lib.qm_latent_expanded_bytes(self.n, self.heads, self.dim, self.rot, self.vdim, up_rows)
+        expanded = torch.full((nbytes // 2,), float("nan"), device=dev, dtype=torch.bfloat16)
+        got, norms, at = [], [], 0
+        for rows in portions:
+            where = torch.tensor([at], dtype=torch.int32, device=dev)
+            latent_q = torch.full((rows, 128), 7.0, device=dev, dtype=dtype)
+            keep = decoder.LatentRows(proj=proj.data_ptr() + 4 * self.proj.shape[1] * at, q_norm=q_norm.data_ptr(), kv_norm=kv_norm.data_ptr(),
+                                      frequency=freq.data_ptr(), q_latent=latent_q.data_ptr(), latent_cache=latent.data_ptr(), key_cache=keys.data_ptr(),
+                                      ld_proj=self.proj.shape[1], ld_q=128, ld_latent=ld, position=at, rows=rows, q_rank=20, kv_rank=self.rank,
+                                      rot_dim=self.rot, key_stride=key_stride, q_column=0, kv_column=self.kv_at, eps=self.eps, magnitude=magnitude)
+            assert lib.qm_latent_rows_norm(C.byref(keep), int(f32), stream) == 0
+            norms.append(get(latent_q))
+            out = torch.full((rows, ld_out), 7.0, device=dev, dtype=dtype)
+            op = decoder.LatentAttention(q=q.data_ptr() + 4 * self.q.shape[1] * at, frequency=freq.data_ptr(), up_k=up.data_ptr(),
+                                         up_v=up.data_ptr() + 2 * v_row * ld, latent_cache=latent.data_ptr(), key_cache=keys.data_ptr(), out=out.data_ptr(),
+                                         q_scratch=q_scratch.data_ptr(), ml=ml.data_ptr(), acc=acc.data_ptr(), expanded=expanded.data_ptr(),
+                                         ld_query=self.q.shape[1], ld_latent=ld, ld_out=ld_out, expanded_bytes=nbytes, position=at, rows=rows,
+                                         heads=self.heads, dim=self.dim, rot_dim=self.rot, vdim=self.vdim, kv_rank=self.rank, key_stride=key_stride,
+                                         splits=splits, up_rows=up_rows, up_v_row=v_row, options=decoder.ATTENTION_ROWS if rows_only else 0,
+                                         scale=self.scale, magnitude=magnitude)
+            if rows == 1:
+                op.position, op.position_dev = 0, where.data_ptr()
+            assert lib.qm_latent_attention_rows(C.byref(op), int(f32), stream) == 0
+            out = get(out)
+            assert np.all(out[:, n_out:] == 0)
+            got.append(out[:, :n_out])
+            at += rows
+        return np.concatenate(got), np.concatenate(norms), get(latent), get(keys)
+
+
+@pytest.mark.parametrize("shape", LATENT)
+def test_latent_attention(decoder, dev, shape):
+    case = LatentCase(shape, 230)
+    want, (latent, key_part) = case.want(), case.kept()
+    q_latent = plain.rms_norm(case.proj[:, :20].astype(np.float64), case.q_norm, case.eps)
+    for portions in ([230], [100, 2, 28, 1, 1, 17, 3, 16, 62], [1] * 8 + [222], [60, 15, 2, 2, 2, 2] + [1] * 60 + [87]):
+        got, norms, c, k = case.run(decoder, dev, True, portions)
+        close(got, want, True, tol32=2e-5)
+        close(norms[:, :20], q_latent, True, tol32=3e-6)
+        close(c[:, :case.rank], latent, True, tol32=3e-6)
+        close(k[:, :case.rot], key_part, True, tol32=3e-6)
+        assert np.all(norms[:, 20:] == 0) and np.all(c[:, case.rank:] == 0) and np.all(k[:, case.rot:] == 0)
+        for rows_only in (False, True):
+            got, norms, c, k = case.run(decoder, dev, False, portions, rows_only=rows_only)
+            close(got, want, False, tol16=3e-2)
+            close(c[:, :case.rank], latent, False)
+
+
+@pytest.mark.parametrize("splits", [1, 2, 32, 64])
+def test_latent_attention_splits(decoder, dev, splits):
+    case = LatentCase((6, 24, 8, 16, 72, None), 700, seed=2)
+    want = case.want()
+    portions = [570, 1, 1, 5] + [1] * 70 + [15, 38]
+    close(case.run(decoder, dev, True, portions, splits=splits)[0], want, True, tol32=2e-5)
+    for rows_only in (False, True):
+        close(case.run(decoder, dev, False, portions, splits=splits, rows_only=rows_only)[0], want, False, tol16=3e-2)
+
+
+def test_many_positions_are_expanded_in_several_linears(decoder, dev):
+    case = LatentCase((2, 16, 8, 16, 32, None), 4400, seed=3)
+    close(case.run(decoder, dev, False, [2100, 2300])[0], case.want(), False, tol16=3e-2)
+
+
+@pytest.mark.parametrize("f32", [True, False])
+@pytest.mark.parametrize("rows", [1, 2, 5, 16, 40, 300])
+@pytest.mark.parametrize("experts,top,width,ff", [(8, 4, 192, 64), (1, 1, 128, 128), (5, 5, 100, 200), (70, 6, 130, 40), (300, 3, 128, 96), (3, 1, 256, 384)])
+def test_experts(decoder, dev, f32, rows, experts, top, width, ff):
+    import torch
+    rng = np.random.default_rng(experts + rows)
+    up128 = lambda n: (n + 127) // 128 * 128
+    wp, fp = up128(width), up128(ff)
+    x = cases.bf16(rng.standard_normal((rows, width)))
+    router = rng.standard_normal((experts, width)) * width ** -0.5
+    logits = (x @ router.T).astype(np.float32)
+    if experts > 1:
+        logits[0, 1] = logits[0, 0]                                   # equals: the lower number first
+    if rows > 30:
+        logits[:, -1] += 4.0                                          # an expert that nearly every row takes
+    gate, up, down = (cases.bf16(rng.standard_normal(s) * s[2] ** -0.5) for s in ((experts, ff, width), (experts, ff, width), (experts, width, ff)))
+
+    def padded(a, *shape):
+        out = np.zeros(shape, np.float32)
+        out[tuple(slice(0, n) for n in a.shape)] = a
+        return out
+
+    xd = put(padded(x, rows, wp), dev, activation(f32))
+    ld = experts + 5
+    ld_logits = put(padded(logits, rows, ld), dev)
+    wd = [put(padded(a, experts, *s), dev, torch.bfloat16) for a, s in ((gate, (fp, wp)), (up, (fp, wp)), (down, (wp, fp)))]
+    want = np.zeros((rows, width))
+    score = plain.sigmoid(logits.astype(np.float64))
+    for t in range(rows):
+        for e in np.argsort(-logits[t], kind="stable")[:top]:
+            want[t] += score[t, e] * plain.gated_mlp(x[t:t + 1].astype(np.float64), *(w[e].astype(np.float64) for w in (gate, up, down)))[0]
+    for options in (0, decoder.EXPERTS_ROWS):
+        nbytes = decoder.lib().qm_expert_scratch_bytes(rows, experts, top, wp, fp, int(f32))
+        scratch = torch.full((nbytes // 4,), float("nan"), device=dev)
+        out = torch.full((rows, wp), 7.0, device=dev)
+        op = decoder.Experts(x=xd.data_ptr(), logits=ld_logits.data_ptr(), gate=wd[0].data_ptr(), up=wd[1].data_ptr(), down=wd[2].data_ptr(),
+                             out32=out.data_ptr(), scratch=scratch.data_ptr(), ld_logits=ld, scratch_bytes=nbytes, rows=rows, experts=experts, top=top,
+                             width_p=wp, ff_p=fp, options=options)
+        assert decoder.lib().qm_expert_rows(C.byref(op), int(f32), torch.cuda.current_stream().cuda_stream) == 0
+        got = get(out)
+        close(got[:, :width], want, f32, tol32=5e-6, tol16=2e-2)
+        assert np.all(got[:, width:] == 0)
