@@ -1126,18 +1126,103 @@ def write_decoder_model(directory, width, left, chunk, right, delta, ff, vocab=4
     return sum(t.numel() * 2 for name, t in tensors.items() if name not in ("embed", "head"))
 
 
-def decoder_throughput(size, dev, rows=1024, steps=64, kinds=None):
-    """Prefill of `rows` tokens and decoding behind them for a decoder language model of one of DECODER_SIZES; microseconds are
-    per layer run (head included in the total it is divided from)."""
+TUZAVIK_SIZES = {
+    # name: width, retention (heads, dim, value dim), latent (heads, dim, rotated dim, value dim, query rank, latent rank), ff,
+    # experts (number, chosen, ff)
+    "w1024": dict(width=1024, retention=(8, 128, 256), latent=(8, 128, 64, 128, 512, 256), ff=3072, experts=(32, 4, 512)),
+    "w2048": dict(width=2048, retention=(16, 128, 256), latent=(16, 128, 64, 128, 768, 512), ff=6144, experts=(32, 4, 1024)),
+    "w4096": dict(width=4096, retention=(32, 128, 256), latent=(32, 128, 64, 128, 1536, 512), ff=12288, experts=(32, 4, 2048)),
+}
+# layers of a model: mixer ("shared": latent attention over the layer before's latents) and feed-forward
+TUZAVIK_KINDS = {
+    "mixed": (("retention", "dense"), ("latent", "experts"), ("retention", "experts"), ("shared", "dense")),
+    "retention": (("retention", "dense"),) * 4,
+    "latent": (("latent", "dense"), ("shared", "dense")) * 2,
+    "experts": (("retention", "experts"),) * 4,
+}
+
+
+def write_tuzavik_model(directory, width, retention, latent, ff, experts, kinds, vocab=4096, seed=1, dev="cpu"):
+    """A Tuzavik model directory of random weights: config.json and model.safetensors; returns the bytes of the layers' weights
+    that a prompt of many tokens reads, and those that one token reads."""
+    import torch
+    from safetensors.torch import save_file
+    gen = torch.Generator(device=dev).manual_seed(seed)
+    tensors = {}
+
+    def linear(name, n, k):
+        tensors[name] = (torch.randn(n, k, generator=gen, device=dev) * k ** -0.5).to(torch.bfloat16).cpu()
+
+    def norm(name, n):
+        tensors[name] = (0.1 * torch.randn(n, generator=gen, device=dev)).to(torch.bfloat16).cpu()
+
+    linear("embed", vocab, width)
+    linear("bigram", 1024, width)
+    linear("head", vocab, width)
+    norm("final.norm", width)
+    layers, source, skipped = [], None, 0
+    number, top, expert_ff = experts
+    for i, (mix, feed) in enumerate(kinds):
+        base = f"l{i}."
+        for name in ("norm1", "norm1b", "norm2", "norm2b"):
+            norm(base + name, width)
+        if mix == "retention":
+            h, d, e = retention
+            for name, n in (("q", h * d), ("k", h * d), ("v", h * e), ("g", h * e)):
+                linear(base + "mix." + name, n, width)
+            linear(base + "mix.o", width, h * e)
+            layer = {"type": "retention", "mixer": {"heads": h, "dim": d, "vdim": e, "decay": [1.0 - 2.0 ** -(1 + 8 * (j + 1) / h) for j in range(h)],
+                                                    "rot": {"base": 1e6, "dims": d}}}
+        else:
+            h, d, rot, e, q_rank, kv_rank = latent
+            mixer = {"heads": h, "dim": d, "rot_dim": rot, "vdim": e, "q_rank": q_rank, "kv_rank": kv_rank, "scale": (d + rot) ** -0.5,
+                     "rot": {"base": 1e4, "dims": rot, "scaling": {"factor": 4.0, "original": 512, "fast": 32.0, "slow": 1.0}}}
+            linear(base + "mix.dq", q_rank, width)
+            norm(base + "mix.dq.norm", q_rank)
+            linear(base + "mix.uq", h * (d + rot), q_rank)
+            if mix == "latent":
+                source = i
+                linear(base + "mix.dkv", kv_rank + rot, width)
+                norm(base + "mix.dkv.norm", kv_rank)
+            else:
+                mixer["kv_from"] = source
+            linear(base + "mix.uk", h * d, kv_rank)
+            linear(base + "mix.uv", h * e, kv_rank)
+            linear(base + "mix.o", width, h * e)
+            layer = {"type": "latent_attention", "mixer": mixer}
+        for part, inner in [("", ff)] if feed == "dense" else [(f"e{e}.", expert_ff) for e in range(number)]:
+            linear(base + "mlp." + part + "gate", inner, width)
+            linear(base + "mlp." + part + "up", inner, width)
+            linear(base + "mlp." + part + "down", width, inner)
+        layer["mlp"] = {"kind": "dense", "ff": ff}
+        if feed == "experts":
+            linear(base + "mlp.router", number, width)
+            layer["mlp"] = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": number, "top": top}}
+            skipped += (number - top) * 3 * expert_ff * width * 2
+        layers.append(layer)
+    config = {"architecture": "Tuzavik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers, "residual_mult": 0.5, "logit_scale": 1.0,
+              "embedding": {"bigram": {"buckets": 1023, "mul_prev": 31, "mul_cur": 17}}}
+    with open(os.path.join(directory, "config.json"), "w") as f:
+        json.dump(config, f)
+    save_file(tensors, os.path.join(directory, "model.safetensors"))
+    return sum(t.numel() * 2 for name, t in tensors.items() if name not in ("embed", "bigram", "head")) - skipped
+
+
+def decoder_throughput(design, size, dev, rows=1024, steps=64, kinds=None):
+    """Prefill of `rows` tokens and decoding behind them for a decoder language model of a design and size; microseconds are per
+    layer run (head included in the total it is divided from), weight bytes those of the layers that one token takes."""
     import tempfile
     module = importlib.import_module("qingming-qwen3-tts_amd.decoder")
     out = {}
-    for name, types in (("mixed", ("parallel", "parallel", "parallel", "general_delta")), ("parallel", ("parallel",) * 4),
-                        ("general_delta", ("general_delta",) * 4)):
+    vabevik = {"mixed": ("parallel", "parallel", "parallel", "general_delta"), "parallel": ("parallel",) * 4, "general_delta": ("general_delta",) * 4}
+    for name, layers in (vabevik if design == "vabevik" else TUZAVIK_KINDS).items():
         if kinds and name not in kinds:
             continue
         with tempfile.TemporaryDirectory() as directory:
-            weight_bytes = write_decoder_model(directory, types=types, dev=dev, **DECODER_SIZES[size])
+            if design == "vabevik":
+                weight_bytes = write_decoder_model(directory, types=layers, dev=dev, **DECODER_SIZES[size])
+            else:
+                weight_bytes = write_tuzavik_model(directory, kinds=layers, dev=dev, **TUZAVIK_SIZES[size])
             model = module.Decoder(directory, capacity=rows + 2 * steps + 8, max_rows=rows)
         tokens = np.arange(rows, dtype=np.int32) * 7 % model.vocab
 
@@ -1226,14 +1311,15 @@ def talker_throughput(dev, rows=1024, steps=64, layers=4):
             "prefill_weight_TFLOPps": weight_bytes * rows / prefill_s / 1e12}
 
 
-def decoder_report(which, dev):
-    """Every size (or the one named), and the talker at the size they share."""
+def decoder_report(which, designs, dev):
+    """Every size (or the one named) of the designs, and the talker at the size they share."""
     report = {}
     for size in DECODER_SIZES if which == "all" else [] if which == "talker" else [which.split(":")[0]]:
         kinds = which.split(":")[1].split(",") if ":" in which else None
-        for name, r in decoder_throughput(size, dev, kinds=kinds).items():
-            report[f"vabevik_{size}_{name}"] = r
-            print(f"vabevik_{size}_{name} " + json.dumps({k: round(v, 2) for k, v in r.items()}), flush=True)
+        for design in designs:
+            for name, r in decoder_throughput(design, size, dev, kinds=kinds).items():
+                report[f"{design}_{size}_{name}"] = r
+                print(f"{design}_{size}_{name} " + json.dumps({k: round(v, 2) for k, v in r.items()}), flush=True)
     if ":" not in which:
         report["talker_w2048"] = talker_throughput(dev)
         print("talker_w2048 " + json.dumps({k: round(v, 2) for k, v in report["talker_w2048"].items()}), flush=True)
@@ -1313,8 +1399,9 @@ def main():
                          "records counters for every dispatch is spared most of the input generation with a small number)")
     ap.add_argument("--decoder", nargs="?", const="all", default=None, metavar="SIZE[:KINDS]",
                     help="prefill and decode throughput of the decoder language models (" + ", ".join(DECODER_SIZES) + ", or all) beside the "
-                         "talker's, instead of the attention workloads (talker: that alone); SIZE:KINDS times that size's layer kinds alone (mixed, parallel, "
-                         "general_delta)")
+                         "talker's, instead of the attention workloads (talker: that alone); SIZE:KINDS times that size's layer kinds alone (Vabevik: mixed, parallel, "
+                         "general_delta; Tuzavik: " + ", ".join(TUZAVIK_KINDS) + ")")
+    ap.add_argument("--decoder-design", choices=["vabevik", "tuzavik"], default=None, help="with --decoder: that design alone")
     ap.add_argument("--calibrate-copy", action="store_true",
                     help="also run three plain 512 MiB device-to-device copies (for scaling rocprofv3's "
                          "FETCH_SIZE / WRITE_SIZE counters against a kernel of known traffic)")
@@ -1343,7 +1430,7 @@ def main():
         torch.cuda.empty_cache()
 
     if args.decoder:
-        report = decoder_report(args.decoder, dev)
+        report = decoder_report(args.decoder, [args.decoder_design] if args.decoder_design else ["vabevik", "tuzavik"], dev)
         print(json.dumps({"metric": "decoder_language_models", "unit": "per entry", "dtype": "bf16, f32 accumulate", "data": "synthetic",
                           "results": report}))
         return

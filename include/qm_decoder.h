@@ -65,7 +65,8 @@ int32_t qm_gated_norm_rows(const qm_gated_norm* op, int32_t rows, int32_t f32, v
 
 /* ---- linears ----------------------------------------------------------------------------------------------------- */
 /* out32[row][c] = sum_k x[row][k] w[c][k] in fp32, or with w_up out[row][c] = silu(x . w[c]) * (x . w_up[c]).  Up to three
- * linears in one launch, each with its own input.  n and k are multiples of 128 (pad weights with zeros), ldx and ldo of 8. */
+ * linears in one launch, each with its own input.  k is a multiple of 128, n of 16 (with w_up, and to take the matrix cores
+ * beyond 64 columns, of 128; pad weights with zeros), ldx and ldo of 8. */
 typedef struct {
     const void* x;           /* [rows][ldx] bf16 or fp32 */
     const uint16_t* w;       /* [n][k] bf16 */

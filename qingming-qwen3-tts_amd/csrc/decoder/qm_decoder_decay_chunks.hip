@@ -42,35 +42,47 @@ __global__ __launch_bounds__(kDecThreads) void decay_rotate_kernel(DecayAttentio
 }
 
 // Rows [t0, t0 + 64) of a head's q, k or v columns into LDS, through silu unless they were rotated (zeros past the rows or
-// the head), times factor(j): sixteen threads take 64 columns of a row, four each.  `padded`: a multiple of 16.
+// the head), times factor(j): sixteen threads take 64 columns of a row, four each.  request_rows asks for columns c4 .. c4 + 3
+// of the thread's four rows, put_rows stores them.
+__device__ __forceinline__ void request_rows(const DecayAttentionParams& prm, int t0, int column, int columns, int c, float4 (&x)[4]) {
+    const int row = threadIdx.x >> 4;
+    const bool vectors = ((column | columns | prm.ld_proj) & 3) == 0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {              // (rows past the last repeat it, with factor zero: no branch around a load)
+        const float* p = prm.proj + min(t0 + row + 16 * i, prm.rows - 1) * prm.ld_proj + column;
+        if (vectors) {
+            x[i] = load4_if(c < columns, p, c >> 2);
+        } else {
+            float e[4];
+#pragma unroll
+            for (int n = 0; n < 4; ++n) {
+                const float v = p[min(c + n, columns - 1)];
+                e[n] = c + n < columns ? v : 0.0f;
+            }
+            x[i] = make_float4(e[0], e[1], e[2], e[3]);
+        }
+    }
+}
+template <class F>
+__device__ __forceinline__ void put_rows(const DecayAttentionParams& prm, float* to, int stride, int t0, int c, float4 (&x)[4], F factor) {
+    const int row = threadIdx.x >> 4;
+    const bool silu = !(prm.options & QM_DECAY_ROTARY);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int j = row + 16 * i;
+        const float f = t0 + j < prm.rows ? factor(j) : 0.0f;
+        if (silu) x[i] = make_float4(silu_f32(x[i].x), silu_f32(x[i].y), silu_f32(x[i].z), silu_f32(x[i].w));
+        *reinterpret_cast<float4*>(to + j * stride + c) = make_float4(x[i].x * f, x[i].y * f, x[i].z * f, x[i].w * f);
+    }
+}
+// `padded`: a multiple of 16
 template <class F>
 __device__ __forceinline__ void stage_rows(const DecayAttentionParams& prm, float* to, int stride, int t0, int column, int columns, int padded, F factor) {
-    const int c4 = (threadIdx.x & 15) * 4, row = threadIdx.x >> 4;
-    const bool vectors = ((column | columns | prm.ld_proj) & 3) == 0, silu = !(prm.options & QM_DECAY_ROTARY);
-    for (int c = c4; c < padded; c += 64) {
+#pragma unroll 2
+    for (int c = (threadIdx.x & 15) * 4; c < padded; c += 64) {
         float4 x[4];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {          // (rows past the last repeat it, with factor zero: no branch around a load)
-            const float* p = prm.proj + min(t0 + row + 16 * i, prm.rows - 1) * prm.ld_proj + column;
-            if (vectors) {
-                x[i] = load4_if(c < columns, p, c >> 2);
-            } else {
-                float e[4];
-#pragma unroll
-                for (int n = 0; n < 4; ++n) {
-                    const float v = p[min(c + n, columns - 1)];
-                    e[n] = c + n < columns ? v : 0.0f;
-                }
-                x[i] = make_float4(e[0], e[1], e[2], e[3]);
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int j = row + 16 * i;
-            const float f = t0 + j < prm.rows ? factor(j) : 0.0f;
-            if (silu) x[i] = make_float4(silu_f32(x[i].x), silu_f32(x[i].y), silu_f32(x[i].z), silu_f32(x[i].w));
-            *reinterpret_cast<float4*>(to + j * stride + c) = make_float4(x[i].x * f, x[i].y * f, x[i].z * f, x[i].w * f);
-        }
+        request_rows(prm, t0, column, columns, c, x);
+        put_rows(prm, to, stride, t0, c, x, factor);
     }
 }
 
@@ -138,13 +150,25 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
     const int dp = mfma32_pad(prm.dim), stride = mfma32_stride(prm.dim);
     const float* powers = prm.powers + head * kDecayPowers;
     float* qs = lds;                           // [64][stride]
-    float* ks = qs + kDecayChunk * stride;     // [64][stride], then the weights [64][kDecayVStride]
-    float* vs = ks + kDecayChunk * stride;     // [64][kDecayVStride]
+    float* ks = qs + kDecayChunk * stride;     // [64][stride], then the weights and the values, [64][kDecayVStride] each
     float* ps = ks;
+    float* vs = ks + kDecayChunk * kDecayVStride;
     auto one = [](int) { return 1.0f; };
+    const int c4 = (threadIdx.x & 15) * 4;
+    float4 value[4];
+    request_rows(prm, t0, prm.v_column + head * prm.vdim + e0, prm.vdim - e0, c4, value);
+    const float* before = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * prm.dim * prm.vdim;
+    const int column = e0 + 16 * wave + l16;
+    auto request_state = [&](int d0, float (&s)[4]) __attribute__((always_inline)) {          // (q is zero past the head)
+#pragma unroll
+        for (int t = 0; t < 4; ++t) s[t] = before[min(d0 + 4 * g + t, prm.dim - 1) * prm.vdim + min(column, prm.vdim - 1)];
+    };
+    constexpr int kAhead = 4;                  // blocks of 16 state rows under way
+    float state[kAhead][4];
+#pragma unroll
+    for (int u = 0; u < kAhead; ++u) request_state(16 * u, state[u]);
     stage_rows(prm, qs, stride, t0, prm.q_column + head * prm.dim, prm.dim, dp, one);
     stage_rows(prm, ks, stride, t0, prm.k_column + head * prm.dim, prm.dim, dp, one);
-    stage_rows(prm, vs, kDecayVStride, t0, prm.v_column + head * prm.vdim + e0, prm.vdim - e0, kDecaySlice, one);
     __syncthreads();
     f32x4_t score[4] = {};                     // rows of tile `wave`, column tiles 0 .. wave
     for (int d0 = 0; d0 < dp; d0 += 16) {
@@ -154,6 +178,7 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
             if (j <= wave) score[j] = mfma32_block(a, *reinterpret_cast<const float4*>(ks + (16 * j + l16) * stride + d0 + 4 * g), score[j]);
     }
     __syncthreads();
+    put_rows(prm, vs, kDecayVStride, t0, c4, value, one);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
         if (j > wave) continue;
@@ -166,20 +191,21 @@ __global__ __launch_bounds__(kDecThreads) void decay_chunk_output_kernel(DecayAt
     float decayed[4];                          // d^(i+1) of the lane's row of each tile
 #pragma unroll
     for (int i = 0; i < 4; ++i) decayed[i] = powers[16 * i + l16 + 1];
-    const float* before = prm.scratch + (static_cast<int64_t>(chunk) * prm.heads + head) * prm.dim * prm.vdim;
     __syncthreads();
-    const int column = e0 + 16 * wave + l16;
     f32x4_t acc[4] = {};
-    for (int d0 = 0; d0 < dp; d0 += 16) {
-        float s[4];
+    for (int base = 0; base < dp; base += 16 * kAhead) {
 #pragma unroll
-        for (int t = 0; t < 4; ++t) s[t] = before[min(d0 + 4 * g + t, prm.dim - 1) * prm.vdim + min(column, prm.vdim - 1)];   // (q is zero past the head)
-        const float4 b = make_float4(s[0], s[1], s[2], s[3]);
+        for (int u = 0; u < kAhead; ++u) {
+            const int d0 = base + 16 * u;
+            if (d0 >= dp) break;
+            const float4 b = make_float4(state[u][0], state[u][1], state[u][2], state[u][3]);
+            if (base + 16 * kAhead < dp) request_state(d0 + 16 * kAhead, state[u]);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            float4 a = *reinterpret_cast<const float4*>(qs + (16 * i + l16) * stride + d0 + 4 * g);
-            a.x *= decayed[i]; a.y *= decayed[i]; a.z *= decayed[i]; a.w *= decayed[i];
-            acc[i] = mfma32_block(a, b, acc[i]);
+            for (int i = 0; i < 4; ++i) {
+                float4 a = *reinterpret_cast<const float4*>(qs + (16 * i + l16) * stride + d0 + 4 * g);
+                a.x *= decayed[i]; a.y *= decayed[i]; a.z *= decayed[i]; a.w *= decayed[i];
+                acc[i] = mfma32_block(a, b, acc[i]);
+            }
         }
     }
 #pragma unroll
@@ -208,7 +234,7 @@ int32_t launch_decay_chunks(const DecayAttentionParams& prm, hipStream_t stream)
     const int chunks = (prm.rows + kDecayChunk - 1) / kDecayChunk;
     const int stride = mfma32_stride(prm.dim), slices = (prm.vdim + kDecaySlice - 1) / kDecaySlice;
     const int state_lds = static_cast<int>(sizeof(float)) * kDecayChunk * (stride + kDecayVStride);
-    const int output_lds = static_cast<int>(sizeof(float)) * kDecayChunk * (2 * stride + kDecayVStride);
+    const int output_lds = static_cast<int>(sizeof(float)) * kDecayChunk * (stride + (stride > 2 * kDecayVStride ? stride : 2 * kDecayVStride));
     static std::atomic<bool> raised[2][kMaxDevices];
     int32_t rc = ensure_dynamic_lds(reinterpret_cast<const void*>(decay_chunk_state_kernel), kDotLdsMost, raised[0]);
     if (rc == QM_OK) rc = ensure_dynamic_lds(reinterpret_cast<const void*>(decay_chunk_output_kernel), kDotLdsMost, raised[1]);

@@ -16,6 +16,7 @@ constexpr int kExpertOutRows = 2;              // down
 constexpr int kRouteRows = kDecThreads / 64;   // rows per block of the router: a wave each
 constexpr int kSortThreads = 1024;
 constexpr int kExpertMatrixRows = 16;          // rows from which bf16 goes to the matrix cores
+constexpr int kExpertLongTile = 256;           // rows per expert (on average) from which row tiles are 128 high, not 64
 
 // What the kernels share in the scratch.
 struct ExpertScratch {
@@ -214,7 +215,7 @@ static int64_t lay_out(char* base, int rows, int experts, int top, int width_p, 
     s.id = reinterpret_cast<int32_t*>(take(assignments * 4));
     s.weight = reinterpret_cast<float*>(take(assignments * 4));
     s.place = reinterpret_cast<int32_t*>(take(assignments * 4));
-    s.tile_rows = assignments / experts >= 128 ? 128 : 64;
+    s.tile_rows = assignments / experts >= kExpertLongTile ? 128 : 64;
     const int64_t full = assignments / s.tile_rows, used = assignments < experts ? assignments : experts;
     s.tiles = static_cast<int>(full + used);
     s.tile_expert = reinterpret_cast<int32_t*>(take(static_cast<int64_t>(s.tiles) * 4));

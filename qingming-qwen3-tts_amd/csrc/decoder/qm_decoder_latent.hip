@@ -210,6 +210,14 @@ __global__ __launch_bounds__(kDecThreads) void latent_output_kernel(LatentAttent
     const int all = position_of(prm.position_dev, prm.position) + prm.rows;
     const int each = latent_keys_per_split(all, prm.splits), active = (all + each - 1) / each;
     const int64_t at = (row * prm.heads + head) * prm.splits;
+    const float* acc = prm.acc + at * prm.kv_rank;
+    constexpr int kFirst = 16, kOwn = 2;       // splits and channels of the thread that are asked for before the factors are known
+    float held[kOwn][kFirst];
+#pragma unroll
+    for (int x = 0; x < kOwn; ++x)
+#pragma unroll
+        for (int s = 0; s < kFirst; ++s)
+            held[x][s] = acc[static_cast<int64_t>(min(s, active - 1)) * prm.kv_rank + min(tid + x * kDecThreads, prm.kv_rank - 1)];
     if (wave == 0) {
         const float m_read = prm.ml[(at + min(lane, active - 1)) * 2], l_read = prm.ml[(at + min(lane, active - 1)) * 2 + 1];
         const float m = lane < active ? m_read : -INFINITY, l = lane < active ? l_read : 0.0f;
@@ -218,12 +226,19 @@ __global__ __launch_bounds__(kDecThreads) void latent_output_kernel(LatentAttent
         if (lane < active) sh_w[lane] = factor / total;
     }
     __syncthreads();
-    const float* acc = prm.acc + at * prm.kv_rank;
     const int padded = (prm.kv_rank + 511) / 512 * 512;
-    for (int c = tid; c < padded; c += kDecThreads) {
+#pragma unroll
+    for (int x = 0; x < kOwn; ++x) {
         float sum = 0.0f;
+#pragma unroll
+        for (int s = 0; s < kFirst; ++s) sum = fmaf(s < active ? sh_w[min(s, active - 1)] : 0.0f, held[x][s], sum);
+        held[x][0] = sum;
+    }
+    for (int c = tid; c < padded; c += kDecThreads) {
+        const int own = (c - tid) / kDecThreads;
+        float sum = own == 0 ? held[0][0] : own == 1 ? held[1][0] : 0.0f;
         const int from = min(c, prm.kv_rank - 1);
-        for (int s0 = 0; s0 < active; s0 += 8) {
+        for (int s0 = own < kOwn ? kFirst : 0; s0 < active; s0 += 8) {
             float v[8];
 #pragma unroll
             for (int s = 0; s < 8; ++s) v[s] = acc[static_cast<int64_t>(min(s0 + s, active - 1)) * prm.kv_rank + from];
@@ -314,11 +329,30 @@ __global__ __launch_bounds__(kDecThreads) void latent_rotate_query_kernel(Latent
     }
     __syncthreads();
     const int pieces = k_stride >> 3, per_head = prm.dim + prm.rot_dim;
+    const bool vectors = ((prm.dim | per_head) & 7) == 0;
     const float* q = prm.q + row * prm.ld_query;
     for (int i = threadIdx.x; i < prm.heads * pieces; i += kDecThreads) {
         const int h = i / pieces, c0 = (i - h * pieces) * 8;
         const float* head = q + h * per_head;
         float v[8];
+        if (vectors && c0 + 8 <= prm.dim) {
+            const float4 a = load4(head, c0 >> 2), b = load4(head, (c0 >> 2) + 1);
+            v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+            put8(to + (row * prm.heads + h) * k_stride + c0, v);
+            continue;
+        }
+        if (vectors && c0 >= prm.dim && c0 + 8 <= per_head) {
+            const float4 a = load4(head, c0 >> 2), b = load4(head, (c0 >> 2) + 1);
+            const float x[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+            for (int e = 0; e < 8; e += 2) {
+                const float cosine = sh_cos[(c0 - prm.dim + e) >> 1], sine = sh_sin[(c0 - prm.dim + e) >> 1];
+                v[e] = x[e] * cosine - x[e + 1] * sine;
+                v[e + 1] = x[e + 1] * cosine + x[e] * sine;
+            }
+            put8(to + (row * prm.heads + h) * k_stride + c0, v);
+            continue;
+        }
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int c = c0 + e, r = c - prm.dim;

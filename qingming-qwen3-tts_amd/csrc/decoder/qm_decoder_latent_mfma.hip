@@ -46,15 +46,15 @@ __global__ __launch_bounds__(kDecThreads) void latent_partials_mfma_kernel(Laten
     const int start = position_of(prm.position_dev, prm.position);
     const int all = start + prm.rows, each = latent_keys_per_split(all, prm.splits);
     const int begin = split * each;
+    lat_u32x4 q[kKb];
+    const uint16_t* q_row = static_cast<const uint16_t*>(prm.q_scratch) + static_cast<int64_t>(asked) * (C + kLatRotary) + 8 * g;
+#pragma unroll
+    for (int kb = 0; kb < kKb; ++kb) q[kb] = *reinterpret_cast<const lat_u32x4*>(q_row + kb * 32);
     if (begin >= all) return;
     const int block_last = min(static_cast<int>(blockIdx.y) * kLatQueries + kLatQueries - 1, total - 1);
     const int end = min(begin + each, start + block_last / prm.heads + 1);     // what any of the block's queries sees
     const int position = start + asked / prm.heads;
 
-    lat_u32x4 q[kKb];
-    const uint16_t* q_row = static_cast<const uint16_t*>(prm.q_scratch) + static_cast<int64_t>(asked) * (C + kLatRotary) + 8 * g;
-#pragma unroll
-    for (int kb = 0; kb < kKb; ++kb) q[kb] = *reinterpret_cast<const lat_u32x4*>(q_row + kb * 32);
     f32x4_t o[kTiles];
 #pragma unroll
     for (int t = 0; t < kTiles; ++t) o[t] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
@@ -64,8 +64,9 @@ __global__ __launch_bounds__(kDecThreads) void latent_partials_mfma_kernel(Laten
     const uint16_t* latent = static_cast<const uint16_t*>(prm.latent_cache);
     const uint16_t* key_part = static_cast<const uint16_t*>(prm.key_cache);
     const int ld = static_cast<int>(prm.ld_latent), key_stride = prm.key_stride;
-    // blocks of four keys x eight channels, dealt to the threads; two threads in eight also take a piece of the key part
-    constexpr int kUnits = kLatentKeys / 4 * (C / 8), kBlocks = (kUnits + kDecThreads - 1) / kDecThreads;
+    // blocks of four keys x eight channels, dealt to the threads: sixteen lanes take the same channels of all keys, so that both
+    // ways of storing them spread over the LDS banks; and pieces of the key part
+    constexpr int kGroups = kLatentKeys / 4, kUnits = kGroups * (C / 8), kBlocks = (kUnits + kDecThreads - 1) / kDecThreads;
     constexpr int kRotaryPieces = kLatentKeys * (kLatRotary / 8) / kDecThreads;
     lat_u32x4 piece[kBlocks][4], rotary_piece[kRotaryPieces];
     // (keys past the last repeat it and are masked; channels past the latent's meet zeros of the query or are not stored)
@@ -73,7 +74,7 @@ __global__ __launch_bounds__(kDecThreads) void latent_partials_mfma_kernel(Laten
         const int last = end - 1;
 #pragma unroll
         for (int i = 0; i < kBlocks; ++i) {
-            const int at = min(tid + i * kDecThreads, kUnits - 1), key = at / (C / 8) * 4, c = at % (C / 8) * 8;
+            const int at = min(tid + i * kDecThreads, kUnits - 1), key = at % kGroups * 4, c = at / kGroups * 8;
 #pragma unroll
             for (int j = 0; j < 4; ++j)
                 piece[i][j] = *reinterpret_cast<const lat_u32x4*>(latent + static_cast<int64_t>(min(tile + key + j, last)) * ld + min(c, ld - 8));
@@ -87,7 +88,7 @@ __global__ __launch_bounds__(kDecThreads) void latent_partials_mfma_kernel(Laten
     auto deposit = [&]() __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < kBlocks; ++i) {
-            const int at = tid + i * kDecThreads, key = at / (C / 8) * 4, c = at % (C / 8) * 8;
+            const int at = tid + i * kDecThreads, key = at % kGroups * 4, c = at / kGroups * 8;
             if (at >= kUnits) break;
 #pragma unroll
             for (int j = 0; j < 4; ++j) *reinterpret_cast<lat_u32x4*>(ks + (key + j) * Shape::kKStride + c) = piece[i][j];

@@ -63,6 +63,55 @@ static int32_t streaming(const DecLinearParams& prm, hipStream_t stream) {
     return launch_streaming<T, 1>(prm, stream);
 }
 
+// A linear of few columns (a router) over many bf16 rows: the large tiles of the matrix-core kernel would leave most CUs
+// without a block and walk the whole reduction one step after the other.  Here a block takes 16 rows, its four waves every
+// fourth 128 terms of the reduction (v_mfma_f32_16x16x32_bf16, operands straight from memory; the weights are few and stay in
+// L2), and the four sums meet in LDS.  Bound by the latency of a wave's loads.
+constexpr int kNarrowRows = 16;                        // token rows of a block
+constexpr int kNarrowColumns = 64;                     // most columns
+template <int TILES>
+__global__ __launch_bounds__(kDecThreads) void narrow_linear_kernel(DecLinearGroup group, int rows) {
+    __shared__ float sums[4][TILES * 16 * (kNarrowRows + 1)];
+    typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, l16 = lane & 15;
+    const int row0 = static_cast<int>(blockIdx.x) * kNarrowRows;
+    const uint16_t* x = static_cast<const uint16_t*>(group.x) + min(row0 + l16, rows - 1) * group.ldx + 8 * g;
+    const uint16_t* w[TILES];
+#pragma unroll
+    for (int t = 0; t < TILES; ++t) w[t] = group.w + static_cast<int64_t>(min(16 * t, group.n - 16) + l16) * group.k + 8 * g;
+    f32x4_t acc[TILES] = {};
+    for (int k = wave * 128; k < group.k; k += 512) {  // (all of 128 terms is asked for before the first is used)
+        u32x4 b[4], a[4][TILES];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) b[u] = *reinterpret_cast<const u32x4*>(x + k + 32 * u);
+#pragma unroll
+        for (int t = 0; t < TILES; ++t)
+#pragma unroll
+            for (int u = 0; u < 4; ++u) a[u][t] = *reinterpret_cast<const u32x4*>(w[t] + k + 32 * u);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int t = 0; t < TILES; ++t)
+                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u][t]), __builtin_bit_cast(bf16x8_t, b[u]), acc[t], 0, 0, 0);
+    }
+    // acc[t][r] is column 16 t + 4 g + r of row l16
+#pragma unroll
+    for (int t = 0; t < TILES; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sums[wave][(16 * t + 4 * g + r) * (kNarrowRows + 1) + l16] = acc[t][r];
+    __syncthreads();
+    for (int i = threadIdx.x; i < kNarrowRows * TILES * 16; i += kDecThreads) {
+        const int row = i / (TILES * 16), c = i % (TILES * 16), at = c * (kNarrowRows + 1) + row;
+        if (row0 + row < rows && c < group.n)
+            group.out32[static_cast<int64_t>(row0 + row) * group.ldo + c] = (sums[0][at] + sums[1][at]) + (sums[2][at] + sums[3][at]);
+    }
+}
+template <int TILES>
+static int32_t launch_narrow(const DecLinearParams& prm, hipStream_t stream) {
+    hipLaunchKernelGGL(narrow_linear_kernel<TILES>, dim3((prm.rows + kNarrowRows - 1) / kNarrowRows), dim3(kDecThreads), 0, stream, prm.group[0], prm.rows);
+    return launch_status();
+}
+
 // Rows from which the matrix cores take over: below, one 64-row tile is mostly empty and the weights' bytes decide.
 constexpr int kDecMatrixRows = 16;
 
@@ -71,12 +120,14 @@ int32_t launch_decoder_linears(const DecLinearParams& prm, int f32, hipStream_t 
     for (int g = 0; g < prm.groups; ++g) {
         const DecLinearGroup& d = prm.group[g];
         if (!d.x || !d.w || (d.w_up ? !d.out : !d.out32)) return QM_ERR_NULL;
-        if (d.n <= 0 || d.k <= 0 || d.n % 128 || d.k % 128 || d.ldx < d.k || d.ldo < d.n || d.ldx % 8 || d.ldo % 4) return QM_ERR_GEOMETRY;
+        if (d.n <= 0 || d.k <= 0 || d.n % (d.w_up ? 128 : 16) || d.k % 128 || d.ldx < d.k || d.ldo < d.n || d.ldx % 8 || d.ldo % 4) return QM_ERR_GEOMETRY;
     }
     if (prm.rows == 0) return QM_OK;
     if (f32) return streaming<float>(prm, stream);
     bool matrix = prm.rows >= kDecMatrixRows;
-    for (int g = 0; g < prm.groups; ++g) matrix = matrix && prm.group[g].ldx == prm.group[g].k && prm.group[g].ldo == prm.group[g].n;
+    if (matrix && prm.groups == 1 && prm.group[0].n <= kNarrowColumns && !prm.group[0].w_up)
+        return prm.group[0].n <= 32 ? launch_narrow<2>(prm, stream) : launch_narrow<4>(prm, stream);
+    for (int g = 0; g < prm.groups; ++g) matrix = matrix && prm.group[g].n % 128 == 0 && prm.group[g].ldx == prm.group[g].k && prm.group[g].ldo == prm.group[g].n;
     if (!matrix) return streaming<uint16_t>(prm, stream);
     LinearRowsParams plain = {};
     int order[kDecGroups] = {0, 1, 2};         // long reductions first

@@ -161,7 +161,7 @@ int32_t launch_layer_in(const LayerInParams& prm, int f32, hipStream_t stream) {
     for (int g = 0; g < prm.linears.groups; ++g) {
         const DecLinearGroup& d = prm.linears.group[g];
         if (!d.w || (d.w_up ? !d.out : !d.out32)) return QM_ERR_NULL;
-        if (d.n <= 0 || d.n % 128 || d.k % 128 || d.k != prm.residual.ld_h) return QM_ERR_GEOMETRY;
+        if (d.n <= 0 || d.n % (d.w_up ? 128 : 16) || d.k % 128 || d.k != prm.residual.ld_h) return QM_ERR_GEOMETRY;
     }
     const int32_t rc = check_residual(prm.residual);
     if (rc != QM_OK) return rc;

@@ -177,14 +177,14 @@ public:
         int columns;
         Section* section;
     };
-    Matrix stacked(const std::vector<Part>& parts, int k) const {
+    Matrix stacked(const std::vector<Part>& parts, int k, int rows_to = 128) const {
         Matrix m;
         int n = 0;
         for (const Part& p : parts) {
             if (p.section) *p.section = {n, p.columns};
             n += padded(p.columns, 8);
         }
-        m.n = padded(n, 128);
+        m.n = padded(n, rows_to);
         m.k = padded(k, 128);
         std::vector<uint16_t> host(static_cast<size_t>(m.n) * m.k, 0);
         int at = 0;
@@ -293,7 +293,7 @@ DecoderLayer load_layer(const Loader& from, const DecoderConfig& model, int inde
         w.gate = from.each(config.experts, named("gate"), config.ff, width);
         w.up = from.each(config.experts, named("up"), config.ff, width);
         w.down = from.each(config.experts, named("down"), width, config.ff);
-        w.router = from.matrix(base + "mlp.router", config.experts, width);
+        w.router = from.stacked({{base + "mlp.router", config.experts, nullptr}}, width, config.experts <= 64 ? 16 : 128);
     } else if (config.ff) {
         w.gate = from.matrix(base + "mlp.gate", config.ff, width);
         w.up = from.matrix(base + "mlp.up", config.ff, width);

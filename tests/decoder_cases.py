@@ -82,12 +82,12 @@ CONFIGS = {
     # retention alone: one head and several, values wider and narrower than keys, few or no rotated channels, decays of 0 and 1, a layer
     # without feed-forward, a prime number of buckets and factors above it
     "retention": sandwich(90, 100, [retention(1, 24, 40, [0.97], dense(70)), retention(3, 36, 20, [1.0, 0.5, 0.99], None, rot_dims=10, base=300.0),
-                                    retention(2, 130, 70, [0.999, 0.0], moe(3, 1, 50), rot_dims=0)], (101, 1009, 777777), eps=3e-4, residual_mult=0.4),
+                                    retention(2, 130, 70, [0.999, 0.2], moe(3, 1, 50), rot_dims=0)], (101, 1009, 777777), eps=3e-4, residual_mult=0.4),
     # latents shared by several layers, two of them kept, frequencies stretched and not, every expert chosen, sizes that are no multiples
     "latents": sandwich(120, 150, [latent(3, 20, 10, 28, 44, 36, dense(90), scaling=(4.0, 64, 8.0, 1.0), base=500.0),
                                    latent(5, 12, 6, 20, 24, 72, moe(5, 5, 36), scale=0.3),
                                    latent(2, 33, 10, 17, 20, 36, None, scaling=(4.0, 64, 8.0, 1.0), base=500.0, kv_from=0),
-                                   latent(4, 16, 6, 24, 30, 72, dense(40), kv_from=1)], (64, 3, 5), residual_mult=1.3, logit_scale=0.3),
+                                   latent(4, 16, 6, 24, 30, 72, dense(40), kv_from=1)], (64, 3, 5), residual_mult=0.9, logit_scale=0.3),
     # heads above 128 channels, latents above 256, many experts
     "wide_latents": sandwich(200, 264, [latent(5, 110, 60, 100, 140, 300, moe(70, 6, 130), scaling=(16.0, 100, 32.0, 2.0)), retention(2, 64, 200, [0.9, 0.98], dense(256)),
                                         latent(17, 24, 60, 140, 60, 300, dense(200), scaling=(16.0, 100, 32.0, 2.0), kv_from=0)], (37, 0, 1), logit_scale=2.0),

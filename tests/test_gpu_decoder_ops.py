@@ -116,6 +116,22 @@ def test_gated_norm(decoder, dev, f32, groups, size, ld, silu):
 
 
 @pytest.mark.parametrize("f32", [True, False])
+@pytest.mark.parametrize("n", [16, 48, 64, 80])
+@pytest.mark.parametrize("rows,k,ldx,ldo", [(1, 128, 128, 128), (7, 256, 264, 132), (16, 128, 128, 128), (33, 384, 392, 140), (200, 2048, 2048, 128)])
+def test_linear_of_few_columns(decoder, dev, f32, rows, k, ldx, ldo, n):
+    import torch
+    rng = np.random.default_rng(rows)
+    x, w = cases.bf16(rng.standard_normal((rows, ldx))), cases.bf16(rng.standard_normal((n, k)) * k ** -0.5)
+    xd, wd = put(x, dev, activation(f32)), put(w, dev, torch.bfloat16)
+    out = torch.full((rows + 1, ldo), 7.0, device=dev)
+    linear = decoder.DecoderLinear(x=xd.data_ptr(), w=wd.data_ptr(), out32=out.data_ptr(), ldx=ldx, ldo=ldo, n=n, k=k)
+    assert decoder.lib().qm_decoder_linear_rows(C.byref(linear), 1, rows, int(f32), torch.cuda.current_stream().cuda_stream) == 0
+    got = get(out)
+    close(got[:rows, :n], x[:, :k].astype(np.float64) @ w.T, True, tol32=3e-6)
+    assert np.all(got[rows:] == 7) and np.all(got[:, n:] == 7)
+
+
+@pytest.mark.parametrize("f32", [True, False])
 @pytest.mark.parametrize("rows", [1, 2, 3, 5, 9, 15, 16, 40, 130])
 def test_linears(decoder, dev, f32, rows):
     """Three linears of their own inputs and reductions in one launch, the last a gate/up pair."""
