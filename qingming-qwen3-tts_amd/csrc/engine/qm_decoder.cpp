@@ -305,9 +305,8 @@ DecoderLayer load_layer(const Loader& from, const DecoderConfig& model, int inde
 int ring_of(const qm_decoder& d, const ChunkAttentionConfig& a) { return std::min<int64_t>(d.capacity, static_cast<int64_t>(a.chunk) + d.max_rows); }
 int chunk_of(const qm_decoder& d, const ChunkAttentionConfig& a) { return std::min(a.chunk, d.capacity); }
 
-// Key splits of one token's attention over latents: passes of 64 keys, at most 32 splits (their sums are combined by every
-// block behind them).
-int latent_splits(int capacity) { return std::clamp((capacity + 63) / 64, 1, 32); }
+// Key splits of one token's attention over latents: passes of 64 keys, as many splits as there may be.
+int latent_splits(int capacity) { return std::clamp((capacity + qm::kLatentKeys - 1) / qm::kLatentKeys, 1, qm::kDecMaxSplits); }
 
 // A chunk's keys in at most 16 splits of whole passes of 128 keys.
 int keys_per_split(int chunk) { return padded(std::max(128, (chunk + 15) / 16), 128); }
