@@ -1176,7 +1176,7 @@ def write_tuzavik_model(directory, width, retention, latent, ff, experts, kinds,
         else:
             h, d, rot, e, q_rank, kv_rank = latent
             mixer = {"heads": h, "dim": d, "rot_dim": rot, "vdim": e, "q_rank": q_rank, "kv_rank": kv_rank, "scale": (d + rot) ** -0.5,
-                     "rot": {"base": 1e4, "dims": rot, "scaling": {"factor": 4.0, "original": 512, "fast": 32.0, "slow": 1.0}}}
+                     "rot": {"base": 1e4, "dims": rot, "scaling": {"factor": 4.0, "original": 256, "fast": 24.0, "slow": 2.0}}}
             linear(base + "mix.dq", q_rank, width)
             norm(base + "mix.dq.norm", q_rank)
             linear(base + "mix.uq", h * (d + rot), q_rank)
@@ -1201,7 +1201,7 @@ def write_tuzavik_model(directory, width, retention, latent, ff, experts, kinds,
             skipped += (number - top) * 3 * expert_ff * width * 2
         layers.append(layer)
     config = {"architecture": "Tuzavik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers, "residual_mult": 0.5, "logit_scale": 1.0,
-              "embedding": {"bigram": {"buckets": 1023, "mul_prev": 31, "mul_cur": 17}}}
+              "embedding": {"bigram": {"buckets": 1023, "mul_prev": 29, "mul_cur": 13}}}
     with open(os.path.join(directory, "config.json"), "w") as f:
         json.dump(config, f)
     save_file(tensors, os.path.join(directory, "model.safetensors"))

@@ -155,12 +155,12 @@ def test_operators_check_their_arguments(decoder):
     for change in (dict(rot_dims=18), dict(rot_dims=3, frequency=at), dict(rot_dims=8), dict(position=-1)):
         assert lib.qm_decay_attention_rows(C.byref(decoder.DecayAttention(**{**decay, "options": decoder.DECAY_ROTARY, **change})), None) < 0, change
     rows = dict(proj=at, q_norm=at, kv_norm=at, frequency=at, q_latent=at, latent_cache=at, key_cache=at, ld_proj=200, ld_q=128, ld_latent=128, rows=0,
-                q_rank=40, kv_rank=64, rot_dim=16, key_stride=16)
+                q_rank=40, kv_rank=72, rot_dim=16, key_stride=16)
     assert lib.qm_latent_rows_norm(C.byref(decoder.LatentRows(**rows)), 0, None) == 0
     for change in (dict(kv_rank=129), dict(kv_rank=0), dict(rot_dim=15), dict(key_stride=8), dict(ld_q=30), dict(position=-1), dict(key_cache=None)):
         assert lib.qm_latent_rows_norm(C.byref(decoder.LatentRows(**{**rows, **change})), 0, None) < 0, change
     latent = dict(q=at, frequency=at, up_k=at, up_v=at, latent_cache=at, key_cache=at, out=at, q_scratch=at, ml=at, acc=at, ld_query=200, ld_latent=128,
-                  ld_out=128, rows=0, heads=4, dim=32, rot_dim=16, vdim=32, kv_rank=64, key_stride=16, splits=4)
+                  ld_out=128, rows=0, heads=3, dim=40, rot_dim=16, vdim=36, kv_rank=72, key_stride=16, splits=4)
     assert lib.qm_latent_attention_rows(C.byref(decoder.LatentAttention(**latent)), 0, None) == 0
     for change in (dict(heads=0), dict(kv_rank=2000), dict(ld_latent=60), dict(ld_query=100), dict(ld_out=100), dict(splits=65), dict(splits=0),
                    dict(key_stride=8), dict(rot_dim=3), dict(position=-1), dict(acc=None)):
@@ -241,14 +241,14 @@ def test_neighbours_turn_together():
 
 
 def test_stretched_frequencies():
-    f, magnitude = plain.yarn(16, 10000.0, dict(factor=8.0, original=512, fast=32.0, slow=1.0))
+    f, magnitude = plain.yarn(16, 10000.0, dict(factor=6.0, original=300, fast=20.0, slow=1.0))
     unstretched, one = plain.yarn(16, 10000.0, None)
-    assert one == 1 and np.isclose(magnitude, 0.1 * np.log(8) + 1)
+    assert one == 1 and np.isclose(magnitude, 0.1 * np.log(6) + 1)
     # pairs that turn often keep their frequency, those that turn less than once are stretched whole
-    turns = 512 * unstretched / (2 * np.pi)
-    assert np.allclose(f[turns > 32], unstretched[turns > 32]) and np.allclose(f[-1], unstretched[-1] / 8)
-    assert np.all(f <= unstretched + 1e-15) and np.all(f >= unstretched / 8 - 1e-15)
-    f, magnitude = plain.yarn(16, 10000.0, dict(factor=1.0, original=512, fast=32.0, slow=1.0))
+    turns = 300 * unstretched / (2 * np.pi)
+    assert np.allclose(f[turns > 20], unstretched[turns > 20]) and np.allclose(f[-1], unstretched[-1] / 6)
+    assert np.all(f <= unstretched + 1e-15) and np.all(f >= unstretched / 6 - 1e-15)
+    f, magnitude = plain.yarn(16, 10000.0, dict(factor=1.0, original=300, fast=20.0, slow=1.0))
     assert np.allclose(f, unstretched) and magnitude == 1
 
 

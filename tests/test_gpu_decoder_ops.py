@@ -360,7 +360,7 @@ def test_retention(decoder, dev, chunked, heads, dim, vdim, rot_dims):
 
 LATENT = [
     # heads, dim, rot_dim, vdim, kv_rank, scaling
-    (3, 16, 8, 24, 40, None), (8, 32, 16, 32, 64, (8.0, 100, 32.0, 1.0)), (5, 20, 6, 28, 100, None), (16, 64, 32, 64, 256, None), (17, 128, 64, 128, 512, None),
+    (3, 16, 8, 24, 40, None), (7, 48, 12, 40, 64, (3.0, 100, 20.0, 1.5)), (5, 20, 6, 28, 100, None), (16, 64, 32, 64, 256, None), (17, 128, 64, 128, 512, None),
     (1, 33, 10, 17, 300, (4.0, 50, 8.0, 0.5)), (2, 40, 64, 72, 128, None), (2, 200, 80, 24, 560, None), (2, 16, 70, 300, 96, None), (40, 8, 2, 8, 24, None),
 ]
 
@@ -482,7 +482,7 @@ def test_many_positions_are_expanded_in_several_linears(decoder, dev):
 
 @pytest.mark.parametrize("f32", [True, False])
 @pytest.mark.parametrize("rows", [1, 2, 5, 16, 40, 300])
-@pytest.mark.parametrize("experts,top,width,ff", [(8, 4, 192, 64), (1, 1, 128, 128), (5, 5, 100, 200), (70, 6, 130, 40), (300, 3, 128, 96), (3, 1, 256, 384)])
+@pytest.mark.parametrize("experts,top,width,ff", [(9, 3, 200, 72), (1, 1, 128, 128), (5, 5, 100, 200), (70, 6, 130, 40), (300, 3, 128, 96), (3, 1, 256, 384)])
 def test_experts(decoder, dev, f32, rows, experts, top, width, ff):
     import torch
     rng = np.random.default_rng(experts + rows)
